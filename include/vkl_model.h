@@ -50,6 +50,20 @@ int vkl_model_create (int dev, const vkl_model_hparams *hp,
  * collected into the maps Model::init takes, the weights are uploaded, and
  * the mapping is released before this returns. */
 int vkl_model_load_gguf (int dev, const char *path_h, vkl_model **out);
+/* A model of any family from a path: a GGUF file, or a folder with config.json
+ * (whose "architecture" picks the class) and model.safetensors.  dtype_h:
+ * "bfloat16" or "float32" (everything in 32-bit) for models that run in either,
+ * NULL for the model's own format; families with a fixed format refuse another
+ * (12, unimplemented).  max_tokens: cache rows of a model whose files name no
+ * context length (0: 4096). */
+int vkl_model_load (int dev, const char *path_h, const char *dtype_h,
+                    size_t max_tokens, vkl_model **out);
+/* The same from a configuration text and tensors in memory (type 30 = BF16;
+ * dim1 = 0: a vector). */
+int vkl_model_create_config (int dev, const char *config_h,
+                             const vkl_tensor_desc *tensors, size_t n_tensors,
+                             const char *dtype_h, size_t max_tokens,
+                             vkl_model **out);
 void vkl_model_destroy (vkl_model *m);
 const char *vkl_model_last_error (const vkl_model *m);
 size_t vkl_model_vocab (const vkl_model *m);
@@ -58,6 +72,18 @@ size_t vkl_model_vocab (const vkl_model *m);
  * (vocab floats) */
 int vkl_model_forward (vkl_model *m, const uint32_t *toks_h, size_t n_toks,
                        size_t offset, float *logits_h);
+/* the same with the logits of the given rows of toks_h (may be none): logits_h
+ * [n_rows, vocab].  Families that give the last row's only refuse others. */
+int vkl_model_forward_rows (vkl_model *m, const uint32_t *toks_h,
+                            size_t n_toks, size_t offset,
+                            const uint32_t *rows_h, size_t n_rows,
+                            float *logits_h);
+size_t vkl_model_context_length (const vkl_model *m);
+/* testing aid for models with an fp32 residual stream: the stream after every
+ * layer run of a pass on the operator chain, n = runs * n_toks * width floats */
+int vkl_model_residual_streams (vkl_model *m, const uint32_t *toks_h,
+                                size_t n_toks, size_t offset, float *out_h,
+                                size_t n);
 /* the greedy loop of app/llama2_infer.cpp:140-218; times in milliseconds */
 int vkl_model_generate_greedy (vkl_model *m, const uint32_t *prompt_h,
                                size_t n_prompt, size_t n_gen,
@@ -116,6 +142,8 @@ int vkl_model_phase_replay (vkl_model *m, int kind, size_t pos, int rounds,
 void vkl_synth_normal_f32 (uint64_t seed, size_t n, float std, float *out_h);
 void vkl_synth_normal_f16 (uint64_t seed, size_t n, float std,
                            uint16_t *out_h);
+void vkl_synth_normal_bf16 (uint64_t seed, size_t n, float std,
+                            uint16_t *out_h);
 /* rows x K matrix of N(0, std) quantised to Q8_0 GGUF blocks */
 void vkl_synth_normal_q8_0 (uint64_t seed, size_t rows, size_t K, float std,
                             uint8_t *out_h);

@@ -1,0 +1,156 @@
+/*
+ * C ABI of decoder stacks whose layers differ from one another (in
+ * libvkllama_hip.so): bf16 weights, an fp32 residual stream, layers with one
+ * norm whose output feeds the token mixer and the feed-forward part in
+ * parallel, and mixers whose values are their keys - attention over shared
+ * key/value rows, and latent attention, where the shared row is the normed
+ * latent of a token.  No counterpart in the reference, which runs Llama-2
+ * blocks only.
+ *
+ * Two number formats (`type` arguments, GGML numbers):
+ *   30 BF16: matrix products and stored activations in bf16 with fp32 sums
+ *    0 F32:  activations, caches and products in true 32-bit
+ * Weights are bf16 in both.  In both, positions, attention scores and weights,
+ * norms, gates and the residual stream are fp32.
+ *
+ * Conventions are those of vkl_hip.h.  Row sizes: a row that a product reads
+ * is padded with zeros to a multiple of 64 values, a head to a multiple of 32.
+ */
+#ifndef VKL_STACK_H
+#define VKL_STACK_H
+#include <stddef.h>
+#include <stdint.h>
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+#define VKL_TYPE_F32 0
+#define VKL_TYPE_BF16 30
+
+/* ---- operators (any number of token rows) -------------------------------- */
+
+/* The output columns of a product fall into segments, each with its own
+ * destination: projections that share an input are one matrix. */
+typedef struct
+{
+  int n0;                /* first column (row of w), a multiple of 8 */
+  int n;                 /* columns written; up to the next segment: padding */
+  void *y;               /* [M, n], row stride ys (elements) */
+  size_t ys;
+  int type;              /* VKL_TYPE_F32 or VKL_TYPE_BF16 */
+  int act;               /* 0 none, 2 the square of relu */
+  const float *residual; /* F32 only, layout of y: y = residual + v */
+  float cap;             /* > 0: y = cap * tanh (v / cap) */
+} vkl_out_seg;
+
+/* y = x W^T, W bf16 [N, K], K % 64 == 0, at most 4 segments.  x bf16: matrix
+ * cores; x fp32: products and sums in 32-bit. */
+int vkl_project_bf16w (const void *x, int xtype, size_t xs, const void *w,
+                       int M, int N, int K, const vkl_out_seg *segs, int nseg,
+                       void *stream);
+/* out[i, :W] = rms_norm (table[toks[i]]) * w (w null: the plain rows), fp32 rows
+ * of stride os; table bf16 [VH, K] of which the first W columns are valid;
+ * ids >= VH read row 0.  Columns W .. os-1 are not written. */
+int vkl_embed_norm_bf16 (const void *table, uint32_t VH, int K, int W,
+                         const uint32_t *toks, uint32_t n, const float *w,
+                         float eps, float *out, size_t os, void *stream);
+/* out[i, :W] = x[r] / sqrt (mean (x[r]^2) + eps) * w for r = rows ? rows[i] : i;
+ * columns W .. Wp-1 of out are set to zero */
+int vkl_rmsnorm_f32 (const float *x, size_t xs, const uint32_t *rows, int n,
+                     int W, const float *w, float eps, void *out, int otype,
+                     size_t os, int Wp, void *stream);
+/* Causal attention of many query rows on the matrix cores, bf16: q [S, H*hd],
+ * k and v [L, G*hd] (they may be the same rows), query head h reads head
+ * h / (H/G); query row s is at position s + L - S and its scores are
+ * q.k * scale * (1 + temp_coef * ln (floor ((p + 1) / temp_every) + 1)); gate:
+ * optional fp32 [S, gs], head h's output times sigmoid (gate[s, h]).  hd a
+ * multiple of 32 up to 256. */
+int vkl_attn_prefill_causal_bf16 (const void *q, const void *k, const void *v,
+                                  int H, int G, int S, int L, int hd,
+                                  size_t qhs, size_t khs, size_t vhs,
+                                  float scale, float temp_coef, int temp_every,
+                                  const float *gate, size_t gs, void *out,
+                                  size_t ors, void *stream);
+/* The same where the values ARE the keys, all sums in fp32, for few query rows
+ * (decode) and for the 32-bit format: q [S, H*dim] and out in qtype / otype,
+ * rows [>= pos0 + S, G*dim] in ctype; query row s is at position pos0 + s.  One
+ * pass over the rows: a row is used for the score and for the output while it
+ * is in registers.  The context is split over workgroups, the last of which
+ * combines the parts (scratch from vkl_attn_rows_scratch_bytes, zeroed once).
+ * dim a multiple of 32 up to 1024. */
+int vkl_attn_rows (const void *q, int qtype, size_t qs, const void *rows,
+                   int ctype, size_t rs, int H, int G, int dim, int S,
+                   uint32_t pos0, float scale, float temp_coef, int temp_every,
+                   void *out, int otype, size_t os, void *scratch,
+                   void *stream);
+size_t vkl_attn_rows_scratch_bytes (int H, int G, int dim, int S);
+/* y[s, h*yh + r] = f * sum_k w[h, r, k] x[s, h*xh + k], w bf16 [H, R, K], f = 1 or
+ * sigmoid (gate[s*gs + h]); K a multiple of 32 */
+int vkl_head_matvec (const void *w, int H, int R, int K, const void *x,
+                     int xtype, size_t xs, size_t xh, void *y, int ytype,
+                     size_t ys, size_t yh, const float *gate, size_t gs, int S,
+                     void *stream);
+
+/* ---- the one-token step ---------------------------------------------------- */
+/* mixers */
+#define VKL_MIX_SHARED_KV 0 /* q.k over rows that are keys and values */
+#define VKL_MIX_LATENT 1    /* q -> W_uk^T q, attention over latents, W_uv */
+
+/* One layer run: a layer that runs several times appears once per run, with
+ * the same weights and a cache of its own. */
+typedef struct
+{
+  int mixer;
+  int H, G;             /* query heads, key/value heads (latent: 1) */
+  int dim, vdim;        /* padded head sizes of queries/keys and values */
+  int rank, rank_p;     /* latent size, padded (latent) */
+  float scale, temp_coef;
+  int temp_every;
+  int ff;               /* feed-forward rows, 0: none */
+  const float *norm;    /* [width_p] */
+  const void *w_in;     /* bf16 [n_in, width_p]: q | k or down-projection | gate | up */
+  int n_in;
+  int kv0, g0, up0;     /* first rows of those parts (multiples of 8); q at 0 */
+  const void *w_out;    /* bf16 [width, k_out]: columns of the heads | feed-forward */
+  int k_out, ff_col;
+  const void *w_ukt;    /* latent: bf16 [H, rank_p, dim] (transposed) */
+  const void *w_uv;     /* latent: bf16 [H, vdim, rank_p] */
+  const float *c_norm;  /* latent: [rank_p] */
+  void *cache;          /* [maxlen, G*dim] or [maxlen, rank_p] */
+} vkl_stack_layer;
+
+typedef struct
+{
+  int width, width_p, vocab, maxlen, n_runs;
+  int ctype;             /* type of the caches */
+  float eps, logit_cap;  /* logit_cap 0: none */
+  const vkl_stack_layer *layers_h; /* HOST array [n_runs] */
+  const void *embed;     /* bf16 [vocab, width_p], also the output matrix */
+  const float *embed_norm, *final_norm; /* [width_p] */
+  void *scratch;         /* vkl_stack_scratch_bytes, zeroed once */
+} vkl_stack_model;
+
+size_t vkl_stack_scratch_bytes (const vkl_stack_model *m);
+/* 1 if the step covers this model (rows of up to 32768 values, sizes padded as
+ * above), else 0; the operators above serve every model */
+int vkl_stack_supported (const vkl_stack_model *m);
+/* One token at position pos: 3 launches per shared-row layer (norm + all
+ * projections; attention; output + feed-forward + residual), 5 per latent one.
+ * Arguments as for vkl_decode_step. */
+int vkl_stack_step (const vkl_stack_model *m, const uint32_t *tok,
+                    uint32_t pos, float *logits32, uint32_t *next_tok,
+                    void *stream);
+/* vkl_decode_loop / vkl_decode_loop_sampled for such a stack */
+int vkl_stack_loop (const vkl_stack_model *m, uint32_t *ids, uint32_t pos0,
+                    int n_steps, float *logits32, void *stream);
+int vkl_stack_loop_sampled (const vkl_stack_model *m, uint32_t *ids,
+                            uint32_t pos0, int n_steps, float *logits32,
+                            int topk, float topp, uint64_t seed, void *stream);
+/* drops the captured step of this model, if there is one */
+void vkl_stack_release (const vkl_stack_model *m);
+
+#ifdef __cplusplus
+}
+#endif
+#endif

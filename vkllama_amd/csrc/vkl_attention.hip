@@ -32,6 +32,12 @@
 // 16t + 8*(j/4) + 4h + j%4 of the block), so the A operand of the second
 // product is one 16-byte LDS read.
 //
+// The element type is a template parameter: fp16 (Llama-2, the score rounded
+// to fp16 as above) or bf16 (scores stay in fp32; weights are rounded once, as
+// the operand of the second product).  Query heads may share key/value heads,
+// the score factor may grow with the query's position, and a head's output may
+// be scaled by the sigmoid of a per-token gate.
+//
 // A second, small kernel in this file prepares the inputs of the first from
 // the projection outputs: RoPE of Q (in place) and K, and the K/V cache write.
 #include "../../include/vkl_hip.h"
@@ -40,6 +46,7 @@
 namespace
 {
 typedef _Float16 half8 __attribute__ ((ext_vector_type (8)));
+typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
 typedef float float16v __attribute__ ((ext_vector_type (16)));
 typedef uint32_t u32x2 __attribute__ ((ext_vector_type (2)));
 
@@ -55,6 +62,46 @@ struct AttnArgs
   int H, S, L, ntq;
   size_t qcs, qhs, kcs, khs, vcs, vhs, ors, ohs;
   float scale;
+  int rep;            // query heads per key/value head
+  float temp_coef;    // != 0: scale times 1 + coef ln (floor ((pos + 1) / every) + 1)
+  int temp_every;
+  const float *gate;  // optional [S, gs]: head h's output times sigmoid (gate[s, h])
+  size_t gs;
+};
+
+// the two element types of the operands
+struct F16Elem
+{
+  typedef half8 v8;
+  static constexpr bool round_scores = true;
+  static __device__ __forceinline__ float16v
+  mfma (v8 a, v8 b, float16v c)
+  {
+    return __builtin_amdgcn_mfma_f32_32x32x16_f16 (a, b, c, 0, 0, 0);
+  }
+  static __device__ __forceinline__ uint16_t
+  bits (float f)
+  {
+    return vkl::f2h (f);
+  }
+  typedef _Float16 t;
+};
+
+struct Bf16Elem
+{
+  typedef bf8 v8;
+  static constexpr bool round_scores = false;
+  static __device__ __forceinline__ float16v
+  mfma (v8 a, v8 b, float16v c)
+  {
+    return __builtin_amdgcn_mfma_f32_32x32x16_bf16 (a, b, c, 0, 0, 0);
+  }
+  static __device__ __forceinline__ uint16_t
+  bits (float f)
+  {
+    return vkl::f2bf (f);
+  }
+  typedef __bf16 t;
 };
 
 __device__ __align__ (16) const uint32_t g_zero16[4] = { 0, 0, 0, 0 };
@@ -65,17 +112,15 @@ fast_exp (float x)
   return __builtin_amdgcn_exp2f (x * 1.44269504088896340736f);
 }
 
-__device__ __forceinline__ half8
-as_half8 (const uint4 v)
-{
-  return __builtin_bit_cast (half8, v);
-}
 
 template <int HD> struct Tile
 {
   static constexpr int CPR = HD / 8;                       // 16-byte chunks per row
-  static constexpr int KCH = kBKey * CPR / kThreads;       // K chunks per thread
-  static constexpr int VIT = (kBKey / 2) * CPR / kThreads; // (key pair, chunk) items per thread
+  static constexpr int KALL = kBKey * CPR, VALL = (kBKey / 2) * CPR;
+  static constexpr int KCH = (KALL + kThreads - 1) / kThreads; // K chunks per thread
+  static constexpr int VIT = (VALL + kThreads - 1) / kThreads; // (key pair, chunk) items per thread
+  // item numbers past the last exist where the tile is not a multiple of the workgroup
+  static constexpr bool KRAG = KALL % kThreads != 0, VRAG = VALL % kThreads != 0;
   uint4 k[KCH];
   uint4 v[VIT][2];
 };
@@ -92,7 +137,7 @@ load_k (const AttnArgs &a, const uint16_t *kb, int t, Tile<HD> &r)
     {
       const int c = threadIdx.x + i * kThreads;
       const int row = t * kBKey + c / CPR;
-      r.k[i] = vkl::ldg4 (row < a.L ? (const void *)(kb + (size_t)row * a.khs + (c % CPR) * 8)
+      r.k[i] = vkl::ldg4 (row < a.L && (!Tile<HD>::KRAG || c < Tile<HD>::KALL) ? (const void *)(kb + (size_t)row * a.khs + (c % CPR) * 8)
                                     : zeros);
     }
 }
@@ -117,8 +162,9 @@ load_v (const AttnArgs &a, const uint16_t *vb, int t, Tile<HD> &r)
       const int pair = it & 31, dc = it >> 5;
       // slots 2*pair and 2*pair+1 hold two adjacent keys
       const int row = t * kBKey + slot_key (2 * pair);
-      r.v[i][0] = vkl::ldg4 (row < a.L ? (const void *)(vb + (size_t)row * a.vhs + dc * 8) : zeros);
-      r.v[i][1] = vkl::ldg4 (row + 1 < a.L ? (const void *)(vb + (size_t)(row + 1) * a.vhs + dc * 8)
+      const bool in = !Tile<HD>::VRAG || it < Tile<HD>::VALL;
+      r.v[i][0] = vkl::ldg4 (row < a.L && in ? (const void *)(vb + (size_t)row * a.vhs + dc * 8) : zeros);
+      r.v[i][1] = vkl::ldg4 (row + 1 < a.L && in ? (const void *)(vb + (size_t)(row + 1) * a.vhs + dc * 8)
                                            : zeros);
     }
 }
@@ -132,6 +178,8 @@ store_k (const Tile<HD> &r, uint16_t *Ks)
   for (int i = 0; i < Tile<HD>::KCH; ++i)
     {
       const int c = threadIdx.x + i * kThreads;
+      if (Tile<HD>::KRAG && c >= Tile<HD>::KALL)
+        continue;
       *(uint4 *)(Ks + (c / CPR) * LDK + (c % CPR) * 8) = r.k[i];
     }
 }
@@ -148,6 +196,8 @@ store_v (const Tile<HD> &r, uint16_t *Vt)
     {
       const int it = threadIdx.x + i * kThreads;
       const int pair = it & 31, dc = it >> 5;
+      if (Tile<HD>::VRAG && it >= Tile<HD>::VALL)
+        continue;
       const uint32_t va[4] = { r.v[i][0].x, r.v[i][0].y, r.v[i][0].z, r.v[i][0].w };
       const uint32_t vb[4] = { r.v[i][1].x, r.v[i][1].y, r.v[i][1].z, r.v[i][1].w };
       uint32_t *dst = (uint32_t *)(Vt + (size_t)(dc * 8) * LDV + 2 * pair);
@@ -161,9 +211,9 @@ store_v (const Tile<HD> &r, uint16_t *Vt)
 }
 
 // S^T of one 32-key block: rows = keys 32*blk .. +31 of the tile in LDS
-template <int HD>
+template <int HD, class E>
 __device__ __forceinline__ float16v
-score_block (const uint16_t *Ks, int blk, const half8 (&qf)[HD / 16], int lane)
+score_block (const uint16_t *Ks, int blk, const typename E::v8 (&qf)[HD / 16], int lane)
 {
   constexpr int LDK = HD + 8;
   float16v acc;
@@ -173,15 +223,16 @@ score_block (const uint16_t *Ks, int blk, const half8 (&qf)[HD / 16], int lane)
   const uint16_t *kp = Ks + (32 * blk + (lane & 31)) * LDK + (lane >> 5) * 8;
 #pragma unroll
   for (int kt = 0; kt < HD / 16; ++kt)
-    acc = __builtin_amdgcn_mfma_f32_32x32x16_f16 (*(const half8 *)(kp + kt * 16), qf[kt], acc,
-                                                  0, 0, 0);
+    acc = E::mfma (*(const typename E::v8 *)(kp + kt * 16), qf[kt], acc);
   return acc;
 }
 
-template <int HD>
-__global__ __launch_bounds__ (kThreads, 2) void
+// (heads wider than 128 values: one workgroup per compute unit, twice the registers)
+template <int HD, class E>
+__global__ __launch_bounds__ (kThreads, HD <= 128 ? 2 : 1) void
 attn_prefill_kernel (const AttnArgs a)
 {
+  typedef typename E::v8 v8;
   constexpr int KT = HD / 16, DB = HD / 32;
   constexpr int LDK = HD + 8, LDV = kBKey + 8;
   __shared__ __align__ (16) uint16_t Ks[kBKey * LDK];
@@ -215,15 +266,20 @@ attn_prefill_kernel (const AttnArgs a)
   const int kmax = min (a.L, q0 + kBQ + shift);
   const int ntile = (kmax + kBKey - 1) / kBKey;
   const int wave_last = q0 + wave * 32 + 31 + shift; // last key any query of the wave sees
-  const uint16_t *kb = a.k + (size_t)head * a.kcs;
-  const uint16_t *vb = a.v + (size_t)head * a.vcs;
+  const int kvh = E::round_scores ? head : head / a.rep;
+  const uint16_t *kb = a.k + (size_t)kvh * a.kcs;
+  const uint16_t *vb = a.v + (size_t)kvh * a.vcs;
+  // this query's score factor
+  float scale = a.scale;
+  if (!E::round_scores && a.temp_coef != 0.f)
+    scale *= 1.0f + a.temp_coef * logf ((float)((qrow + shift + 1) / a.temp_every + 1));
 
-  half8 qf[KT];
+  v8 qf[KT];
   {
     const uint16_t *qp = a.q + (size_t)head * a.qcs + (size_t)min (qrow, a.S - 1) * a.qhs + hh * 8;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt)
-      qf[kt] = as_half8 (vkl::ldg4 (qp + kt * 16));
+      qf[kt] = __builtin_bit_cast (v8, vkl::ldg4 (qp + kt * 16));
   }
 
   Tile<HD> tl;
@@ -260,13 +316,13 @@ attn_prefill_kernel (const AttnArgs a)
 #pragma unroll
       for (int blk = 0; blk < 2; ++blk)
         {
-          const float16v acc = score_block<HD> (Ks, blk, qf, lane);
+          const float16v acc = score_block<HD, E> (Ks, blk, qf, lane);
           const int key0 = t * kBKey + 32 * blk + 4 * hh;
 #pragma unroll
           for (int r = 0; r < 16; ++r)
             {
               const int key = key0 + 8 * (r >> 2) + (r & 3);
-              const float sc = vkl::h2f (vkl::f2h (acc[r] * a.scale));
+              const float sc = E::round_scores ? vkl::h2f (vkl::f2h (acc[r] * scale)) : acc[r] * scale;
               sv[blk][r] = inner || key <= qrow + shift ? sc : kNeg;
               bm = fmaxf (bm, sv[blk][r]);
             }
@@ -286,7 +342,7 @@ attn_prefill_kernel (const AttnArgs a)
               oacc[db][r] *= alpha;
           m = mn;
         }
-      half8 pf[2][2];
+      v8 pf[2][2];
 #pragma unroll
       for (int blk = 0; blk < 2; ++blk)
 #pragma unroll
@@ -295,7 +351,7 @@ attn_prefill_kernel (const AttnArgs a)
             // exp (kNeg - m) = 0.  The sum takes the weight as the product
             // below consumes it, rounded to fp16: the weights then add up to
             // one exactly.
-            const _Float16 e = (_Float16)fast_exp (sv[blk][r] - m);
+            const typename E::t e = (typename E::t)fast_exp (sv[blk][r] - m);
             sum += (float)e;
             pf[blk][r >> 3][r & 7] = e;
           }
@@ -307,13 +363,14 @@ attn_prefill_kernel (const AttnArgs a)
           for (int blk = 0; blk < 2; ++blk)
 #pragma unroll
             for (int t2 = 0; t2 < 2; ++t2)
-              oacc[db] = __builtin_amdgcn_mfma_f32_32x32x16_f16 (
-                  *(const half8 *)(vp + 32 * blk + 16 * t2), pf[blk][t2], oacc[db], 0, 0, 0);
+              oacc[db] = E::mfma (*(const v8 *)(vp + 32 * blk + 16 * t2), pf[blk][t2], oacc[db]);
         }
     }
   // the other half of the lanes has summed the other keys of the same query
   sum += __shfl_xor (sum, 32, 64);
-  const float inv = 1.0f / sum;
+  float inv = 1.0f / sum;
+  if (!E::round_scores && a.gate)
+    inv = inv / (1.0f + expf (-vkl::ldg (a.gate + (size_t)min (qrow, a.S - 1) * a.gs + head)));
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -330,9 +387,9 @@ attn_prefill_kernel (const AttnArgs a)
       {
         const int d = 32 * db + 8 * g + 4 * hh;
         u32x2 w;
-        w.x = (uint32_t)vkl::f2h (oacc[db][4 * g]) | ((uint32_t)vkl::f2h (oacc[db][4 * g + 1]) << 16);
-        w.y = (uint32_t)vkl::f2h (oacc[db][4 * g + 2])
-              | ((uint32_t)vkl::f2h (oacc[db][4 * g + 3]) << 16);
+        w.x = (uint32_t)E::bits (oacc[db][4 * g]) | ((uint32_t)E::bits (oacc[db][4 * g + 1]) << 16);
+        w.y = (uint32_t)E::bits (oacc[db][4 * g + 2])
+              | ((uint32_t)E::bits (oacc[db][4 * g + 3]) << 16);
         *(VKL_GLOBAL u32x2 *)(op + d) = w;
       }
 }
@@ -449,7 +506,8 @@ vkl_attn_prefill_causal_f16 (const void *q, const void *k, const void *v,
                  && ((uintptr_t)out % 8) == 0);
   VKL_CHECK_ARG ((qcs % 8) == 0 && (qhs % 8) == 0 && (kcs % 8) == 0 && (khs % 8) == 0
                  && (vcs % 8) == 0 && (vhs % 8) == 0 && (ors % 4) == 0 && (ohs % 4) == 0);
-  AttnArgs a;
+  AttnArgs a = {};
+  a.rep = 1;
   a.q = (const uint16_t *)q, a.k = (const uint16_t *)k, a.v = (const uint16_t *)v;
   a.out = (uint16_t *)out;
   a.H = H, a.S = S, a.L = L, a.ntq = (S + kBQ - 1) / kBQ;
@@ -457,8 +515,47 @@ vkl_attn_prefill_causal_f16 (const void *q, const void *k, const void *v,
   a.ors = ors, a.ohs = ohs, a.scale = scale;
   const dim3 grid ((unsigned)(a.ntq * H));
   if (hd == 128)
-    attn_prefill_kernel<128><<<grid, dim3 (kThreads), 0, (hipStream_t)stream>>> (a);
+    attn_prefill_kernel<128, F16Elem><<<grid, dim3 (kThreads), 0, (hipStream_t)stream>>> (a);
   else
-    attn_prefill_kernel<64><<<grid, dim3 (kThreads), 0, (hipStream_t)stream>>> (a);
+    attn_prefill_kernel<64, F16Elem><<<grid, dim3 (kThreads), 0, (hipStream_t)stream>>> (a);
+  return vkl_launch_status ();
+}
+
+extern "C" int
+vkl_attn_prefill_causal_bf16 (const void *q, const void *k, const void *v, int H, int G, int S, int L, int hd,
+                              size_t qhs, size_t khs, size_t vhs, float scale, float temp_coef,
+                              int temp_every, const float *gate, size_t gs, void *out, size_t ors,
+                              void *stream)
+{
+  VKL_CHECK_ARG (q && k && v && out);
+  VKL_CHECK_ARG (H > 0 && G > 0 && (H % G) == 0 && S > 0 && L >= S);
+  VKL_CHECK_ARG (hd > 0 && (hd % 32) == 0 && hd <= 256);
+  VKL_CHECK_ARG (temp_coef == 0.f || temp_every > 0);
+  VKL_CHECK_ARG (((uintptr_t)q % 16) == 0 && ((uintptr_t)k % 16) == 0 && ((uintptr_t)v % 16) == 0
+                 && ((uintptr_t)out % 8) == 0);
+  VKL_CHECK_ARG ((qhs % 8) == 0 && (khs % 8) == 0 && (vhs % 8) == 0 && (ors % 4) == 0);
+  VKL_CHECK_ARG (qhs >= (size_t)H * hd && khs >= (size_t)G * hd && vhs >= (size_t)G * hd
+                 && ors >= (size_t)H * hd && (!gate || gs >= (size_t)H));
+  AttnArgs a = {};
+  a.q = (const uint16_t *)q, a.k = (const uint16_t *)k, a.v = (const uint16_t *)v;
+  a.out = (uint16_t *)out;
+  a.H = H, a.S = S, a.L = L, a.ntq = (S + kBQ - 1) / kBQ;
+  a.qcs = a.kcs = a.vcs = a.ohs = (size_t)hd;
+  a.qhs = qhs, a.khs = khs, a.vhs = vhs, a.ors = ors;
+  a.scale = scale, a.rep = H / G, a.temp_coef = temp_coef, a.temp_every = temp_every;
+  a.gate = gate, a.gs = gs;
+  const dim3 grid ((unsigned)(a.ntq * H)), block (kThreads);
+  hipStream_t s = (hipStream_t)stream;
+  switch (hd)
+    {
+    case 32: attn_prefill_kernel<32, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 64: attn_prefill_kernel<64, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 96: attn_prefill_kernel<96, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 128: attn_prefill_kernel<128, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 160: attn_prefill_kernel<160, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 192: attn_prefill_kernel<192, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    case 224: attn_prefill_kernel<224, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    default: attn_prefill_kernel<256, Bf16Elem><<<grid, block, 0, s>>> (a); break;
+    }
   return vkl_launch_status ();
 }

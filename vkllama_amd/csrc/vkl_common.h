@@ -179,6 +179,19 @@ f2h (float f)
   return __builtin_bit_cast (uint16_t, (h16)f); // v_cvt_f16_f32: RNE
 }
 
+// bf16: the upper half of a float, rounded to nearest even on the way down
+__device__ __forceinline__ float
+bf2f (uint16_t bits)
+{
+  return __uint_as_float ((uint32_t)bits << 16);
+}
+
+__device__ __forceinline__ uint16_t
+f2bf (float f)
+{
+  return __builtin_bit_cast (uint16_t, (__bf16)f);
+}
+
 __device__ __forceinline__ float
 silu (float v)
 {

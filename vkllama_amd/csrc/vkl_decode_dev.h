@@ -37,5 +37,11 @@ st_coherent_u32 (uint32_t *p, uint32_t v)
 {
   __hip_atomic_store (p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
+
+// vkl_sample.hip: the draw that ends a step of a replayed loop; dev_params =
+// {k, bits of p, seed low, seed high} in device memory, loop = {index,
+// position}: writes ids[index + 1] and advances both loop words
+int sample_loop_launch (const float *logits, int V, const uint32_t *dev_params, uint32_t *loop,
+                        uint32_t *ids, hipStream_t s);
 } // namespace vkl
 #endif

@@ -574,10 +574,5 @@ int launch_layer (const Params &p, const vkl_layer_weights &lw, int layer, int G
 // the token's embedding row -> residual stream (one small launch in front of layer 0)
 int launch_embed_row (const Params &p, hipStream_t s);
 } // namespace dec
-// vkl_sample.hip: the draw that ends a step of a replayed loop; dev_params =
-// {k, bits of p, seed low, seed high} in device memory, loop = {index,
-// position}: writes ids[index + 1] and advances both loop words
-int sample_loop_launch (const float *logits, int V, const uint32_t *dev_params, uint32_t *loop,
-                        uint32_t *ids, hipStream_t s);
 } // namespace vkl
 #endif

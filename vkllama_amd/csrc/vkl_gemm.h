@@ -37,6 +37,35 @@ struct GemmArgs
   size_t workspace_bytes; // size of `workspace` (checked before every use)
 };
 
+// A product whose output columns fall into segments, each with a destination, a
+// type, an activation and possibly a residual of its own: the projections that
+// share one input (queries, keys, gates, the feed-forward part of a parallel
+// layer) are one matrix, and so are those that add into one residual row.
+// bf16 weights; x in bf16 (matrix cores' bf16 products) or fp32 (products in
+// true 32-bit).  K is a multiple of 64 (columns beyond the valid ones hold
+// zeros on both sides); segments start at multiples of 8.
+constexpr int kGemmSegs = 4;
+struct GemmSeg
+{
+  int n0, n;             // first column, columns that are written
+  void *y;               // [M, n], row stride ys
+  size_t ys;
+  int f32;               // y in fp32, else bf16
+  int act;               // 0 none, 2 the square of relu
+  const float *residual; // fp32 y only: y = residual + v
+  float cap;             // > 0: cap * tanh (v / cap)
+  int vec;               // rows of y allow vector stores
+};
+struct GemmSegArgs : GemmArgs
+{
+  const float *xf; // fp32 x (x is null then)
+  int nseg;
+  GemmSeg seg[kGemmSegs];
+};
+// the fp32 product (vkl_gemm_f32.hip) and the bf16 one (vkl_gemm_wide.hip)
+int gemm_f32_launch (const GemmSegArgs &a, hipStream_t s);
+int gemm_wide_bf16_launch (const GemmSegArgs &a, hipStream_t s);
+
 // smallest M for which the matrix-core kernels beat one weight-streaming pass
 // per token row (measured on the 7B shapes): Q8_0 weights, fp16 weights, and
 // batched fp16 products (one small matrix per head)

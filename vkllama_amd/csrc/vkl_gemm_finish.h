@@ -98,5 +98,99 @@ gemm_finish8 (const GemmArgs &a, float (&v)[8], const float (&g)[8], int m, int 
         y32[e] = h2f (he);
     }
 }
+// The value that a segment stores for a sum
+__device__ __forceinline__ float
+seg_value (const GemmSeg &sg, float v)
+{
+  if (sg.act == 2)
+    {
+      v = fmaxf (v, 0.f);
+      v = v * v;
+    }
+  if (sg.cap > 0.f)
+    v = sg.cap * tanhf (v / sg.cap);
+  return v;
+}
+
+// The same for a product with segments: v the sums of row m from column ncol0
+// (a multiple of 8) on; segments start at multiples of 8, so all eight columns
+// belong to one.
+template <bool UPGATE>
+__device__ __forceinline__ void
+gemm_finish8 (const GemmSegArgs &a, float (&v)[8], const float (&)[8], int m, int ncol0, int, int, float *part)
+{
+  typedef float f32x4 __attribute__ ((ext_vector_type (4)));
+  if (m >= a.M || ncol0 >= a.N)
+    return;
+  if (part)
+    {
+      // (N is a multiple of 8 here or the tail is written one by one)
+      float *dst = part + (size_t)m * a.N + ncol0;
+      if ((a.N % 8) == 0)
+        {
+          f32x4 w0 = { v[0], v[1], v[2], v[3] }, w1 = { v[4], v[5], v[6], v[7] };
+          *(VKL_GLOBAL f32x4 *)dst = w0;
+          *(VKL_GLOBAL f32x4 *)(dst + 4) = w1;
+        }
+      else
+        for (int e = 0; e < 8 && ncol0 + e < a.N; ++e)
+          dst[e] = v[e];
+      return;
+    }
+  int si = 0;
+#pragma unroll
+  for (int i = 1; i < kGemmSegs; ++i)
+    if (i < a.nseg && ncol0 >= a.seg[i].n0)
+      si = i;
+#pragma unroll
+  for (int i = 0; i < kGemmSegs; ++i)
+    {
+      if (i != si)
+        continue;
+      const GemmSeg &sg = a.seg[i];
+      const int c = ncol0 - sg.n0;
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        v[e] = seg_value (sg, v[e]);
+      const bool whole = sg.vec && c + 8 <= sg.n;
+      if (sg.f32)
+        {
+          float *y = (float *)sg.y + (size_t)m * sg.ys + c;
+          const float *r = sg.residual ? sg.residual + (size_t)m * sg.ys + c : nullptr;
+          if (whole)
+            {
+              f32x4 w0 = { v[0], v[1], v[2], v[3] }, w1 = { v[4], v[5], v[6], v[7] };
+              if (r)
+                {
+                  w0 += *(const VKL_GLOBAL f32x4 *)r;
+                  w1 += *(const VKL_GLOBAL f32x4 *)(r + 4);
+                }
+              *(VKL_GLOBAL f32x4 *)y = w0;
+              *(VKL_GLOBAL f32x4 *)(y + 4) = w1;
+            }
+          else
+            for (int e = 0; e < 8 && c + e < sg.n; ++e)
+              y[e] = r ? r[e] + v[e] : v[e];
+        }
+      else
+        {
+          uint16_t *y = (uint16_t *)sg.y + (size_t)m * sg.ys + c;
+          uint16_t h[8];
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            h[e] = f2bf (v[e]);
+          if (whole)
+            {
+              vkl_u32x4 pk;
+              pk.x = h[0] | ((uint32_t)h[1] << 16), pk.y = h[2] | ((uint32_t)h[3] << 16);
+              pk.z = h[4] | ((uint32_t)h[5] << 16), pk.w = h[6] | ((uint32_t)h[7] << 16);
+              *(VKL_GLOBAL vkl_u32x4 *)y = pk;
+            }
+          else
+            for (int e = 0; e < 8 && c + e < sg.n; ++e)
+              y[e] = h[e];
+        }
+    }
+}
 } // namespace vkl
 #endif

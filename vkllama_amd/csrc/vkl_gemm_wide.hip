@@ -23,6 +23,7 @@
 // Measured on the 7B shapes at 2048 rows: matrix cores busy 63 % of the cycles
 // (the tile kernel of vkl_gemm_mfma.hip, which stages through registers:
 // 30-39 %).
+#include "../../include/vkl_stack.h"
 #include "vkl_common.h"
 #include "vkl_gemm.h"
 #include "vkl_gemm_finish.h"
@@ -32,6 +33,7 @@ namespace vkl
 namespace
 {
 typedef _Float16 half8 __attribute__ ((ext_vector_type (8)));
+typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
 typedef float float16v __attribute__ ((ext_vector_type (16)));
 #define VKL_LDS __attribute__ ((address_space (3)))
 
@@ -41,6 +43,27 @@ constexpr int WWAVES = 4;                       // 2 x 2
 constexpr int WTN = WBN / 2 / 32;
 constexpr int WROWB = WBK * 2;                  // bytes of a tile row
 
+
+// element type of the dense kernel by its argument block: fp16 for the products
+// with one plain epilogue, bf16 for those with segments
+template <class Args> struct WideElem
+{
+  typedef half8 v8;
+  static __device__ __forceinline__ float16v
+  mfma (v8 a, v8 b, float16v c)
+  {
+    return __builtin_amdgcn_mfma_f32_32x32x16_f16 (a, b, c, 0, 0, 0);
+  }
+};
+template <> struct WideElem<GemmSegArgs>
+{
+  typedef bf8 v8;
+  static __device__ __forceinline__ float16v
+  mfma (v8 a, v8 b, float16v c)
+  {
+    return __builtin_amdgcn_mfma_f32_32x32x16_bf16 (a, b, c, 0, 0, 0);
+  }
+};
 
 // Issue order of one quarter of a k-step: after product Q one fragment read
 // (the first NR products) and an even share of the quarter's LQ loads.
@@ -73,9 +96,9 @@ template <int V> struct WideInt
 // l%32 of its 32 x 32 block.
 constexpr int kWideParkLd = 68; // floats per parked row: 16-byte aligned, rows 4 banks apart
 
-template <bool UPGATE, int TM>
+template <bool UPGATE, int TM, class Args>
 __device__ __forceinline__ void
-wide_epilogue (const GemmArgs &a, const float16v (&acc)[TM][WTN], uint8_t *wide_lds, int wave, int lane,
+wide_epilogue (const Args &a, const float16v (&acc)[TM][WTN], uint8_t *wide_lds, int wave, int lane,
                int m0, int n0, int zmat, int vec, float *part)
 {
   // waves are numbered row block first: wave = 2 wm + wn, TM x 32 rows by 64 columns each
@@ -169,10 +192,11 @@ wide_lds_f16 ()
 
 // BM: token rows of a tile, 256 or (where 256-row tiles would be too few to
 // occupy the compute units) 128, i.e. 64 x 64 per wave.
-template <int BM, bool UPGATE>
+template <int BM, bool UPGATE, class Args = GemmArgs>
 __global__ __launch_bounds__ (WWAVES * 64) void
-gemm_wide_f16_kernel (const GemmArgs a, int tiles_m, int tiles_n, int per_xcd, int vec, int ksplit, float *ws)
+gemm_wide_f16_kernel (const Args a, int tiles_m, int tiles_n, int per_xcd, int vec, int ksplit, float *ws)
 {
+  typedef typename WideElem<Args>::v8 v8;
   constexpr int TM = BM / 2 / 32;                    // 32-row accumulators per wave
   constexpr int STAGE_BYTES = (BM + WBN) * WROWB;
   constexpr int GPW = (BM + WBN) / 8 / WWAVES;       // 1 KiB load instructions per wave and k-step
@@ -258,17 +282,17 @@ gemm_wide_f16_kernel (const GemmArgs a, int tiles_m, int tiles_n, int per_xcd, i
   for (int p = 0; p < WSTAGES - 1; ++p)
     issue_part (p < nk ? p : nk - 1, p, 0, GPW);
 
-  half8 af[2][TM], bf[2][WTN];
+  v8 af[2][TM], bf[2][WTN];
   // in the order the products need them
   auto read_frags = [&] (int st, int ks, int buf) {
     const uint8_t *sb = wide_lds + st * STAGE_BYTES;
-    af[buf][0] = *(const half8 *)(sb + aoff[ks]);
+    af[buf][0] = *(const v8 *)(sb + aoff[ks]);
 #pragma unroll
     for (int jn = 0; jn < WTN; ++jn)
-      bf[buf][jn] = *(const half8 *)(sb + boff[ks] + jn * BJ);
+      bf[buf][jn] = *(const v8 *)(sb + boff[ks] + jn * BJ);
 #pragma unroll
     for (int i = 1; i < TM; ++i)
-      af[buf][i] = *(const half8 *)(sb + aoff[ks] + i * 32 * WROWB);
+      af[buf][i] = *(const v8 *)(sb + aoff[ks] + i * 32 * WROWB);
   };
   // s_waitcnt immediates: vmcnt = the loads of the newest k-step may stay in
   // flight; the second one also waits for the wave's own LDS reads
@@ -306,7 +330,7 @@ gemm_wide_f16_kernel (const GemmArgs a, int tiles_m, int tiles_n, int per_xcd, i
         for (int i = 0; i < TM; ++i)
 #pragma unroll
           for (int jn = 0; jn < WTN; ++jn)
-            acc[i][jn] = __builtin_amdgcn_mfma_f32_32x32x16_f16 (af[ks & 1][i], bf[ks & 1][jn], acc[i][jn], 0, 0, 0);
+            acc[i][jn] = WideElem<Args>::mfma (af[ks & 1][i], bf[ks & 1][jn], acc[i][jn]);
         if (ks == 0)
           WideOrder<0, NP, NR, LB1>::run ();
         else if (ks == 1)
@@ -762,4 +786,124 @@ gemm_wide_launch (const GemmArgs &a, hipStream_t s)
     return gemm_reduce_parts (a, ws, ksplit, a.M, s);
   return (int)hipGetLastError ();
 }
+
+// ---------------------------------------------------------------------------
+// bf16 operands, output columns in segments
+// ---------------------------------------------------------------------------
+namespace
+{
+// adds the parts of a split k range in order and applies the segments' epilogue
+__global__ __launch_bounds__ (256) void
+wide_reduce_seg_kernel (const GemmSegArgs a, const float *ws, int parts)
+{
+  const int n8 = (a.N + 7) / 8;
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (size_t)a.M * n8)
+    return;
+  const int m = (int)(i / n8), n = (int)(i % n8) * 8;
+  float v[8], g[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+    v[e] = 0.f, g[e] = 0.f;
+  for (int p = 0; p < parts; ++p)
+    {
+      const float *src = ws + ((size_t)p * a.M + m) * a.N;
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        v[e] += ldg (src + min (n + e, a.N - 1));
+    }
+  gemm_finish8<false> (a, v, g, m, n, 0, 0, nullptr);
+}
+
+// As wide_plan (the same cost model; it holds for bf16), with every row count
+// allowed and, where the tiles are few, up to 16 parts of at least 4 k-steps:
+// with few token rows the workgroups exist to stream the weights.
+WidePlan
+wide_plan_bf16 (const GemmSegArgs &a)
+{
+  WidePlan best = { 0, 1 };
+  double best_cost = 0;
+  const int nk = a.K / WBK;
+  for (int bm = 128; bm <= WBM; bm *= 2)
+    for (int ks = 1; ks <= 16; ks *= 2)
+      {
+        if (a.M < bm && bm > 128)
+          continue;
+        if (ks > 1
+            && (nk / ks < 4 || (size_t)ks * a.M * a.N * sizeof (float) > gemm_stream_workspace_bytes ()))
+          continue;
+        const long groups = (long)((a.M + bm - 1) / bm) * ((a.N + WBN - 1) / WBN) * ks;
+        const double round = (bm == WBM ? 0.95 : 0.55) * nk / ks + (bm == WBM ? 8 : 6);
+        const double reduce = ks > 1 ? 5 + (double)ks * a.M * a.N * sizeof (float) / 2.5e6 : 0;
+        const double cost = (double)((groups + 255) / 256) * round + reduce;
+        if (!best.bm || cost < best_cost)
+          best = { bm, ks }, best_cost = cost;
+      }
+  return best;
+}
+
+template <int BM>
+int
+launch_wide_bf16 (const GemmSegArgs &a, int ksplit, hipStream_t s)
+{
+  static LdsLimit limit;
+  constexpr size_t lds = wide_lds_f16<BM> ();
+  const auto kernel = gemm_wide_f16_kernel<BM, false, GemmSegArgs>;
+  if (int e = limit.raise ((const void *)kernel, lds))
+    return e;
+  float *ws = nullptr;
+  if (ksplit > 1 && !(ws = gemm_stream_workspace (s)))
+    ksplit = 1;
+  const int tiles_m = (a.M + BM - 1) / BM, tiles_n = (a.N + WBN - 1) / WBN;
+  const int per_xcd = (tiles_m * tiles_n * ksplit + 7) / 8;
+  kernel<<<dim3 ((unsigned)(per_xcd * 8)), dim3 (WWAVES * 64), lds, s>>> (a, tiles_m, tiles_n, per_xcd, 1, ksplit, ws);
+  if (ksplit > 1)
+    {
+      const size_t total = (size_t)a.M * ((a.N + 7) / 8);
+      wide_reduce_seg_kernel<<<dim3 ((unsigned)((total + 255) / 256)), dim3 (256), 0, s>>> (a, ws, ksplit);
+    }
+  return (int)hipGetLastError ();
+}
+} // namespace
+
+int
+gemm_wide_bf16_launch (const GemmSegArgs &a, hipStream_t s)
+{
+  const WidePlan p = wide_plan_bf16 (a);
+  return p.bm == WBM ? launch_wide_bf16<WBM> (a, p.ksplit, s) : launch_wide_bf16<128> (a, p.ksplit, s);
+}
 } // namespace vkl
+
+extern "C" int
+vkl_project_bf16w (const void *x, int xtype, size_t xs, const void *w, int M, int N, int K,
+                   const vkl_out_seg *segs, int nseg, void *stream)
+{
+  VKL_CHECK_ARG (x && w && segs && M > 0 && N > 0 && K > 0 && (K % 64) == 0 && xs >= (size_t)K);
+  VKL_CHECK_ARG (nseg > 0 && nseg <= vkl::kGemmSegs && (xtype == VKL_TYPE_F32 || xtype == VKL_TYPE_BF16));
+  VKL_CHECK_ARG ((xs % 8) == 0 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0);
+  vkl::GemmSegArgs a = {};
+  if (xtype == VKL_TYPE_F32)
+    a.xf = (const float *)x;
+  else
+    a.x = (const uint16_t *)x;
+  a.xs = xs, a.M = M, a.N = N, a.K = K, a.Kp = K, a.wtype = 1, a.batch = 1, a.nmat = 1, a.scale = 1.f;
+  a.wh[0] = a.wh[1] = a.wh[2] = (const uint16_t *)w;
+  a.ws = (size_t)K;
+  a.nseg = nseg;
+  int end = 0;
+  for (int i = 0; i < nseg; ++i)
+    {
+      const vkl_out_seg &o = segs[i];
+      VKL_CHECK_ARG (o.y && o.n > 0 && o.n0 >= end && (o.n0 % 8) == 0 && o.n0 + o.n <= N && o.ys >= (size_t)o.n);
+      VKL_CHECK_ARG (i > 0 || o.n0 == 0);
+      VKL_CHECK_ARG (o.act == 0 || o.act == 2);
+      VKL_CHECK_ARG (o.type == VKL_TYPE_F32 || (o.type == VKL_TYPE_BF16 && !o.residual));
+      vkl::GemmSeg &g = a.seg[i];
+      g.n0 = o.n0, g.n = o.n, g.y = o.y, g.ys = o.ys, g.f32 = o.type == VKL_TYPE_F32;
+      g.act = o.act, g.residual = o.residual, g.cap = o.cap;
+      g.vec = (o.ys % 8) == 0 && ((uintptr_t)o.y % 16) == 0 && (!o.residual || ((uintptr_t)o.residual % 16) == 0);
+      end = o.n0 + o.n;
+    }
+  return xtype == VKL_TYPE_F32 ? vkl::gemm_f32_launch (a, (hipStream_t)stream)
+                               : vkl::gemm_wide_bf16_launch (a, (hipStream_t)stream);
+}

@@ -1,0 +1,1443 @@
+// Operators and the one-token step of decoder stacks with bf16 weights, an
+// fp32 residual stream and mixers whose values are their keys
+// (include/vkl_stack.h).
+//
+// The step of one token streams every weight once, so its kernels are built
+// like those of vkl_decode.hip: workgroups of 8 waves, two per compute unit,
+// every wave over whole weight rows with two 8 KiB items in flight, the
+// activation row normed and staged in LDS while the first weights travel.
+// Activations are fp32 in LDS (a bf16 weight is widened by a shift; the vector
+// units have three times the throughput the stream needs), so the step serves
+// both number formats; only the caches differ in type.
+//   1. norm + all projections of the layer input: queries, keys or latent,
+//      gates, feed-forward up (parallel layers: one norm feeds both parts);
+//      keys go straight to their cache row
+//   2. attention over the cache, split over workgroups
+//      (latent: queries through W_uk^T first, which also norms the new latent
+//      into the cache; the output through W_uv and the gate)
+//   3. output projection and feed-forward down as ONE product over the
+//      concatenated inputs, added into the residual row
+// then final norm + tied output matrix + soft cap + arg-max.
+#include "../../include/vkl_stack.h"
+#include "vkl_common.h"
+#include "vkl_decode_dev.h"
+#include "vkl_gemm.h"
+#include <algorithm>
+#include <mutex>
+#include <vector>
+
+namespace vkl
+{
+namespace
+{
+// a position known on the host, or kept on the device by a replayed loop
+// ({index into the ids, position})
+struct StepPos
+{
+  const uint32_t *loop;
+  uint32_t val;
+  __device__ __forceinline__ uint32_t
+  get () const
+  {
+    return loop ? ldg (loop + 1) : val;
+  }
+};
+
+__device__ __forceinline__ void
+widen8 (const uint4 w, float (&f)[8])
+{
+  const uint32_t u[4] = { w.x, w.y, w.z, w.w };
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    {
+      f[2 * i] = __uint_as_float (u[i] << 16);
+      f[2 * i + 1] = __uint_as_float (u[i] & 0xffff0000u);
+    }
+}
+
+__device__ __forceinline__ float
+sigmoid (float z)
+{
+  return 1.0f / (1.0f + expf (-z));
+}
+
+__device__ __forceinline__ float
+load_elem (const void *p, int type, size_t i)
+{
+  return type == VKL_TYPE_F32 ? ldg ((const float *)p + i) : bf2f (ldg ((const uint16_t *)p + i));
+}
+
+__device__ __forceinline__ void
+store_elem (void *p, int type, size_t i, float v)
+{
+  if (type == VKL_TYPE_F32)
+    stg ((float *)p + i, v);
+  else
+    stg ((uint16_t *)p + i, f2bf (v));
+}
+
+// sum over a workgroup of 256 or 512 threads; red: 8 floats of LDS
+__device__ __forceinline__ float
+group_sum (float v, float *red)
+{
+  v = wave_sum (v);
+  if ((threadIdx.x & 63) == 0)
+    red[threadIdx.x >> 6] = v;
+  __syncthreads ();
+  float s = 0.f;
+  for (unsigned i = 0; i < blockDim.x / 64; ++i)
+    s += red[i];
+  __syncthreads ();
+  return s;
+}
+
+// ---------------------------------------------------------------------------
+// embedding and norms
+// ---------------------------------------------------------------------------
+struct EmbedArgs
+{
+  const uint16_t *table;
+  uint32_t VH;
+  int K, W;
+  const uint32_t *toks;
+  const uint32_t *loop; // replayed loop: the token is toks[loop[0]]
+  const float *w;
+  float eps;
+  float *out;
+  size_t os;
+};
+
+__global__ __launch_bounds__ (256) void
+embed_norm_kernel (const EmbedArgs a)
+{
+  __shared__ float red[8];
+  const uint32_t i = blockIdx.x;
+  uint32_t id = ldg (a.toks + (a.loop ? ldg (a.loop) : i));
+  id = id < a.VH ? id : 0;
+  const uint16_t *row = a.table + (size_t)id * a.K;
+  float alpha = 1.f;
+  if (a.w)
+    {
+      float ss = 0.f;
+      for (int c = threadIdx.x; c < a.W; c += 256)
+        {
+          const float v = bf2f (ldg (row + c));
+          ss = __builtin_fmaf (v, v, ss);
+        }
+      alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
+    }
+  for (int c = threadIdx.x; c < a.W; c += 256)
+    {
+      const float v = bf2f (ldg (row + c));
+      stg (a.out + (size_t)i * a.os + c, a.w ? v * alpha * ldg (a.w + c) : v);
+    }
+}
+
+struct NormArgs
+{
+  const float *x;
+  size_t xs;
+  const uint32_t *rows;
+  int W, Wp;
+  const float *w;
+  float eps;
+  void *out;
+  int otype;
+  size_t os;
+};
+
+__global__ __launch_bounds__ (256) void
+rmsnorm_f32_kernel (const NormArgs a)
+{
+  __shared__ float red[8];
+  const size_t r = a.rows ? ldg (a.rows + blockIdx.x) : blockIdx.x;
+  const float *x = a.x + r * a.xs;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < a.W; c += 256)
+    {
+      const float v = ldg (x + c);
+      ss = __builtin_fmaf (v, v, ss);
+    }
+  const float alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
+  for (int c = threadIdx.x; c < a.Wp; c += 256)
+    store_elem (a.out, a.otype, blockIdx.x * a.os + c, c < a.W ? ldg (x + c) * alpha * ldg (a.w + c) : 0.f);
+}
+
+// ---------------------------------------------------------------------------
+// attention over rows that are keys and values
+// ---------------------------------------------------------------------------
+constexpr int kRowThreads = 256;
+constexpr int kRowUnroll = 4;
+constexpr int kRowSplits = 64;
+constexpr int kRowTarget = 512; // workgroups a launch aims for
+constexpr float kNoKey = -1.0e30f;
+
+struct RowAttnArgs
+{
+  const void *q;
+  int qtype;
+  size_t qs;
+  const void *rows;
+  size_t rs;
+  int G, D, rep, tiles; // rep: query heads per group; tiles: head tiles per group
+  StepPos pos;
+  float scale, tcoef;
+  int tevery;
+  void *out;
+  int otype;
+  size_t os;
+  int nsplit;
+  float *pm, *pl, *pacc; // parts of a split context: [S][G*tiles][nsplit][HT] (x D)
+  uint32_t *cnt;         // [S][G*tiles]
+};
+
+template <int LPR>
+__device__ __forceinline__ float
+lanes_sum (float v)
+{
+  v = row_sum<(LPR < 16 ? LPR : 16)> (v);
+  if (LPR >= 32)
+    v += __shfl_xor (v, 16, 64);
+  if (LPR >= 64)
+    v += __shfl_xor (v, 32, 64);
+  return v;
+}
+
+template <typename CT> struct RowVec; // 8 elements of a row as they lie
+template <> struct RowVec<uint16_t>
+{
+  uint4 a;
+  __device__ __forceinline__ void
+  load (const uint16_t *p)
+  {
+    a = ldg4 (p);
+  }
+  __device__ __forceinline__ void
+  get (float (&f)[8]) const
+  {
+    widen8 (a, f);
+  }
+  static __device__ __forceinline__ float
+  exponential (float x)
+  {
+    return __builtin_amdgcn_exp2f (x * 1.44269504088896340736f);
+  }
+};
+template <> struct RowVec<float>
+{
+  uint4 a, b;
+  __device__ __forceinline__ void
+  load (const float *p)
+  {
+    a = ldg4 (p), b = ldg4 (p + 4);
+  }
+  __device__ __forceinline__ void
+  get (float (&f)[8]) const
+  {
+    const uint32_t u[8] = { a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w };
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+      f[e] = __uint_as_float (u[e]);
+  }
+  static __device__ __forceinline__ float
+  exponential (float x)
+  {
+    return expf (x);
+  }
+};
+
+// LPR lanes share a row, NCH chunks of 8 values per lane; HT query heads per
+// workgroup.  Every group of LPR lanes walks rows of its own with a running
+// maximum; the groups' results meet in LDS at the end.
+template <typename CT, int LPR, int NCH, int HT>
+__global__ __launch_bounds__ (kRowThreads) void
+attn_rows_kernel (const RowAttnArgs a)
+{
+  constexpr int RPW = 64 / LPR, RPS = 4 * RPW, U = kRowUnroll, STEP = RPS * U;
+  constexpr int NS = kRowThreads / LPR; // lane groups
+  constexpr int DA = LPR * 8 * NCH;     // values of a row the lanes cover
+  extern __shared__ __align__ (16) float lds_rows[]; // [NS][HT][DA]
+  __shared__ float sm[NS][HT], sl[NS][HT], wgt[HT][kRowSplits];
+  __shared__ uint32_t last_s;
+  const int s = blockIdx.z, gt = blockIdx.y;
+  const int g = gt / a.tiles, t = gt - g * a.tiles;
+  const uint32_t pos = a.pos.get () + (uint32_t)s;
+  const int L = (int)pos + 1;
+  int chunk = (L + a.nsplit - 1) / a.nsplit;
+  chunk = (chunk + STEP - 1) / STEP * STEP;
+  const int active = (L + chunk - 1) / chunk;
+  const int c = blockIdx.x;
+  if (c >= active)
+    return;
+  const int l0 = c * chunk, l1 = min (L, l0 + chunk);
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int sub = lane % LPR, grp = lane / LPR, slot = tid / LPR;
+
+  const int col[2] = { sub * 8, LPR * 8 + sub * 8 };
+  const CT *base = (const CT *)a.rows + (size_t)g * a.D;
+  int cc[NCH]; // columns clamped into the row (lanes past its end contribute q = 0)
+#pragma unroll
+  for (int n = 0; n < NCH; ++n)
+    cc[n] = min (col[n], a.D - 8);
+
+  const int h0 = g * a.rep + t * HT;
+  float q[HT][NCH * 8];
+  {
+    float f = a.scale;
+    if (a.tcoef != 0.f)
+      f *= 1.0f + a.tcoef * logf ((float)((pos + 1u) / (uint32_t)a.tevery + 1u));
+#pragma unroll
+    for (int h = 0; h < HT; ++h)
+      {
+        const size_t qo = (size_t)s * a.qs + (size_t)(g * a.rep + min (t * HT + h, a.rep - 1)) * a.D;
+#pragma unroll
+        for (int n = 0; n < NCH; ++n)
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            q[h][n * 8 + e] = col[n] < a.D ? load_elem (a.q, a.qtype, qo + cc[n] + e) * f : 0.f;
+      }
+  }
+  float m[HT], l[HT], acc[HT][NCH * 8];
+#pragma unroll
+  for (int h = 0; h < HT; ++h)
+    {
+      m[h] = kNoKey, l[h] = 0.f;
+#pragma unroll
+      for (int e = 0; e < NCH * 8; ++e)
+        acc[h][e] = 0.f;
+    }
+
+  RowVec<CT> nx[U][NCH];
+  auto issue = [&] (int lb) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int n = 0; n < NCH; ++n)
+        nx[u][n].load (base + (size_t)min (lb + (u * 4 + wave) * RPW + grp, l1 - 1) * a.rs + cc[n]);
+  };
+  issue (l0);
+  for (int lb = l0; lb < l1; lb += STEP)
+    {
+      float row[U][NCH * 8];
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int n = 0; n < NCH; ++n)
+          {
+            float f[8];
+            nx[u][n].get (f);
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+              row[u][n * 8 + e] = f[e];
+          }
+      issue (min (lb + STEP, l1 - 1));
+#pragma unroll
+      for (int h = 0; h < HT; ++h)
+        {
+          float sc[U], mx = m[h];
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            {
+              float d = 0.f;
+#pragma unroll
+              for (int e = 0; e < NCH * 8; ++e)
+                d = __builtin_fmaf (q[h][e], row[u][e], d);
+              d = lanes_sum<LPR> (d);
+              sc[u] = lb + (u * 4 + wave) * RPW + grp < l1 ? d : kNoKey;
+              mx = fmaxf (mx, sc[u]);
+            }
+          const float al = RowVec<CT>::exponential (m[h] - mx);
+          m[h] = mx;
+          l[h] *= al;
+#pragma unroll
+          for (int e = 0; e < NCH * 8; ++e)
+            acc[h][e] *= al;
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            {
+              // (a group that has seen no row yet has mx = kNoKey: the guard
+              // keeps its weights at zero)
+              const float p = sc[u] > kNoKey ? RowVec<CT>::exponential (sc[u] - mx) : 0.f;
+              l[h] += p;
+#pragma unroll
+              for (int e = 0; e < NCH * 8; ++e)
+                acc[h][e] = __builtin_fmaf (p, row[u][e], acc[h][e]);
+            }
+        }
+    }
+
+  // the lane groups' parts
+  if (sub == 0)
+#pragma unroll
+    for (int h = 0; h < HT; ++h)
+      sm[slot][h] = m[h];
+  __syncthreads ();
+  float M[HT];
+#pragma unroll
+  for (int h = 0; h < HT; ++h)
+    {
+      float v = kNoKey;
+      for (int i = 0; i < NS; ++i)
+        v = fmaxf (v, sm[i][h]);
+      M[h] = v;
+      const float f = expf (m[h] - v);
+      if (sub == 0)
+        sl[slot][h] = l[h] * f;
+#pragma unroll
+      for (int n = 0; n < NCH; ++n)
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          lds_rows[(slot * HT + h) * DA + col[n] + e] = acc[h][n * 8 + e] * f;
+    }
+  __syncthreads ();
+  const int nh = min (HT, a.rep - t * HT); // heads of this tile
+  const size_t pbase = ((size_t)s * gridDim.y + gt) * a.nsplit;
+  for (int o = tid; o < nh * a.D; o += kRowThreads)
+    {
+      const int h = o / a.D, d = o - h * a.D;
+      float v = 0.f, S = 0.f;
+      for (int i = 0; i < NS; ++i)
+        v += lds_rows[(i * HT + h) * DA + d];
+      if (active == 1)
+        {
+          for (int i = 0; i < NS; ++i)
+            S += sl[i][h];
+          store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d, v / S);
+        }
+      else
+        {
+          // (write-through: the workgroup that combines may be on another XCD)
+          st_coherent_u32 ((uint32_t *)a.pacc + ((pbase + c) * HT + h) * a.D + d, __float_as_uint (v));
+        }
+    }
+  if (active == 1)
+    return;
+  if (tid < nh)
+    {
+      float S = 0.f, mm = kNoKey;
+      for (int i = 0; i < NS; ++i)
+        S += sl[i][tid], mm = fmaxf (mm, sm[i][tid]);
+      st_coherent_u32 ((uint32_t *)a.pm + (pbase + c) * HT + tid, __float_as_uint (mm));
+      st_coherent_u32 ((uint32_t *)a.pl + (pbase + c) * HT + tid, __float_as_uint (S));
+    }
+  // count in once this workgroup's parts are in memory; the last one combines
+  __builtin_amdgcn_s_waitcnt (0);
+  __syncthreads ();
+  if (tid == 0)
+    {
+      uint32_t *cnt = a.cnt + (size_t)s * gridDim.y + gt;
+      const uint32_t old = __hip_atomic_fetch_add (cnt, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      const bool last = old + 1u == (uint32_t)active;
+      if (last)
+        st_coherent_u32 (cnt, 0u);
+      last_s = last ? 1u : 0u;
+    }
+  __syncthreads ();
+  if (last_s == 0u)
+    return;
+  for (int i = tid; i < nh * active; i += kRowThreads)
+    {
+      const int h = i / active, p = i - h * active;
+      wgt[h][p] = __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pm + (pbase + p) * HT + h));
+    }
+  __syncthreads ();
+  float *sums = &sl[0][0]; // [nh], free by now
+  if (tid < nh)
+    {
+      float mm = kNoKey, S = 0.f;
+      for (int p = 0; p < active; ++p)
+        mm = fmaxf (mm, wgt[tid][p]);
+      for (int p = 0; p < active; ++p)
+        {
+          const float f = expf (wgt[tid][p] - mm);
+          wgt[tid][p] = f;
+          S += f * __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pl + (pbase + p) * HT + tid));
+        }
+      sums[tid] = S;
+    }
+  __syncthreads ();
+  for (int o = tid; o < nh * a.D; o += kRowThreads)
+    {
+      const int h = o / a.D, d = o - h * a.D;
+      float v = 0.f;
+      for (int p0 = 0; p0 < active; p0 += 8)
+        {
+          float pv[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j)
+            pv[j] = __uint_as_float (ld_coherent_u32 (
+                (const uint32_t *)a.pacc + ((pbase + min (p0 + j, active - 1)) * HT + h) * a.D + d));
+#pragma unroll
+          for (int j = 0; j < 8; ++j)
+            v += p0 + j < active ? wgt[h][min (p0 + j, active - 1)] * pv[j] : 0.f;
+        }
+      store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d, v / sums[h]);
+    }
+}
+
+// heads per workgroup: as many as share a row, within the registers
+int
+row_head_tile (int rep, int D)
+{
+  const int cap = D > 512 ? 4 : 8;
+  int ht = 1;
+  while (ht * 2 <= cap && ht < rep)
+    ht *= 2;
+  return ht;
+}
+
+struct RowPlan
+{
+  int ht, tiles, nsplit;
+  size_t parts; // entries of pm / pl
+};
+
+RowPlan
+row_plan (int H, int G, int D, int S)
+{
+  RowPlan p;
+  const int rep = H / G;
+  p.ht = row_head_tile (rep, D);
+  p.tiles = (rep + p.ht - 1) / p.ht;
+  const long groups = (long)G * p.tiles * S;
+  p.nsplit = (int)std::max (1L, std::min ((long)kRowSplits, kRowTarget / groups));
+  p.parts = (size_t)groups * p.nsplit * p.ht;
+  return p;
+}
+
+template <typename CT, int LPR, int NCH, int HT>
+int
+launch_rows_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
+{
+  static LdsLimit limit;
+  const size_t lds = (size_t)kRowThreads * 8 * NCH * HT * sizeof (float);
+  if (int e = limit.raise ((const void *)attn_rows_kernel<CT, LPR, NCH, HT>, lds))
+    return e;
+  attn_rows_kernel<CT, LPR, NCH, HT><<<grid, dim3 (kRowThreads), lds, s>>> (a);
+  return (int)hipGetLastError ();
+}
+
+template <typename CT, int LPR, int NCH>
+int
+launch_rows_ht (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
+{
+  switch (ht)
+    {
+    case 1: return launch_rows_k<CT, LPR, NCH, 1> (a, grid, s);
+    case 2: return launch_rows_k<CT, LPR, NCH, 2> (a, grid, s);
+    case 4: return launch_rows_k<CT, LPR, NCH, 4> (a, grid, s);
+    default:
+      if constexpr (NCH == 1)
+        return launch_rows_k<CT, LPR, NCH, 8> (a, grid, s);
+      return (int)hipErrorInvalidValue;
+    }
+}
+
+template <typename CT>
+int
+launch_rows (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
+{
+  if (a.D <= 32)
+    return launch_rows_ht<CT, 4, 1> (a, ht, grid, s);
+  if (a.D <= 64)
+    return launch_rows_ht<CT, 8, 1> (a, ht, grid, s);
+  if (a.D <= 128)
+    return launch_rows_ht<CT, 16, 1> (a, ht, grid, s);
+  if (a.D <= 256)
+    return launch_rows_ht<CT, 32, 1> (a, ht, grid, s);
+  if (a.D <= 512)
+    return launch_rows_ht<CT, 64, 1> (a, ht, grid, s);
+  return launch_rows_ht<CT, 64, 2> (a, ht, grid, s);
+}
+
+// The counters lie in front of the parts, in a block of fixed size, so that a
+// scratch area may serve launches of different shapes (each leaves its counters
+// at zero): only a split context has them, and there are at most kRowTarget / 2
+// of those workgroup rows then.
+constexpr size_t kRowCounterBytes = 4096;
+static_assert (kRowTarget / 2 * sizeof (uint32_t) <= kRowCounterBytes, "a counter per workgroup row");
+
+size_t
+row_scratch_bytes (int H, int G, int D, int S)
+{
+  const RowPlan p = row_plan (H, G, D, S);
+  return kRowCounterBytes + (p.nsplit > 1 ? p.parts * (2 + (size_t)D) * sizeof (float) : 0) + 256;
+}
+
+int
+rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype, size_t rs, int H, int G, int D,
+                int S, StepPos pos, float scale, float tcoef, int tevery, void *out, int otype, size_t os,
+                void *scratch, hipStream_t s)
+{
+  const RowPlan p = row_plan (H, G, D, S);
+  RowAttnArgs a = {};
+  a.q = q, a.qtype = qtype, a.qs = qs, a.rows = rows, a.rs = rs;
+  a.G = G, a.D = D, a.rep = H / G, a.tiles = p.tiles;
+  a.pos = pos, a.scale = scale, a.tcoef = tcoef, a.tevery = tevery;
+  a.out = out, a.otype = otype, a.os = os, a.nsplit = p.nsplit;
+  a.cnt = (uint32_t *)scratch;
+  a.pm = (float *)((uint8_t *)scratch + kRowCounterBytes);
+  a.pl = a.pm + p.parts;
+  a.pacc = a.pl + p.parts;
+  const dim3 grid ((unsigned)p.nsplit, (unsigned)(G * p.tiles), (unsigned)S);
+  return ctype == VKL_TYPE_F32 ? launch_rows<float> (a, p.ht, grid, s) : launch_rows<uint16_t> (a, p.ht, grid, s);
+}
+
+// ---------------------------------------------------------------------------
+// one small matrix per head
+// ---------------------------------------------------------------------------
+struct HeadArgs
+{
+  const uint16_t *w;
+  int R, K, bph; // bph: workgroups per head
+  int heads;
+  const void *x;
+  int xtype;
+  size_t xs, xh;
+  void *y;
+  int ytype;
+  size_t ys, yh;
+  const float *gate;
+  size_t gs;
+  // an extra workgroup norms a row of fp32 values into a cache row (the new
+  // token's latent), null: none
+  const float *nx;
+  const float *nw;
+  int nW, nWp;
+  float neps;
+  void *ncache;
+  int ntype;
+  StepPos pos;
+};
+
+constexpr int kHeadRows = 4; // row groups per wave
+
+template <int LPR>
+__global__ __launch_bounds__ (256) void
+head_matvec_kernel (const HeadArgs a)
+{
+  __shared__ float red[8];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  if ((int)blockIdx.x == a.heads * a.bph)
+    {
+      float ss = 0.f;
+      for (int c = tid; c < a.nW; c += 256)
+        {
+          const float v = ldg (a.nx + c);
+          ss = __builtin_fmaf (v, v, ss);
+        }
+      const float alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.nW + a.neps);
+      const size_t o = (size_t)a.pos.get () * a.nWp;
+      for (int c = tid; c < a.nWp; c += 256)
+        store_elem (a.ncache, a.ntype, o + c, c < a.nW ? ldg (a.nx + c) * alpha * ldg (a.nw + c) : 0.f);
+      return;
+    }
+  const int h = blockIdx.x / a.bph, b = blockIdx.x - h * a.bph, s = blockIdx.y;
+  constexpr int RPW = 64 / LPR;
+  const int sub = lane % LPR, grp = lane / LPR;
+  const int r0 = (b * 4 + wave) * RPW * kHeadRows + grp; // rows r0 + i * RPW
+  const uint16_t *w = a.w + (size_t)h * a.R * a.K;
+  const size_t xo = (size_t)s * a.xs + (size_t)h * a.xh;
+  float acc[kHeadRows] = {};
+  for (int k0 = 0; k0 < a.K; k0 += LPR * 8)
+    {
+      const int k = k0 + sub * 8, kc = min (k, a.K - 8);
+      uint4 wv[kHeadRows];
+#pragma unroll
+      for (int i = 0; i < kHeadRows; ++i)
+        wv[i] = ldg4 (w + (size_t)min (r0 + i * RPW, a.R - 1) * a.K + kc);
+      float xv[8];
+      if (a.xtype == VKL_TYPE_F32)
+        {
+          RowVec<float> v;
+          v.load ((const float *)a.x + xo + kc);
+          v.get (xv);
+        }
+      else
+        {
+          RowVec<uint16_t> v;
+          v.load ((const uint16_t *)a.x + xo + kc);
+          v.get (xv);
+        }
+      if (k >= a.K)
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          xv[e] = 0.f;
+#pragma unroll
+      for (int i = 0; i < kHeadRows; ++i)
+        {
+          float f[8];
+          widen8 (wv[i], f);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            acc[i] = __builtin_fmaf (f[e], xv[e], acc[i]);
+        }
+    }
+  const float f = a.gate ? sigmoid (ldg (a.gate + (size_t)s * a.gs + h)) : 1.0f;
+#pragma unroll
+  for (int i = 0; i < kHeadRows; ++i)
+    {
+      const float v = lanes_sum<LPR> (acc[i]);
+      if (sub == 0 && r0 + i * RPW < a.R)
+        store_elem (a.y, a.ytype, (size_t)s * a.ys + (size_t)h * a.yh + r0 + i * RPW, v * f);
+    }
+}
+
+int
+head_matvec (HeadArgs a, int S, hipStream_t s)
+{
+  const int lpr = a.K <= 32 ? 4 : a.K <= 64 ? 8 : a.K <= 128 ? 16 : a.K <= 256 ? 32 : 64;
+  const int rows = 4 * (64 / lpr) * kHeadRows;
+  a.bph = (a.R + rows - 1) / rows;
+  const dim3 grid ((unsigned)(a.heads * a.bph + (a.nx ? 1 : 0)), (unsigned)S), block (256);
+  switch (lpr)
+    {
+    case 4: head_matvec_kernel<4><<<grid, block, 0, s>>> (a); break;
+    case 8: head_matvec_kernel<8><<<grid, block, 0, s>>> (a); break;
+    case 16: head_matvec_kernel<16><<<grid, block, 0, s>>> (a); break;
+    case 32: head_matvec_kernel<32><<<grid, block, 0, s>>> (a); break;
+    default: head_matvec_kernel<64><<<grid, block, 0, s>>> (a); break;
+    }
+  return (int)hipGetLastError ();
+}
+
+// ---------------------------------------------------------------------------
+// the weight-streaming product of the step
+// ---------------------------------------------------------------------------
+constexpr int kGvThreads = 512, kGvWaves = 8;
+constexpr int kGvSpan = 2048; // columns of an item: 4 loads of 512 columns per row
+constexpr int kGvRows = 2;    // rows of an item
+
+enum
+{
+  GV_SEGS = 0,  // outputs by segment
+  GV_ADD = 1,   // y[n] += sum
+  GV_LOGITS = 2 // y[n] = soft cap, arg-max partials
+};
+
+struct GvSeg
+{
+  int n0, n;
+  void *y;
+  int f32, act;
+  size_t pos_stride; // y moves by this per position (a cache row)
+};
+
+struct GvArgs
+{
+  const uint16_t *w;
+  int N, K;
+  const float *x;    // [K]
+  const float *norm; // [K] (zero beyond W), RMS norm over W values
+  int W;
+  float eps;
+  int nseg;
+  GvSeg seg[kGemmSegs];
+  StepPos pos;
+  float *y;
+  float cap;
+  // arg-max: partials [grid] of (value, id), the counter, where the id goes
+  float *amax_v;
+  uint32_t *amax_i, *amax_cnt;
+  uint32_t *next_tok; // optional
+  uint32_t *loop, *ids; // replayed loop: ids[index + 1], then both words advance
+  int pick;
+};
+
+__device__ __forceinline__ bool
+amax_better (float v, uint32_t i, float bv, uint32_t bi)
+{
+  return v > bv || (v == bv && i < bi);
+}
+
+// XV: float4 per thread that hold the activation row while the first weights
+// are requested; 0: a row of any length, staged before them
+template <int MODE, int XV>
+__global__ __launch_bounds__ (kGvThreads) void
+stack_gemv_kernel (const GvArgs a)
+{
+  // column c of the row: block c / 512, first or second half of lane (c % 512) / 8
+  extern __shared__ __align__ (16) float xl[];
+  __shared__ float red[16];
+  __shared__ float bv_s[kGvWaves];
+  __shared__ uint32_t bi_s[kGvWaves + 1];
+  constexpr bool NORM = MODE != GV_ADD;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane (tid >> 6);
+  const int nspan = (a.K + kGvSpan - 1) / kGvSpan;
+  const int units = (a.N + kGvRows - 1) / kGvRows;
+  const int w0 = blockIdx.x * kGvWaves + wave, nw = gridDim.x * kGvWaves;
+  const int mine = w0 < units ? (units - w0 + nw - 1) / nw : 0;
+  const int items = mine * nspan;
+
+  uint4 bufa[kGvRows * 4], bufb[kGvRows * 4];
+  auto issue = [&] (int it, uint4 (&b)[kGvRows * 4]) {
+    const int ic = min (it, max (items - 1, 0));
+    const int un = ic / nspan, sp = ic - un * nspan;
+    const int row0 = min (w0 + un * nw, units - 1) * kGvRows;
+#pragma unroll
+    for (int r = 0; r < kGvRows; ++r)
+      {
+        const uint16_t *p = a.w + (size_t)min (row0 + r, a.N - 1) * a.K;
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          b[r * 4 + u] = ldg4_stream (p + min (sp * kGvSpan + u * 512 + lane * 8, a.K - 8));
+      }
+  };
+  auto put = [&] (int c, const float4 v) { // c: a multiple of 4
+    const int o = (c >> 9) * 512 + ((c >> 2) & 1) * 256 + ((c & 511) >> 3) * 4;
+    *(float4 *)(xl + o) = v;
+  };
+  const int kpad = nspan * kGvSpan;
+  if constexpr (XV > 0)
+    {
+      float4 xv[XV], nv[XV];
+#pragma unroll
+      for (int j = 0; j < XV; ++j)
+        {
+          const int c = min ((tid + j * kGvThreads) * 4, a.K - 4);
+          xv[j] = __builtin_bit_cast (float4, ldg4 (a.x + c));
+          if (NORM)
+            nv[j] = __builtin_bit_cast (float4, ldg4 (a.norm + c));
+        }
+      __builtin_amdgcn_sched_barrier (0);
+      issue (0, bufa);
+      __builtin_amdgcn_sched_barrier (0);
+      float alpha = 1.f;
+      if (NORM)
+        {
+          float ss = 0.f;
+#pragma unroll
+          for (int j = 0; j < XV; ++j)
+            if ((tid + j * kGvThreads) * 4 < a.K)
+              {
+                ss = __builtin_fmaf (xv[j].x, xv[j].x, ss), ss = __builtin_fmaf (xv[j].y, xv[j].y, ss);
+                ss = __builtin_fmaf (xv[j].z, xv[j].z, ss), ss = __builtin_fmaf (xv[j].w, xv[j].w, ss);
+              }
+          alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
+        }
+#pragma unroll
+      for (int j = 0; j < XV; ++j)
+        {
+          const int c = (tid + j * kGvThreads) * 4;
+          float4 v = xv[j];
+          if (NORM)
+            {
+              v.x = v.x * alpha * nv[j].x, v.y = v.y * alpha * nv[j].y;
+              v.z = v.z * alpha * nv[j].z, v.w = v.w * alpha * nv[j].w;
+            }
+          if (c >= a.K)
+            v = make_float4 (0.f, 0.f, 0.f, 0.f);
+          if (c < kpad)
+            put (c, v);
+        }
+    }
+  else
+    {
+      float alpha = 1.f;
+      if (NORM)
+        {
+          float ss = 0.f;
+          for (int c = tid; c < a.K; c += kGvThreads)
+            {
+              const float v = ldg (a.x + c);
+              ss = __builtin_fmaf (v, v, ss);
+            }
+          alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
+        }
+      for (int c = tid * 4; c < kpad; c += kGvThreads * 4)
+        {
+          float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
+          if (c < a.K)
+            {
+              v = __builtin_bit_cast (float4, ldg4 (a.x + c));
+              if (NORM)
+                {
+                  const float4 n = __builtin_bit_cast (float4, ldg4 (a.norm + c));
+                  v.x = v.x * alpha * n.x, v.y = v.y * alpha * n.y;
+                  v.z = v.z * alpha * n.z, v.w = v.w * alpha * n.w;
+                }
+            }
+          put (c, v);
+        }
+      issue (0, bufa);
+    }
+  __syncthreads ();
+
+  const uint32_t pos = MODE == GV_SEGS ? a.pos.get () : 0u;
+  float sum[kGvRows];
+#pragma unroll
+  for (int r = 0; r < kGvRows; ++r)
+    sum[r] = 0.f;
+  float best_v = -INFINITY;
+  uint32_t best_i = 0xffffffffu;
+  auto compute = [&] (int it, const uint4 (&b)[kGvRows * 4]) {
+    const int un = it / nspan, sp = it - un * nspan;
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      {
+        const float *xp = xl + (sp * 4 + u) * 512 + lane * 4;
+        const float4 x0 = *(const float4 *)xp, x1 = *(const float4 *)(xp + 256);
+        const float xv[8] = { x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w };
+#pragma unroll
+        for (int r = 0; r < kGvRows; ++r)
+          {
+            float f[8];
+            widen8 (b[r * 4 + u], f);
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+              sum[r] = __builtin_fmaf (f[e], xv[e], sum[r]);
+          }
+      }
+    if (sp != nspan - 1)
+      return;
+    const int row0 = (w0 + un * nw) * kGvRows;
+#pragma unroll
+    for (int r = 0; r < kGvRows; ++r)
+      {
+        float v = wave_sum (sum[r]);
+        sum[r] = 0.f;
+        const int n = row0 + r;
+        if (n >= a.N)
+          continue;
+        if (MODE == GV_ADD)
+          {
+            if (lane == 0)
+              stg (a.y + n, ldg (a.y + n) + v);
+          }
+        else if (MODE == GV_LOGITS)
+          {
+            if (a.cap > 0.f)
+              v = a.cap * tanhf (v / a.cap);
+            if (lane == 0)
+              stg (a.y + n, v);
+            if (amax_better (v, (uint32_t)n, best_v, best_i))
+              best_v = v, best_i = (uint32_t)n;
+          }
+        else
+          {
+#pragma unroll
+            for (int i = 0; i < kGemmSegs; ++i)
+              if (i < a.nseg && n >= a.seg[i].n0 && n < a.seg[i].n0 + a.seg[i].n)
+                {
+                  const GvSeg &sg = a.seg[i];
+                  float y = v;
+                  if (sg.act == 2)
+                    {
+                      y = fmaxf (y, 0.f);
+                      y = y * y;
+                    }
+                  if (lane == 0)
+                    store_elem (sg.y, sg.f32 ? VKL_TYPE_F32 : VKL_TYPE_BF16,
+                                (size_t)pos * sg.pos_stride + (n - sg.n0), y);
+                }
+          }
+      }
+  };
+  for (int it = 0; it < items; it += 2)
+    {
+      issue (it + 1, bufb);
+      compute (it, bufa);
+      issue (it + 2, bufa);
+      if (it + 1 < items)
+        compute (it + 1, bufb);
+    }
+  if (MODE != GV_LOGITS || !a.pick)
+    return;
+  // arg-max: the workgroup's best, then the last workgroup over all of them
+  if (lane == 0)
+    bv_s[wave] = best_v, bi_s[wave] = best_i;
+  __syncthreads ();
+  if (tid == 0)
+    {
+      for (int i = 1; i < kGvWaves; ++i)
+        if (amax_better (bv_s[i], bi_s[i], best_v, best_i))
+          best_v = bv_s[i], best_i = bi_s[i];
+      st_coherent_u32 ((uint32_t *)a.amax_v + blockIdx.x, __float_as_uint (best_v));
+      st_coherent_u32 (a.amax_i + blockIdx.x, best_i);
+      __builtin_amdgcn_s_waitcnt (0);
+      const uint32_t old = __hip_atomic_fetch_add (a.amax_cnt, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      const bool last = old + 1u == gridDim.x;
+      if (last)
+        st_coherent_u32 (a.amax_cnt, 0u);
+      bi_s[kGvWaves] = last ? 1u : 0u;
+    }
+  __syncthreads ();
+  if (bi_s[kGvWaves] == 0u || tid >= 64)
+    return;
+  best_v = -INFINITY, best_i = 0xffffffffu;
+  for (int i = lane; i < (int)gridDim.x; i += 64)
+    {
+      const float v = __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.amax_v + i));
+      const uint32_t id = ld_coherent_u32 (a.amax_i + i);
+      if (amax_better (v, id, best_v, best_i))
+        best_v = v, best_i = id;
+    }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1)
+    {
+      const float ov = __shfl_xor (best_v, o, 64);
+      const uint32_t oi = __shfl_xor (best_i, o, 64);
+      if (amax_better (ov, oi, best_v, best_i))
+        best_v = ov, best_i = oi;
+    }
+  if (lane == 0)
+    {
+      const uint32_t id = best_i == 0xffffffffu ? 0u : best_i;
+      if (a.next_tok)
+        *a.next_tok = id;
+      if (a.loop)
+        {
+          const uint32_t index = a.loop[0];
+          a.ids[index + 1] = id;
+          a.loop[0] = index + 1u, a.loop[1] += 1u;
+        }
+    }
+}
+
+constexpr int kGvMaxLds = 128 << 10;
+
+bool
+gv_supported (int K)
+{
+  return (size_t)((K + kGvSpan - 1) / kGvSpan) * kGvSpan * sizeof (float) <= (size_t)kGvMaxLds;
+}
+
+template <int MODE, int XV>
+int
+launch_gv_k (const GvArgs &a, int grid, size_t lds, hipStream_t s)
+{
+  static LdsLimit limit;
+  if (int e = limit.raise ((const void *)stack_gemv_kernel<MODE, XV>, lds))
+    return e;
+  stack_gemv_kernel<MODE, XV><<<dim3 ((unsigned)grid), dim3 (kGvThreads), lds, s>>> (a);
+  return (int)hipGetLastError ();
+}
+
+template <int MODE>
+int
+launch_gv (const GvArgs &a, int n_cu, hipStream_t s)
+{
+  if (!gv_supported (a.K))
+    return (int)hipErrorInvalidValue;
+  const int units = (a.N + kGvRows - 1) / kGvRows;
+  const int grid = std::min (2 * n_cu, (units + kGvWaves - 1) / kGvWaves);
+  const size_t lds = (size_t)((a.K + kGvSpan - 1) / kGvSpan) * kGvSpan * sizeof (float);
+  if (a.K <= 2048)
+    return launch_gv_k<MODE, 1> (a, grid, lds, s);
+  if (a.K <= 4096)
+    return launch_gv_k<MODE, 2> (a, grid, lds, s);
+  if (a.K <= 8192)
+    return launch_gv_k<MODE, 4> (a, grid, lds, s);
+  if (a.K <= 16384)
+    return launch_gv_k<MODE, 8> (a, grid, lds, s);
+  return launch_gv_k<MODE, 0> (a, grid, lds, s);
+}
+
+// ---------------------------------------------------------------------------
+// the step
+// ---------------------------------------------------------------------------
+struct StackScratch
+{
+  uint32_t *sync; // [0] arg-max counter, [16..17] loop state, [20..23] sampler parameters
+  uint32_t *cnt;  // attention counters and parts
+  float *x, *q, *c, *g, *cat, *qa, *oa, *logits, *amax_v;
+  uint32_t *amax_i;
+  size_t bytes;
+};
+
+constexpr int kMaxGrid = 2048;
+
+StackScratch
+carve_stack (const vkl_stack_model *m)
+{
+  StackScratch s = {};
+  size_t q = 0, c = 0, g = 0, cat = 0, qa = 0, attn = 0;
+  for (int i = 0; i < m->n_runs; ++i)
+    {
+      const vkl_stack_layer &l = m->layers_h[i];
+      q = std::max (q, (size_t)l.H * l.dim);
+      cat = std::max (cat, (size_t)l.k_out);
+      if (l.mixer == VKL_MIX_LATENT)
+        {
+          c = std::max (c, (size_t)l.rank_p), g = std::max (g, (size_t)l.H);
+          qa = std::max (qa, (size_t)l.H * l.rank_p);
+          attn = std::max (attn, row_scratch_bytes (l.H, 1, l.rank_p, 1));
+        }
+      else
+        attn = std::max (attn, row_scratch_bytes (l.H, l.G, l.dim, 1));
+    }
+  uint8_t *base = (uint8_t *)m->scratch;
+  size_t off = 0;
+  auto take = [&] (size_t bytes) {
+    uint8_t *p = base + off;
+    off += (bytes + 255) / 256 * 256;
+    return p;
+  };
+  s.sync = (uint32_t *)take (4096);
+  s.cnt = (uint32_t *)take (attn);
+  s.x = (float *)take ((size_t)m->width_p * 4);
+  s.q = (float *)take (q * 4);
+  s.c = (float *)take (c * 4);
+  s.g = (float *)take (g * 4);
+  s.cat = (float *)take (cat * 4);
+  s.qa = (float *)take (qa * 4);
+  s.oa = (float *)take (qa * 4);
+  s.logits = (float *)take ((size_t)m->vocab * 4);
+  s.amax_v = (float *)take (kMaxGrid * 4);
+  s.amax_i = (uint32_t *)take (kMaxGrid * 4);
+  s.bytes = off;
+  return s;
+}
+
+int
+check_stack (const vkl_stack_model *m)
+{
+  VKL_CHECK_ARG (m && m->layers_h && m->embed && m->final_norm && m->scratch);
+  VKL_CHECK_ARG (m->width > 0 && m->width <= m->width_p && (m->width_p % 64) == 0 && m->vocab > 0 && m->maxlen > 0
+                 && m->n_runs > 0);
+  VKL_CHECK_ARG (m->ctype == VKL_TYPE_F32 || m->ctype == VKL_TYPE_BF16);
+  VKL_CHECK_ARG (gv_supported (m->width_p));
+  for (int i = 0; i < m->n_runs; ++i)
+    {
+      const vkl_stack_layer &l = m->layers_h[i];
+      VKL_CHECK_ARG (l.mixer == VKL_MIX_SHARED_KV || l.mixer == VKL_MIX_LATENT);
+      VKL_CHECK_ARG (l.norm && l.w_in && l.w_out && l.cache && l.H > 0 && l.G > 0 && (l.H % l.G) == 0);
+      VKL_CHECK_ARG (l.dim > 0 && (l.dim % 32) == 0 && l.vdim > 0 && (l.vdim % 32) == 0);
+      VKL_CHECK_ARG ((l.k_out % 64) == 0 && gv_supported (l.k_out) && l.ff >= 0);
+      VKL_CHECK_ARG (l.ff_col >= l.H * l.vdim && l.ff_col + l.ff <= l.k_out);
+      VKL_CHECK_ARG (l.temp_coef == 0.f || l.temp_every > 0);
+      VKL_CHECK_ARG (l.kv0 >= l.H * l.dim);
+      if (l.mixer == VKL_MIX_LATENT)
+        {
+          VKL_CHECK_ARG (l.w_ukt && l.w_uv && l.c_norm && l.rank > 0 && l.rank <= l.rank_p && (l.rank_p % 32) == 0
+                         && l.rank_p <= 1024 && l.G == 1);
+          VKL_CHECK_ARG (l.g0 >= l.kv0 + l.rank && l.up0 >= l.g0 + l.H && l.up0 + l.ff <= l.n_in);
+        }
+      else
+        VKL_CHECK_ARG (l.dim <= 1024 && l.vdim == l.dim && l.up0 >= l.kv0 + l.G * l.dim && l.up0 + l.ff <= l.n_in);
+    }
+  return 0;
+}
+
+struct StepArgs
+{
+  const vkl_stack_model *m;
+  StackScratch s;
+  StepPos pos;
+  const uint32_t *toks; // the token, or the ids of a replayed loop
+  float *logits;
+  uint32_t *next_tok;
+  uint32_t *loop, *ids;
+  bool sampled;
+  int n_cu;
+};
+
+int
+launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
+{
+  const vkl_stack_model &m = *p.m;
+  const bool latent = l.mixer == VKL_MIX_LATENT;
+  GvArgs a = {};
+  a.w = (const uint16_t *)l.w_in, a.N = l.n_in, a.K = m.width_p;
+  a.x = p.s.x, a.norm = l.norm, a.W = m.width, a.eps = m.eps, a.pos = p.pos;
+  int n = 0;
+  a.seg[n++] = { 0, l.H * l.dim, p.s.q, 1, 0, 0 };
+  if (latent)
+    {
+      a.seg[n++] = { l.kv0, l.rank, p.s.c, 1, 0, 0 };
+      a.seg[n++] = { l.g0, l.H, p.s.g, 1, 0, 0 };
+    }
+  else
+    a.seg[n++] = { l.kv0, l.G * l.dim, l.cache, m.ctype == VKL_TYPE_F32, 0, (size_t)l.G * l.dim };
+  if (l.ff)
+    a.seg[n++] = { l.up0, l.ff, p.s.cat + l.ff_col, 1, 2, 0 };
+  a.nseg = n;
+  if (int e = launch_gv<GV_SEGS> (a, p.n_cu, st))
+    return e;
+  if (latent)
+    {
+      HeadArgs h = {};
+      h.w = (const uint16_t *)l.w_ukt, h.heads = l.H, h.R = l.rank_p, h.K = l.dim;
+      h.x = p.s.q, h.xtype = VKL_TYPE_F32, h.xh = (size_t)l.dim;
+      h.y = p.s.qa, h.ytype = VKL_TYPE_F32, h.yh = (size_t)l.rank_p;
+      h.nx = p.s.c, h.nw = l.c_norm, h.nW = l.rank, h.nWp = l.rank_p, h.neps = m.eps;
+      h.ncache = l.cache, h.ntype = m.ctype, h.pos = p.pos;
+      if (int e = head_matvec (h, 1, st))
+        return e;
+      if (int e = rows_attention (p.s.qa, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.rank_p, l.H, 1, l.rank_p, 1,
+                                  p.pos, l.scale, l.temp_coef, l.temp_every, p.s.oa, VKL_TYPE_F32, 0, p.s.cnt, st))
+        return e;
+      HeadArgs v = {};
+      v.w = (const uint16_t *)l.w_uv, v.heads = l.H, v.R = l.vdim, v.K = l.rank_p;
+      v.x = p.s.oa, v.xtype = VKL_TYPE_F32, v.xh = (size_t)l.rank_p;
+      v.y = p.s.cat, v.ytype = VKL_TYPE_F32, v.yh = (size_t)l.vdim;
+      v.gate = p.s.g;
+      if (int e = head_matvec (v, 1, st))
+        return e;
+    }
+  else if (int e = rows_attention (p.s.q, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.G * l.dim, l.H, l.G, l.dim, 1,
+                                   p.pos, l.scale, l.temp_coef, l.temp_every, p.s.cat, VKL_TYPE_F32, 0, p.s.cnt, st))
+    return e;
+  GvArgs o = {};
+  o.w = (const uint16_t *)l.w_out, o.N = m.width, o.K = l.k_out;
+  o.x = p.s.cat, o.y = p.s.x;
+  return launch_gv<GV_ADD> (o, p.n_cu, st);
+}
+
+int
+launch_stack_step (const StepArgs &p, hipStream_t st)
+{
+  const vkl_stack_model &m = *p.m;
+  EmbedArgs e = {};
+  e.table = (const uint16_t *)m.embed, e.VH = (uint32_t)m.vocab, e.K = m.width_p, e.W = m.width;
+  e.toks = p.toks, e.loop = p.loop, e.w = m.embed_norm, e.eps = m.eps, e.out = p.s.x, e.os = (size_t)m.width_p;
+  embed_norm_kernel<<<dim3 (1), dim3 (256), 0, st>>> (e);
+  for (int i = 0; i < m.n_runs; ++i)
+    if (int err = launch_stack_layer (p, m.layers_h[i], st))
+      return err;
+  GvArgs a = {};
+  a.w = (const uint16_t *)m.embed, a.N = m.vocab, a.K = m.width_p;
+  a.x = p.s.x, a.norm = m.final_norm, a.W = m.width, a.eps = m.eps;
+  a.y = p.logits ? p.logits : p.s.logits, a.cap = m.logit_cap;
+  a.amax_v = p.s.amax_v, a.amax_i = p.s.amax_i, a.amax_cnt = p.s.sync;
+  a.pick = (p.next_tok || p.loop) && !p.sampled;
+  a.next_tok = p.next_tok, a.loop = p.loop, a.ids = p.ids;
+  if (int err = launch_gv<GV_LOGITS> (a, p.n_cu, st))
+    return err;
+  if (p.loop && p.sampled)
+    return sample_loop_launch (a.y, m.vocab, p.s.sync + 20, p.loop, p.ids, st);
+  return (int)hipGetLastError ();
+}
+
+int
+compute_units (int *n_cu)
+{
+  int dev = 0;
+  VKL_HIP (hipGetDevice (&dev));
+  VKL_HIP (hipDeviceGetAttribute (n_cu, hipDeviceAttributeMultiprocessorCount, dev));
+  VKL_CHECK_ARG (2 * *n_cu <= kMaxGrid);
+  return 0;
+}
+
+__global__ void
+set_stack_loop_kernel (uint32_t *sync, uint32_t pos, uint32_t k, uint32_t p_bits, uint32_t seed_lo, uint32_t seed_hi)
+{
+  sync[16] = 0u, sync[17] = pos;
+  sync[20] = k, sync[21] = p_bits, sync[22] = seed_lo, sync[23] = seed_hi;
+}
+
+// captured steps, one per (model, buffers, way of picking the token)
+struct StackGraph
+{
+  uint64_t key = 0;
+  const void *scratch = nullptr;
+  hipGraph_t graph = nullptr;
+  hipGraphExec_t exec = nullptr;
+};
+std::vector<StackGraph> g_stack_graphs;
+std::mutex g_stack_mu;
+constexpr size_t kStackGraphs = 8;
+
+void
+drop_stack_graph (StackGraph &g)
+{
+  if (g.exec)
+    (void)hipGraphExecDestroy (g.exec);
+  if (g.graph)
+    (void)hipGraphDestroy (g.graph);
+}
+
+uint64_t
+stack_key (const vkl_stack_model *m, const void *ids, const void *logits, bool sampled)
+{
+  uint64_t h = 1469598103934665603ull;
+  auto mix = [&h] (const void *p, size_t n) {
+    for (size_t i = 0; i < n; ++i)
+      h = (h ^ ((const uint8_t *)p)[i]) * 1099511628211ull;
+  };
+  const void *ptrs[6] = { m->embed, m->embed_norm, m->final_norm, m->scratch, ids, logits };
+  const int dims[6] = { m->width, m->vocab, m->maxlen, m->n_runs, m->ctype, (int)sampled };
+  mix (ptrs, sizeof (ptrs)), mix (dims, sizeof (dims)), mix (&m->eps, 4), mix (&m->logit_cap, 4);
+  mix (m->layers_h, sizeof (vkl_stack_layer) * (size_t)m->n_runs);
+  return h;
+}
+
+int
+stack_loop (const vkl_stack_model *m, uint32_t *ids, uint32_t pos0, int n_steps, float *logits, bool sampled,
+            int topk, float topp, uint64_t seed, hipStream_t st)
+{
+  if (int e = check_stack (m))
+    return e;
+  VKL_CHECK_ARG (ids && n_steps >= 0 && (uint64_t)pos0 + (uint64_t)n_steps <= (uint64_t)m->maxlen);
+  if (n_steps == 0)
+    return 0;
+  StepArgs p = {};
+  p.m = m, p.s = carve_stack (m);
+  if (int e = compute_units (&p.n_cu))
+    return e;
+  p.loop = p.s.sync + 16, p.ids = ids, p.toks = ids;
+  p.pos = { p.loop, 0u };
+  p.logits = logits, p.sampled = sampled;
+  set_stack_loop_kernel<<<dim3 (1), dim3 (1), 0, st>>> (p.s.sync, pos0, (uint32_t)topk,
+                                                        __builtin_bit_cast (uint32_t, topp), (uint32_t)seed,
+                                                        (uint32_t)(seed >> 32));
+  std::lock_guard<std::mutex> lock (g_stack_mu);
+  const uint64_t key = stack_key (m, ids, logits, sampled);
+  StackGraph *g = nullptr;
+  for (StackGraph &c : g_stack_graphs)
+    if (c.key == key && c.scratch == m->scratch)
+      g = &c;
+  if (!g)
+    {
+      StackGraph n;
+      n.key = key, n.scratch = m->scratch;
+      VKL_HIP (hipStreamBeginCapture (st, hipStreamCaptureModeThreadLocal));
+      int err = launch_stack_step (p, st);
+      const hipError_t e = hipStreamEndCapture (st, &n.graph);
+      if (!err && e != hipSuccess)
+        err = (int)e;
+      if (!err)
+        err = (int)hipGraphInstantiate (&n.exec, n.graph, nullptr, nullptr, 0);
+      if (err)
+        {
+          drop_stack_graph (n);
+          return err;
+        }
+      if (g_stack_graphs.size () >= kStackGraphs)
+        {
+          drop_stack_graph (g_stack_graphs.front ());
+          g_stack_graphs.erase (g_stack_graphs.begin ());
+        }
+      g_stack_graphs.push_back (n);
+      g = &g_stack_graphs.back ();
+    }
+  for (int i = 0; i < n_steps; ++i)
+    VKL_HIP (hipGraphLaunch (g->exec, st));
+  return vkl_launch_status ();
+}
+} // namespace
+} // namespace vkl
+
+using namespace vkl;
+
+extern "C" int
+vkl_embed_norm_bf16 (const void *table, uint32_t VH, int K, int W, const uint32_t *toks, uint32_t n, const float *w,
+                     float eps, float *out, size_t os, void *stream)
+{
+  VKL_CHECK_ARG (table && toks && out && VH > 0 && n > 0 && W > 0 && K >= W && os >= (size_t)W);
+  EmbedArgs a = {};
+  a.table = (const uint16_t *)table, a.VH = VH, a.K = K, a.W = W, a.toks = toks, a.w = w, a.eps = eps;
+  a.out = out, a.os = os;
+  embed_norm_kernel<<<dim3 (n), dim3 (256), 0, (hipStream_t)stream>>> (a);
+  return vkl_launch_status ();
+}
+
+extern "C" int
+vkl_rmsnorm_f32 (const float *x, size_t xs, const uint32_t *rows, int n, int W, const float *w, float eps, void *out,
+                 int otype, size_t os, int Wp, void *stream)
+{
+  VKL_CHECK_ARG (x && w && out && n > 0 && W > 0 && Wp >= W && xs >= (size_t)W && os >= (size_t)Wp);
+  VKL_CHECK_ARG (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16);
+  const NormArgs a = { x, xs, rows, W, Wp, w, eps, out, otype, os };
+  rmsnorm_f32_kernel<<<dim3 ((unsigned)n), dim3 (256), 0, (hipStream_t)stream>>> (a);
+  return vkl_launch_status ();
+}
+
+extern "C" size_t
+vkl_attn_rows_scratch_bytes (int H, int G, int dim, int S)
+{
+  if (H <= 0 || G <= 0 || H % G || dim <= 0 || S <= 0)
+    return 0;
+  return row_scratch_bytes (H, G, dim, S);
+}
+
+extern "C" int
+vkl_attn_rows (const void *q, int qtype, size_t qs, const void *rows, int ctype, size_t rs, int H, int G, int dim,
+               int S, uint32_t pos0, float scale, float temp_coef, int temp_every, void *out, int otype, size_t os,
+               void *scratch, void *stream)
+{
+  VKL_CHECK_ARG (q && rows && out && scratch && H > 0 && G > 0 && (H % G) == 0 && S > 0 && S <= 65535);
+  VKL_CHECK_ARG (dim > 0 && (dim % 32) == 0 && dim <= 1024 && rs >= (size_t)G * dim && (rs % 8) == 0);
+  VKL_CHECK_ARG (temp_coef == 0.f || temp_every > 0);
+  VKL_CHECK_ARG (((uintptr_t)rows % 16) == 0 && qs >= (size_t)H * dim && os >= (size_t)H * dim);
+  VKL_CHECK_ARG ((qtype == VKL_TYPE_F32 || qtype == VKL_TYPE_BF16) && (ctype == VKL_TYPE_F32 || ctype == VKL_TYPE_BF16)
+                 && (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16));
+  return rows_attention (q, qtype, qs, rows, ctype, rs, H, G, dim, S, StepPos{ nullptr, pos0 }, scale, temp_coef,
+                         temp_every, out, otype, os, scratch, (hipStream_t)stream);
+}
+
+extern "C" int
+vkl_head_matvec (const void *w, int H, int R, int K, const void *x, int xtype, size_t xs, size_t xh, void *y,
+                 int ytype, size_t ys, size_t yh, const float *gate, size_t gs, int S, void *stream)
+{
+  VKL_CHECK_ARG (w && x && y && H > 0 && R > 0 && K > 0 && (K % 32) == 0 && S > 0 && S <= 65535);
+  VKL_CHECK_ARG ((xtype == VKL_TYPE_F32 || xtype == VKL_TYPE_BF16) && (ytype == VKL_TYPE_F32 || ytype == VKL_TYPE_BF16));
+  VKL_CHECK_ARG (xh >= (size_t)K && yh >= (size_t)R && (xs % 8) == 0 && (xh % 8) == 0 && ((uintptr_t)x % 16) == 0
+                 && ((uintptr_t)w % 16) == 0);
+  VKL_CHECK_ARG (S == 1 || (xs >= (size_t)H * xh && ys >= (size_t)H * yh));
+  HeadArgs a = {};
+  a.w = (const uint16_t *)w, a.heads = H, a.R = R, a.K = K, a.x = x, a.xtype = xtype, a.xs = xs, a.xh = xh;
+  a.y = y, a.ytype = ytype, a.ys = ys, a.yh = yh, a.gate = gate, a.gs = gs;
+  return head_matvec (a, S, (hipStream_t)stream);
+}
+
+extern "C" size_t
+vkl_stack_scratch_bytes (const vkl_stack_model *m)
+{
+  if (!m || !m->layers_h || m->n_runs <= 0)
+    return 0;
+  return carve_stack (m).bytes;
+}
+
+extern "C" int
+vkl_stack_supported (const vkl_stack_model *m)
+{
+  return check_stack (m) == 0 ? 1 : 0;
+}
+
+extern "C" int
+vkl_stack_step (const vkl_stack_model *m, const uint32_t *tok, uint32_t pos, float *logits32, uint32_t *next_tok,
+                void *stream)
+{
+  if (int e = check_stack (m))
+    return e;
+  VKL_CHECK_ARG (tok && pos < (uint32_t)m->maxlen);
+  StepArgs p = {};
+  p.m = m, p.s = carve_stack (m);
+  if (int e = compute_units (&p.n_cu))
+    return e;
+  p.pos = { nullptr, pos }, p.toks = tok, p.logits = logits32, p.next_tok = next_tok;
+  return launch_stack_step (p, (hipStream_t)stream);
+}
+
+extern "C" int
+vkl_stack_loop (const vkl_stack_model *m, uint32_t *ids, uint32_t pos0, int n_steps, float *logits32, void *stream)
+{
+  return stack_loop (m, ids, pos0, n_steps, logits32, false, 1, -1.f, 0, (hipStream_t)stream);
+}
+
+extern "C" int
+vkl_stack_loop_sampled (const vkl_stack_model *m, uint32_t *ids, uint32_t pos0, int n_steps, float *logits32,
+                        int topk, float topp, uint64_t seed, void *stream)
+{
+  VKL_CHECK_ARG (topp >= 0.f || topk >= 1);
+  VKL_CHECK_ARG (topp < 0.f || topp <= 1.0f);
+  return stack_loop (m, ids, pos0, n_steps, logits32, true, topk, topp, seed, (hipStream_t)stream);
+}
+
+extern "C" void
+vkl_stack_release (const vkl_stack_model *m)
+{
+  if (!m)
+    return;
+  std::lock_guard<std::mutex> lock (g_stack_mu);
+  for (size_t i = 0; i < g_stack_graphs.size ();)
+    if (g_stack_graphs[i].scratch == m->scratch)
+      {
+        drop_stack_graph (g_stack_graphs[i]);
+        g_stack_graphs.erase (g_stack_graphs.begin () + (long)i);
+      }
+    else
+      ++i;
+}

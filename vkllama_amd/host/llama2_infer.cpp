@@ -1,13 +1,14 @@
-// Command-line generation from a GGUF file with the drop-in classes: the flow
+// Command-line generation with the C++ classes, from a GGUF file or a folder with
+// config.json and model.safetensors: the flow
 // of the reference's app/llama2_infer.cpp (open the file, collect keys and
 // tensors, Model::init, prompt pass, then one token per step picked on the
 // host by a TopkSampler(1), line 138 there) without the sentencepiece
 // tokenizer, which is not available to C++ in this image: the prompt is given
 // as token ids.
 //
-//   llama2_infer [--topk K | --topp P] [--seed S] MODEL.gguf N_TOKENS ID [ID ...]
-#include "models/gguflib.h"
-#include "models/llama2.h"
+//   llama2_infer [--topk K | --topp P] [--seed S] [--dtype bfloat16|float32]
+//                [--max-tokens N] MODEL N_TOKENS ID [ID ...]
+#include "models/registry.h"
 #include "models/samplers.h"
 #include <cstring>
 #include <memory>
@@ -26,6 +27,7 @@ main (int argc, char **argv)
   float topp = -1.f;
   bool seeded = false;
   uint64_t seed = 0;
+  vkllama::ModelOptions options;
   while (argc > 2 && argv[1][0] == '-' && argv[1][1] == '-')
     {
       if (!strcmp (argv[1], "--topk"))
@@ -34,6 +36,10 @@ main (int argc, char **argv)
         topp = strtof (argv[2], nullptr);
       else if (!strcmp (argv[1], "--seed"))
         seeded = true, seed = strtoull (argv[2], nullptr, 10);
+      else if (!strcmp (argv[1], "--dtype") && (!strcmp (argv[2], "bfloat16") || !strcmp (argv[2], "float32")))
+        options.dtype = argv[2][0] == 'f' ? vkllama::FP32 : vkllama::BF16;
+      else if (!strcmp (argv[1], "--max-tokens"))
+        options.max_tokens = strtoull (argv[2], nullptr, 10);
       else
         break;
       argv += 2, argc -= 2;
@@ -41,7 +47,8 @@ main (int argc, char **argv)
   if (argc < 4 || topk < 1)
     {
       fprintf (stderr,
-               "usage: llama2_infer [--topk K | --topp P] [--seed S] <model.gguf> <predict tokens> "
+               "usage: llama2_infer [--topk K | --topp P] [--seed S] [--dtype bfloat16|float32] "
+               "[--max-tokens N] <model> <predict tokens> "
                "<prompt id> [id ...]\n");
       return 2;
     }
@@ -50,38 +57,18 @@ main (int argc, char **argv)
     sampler.reset (seeded ? new TopPSampler (topp, seed) : new TopPSampler (topp));
   else
     sampler.reset (seeded ? new TopkSampler (topk, seed) : new TopkSampler (topk));
-  gguf_ctx *gguf = gguf_open (argv[1]);
-  if (!gguf)
-    {
-      fprintf (stderr, "cannot read %s as a GGUF file\n", argv[1]);
-      return 1;
-    }
-  std::map<std::string, gguf_key> kv;
-  gguf_key key;
-  while (gguf_get_key (gguf, &key))
-    {
-      fprintf (stderr, "%.*s: [%s]\n", (int)key.namelen, key.name,
-               gguf_get_value_type_name (key.type));
-      kv[std::string (key.name, key.namelen)] = key;
-    }
-  std::map<std::string, gguf_tensor> tensors;
-  gguf_tensor tensor;
-  while (gguf_get_tensor (gguf, &tensor))
-    tensors[std::string (tensor.name, tensor.namelen)] = tensor;
-
   const int predict = atoi (argv[2]);
   std::vector<uint32_t> prompt;
   for (int i = 3; i < argc; ++i)
     prompt.push_back ((uint32_t)strtoul (argv[i], nullptr, 10));
 
-  vkllama::Model model (0);
-  auto ret = model.init (kv, tensors);
-  gguf_close (gguf);
-  if (!ret.ok ())
+  auto loaded = vkllama::load_model (argv[1], options);
+  if (!loaded.ok ())
     {
-      fprintf (stderr, "failed at init model: %s\n", ret.ToString ().c_str ());
+      fprintf (stderr, "failed at init model: %s\n", loaded.status ().ToString ().c_str ());
       return 1;
     }
+  vkllama::CausalModel &model = **loaded;
   fprintf (stderr, "all weights are uploaded to device\n");
 
   using clock = std::chrono::steady_clock;

@@ -1,18 +1,24 @@
 // extern "C" wrappers around vkllama::Model and the synthetic-weight helpers
 // (include/vkl_model.h).
 #include "vkl_model.h"
+#include "models/fazinex.h"
 #include "models/gguflib.h"
 #include "models/llama2.h"
+#include "models/registry.h"
 #include "vkl_decode.h"
 #include "vkl_hip.h"
 #include <cmath>
+#include <cstring>
 #include <map>
 #include <string>
 #include <vector>
 
 struct vkl_model
 {
-  vkllama::Model *model = nullptr;
+  vkllama::CausalModel *model = nullptr;
+  // the family's own calls: null for a model of another family
+  vkllama::Model *llama () const { return dynamic_cast<vkllama::Model *> (model); }
+  vkllama::Fazinex *fazinex () const { return dynamic_cast<vkllama::Fazinex *> (model); }
   std::string last_error;
   std::vector<gguf_value> values;
   std::vector<std::string> names;
@@ -75,10 +81,11 @@ vkl_model_create (int dev, const vkl_model_hparams *hp,
       t.weights_data = (uint8_t *)tensors[i].data;
       ts[m->names.back ()] = t;
     }
-  m->model = new vkllama::Model (dev);
+  auto *llama = new vkllama::Model (dev);
+  m->model = llama;
   try
     {
-      auto s = m->model->init (kv, ts);
+      auto s = llama->init (kv, ts);
       if (!s.ok ())
         return fail (m, s);
     }
@@ -89,36 +96,80 @@ vkl_model_create (int dev, const vkl_model_hparams *hp,
   return 0;
 }
 
-extern "C" int
-vkl_model_load_gguf (int dev, const char *path, vkl_model **out)
+namespace
 {
-  if (!path || !out)
-    return (int)absl::StatusCode::kInvalidArgument;
-  auto *m = new vkl_model ();
-  *out = m;
-  gguf_ctx *g = gguf_open (path);
-  if (!g)
-    return fail (m, absl::NotFoundError (std::string ("not a readable GGUF file: ") + path));
-  std::map<std::string, gguf_key> kv;
-  std::map<std::string, gguf_tensor> ts;
-  gguf_key key;
-  while (gguf_get_key (g, &key))
-    kv[std::string (key.name, key.namelen)] = key;
-  gguf_tensor t;
-  while (gguf_get_tensor (g, &t))
-    ts[std::string (t.name, t.namelen)] = t;
-  m->model = new vkllama::Model (dev);
-  absl::Status s = absl::OkStatus ();
+// runs `make`, which gives a StatusOr<unique_ptr<CausalModel>>, into m
+template <typename F>
+int
+adopt (vkl_model *m, F &&make)
+{
   try
     {
-      s = m->model->init (kv, ts);
+      auto r = make ();
+      if (!r.ok ())
+        return fail (m, r.status ());
+      m->model = r->release ();
     }
   catch (const std::exception &e)
     {
-      s = absl::InternalError (e.what ());
+      return fail (m, absl::InternalError (e.what ()));
     }
-  gguf_close (g); // every weight has been copied to the device by now
-  return s.ok () ? 0 : fail (m, s);
+  return 0;
+}
+
+bool
+parse_options (int dev, const char *dtype, size_t max_tokens, vkllama::ModelOptions &o)
+{
+  o.device = dev, o.max_tokens = max_tokens;
+  if (dtype && !strcmp (dtype, "float32"))
+    o.dtype = vkllama::FP32;
+  else if (dtype && strcmp (dtype, "bfloat16"))
+    return false;
+  return true;
+}
+}
+
+extern "C" int
+vkl_model_load (int dev, const char *path, const char *dtype, size_t max_tokens, vkl_model **out)
+{
+  vkllama::ModelOptions o;
+  if (!path || !out || !parse_options (dev, dtype, max_tokens, o))
+    return (int)absl::StatusCode::kInvalidArgument;
+  auto *m = new vkl_model ();
+  *out = m;
+  return adopt (m, [&] () { return vkllama::load_model (path, o); });
+}
+
+extern "C" int
+vkl_model_load_gguf (int dev, const char *path, vkl_model **out)
+{
+  return vkl_model_load (dev, path, nullptr, 0, out);
+}
+
+extern "C" int
+vkl_model_create_config (int dev, const char *config, const vkl_tensor_desc *tensors, size_t n_tensors,
+                         const char *dtype, size_t max_tokens, vkl_model **out)
+{
+  vkllama::ModelOptions o;
+  if (!config || !out || (!tensors && n_tensors) || !parse_options (dev, dtype, max_tokens, o))
+    return (int)absl::StatusCode::kInvalidArgument;
+  auto *m = new vkl_model ();
+  *out = m;
+  vkllama::WeightSource w;
+  for (size_t i = 0; i < n_tensors; ++i)
+    {
+      const vkl_tensor_desc &t = tensors[i];
+      if (!t.name || !t.data || (t.type != 30 && t.type != 0 && t.type != 1))
+        return fail (m, absl::InvalidArgumentError ("tensor without name or data, or of another type than BF16, F16, F32"));
+      vkllama::WeightView v;
+      v.dtype = t.type == 30 ? vkllama::BF16 : t.type == 1 ? vkllama::FP16 : vkllama::FP32;
+      if (t.dim1)
+        v.shape.push_back ((size_t)t.dim1);
+      v.shape.push_back ((size_t)t.dim0);
+      v.data = (const uint8_t *)t.data, v.bytes = (size_t)t.bsize;
+      w.add (t.name, v);
+    }
+  return adopt (m, [&] () { return vkllama::create_model (config, w, o); });
 }
 
 extern "C" void
@@ -161,6 +212,49 @@ vkl_model_forward (vkl_model *m, const uint32_t *toks, size_t n_toks,
     {
       return fail (m, absl::InternalError (e.what ()));
     }
+  return 0;
+}
+
+extern "C" int
+vkl_model_forward_rows (vkl_model *m, const uint32_t *toks, size_t n_toks, size_t offset, const uint32_t *rows,
+                        size_t n_rows, float *logits)
+{
+  if (!m || !m->model || !toks || (n_rows && (!rows || !logits)))
+    return (int)absl::StatusCode::kInvalidArgument;
+  try
+    {
+      auto r = m->model->forward_rows (std::vector<uint32_t> (toks, toks + n_toks), offset,
+                                       std::vector<uint32_t> (rows, rows + n_rows));
+      if (!r.ok ())
+        return fail (m, r.status ());
+      std::copy (r->begin (), r->end (), logits);
+    }
+  catch (const std::exception &e)
+    {
+      return fail (m, absl::InternalError (e.what ()));
+    }
+  return 0;
+}
+
+extern "C" size_t
+vkl_model_context_length (const vkl_model *m)
+{
+  return m && m->model ? m->model->context_length () : 0;
+}
+
+extern "C" int
+vkl_model_residual_streams (vkl_model *m, const uint32_t *toks, size_t n_toks, size_t offset, float *out, size_t n)
+{
+  if (!m || !m->model || !toks || !out)
+    return (int)absl::StatusCode::kInvalidArgument;
+  if (!m->fazinex ())
+    return fail (m, absl::UnimplementedError ("this model family keeps no fp32 residual stream"));
+  auto r = m->fazinex ()->residual_streams (std::vector<uint32_t> (toks, toks + n_toks), offset);
+  if (!r.ok ())
+    return fail (m, r.status ());
+  if (r->size () != n)
+    return fail (m, absl::OutOfRangeError ("output buffer of the wrong size"));
+  std::copy (r->begin (), r->end (), out);
   return 0;
 }
 
@@ -216,28 +310,22 @@ vkl_model_set_option (vkl_model *m, const char *name, int value)
 {
   if (!m || !m->model || !name)
     return (int)absl::StatusCode::kInvalidArgument;
-  const std::string n (name);
-  if (n == "fused_decode")
-    m->model->set_fused_decode (value != 0);
-  else if (n == "lastblock_rope_quirk")
-    m->model->set_lastblock_rope_quirk (value != 0);
-  else if (n == "operator_attention")
-    m->model->set_operator_attention (value != 0);
-  else if (n == "decode_mode")
-    m->model->set_decode_mode (value);
-  else if (n == "decode_graph")
-    m->model->set_decode_graph (value != 0);
-  else if (n == "phase_timing")
-    vkl_decode_phase_timing (value);
-  else if (n == "fuse_attn_wo" || n == "wait_test" || n == "attn_split_min")
+  if (!strcmp (name, "phase_timing"))
     {
-      // options of this model's fused decode steps (fields of vkl_decode_model)
-      if (!m->model->set_decode_option (name, value))
-        return fail (m, absl::InvalidArgumentError ("option " + n + ": value out of range"));
+      vkl_decode_phase_timing (value);
+      return 0;
     }
-  else
-    return fail (m, absl::InvalidArgumentError ("unknown option " + n));
-  return 0;
+  const auto s = m->model->set_option (name, value);
+  return s.ok () ? 0 : fail (m, s);
+}
+
+namespace
+{
+int
+not_llama (vkl_model *m)
+{
+  return fail (m, absl::UnimplementedError ("only Llama-2 models offer this call"));
+}
 }
 
 extern "C" int
@@ -246,8 +334,10 @@ vkl_model_read_kv_cache (vkl_model *m, size_t layer, int value, uint16_t *out,
 {
   if (!m || !m->model || !out)
     return (int)absl::StatusCode::kInvalidArgument;
+  if (!m->llama ())
+    return not_llama (m);
   std::vector<uint16_t> buf;
-  auto s = m->model->read_kv_cache (layer, value != 0, buf);
+  auto s = m->llama ()->read_kv_cache (layer, value != 0, buf);
   if (!s.ok ())
     return fail (m, s);
   if (n < buf.size ())
@@ -262,7 +352,9 @@ vkl_model_write_kv_cache (vkl_model *m, size_t layer, int value, const uint16_t 
 {
   if (!m || !m->model || !rows)
     return (int)absl::StatusCode::kInvalidArgument;
-  auto s = m->model->write_kv_cache (layer, value != 0, rows, n);
+  if (!m->llama ())
+    return not_llama (m);
+  auto s = m->llama ()->write_kv_cache (layer, value != 0, rows, n);
   return s.ok () ? 0 : fail (m, s);
 }
 
@@ -295,14 +387,16 @@ vkl_model_phase_replay (vkl_model *m, int kind, size_t pos, int rounds,
 {
   if (!m || !m->model || !avg_ms)
     return (int)absl::StatusCode::kInvalidArgument;
-  auto s = m->model->decode_phase_replay (kind, pos, rounds, avg_ms, launches);
+  if (!m->llama ())
+    return not_llama (m);
+  auto s = m->llama ()->decode_phase_replay (kind, pos, rounds, avg_ms, launches);
   return s.ok () ? 0 : fail (m, s);
 }
 
 extern "C" size_t
 vkl_model_phase_bytes (const vkl_model *m, int kind, size_t L)
 {
-  return m && m->model ? m->model->decode_phase_bytes (kind, L) : 0;
+  return m && m->llama () ? m->llama ()->decode_phase_bytes (kind, L) : 0;
 }
 
 // ---------------------------------------------------------------------------
@@ -355,6 +449,19 @@ vkl_synth_normal_f16 (uint64_t seed, size_t n, float std, uint16_t *out)
 #pragma omp parallel for schedule(static)
   for (size_t i = 0; i < n; ++i)
     out[i] = __fp32_to_fp16_rne (normal_at (seed, i, std)).u16;
+}
+
+extern "C" void
+vkl_synth_normal_bf16 (uint64_t seed, size_t n, float std, uint16_t *out)
+{
+#pragma omp parallel for schedule(static)
+  for (size_t i = 0; i < n; ++i)
+    {
+      const float v = normal_at (seed, i, std);
+      uint32_t u;
+      memcpy (&u, &v, 4);
+      out[i] = (uint16_t)((u + 0x7fffu + ((u >> 16) & 1u)) >> 16); // to nearest, ties to even
+    }
 }
 
 extern "C" void

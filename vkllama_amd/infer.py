@@ -1,9 +1,10 @@
-"""Generation from a GGUF model file, the job of app/llama2_infer.cpp of the
-reference:
+"""Generation from a model, a GGUF file or a folder with config.json and
+model.safetensors; the job of app/llama2_infer.cpp of the reference:
 
     python -m vkllama_amd.infer MODEL.gguf N_TOKENS --ids 1 15043 3186
     python -m vkllama_amd.infer MODEL.gguf N_TOKENS --tokenizer tokenizer.model --prompt "Hello"
     python -m vkllama_amd.infer MODEL.gguf N_TOKENS --ids 1 15043 --topk 40 --seed 7
+    python -m vkllama_amd.infer FOLDER N_TOKENS --ids 1 15043 --dtype float32 --max-tokens 8192
 
 The default is the reference's TopkSampler(1), i.e. greedy, which runs with
 the token pick on the device; --topk K / --topp P draw on the host from the
@@ -53,6 +54,10 @@ def main(argv=None):
     ap.add_argument("--seed", type=int, help="seed of the sampler (default: random device)")
     ap.add_argument("--device-sampler", action="store_true",
                     help="draw on the device (no logits download per token); needs --seed or uses seed 0")
+    ap.add_argument("--dtype", choices=("bfloat16", "float32"),
+                    help="number format of a model that runs in either (default: the model's own)")
+    ap.add_argument("--max-tokens", type=int, default=0,
+                    help="cache rows of a model whose files name no context length (default 4096)")
     args = ap.parse_args(argv)
 
     sp = None
@@ -70,7 +75,7 @@ def main(argv=None):
         ap.error("give --ids or --prompt")
 
     from . import model as M
-    m = M.Llama2.from_gguf(args.model, args.device)
+    m = M.CausalModel.load(args.model, args.dtype, args.max_tokens, args.device)
     sampled = args.topp is not None or (args.topk or 1) > 1
     if sampled and args.device_sampler:
         out, prefill_ms, decode_ms = m.generate_sampled(np.array(ids, np.uint32), args.n_tokens, args.topk or 40,

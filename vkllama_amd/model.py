@@ -1,7 +1,8 @@
-"""ctypes binding of include/vkl_model.h (libvkllama_host.so): the llama2
-token loop behind the C++ drop-in classes.  No CPU fallback: a missing
+"""ctypes binding of include/vkl_model.h (libvkllama_host.so): the models
+behind the C++ classes and their token loop.  No CPU fallback: a missing
 library or a failing call raises."""
 import ctypes as C
+import json
 import os
 
 import numpy as np
@@ -24,6 +25,12 @@ class HParams(C.Structure):
 SIGNATURES = {
     "vkl_model_create": (i32, [i32, C.POINTER(HParams), C.POINTER(TensorDesc), sz, C.POINTER(vp)]),
     "vkl_model_load_gguf": (i32, [i32, C.c_char_p, C.POINTER(vp)]),
+    "vkl_model_load": (i32, [i32, C.c_char_p, C.c_char_p, sz, C.POINTER(vp)]),
+    "vkl_model_create_config": (i32, [i32, C.c_char_p, C.POINTER(TensorDesc), sz, C.c_char_p, sz, C.POINTER(vp)]),
+    "vkl_model_forward_rows": (i32, [vp, vp, sz, sz, vp, sz, vp]),
+    "vkl_model_context_length": (sz, [vp]),
+    "vkl_model_residual_streams": (i32, [vp, vp, sz, sz, vp, sz]),
+    "vkl_synth_normal_bf16": (None, [u64, sz, C.c_float, vp]),
     "vkl_model_destroy": (None, [vp]),
     "vkl_model_last_error": (C.c_char_p, [vp]),
     "vkl_model_vocab": (sz, [vp]),
@@ -137,7 +144,129 @@ class Sampler:
             pass
 
 
-class Llama2:
+class CausalModel:
+    """A model of any family through the C ABI: the calls they all offer."""
+
+    _h = None
+    cfg = None
+
+    def _adopt(self, rc, h, what):
+        self._h = h
+        if rc:
+            msg = self._err() if h else "bad argument"
+            self.close()
+            e = capi.VklError("%s failed (%d): %s" % (what, rc, msg))
+            e.code = rc
+            raise e
+        return self
+
+    @classmethod
+    def load(cls, path, dtype=None, max_tokens=0, dev=0):
+        """From a path: a GGUF file, or a folder with config.json and
+        model.safetensors.  dtype: "bfloat16", "float32" or None (the model's
+        own); max_tokens sizes the cache of a model that names no context
+        length."""
+        self, h = cls.__new__(cls), vp()
+        rc = lib().vkl_model_load(dev, str(path).encode(), dtype and dtype.encode(), int(max_tokens), C.byref(h))
+        self._adopt(rc, h, "vkl_model_load")
+        self.cfg = {"vocab": int(lib().vkl_model_vocab(self._h))}
+        return self
+
+    @classmethod
+    def create(cls, config, weights, dtype=None, max_tokens=0, dev=0):
+        """From a configuration (a dict or JSON text) and a dict name -> bf16
+        bits (uint16 arrays)."""
+        text = config if isinstance(config, str) else json.dumps(config)
+        descs, keep = (TensorDesc * len(weights))(), []
+        for i, (name, a) in enumerate(weights.items()):
+            a = np.ascontiguousarray(a)
+            assert a.dtype == np.uint16 and a.ndim in (1, 2), name
+            keep.append(a)
+            descs[i] = TensorDesc(name.encode(), 30, a.shape[-1], a.shape[0] if a.ndim == 2 else 0, a.ctypes.data,
+                                  a.nbytes)
+        self, h = cls.__new__(cls), vp()
+        rc = lib().vkl_model_create_config(dev, text.encode(), descs, len(weights), dtype and dtype.encode(),
+                                           int(max_tokens), C.byref(h))
+        self._adopt(rc, h, "vkl_model_create_config")
+        self.cfg = {"vocab": int(lib().vkl_model_vocab(self._h))}
+        return self
+
+    def _err(self):
+        m = lib().vkl_model_last_error(self._h)
+        return m.decode() if m else "?"
+
+    def _check(self, rc, what):
+        if rc:
+            raise capi.VklError("%s failed (%d): %s" % (what, rc, self._err()))
+
+    def close(self):
+        if self._h:
+            lib().vkl_model_destroy(self._h)
+            self._h = None
+
+    def __del__(self):
+        try:
+            self.close()
+        except Exception:
+            pass
+
+    def set_option(self, name, value):
+        self._check(lib().vkl_model_set_option(self._h, name.encode(), int(value)), "set_option")
+
+    def forward(self, toks, offset):
+        toks = np.ascontiguousarray(toks, np.uint32)
+        logits = np.empty(self.cfg["vocab"], np.float32)
+        self._check(lib().vkl_model_forward(self._h, toks.ctypes.data, toks.size, offset, logits.ctypes.data),
+                    "vkl_model_forward")
+        return logits
+
+    def forward_rows(self, toks, offset, rows):
+        """logits [len(rows), vocab] of those rows of toks"""
+        toks, rows = np.ascontiguousarray(toks, np.uint32), np.ascontiguousarray(rows, np.uint32)
+        logits = np.empty((rows.size, self.cfg["vocab"]), np.float32)
+        self._check(lib().vkl_model_forward_rows(self._h, toks.ctypes.data, toks.size, offset, rows.ctypes.data,
+                                                 rows.size, logits.ctypes.data), "vkl_model_forward_rows")
+        return logits
+
+    def residual_streams(self, toks, offset, runs, width):
+        toks = np.ascontiguousarray(toks, np.uint32)
+        out = np.empty((runs, toks.size, width), np.float32)
+        self._check(lib().vkl_model_residual_streams(self._h, toks.ctypes.data, toks.size, offset, out.ctypes.data,
+                                                     out.size), "vkl_model_residual_streams")
+        return out
+
+    def context_length(self):
+        return int(lib().vkl_model_context_length(self._h))
+
+    def generate_greedy(self, prompt, n_gen):
+        prompt = np.ascontiguousarray(prompt, np.uint32)
+        ids = np.empty(n_gen, np.uint32)
+        t_pre, t_dec = C.c_double(0), C.c_double(0)
+        self._check(lib().vkl_model_generate_greedy(self._h, prompt.ctypes.data, prompt.size, n_gen,
+                                                    ids.ctypes.data, C.byref(t_pre), C.byref(t_dec)),
+                    "vkl_model_generate_greedy")
+        return ids, t_pre.value, t_dec.value
+
+    def generate_sampled(self, prompt, n_gen, topk=40, topp=None, seed=0):
+        """Generation with the token drawn on the device: from the topk largest
+        logits, or (topp given) from the top-p set; seed fixes the sequence."""
+        prompt = np.ascontiguousarray(prompt, np.uint32)
+        ids = np.empty(n_gen, np.uint32)
+        t_pre, t_dec = C.c_double(0), C.c_double(0)
+        self._check(lib().vkl_model_generate_sampled(self._h, prompt.ctypes.data, prompt.size, n_gen, int(topk),
+                                                     -1.0 if topp is None else float(topp), int(seed),
+                                                     ids.ctypes.data, C.byref(t_pre), C.byref(t_dec)),
+                    "vkl_model_generate_sampled")
+        return ids, t_pre.value, t_dec.value
+
+    def decode_recoveries(self):
+        return int(lib().vkl_model_decode_recoveries(self._h))
+
+    def decode_step_bytes(self, L):
+        return int(lib().vkl_model_decode_step_bytes(self._h, L))
+
+
+class Llama2(CausalModel):
     """vkllama::Model through the C ABI.
 
     cfg: dim, n_layers, n_heads, ffn, vocab, maxlen, eps, wtype
@@ -173,67 +302,7 @@ class Llama2:
     def from_gguf(cls, path, dev=0):
         """Loads a GGUF file the way app/llama2_infer.cpp of the reference does
         (keys and tensors through the gguf reader, then Model::init)."""
-        self = cls.__new__(cls)
-        self._h = None
-        h = vp()
-        rc = lib().vkl_model_load_gguf(dev, path.encode(), C.byref(h))
-        self._h = h
-        if rc:
-            msg = self._err()
-            self.close()
-            raise capi.VklError("vkl_model_load_gguf failed (%d): %s" % (rc, msg))
-        self.cfg = {"vocab": int(lib().vkl_model_vocab(self._h))}
-        return self
-
-    def _err(self):
-        m = lib().vkl_model_last_error(self._h)
-        return m.decode() if m else "?"
-
-    def _check(self, rc, what):
-        if rc:
-            raise capi.VklError("%s failed (%d): %s" % (what, rc, self._err()))
-
-    def close(self):
-        if self._h:
-            lib().vkl_model_destroy(self._h)
-            self._h = None
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
-
-    def set_option(self, name, value):
-        self._check(lib().vkl_model_set_option(self._h, name.encode(), int(value)), "set_option")
-
-    def forward(self, toks, offset):
-        toks = np.ascontiguousarray(toks, np.uint32)
-        logits = np.empty(self.cfg["vocab"], np.float32)
-        self._check(lib().vkl_model_forward(self._h, toks.ctypes.data, toks.size, offset, logits.ctypes.data),
-                    "vkl_model_forward")
-        return logits
-
-    def generate_greedy(self, prompt, n_gen):
-        prompt = np.ascontiguousarray(prompt, np.uint32)
-        ids = np.empty(n_gen, np.uint32)
-        t_pre, t_dec = C.c_double(0), C.c_double(0)
-        self._check(lib().vkl_model_generate_greedy(self._h, prompt.ctypes.data, prompt.size, n_gen,
-                                                    ids.ctypes.data, C.byref(t_pre), C.byref(t_dec)),
-                    "vkl_model_generate_greedy")
-        return ids, t_pre.value, t_dec.value
-
-    def generate_sampled(self, prompt, n_gen, topk=40, topp=None, seed=0):
-        """Generation with the token drawn on the device: from the topk largest
-        logits, or (topp given) from the top-p set; seed fixes the sequence."""
-        prompt = np.ascontiguousarray(prompt, np.uint32)
-        ids = np.empty(n_gen, np.uint32)
-        t_pre, t_dec = C.c_double(0), C.c_double(0)
-        self._check(lib().vkl_model_generate_sampled(self._h, prompt.ctypes.data, prompt.size, n_gen, int(topk),
-                                                     -1.0 if topp is None else float(topp), int(seed),
-                                                     ids.ctypes.data, C.byref(t_pre), C.byref(t_dec)),
-                    "vkl_model_generate_sampled")
-        return ids, t_pre.value, t_dec.value
+        return cls.load(path, dev=dev)
 
     def read_kv_cache(self, layer, value):
         c = self.cfg
@@ -248,12 +317,6 @@ class Llama2:
         rows = np.ascontiguousarray(rows, np.float16)
         self._check(lib().vkl_model_write_kv_cache(self._h, layer, int(value), rows.ctypes.data, rows.size),
                     "vkl_model_write_kv_cache")
-
-    def decode_recoveries(self):
-        return int(lib().vkl_model_decode_recoveries(self._h))
-
-    def decode_step_bytes(self, L):
-        return int(lib().vkl_model_decode_step_bytes(self._h, L))
 
     PHASES = ("kqv", "attention", "wo", "upgate", "down", "lm_head", "argmax", "unused", "layer")
 

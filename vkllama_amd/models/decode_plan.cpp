@@ -6,21 +6,8 @@
 
 namespace vkllama
 {
-static absl::Status
-hip_status (const char *what, int e)
-{
-  if (!e)
-    return absl::OkStatus ();
-  if (e == 1)
-    return absl::InvalidArgumentError (
-        absl::StrFormat ("%s: rejected by the HIP layer", what));
-  return absl::InternalError (
-      absl::StrFormat ("%s: %s", what, vkl_error_string (e)));
-}
-
 DecodePlan::DecodePlan ()
-    : gpu_ (nullptr), usable_ (false), mode_ (1), adopted_valid_ (false),
-      vocab_ (0)
+    : usable_ (false), mode_ (1)
 {
   memset (&desc_, 0, sizeof (desc_));
 }
@@ -36,12 +23,7 @@ DecodePlan::build (Model &model, GPUDevice *gpu, InputLayer *in,
                    std::vector<Llama2Block *> &blocks, OutputLayer *out,
                    float eps)
 {
-  gpu_ = gpu;
-  vocab_ = model.vocab_size ();
-  tok_slot_ = Tensor (1, 1, 1, gpu, UINT32, true);
-  VKLLAMA_STATUS_OK (tok_slot_.create ());
-  logits32_ = Tensor (1, 1, (int)vocab_, gpu, FP32, false);
-  VKLLAMA_STATUS_OK (logits32_.create ());
+  VKLLAMA_STATUS_OK (create_buffers (gpu, model.vocab_size ()));
 
   Tensor &emb = in->embedding ()->vocab ();
   auto *attn0 = blocks[0]->attention ();
@@ -149,16 +131,6 @@ DecodePlan::build (Model &model, GPUDevice *gpu, InputLayer *in,
 }
 
 absl::Status
-DecodePlan::step_host_token (uint32_t tok, size_t offset)
-{
-  // the slot may still be read by a queued step
-  VKLLAMA_STATUS_OK (
-      hip_status ("waiting for the stream", vkl_stream_sync (gpu_->stream ())));
-  *(uint32_t *)tok_slot_.host () = tok;
-  return step_device_token ((const uint32_t *)tok_slot_.data (), offset);
-}
-
-absl::Status
 DecodePlan::step_device_token (const uint32_t *tok, size_t offset,
                                uint32_t *next_tok)
 {
@@ -242,48 +214,5 @@ DecodePlan::check ()
                     : "no such launch was in use"));
     }
   return absl::OkStatus ();
-}
-
-absl::Status
-DecodePlan::adopt_logits (Tensor logits32)
-{
-  if (logits32.dtype () != FP32 || logits32.size () < vocab_)
-    return absl::InvalidArgumentError ("logits tensor has the wrong type");
-  adopted_ = logits32;
-  adopted_valid_ = true;
-  return absl::OkStatus ();
-}
-
-absl::Status
-DecodePlan::read_logits (float *dst)
-{
-  const Tensor &src = adopted_valid_ ? adopted_ : logits32_;
-  const float *p = (const float *)src.data () + (src.size () - vocab_);
-  VKLLAMA_STATUS_OK (hip_status (
-      "downloading logits",
-      vkl_memcpy_d2h (dst, p, vocab_ * sizeof (float), gpu_->stream ())));
-  VKLLAMA_STATUS_OK (hip_status ("downloading logits", vkl_stream_sync (gpu_->stream ())));
-  return check ();
-}
-
-absl::Status
-DecodePlan::argmax_logits (uint32_t *dst)
-{
-  const Tensor &src = adopted_valid_ ? adopted_ : logits32_;
-  const float *p = (const float *)src.data () + (src.size () - vocab_);
-  return hip_status ("argmax", vkl_argmax_f32 (p, (int)vocab_, dst,
-                                               gpu_->stream ()));
-}
-
-absl::Status
-DecodePlan::sample_logits (uint32_t *dst, int topk, float topp, uint64_t seed,
-                           uint32_t counter)
-{
-  const Tensor &src = adopted_valid_ ? adopted_ : logits32_;
-  const float *p = (const float *)src.data () + (src.size () - vocab_);
-  return hip_status ("sample",
-                     vkl_sample_f32 (p, (int)vocab_, topk, topp, seed, counter,
-                                     nullptr, dst, nullptr, nullptr, nullptr,
-                                     gpu_->stream ()));
 }
 }

@@ -5,7 +5,6 @@
 #include "models/llama2.h"
 #include "models/decode_plan.h"
 #include "vkl_hip.h"
-#include <chrono>
 #include <stdexcept>
 #include <string.h>
 
@@ -170,10 +169,10 @@ OutputLayer::print_op_cost ()
 
 // ---------------------------------------------------------------------------
 Model::Model (int dev)
-    : dev_ (dev), gpu_ (nullptr), input_command_ (nullptr),
+    : dev_ (dev), input_command_ (nullptr),
       output_command_ (nullptr), input_layer_ (nullptr),
-      output_layer_ (nullptr), vocab_ (0), dim_ (0), ffn_ (0), heads_ (0),
-      maxlen_ (0), wtype_ (Q8_0), fused_decode_ (true), plan_ (nullptr)
+      output_layer_ (nullptr), dim_ (0), ffn_ (0), heads_ (0),
+      wtype_ (Q8_0), plan_ (nullptr)
 {
 }
 
@@ -184,7 +183,7 @@ Model::~Model ()
   delete plan_;
   argmax_.reset ();
   vktoks_ = Tensor ();
-  next_tok_ = Tensor ();
+  release_buffers_ ();
   delete input_layer_;
   delete output_layer_;
   for (auto *block : blocks_)
@@ -384,14 +383,13 @@ Model::set_lastblock_rope_quirk (bool on)
 
 // One pass of the operator chain; returns the fp32 logits tensor [1, 1, V].
 absl::StatusOr<Tensor>
-Model::forward_ (std::vector<uint32_t> const &toks, const size_t offset)
+Model::forward_ (std::vector<uint32_t> const &toks, const size_t offset,
+                 std::vector<uint32_t> const &rows)
 {
-  if (toks.empty ())
-    return absl::InvalidArgumentError ("model called with no tokens");
-  if (offset + toks.size () > maxlen_)
-    return absl::OutOfRangeError (absl::StrFormat (
-        "positions [%zu, %zu) exceed the context length %zu", offset,
-        offset + toks.size (), maxlen_));
+  VKLLAMA_STATUS_OK (check_span_ (toks.size (), offset));
+  // the last block continues with the last row only
+  if (rows.size () != 1 || rows[0] + 1 != toks.size ())
+    return absl::UnimplementedError ("this model gives the logits of the last row of a pass");
   if (vktoks_.width () != toks.size ())
     {
       // the previous buffer may still be read by queued work
@@ -431,39 +429,15 @@ Model::forward_ (std::vector<uint32_t> const &toks, const size_t offset)
   return (*output_layer_) (*X);
 }
 
-absl::StatusOr<std::vector<float> >
-Model::operator() (std::vector<uint32_t> const &toks, const size_t offset)
+StepPlan *
+Model::plan_ptr_ ()
 {
-  if (!plan_)
-    return absl::InternalError ("model used before init()");
-  std::vector<float> buf_logits;
-  if (fused_decode_ && toks.size () == 1 && plan_->usable ())
-    {
-      if (offset + 1 > maxlen_)
-        return absl::OutOfRangeError (absl::StrFormat (
-            "position %zu exceeds the context length %zu", offset, maxlen_));
-      VKLLAMA_STATUS_OK (output_command_->wait ());
-      VKLLAMA_STATUS_OK (plan_->step_host_token (toks[0], offset));
-      buf_logits.resize (vocab_);
-      auto rs = plan_->read_logits (buf_logits.data ());
-      if (absl::IsUnavailable (rs))
-        {
-          // a wait between workgroups gave up; the plan has switched to the
-          // launches that wait for nothing: the same step once more
-          ++decode_recoveries_;
-          VKLLAMA_STATUS_OK (plan_->step_host_token (toks[0], offset));
-          rs = plan_->read_logits (buf_logits.data ());
-        }
-      VKLLAMA_STATUS_OK (rs);
-      return buf_logits;
-    }
-  auto output = forward_ (toks, offset);
-  VKLLAMA_STATUS_OK (output);
-  buf_logits.resize (output->size ());
-  VKLLAMA_STATUS_OK (output_command_->download (*output, buf_logits.data (),
-                                                buf_logits.size ()));
-  VKLLAMA_STATUS_OK (output_command_->end ());
-  VKLLAMA_STATUS_OK (output_command_->submit ());
+  return plan_;
+}
+
+absl::Status
+Model::wait_all_ ()
+{
   VKLLAMA_STATUS_OK (input_command_->wait ());
   for (auto *c : block_commands_)
     VKLLAMA_STATUS_OK (c->wait ());
@@ -474,156 +448,26 @@ Model::operator() (std::vector<uint32_t> const &toks, const size_t offset)
     b->print_op_cost ();
   output_layer_->print_op_cost ();
 #endif
-  return buf_logits;
-}
-
-// the next token from the logits of the last pass: arg-max, or a draw from
-// the top-k / top-p candidates with the uniform number of (seed, position)
-absl::Status
-Model::pick_token_ (uint32_t *dst, size_t position)
-{
-  if (!samp_on_)
-    return plan_->argmax_logits (dst);
-  return plan_->sample_logits (dst, samp_k_, samp_p_, samp_seed_,
-                               (uint32_t)position);
+  return absl::OkStatus ();
 }
 
 absl::Status
-Model::generate_sampled (std::vector<uint32_t> const &prompt, size_t n_gen,
-                         int topk, float topp, uint64_t seed,
-                         std::vector<uint32_t> &out, double *prefill_ms,
-                         double *decode_ms)
+Model::set_option (const std::string &name, int value)
 {
-  if (topp < 0.f && topk < 1)
-    return absl::InvalidArgumentError ("top-k sampling needs k >= 1");
-  if (topp > 1.f)
-    return absl::InvalidArgumentError ("top-p sampling needs p in [0, 1]");
-  samp_on_ = true, samp_k_ = topk, samp_p_ = topp, samp_seed_ = seed;
-  auto s = generate_greedy (prompt, n_gen, out, prefill_ms, decode_ms);
-  samp_on_ = false;
-  return s;
-}
-
-absl::Status
-Model::generate_greedy (std::vector<uint32_t> const &prompt, size_t n_gen,
-                        std::vector<uint32_t> &out, double *prefill_ms,
-                        double *decode_ms)
-{
-  auto s = generate_once_ (prompt, n_gen, out, prefill_ms, decode_ms);
-  if (absl::IsUnavailable (s))
+  if (name == "lastblock_rope_quirk")
+    set_lastblock_rope_quirk (value != 0);
+  else if (name == "operator_attention")
+    set_operator_attention (value != 0);
+  else if (name == "decode_mode")
+    set_decode_mode (value);
+  else if (name == "fuse_attn_wo" || name == "wait_test" || name == "attn_split_min")
     {
-      // a wait between workgroups gave up somewhere in the loop; the plan has
-      // switched to the launches that wait for nothing.  The generation is
-      // repeated from the prompt: KV rows written so far are rewritten with
-      // the same values.
-      ++decode_recoveries_;
-      s = generate_once_ (prompt, n_gen, out, prefill_ms, decode_ms);
-    }
-  return s;
-}
-
-absl::Status
-Model::generate_once_ (std::vector<uint32_t> const &prompt, size_t n_gen,
-                       std::vector<uint32_t> &out, double *prefill_ms,
-                       double *decode_ms)
-{
-  using clock = std::chrono::steady_clock;
-  out.clear ();
-  if (n_gen == 0)
-    return absl::OkStatus ();
-  if (prompt.empty ())
-    return absl::InvalidArgumentError ("empty prompt");
-  if (prompt.size () + n_gen - 1 > maxlen_)
-    return absl::OutOfRangeError (absl::StrFormat (
-        "prompt of %zu + %zu generated tokens exceed the context length %zu",
-        prompt.size (), n_gen, maxlen_));
-  if (!plan_)
-    return absl::InternalError ("model used before init()");
-  // generated ids stay in device memory between steps (the arg-max of step i
-  // is the input token of step i + 1) and are copied out once at the end
-  if (next_tok_.width () < n_gen)
-    {
-      VKLLAMA_STATUS_OK (output_command_->wait ());
-      next_tok_ = Tensor (1, 1, n_gen, gpu_, UINT32, false);
-      VKLLAMA_STATUS_OK (next_tok_.create ());
-    }
-  uint32_t *ids = (uint32_t *)next_tok_.data ();
-  void *s = gpu_->stream ();
-
-  const auto t0 = clock::now ();
-  // prompt pass; arg-max of its fp16 logits becomes ids[0]
-  if (fused_decode_ && prompt.size () == 1 && plan_->usable ())
-    {
-      VKLLAMA_STATUS_OK (plan_->step_host_token (prompt[0], 0));
+      // options of this model's fused decode steps (fields of vkl_decode_model)
+      if (!set_decode_option (name.c_str (), value))
+        return absl::InvalidArgumentError ("option " + name + ": value out of range");
     }
   else
-    {
-      auto logits32 = forward_ (prompt, 0);
-      VKLLAMA_STATUS_OK (logits32);
-      VKLLAMA_STATUS_OK (plan_->adopt_logits (*logits32));
-    }
-  VKLLAMA_STATUS_OK (pick_token_ (ids + 0, prompt.size ()));
-  if (int e = vkl_stream_sync (s))
-    return absl::InternalError (vkl_error_string (e));
-  const auto t1 = clock::now ();
-  size_t n_toks = prompt.size () + 1;
-  size_t i0 = 1;
-  if (fused_decode_ && plan_->usable () && decode_graph_ && n_gen > 1)
-    {
-      // ids[0] is at position prompt.size (); each replay appends one id
-      if (samp_on_)
-        {
-          VKLLAMA_STATUS_OK (plan_->loop_sampled (ids, prompt.size (), n_gen - 1, samp_k_,
-                                                  samp_p_, samp_seed_));
-        }
-      else
-        {
-          VKLLAMA_STATUS_OK (plan_->loop (ids, prompt.size (), n_gen - 1));
-        }
-      i0 = n_gen;
-    }
-  for (size_t i = i0; i < n_gen; ++i, ++n_toks)
-    {
-      if (fused_decode_ && plan_->usable ())
-        {
-          // the step's last launch reduces the arg-max partials into ids[i]
-          VKLLAMA_STATUS_OK (plan_->step_device_token (
-              ids + (i - 1), n_toks - 1, samp_on_ ? nullptr : ids + i));
-          if (samp_on_)
-            VKLLAMA_STATUS_OK (pick_token_ (ids + i, n_toks));
-          continue;
-        }
-      else
-        {
-          uint32_t prev = 0;
-          if (int e = vkl_memcpy_d2h (&prev, ids + (i - 1), sizeof (prev), s))
-            return absl::InternalError (vkl_error_string (e));
-          if (int e = vkl_stream_sync (s))
-            return absl::InternalError (vkl_error_string (e));
-          auto logits32 = forward_ ({ prev }, n_toks - 1);
-          VKLLAMA_STATUS_OK (logits32);
-          VKLLAMA_STATUS_OK (plan_->adopt_logits (*logits32));
-        }
-      VKLLAMA_STATUS_OK (pick_token_ (ids + i, n_toks));
-    }
-  if (int e = vkl_stream_sync (s))
-    return absl::InternalError (vkl_error_string (e));
-  const auto t2 = clock::now ();
-  VKLLAMA_STATUS_OK (plan_->check ());
-  // run deferred work the operator chain may have queued
-  VKLLAMA_STATUS_OK (input_command_->wait ());
-  for (auto *c : block_commands_)
-    VKLLAMA_STATUS_OK (c->wait ());
-  VKLLAMA_STATUS_OK (output_command_->wait ());
-  out.resize (n_gen);
-  if (int e = vkl_memcpy_d2h (out.data (), ids, n_gen * sizeof (uint32_t), s))
-    return absl::InternalError (vkl_error_string (e));
-  if (int e = vkl_stream_sync (s))
-    return absl::InternalError (vkl_error_string (e));
-  if (prefill_ms)
-    *prefill_ms = std::chrono::duration<double, std::milli> (t1 - t0).count ();
-  if (decode_ms)
-    *decode_ms = std::chrono::duration<double, std::milli> (t2 - t1).count ();
+    return CausalModel::set_option (name, value);
   return absl::OkStatus ();
 }
 

@@ -24,6 +24,7 @@ extern "C"{
 }
 // clang-format on
 #include "absl/status/statusor.h"
+#include "models/causal_model.h"
 #include "src/core/command.h"
 #include "src/core/common.h"
 #include "src/core/tensor.h"
@@ -142,22 +143,17 @@ private:
 
 struct DecodePlan; // device pointers of the fused one-token path
 
-class Model
+class Model : public CausalModel
 {
 public:
   Model (int dev = 0);
-  ~Model ();
-  Model (const Model &) = delete;
-  Model &operator= (const Model &) = delete;
+  ~Model () override;
 
   absl::Status init (std::map<std::string, gguf_key> &kv,
                      std::map<std::string, gguf_tensor> &tensors);
 
-  absl::StatusOr<std::vector<float> >
-  operator() (std::vector<uint32_t> const &toks, const size_t offset);
-
+  // (the pass itself, operator() (toks, offset), and generation: CausalModel)
   // ---- additions -----------------------------------------------------------
-  void set_fused_decode (bool on) { fused_decode_ = on; }
   void set_lastblock_rope_quirk (bool on);
   // prompt pass: attention as the reference's three operators (see
   // MultiHeadAttentionV2::set_operator_attention)
@@ -167,25 +163,7 @@ public:
   // options of the fused decode steps: "attn_split_min", "fuse_attn_wo",
   // "wait_test" (DecodePlan::set_option)
   bool set_decode_option (const char *name, int value);
-  // greedy loop replayed from a captured HIP graph (default) or launched
-  // step by step
-  void set_decode_graph (bool on) { decode_graph_ = on; }
-  // Greedy loop of app/llama2_infer.cpp:140-218: prompt at offset 0, then one
-  // token at a time at offset toks.size()-1; n_gen ids are written to out.
-  // The wall-clock times of the two phases are returned in milliseconds.
-  absl::Status generate_greedy (std::vector<uint32_t> const &prompt,
-                                size_t n_gen, std::vector<uint32_t> &out,
-                                double *prefill_ms = nullptr,
-                                double *decode_ms = nullptr);
-  // The same loop with the token drawn on the device from the top-k
-  // (topp < 0) or top-p candidates of every step's logits
-  // (models/samplers.cpp:37-101 as a kernel): logits never leave the device.
-  // The draw at position pos uses the uniform number of (seed, pos).
-  absl::Status generate_sampled (std::vector<uint32_t> const &prompt,
-                                 size_t n_gen, int topk, float topp,
-                                 uint64_t seed, std::vector<uint32_t> &out,
-                                 double *prefill_ms = nullptr,
-                                 double *decode_ms = nullptr);
+  absl::Status set_option (const std::string &name, int value) override;
   // copies one layer's K or V cache, [heads, maxlen, head_dim] fp16 bits
   absl::Status read_kv_cache (size_t layer, bool value,
                               std::vector<uint16_t> &out);
@@ -196,49 +174,31 @@ public:
   // src/ops/update_kv_cache.cpp).
   absl::Status write_kv_cache (size_t layer, bool value, const uint16_t *rows,
                                size_t n);
-  GPUDevice *device () { return gpu_; }
-  size_t vocab_size () const { return vocab_; }
-  size_t context_length () const { return maxlen_; }
   size_t block_count () const { return blocks_.size (); }
-  // algorithmic bytes one decode step at context length L reads and writes
-  size_t decode_step_bytes (size_t L) const;
+  size_t decode_step_bytes (size_t L) const override;
   // algorithmic bytes of one launch of a decode phase (see vkl_decode.h)
   size_t decode_phase_bytes (int kind, size_t L) const;
   absl::Status decode_phase_replay (int kind, size_t pos, int rounds,
                                     double *avg_ms, uint64_t *launches);
-  // how often a decode step or generation was repeated because a wait between
-  // workgroups inside a launch had given up (DecodePlan::check)
-  size_t decode_recoveries () const { return decode_recoveries_; }
 
 private:
   absl::StatusOr<Tensor> forward_ (std::vector<uint32_t> const &toks,
-                                   const size_t offset);
+                                   const size_t offset,
+                                   std::vector<uint32_t> const &rows) override;
+  absl::Status wait_all_ () override;
+  StepPlan *plan_ptr_ () override;
   int dev_;
-  GPUDevice *gpu_;
   Command *input_command_;
   std::vector<Command *> block_commands_;
   Command *output_command_;
   InputLayer *input_layer_;
   OutputLayer *output_layer_;
   std::vector<Llama2Block *> blocks_;
-  size_t vocab_, dim_, ffn_, heads_, maxlen_;
+  size_t dim_, ffn_, heads_;
   DType wtype_;
-  bool fused_decode_;
   Tensor vktoks_;
-  Tensor next_tok_;
   std::unique_ptr<ArgMax> argmax_;
   DecodePlan *plan_;
-  bool decode_graph_ = true;
-  // sampling on the device during generate_*(): off = arg-max
-  bool samp_on_ = false;
-  int samp_k_ = 1;
-  float samp_p_ = -1.f;
-  uint64_t samp_seed_ = 0;
-  size_t decode_recoveries_ = 0;
-  absl::Status pick_token_ (uint32_t *dst, size_t position);
-  absl::Status generate_once_ (std::vector<uint32_t> const &prompt, size_t n_gen,
-                               std::vector<uint32_t> &out, double *prefill_ms,
-                               double *decode_ms);
 };
 
 }

@@ -38,6 +38,7 @@ typedef enum : int
   UINT32,
   INT8,
   Q8_0, // block-wise quantize
+  BF16,
 } DType;
 
 struct ShapeConstant

@@ -12,7 +12,8 @@ get_dtype_property (const DType dtype)
   switch (dtype)
     {
     case FP32: return { 1, sizeof (float) };
-    case FP16: return { 1, sizeof (uint16_t) };
+    case FP16:
+    case BF16: return { 1, sizeof (uint16_t) };
     case UINT32: return { 1, sizeof (uint32_t) };
     case INT8: return { 1, sizeof (int8_t) };
     case Q8_0: return { 32, 34 };
@@ -102,7 +103,8 @@ Tensor::elem_bytes () const
     {
     case FP32: return sizeof (float);
     case UINT32: return sizeof (uint32_t);
-    case FP16: return sizeof (uint16_t);
+    case FP16:
+    case BF16: return sizeof (uint16_t);
     case INT8:
     case Q8_0: return sizeof (int8_t);
     }
