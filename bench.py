@@ -168,8 +168,106 @@ def bench_single_matmul(args):
                          "sample": "%d calls of the oracle's matmul on the first matrix" % n_cpu}}))
 
 
+def fazinex_config(dim, n_layers, heads, kv_heads, head, rank, ffn, vocab):
+    """Layers alternate between shared key/value attention and latent attention."""
+    mlp = {"kind": "dense", "ff": ffn}
+    shared = {"type": "attention", "mlp": mlp,
+              "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": head, "vdim": head, "scale": head ** -0.5,
+                        "q_temp": {"coef": 0.1, "every": 512}}}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": heads, "dim": head, "vdim": head, "kv_rank": rank, "scale": head ** -0.5}}
+    return {"architecture": "Fazinex", "vocab": vocab, "width": dim, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "loop": None, "layers": [shared if i % 2 == 0 else latent for i in range(n_layers)]}
+
+
+def fazinex_weights(cfg, seed):
+    """name -> bf16 bits of N(0, 0.02) matrices and unit norms"""
+    from vkllama_amd import model as M
+    w, V = cfg["width"], cfg["vocab"]
+    shapes = [("embed", (V, w)), ("embed.norm", (w,)), ("final.norm", (w,))]
+    for i, L in enumerate(cfg["layers"]):
+        m, p, f = L["mixer"], "l%d." % i, L["mlp"]["ff"]
+        H = m["heads"]
+        shapes += [(p + "norm1", (w,)), (p + "mix.q", (H * m["dim"], w)), (p + "mix.o", (w, H * m["vdim"])),
+                   (p + "mlp.up", (f, w)), (p + "mlp.down", (w, f))]
+        if L["type"] == "attention":
+            shapes += [(p + "mix.k", (m["kv_heads"] * m["dim"], w))]
+        else:
+            r = m["kv_rank"]
+            shapes += [(p + "mix.dkv", (r, w)), (p + "mix.dkv.norm", (r,)), (p + "mix.uk", (H * m["dim"], r)),
+                       (p + "mix.uv", (H * m["vdim"], r)), (p + "mix.g", (H, w))]
+    out = {}
+    for i, (name, sh) in enumerate(shapes):
+        a = np.full(sh, 0x3F80, np.uint16)
+        if len(sh) == 2:
+            M.lib().vkl_synth_normal_bf16(seed + i, a.size, 0.02, a.ctypes.data)
+        out[name] = a
+    return out
+
+
+# --design fazinex: (width, layers, heads, key/value heads, head size, latent, ff), each beside a Llama-2-shaped model
+# with FP16 weights of the same width, heads, ff and layer count
+DESIGN_SIZES = {"4096": (4096, 8, 32, 8, 128, 512, 11008), "2048": (2048, 8, 16, 4, 128, 512, 5504),
+                "5120": (5120, 6, 40, 8, 128, 512, 13824)}
+
+
+def bench_design(args):
+    """Prompt pass and greedy decoding of a Fazinex model and of a Llama-2-shaped FP16 model of equal size, random
+    weights, one JSON line per size.  The two are timed in turn, each figure is the best of the repetitions."""
+    from vkllama_amd import model as M
+    vocab, steps = 32000, args.steps
+    for name in args.design_sizes.split(","):
+        dim, layers, heads, kvh, head, rank, ffn = DESIGN_SIZES[name]
+        prompts = [int(n) for n in args.design_prompts.split(",")]
+        maxlen = max(prompts) + steps + 8
+        fcfg = fazinex_config(dim, layers, heads, kvh, head, rank, ffn, vocab)
+        models = {}
+        if args.design_only != "llama2":
+            w = fazinex_weights(fcfg, args.seed)
+            models["fazinex"] = M.CausalModel.create(fcfg, w, "bfloat16", maxlen)
+            del w
+        if args.design_only != "fazinex":
+            lcfg = dict(dim=dim, n_layers=layers, n_heads=heads, ffn=ffn, vocab=vocab, maxlen=maxlen, eps=1e-5, wtype=1)
+            w = M.synth_weights(lcfg, seed=args.seed)
+            models["llama2-f16"] = M.Llama2(lcfg, w)
+            del w
+        rng = np.random.default_rng(args.seed)
+        rows = []
+        for n in prompts:
+            prompt = rng.integers(3, vocab, n).astype(np.uint32)
+            best = {}
+            for m in models.values():
+                m.set_option("decode_graph", args.decode_graph)
+                m.generate_greedy(prompt, args.warmup + 1)
+            for _ in range(args.design_repeats):
+                for k, m in models.items():
+                    _, pre, dec = m.generate_greedy(prompt, steps + 1)
+                    b = best.setdefault(k, [pre, dec])
+                    b[0], b[1] = min(b[0], pre), min(b[1], dec)
+            for k, m in models.items():
+                pre, dec = best[k]
+                nbytes = m.decode_step_bytes(n + steps // 2)
+                rows.append({"model": k, "prompt": n, "prefill_tokens_per_second": round(n / pre * 1e3, 1),
+                             "decode_tokens_per_second": round(steps / dec * 1e3, 2),
+                             "decode_bytes_per_step": int(nbytes),
+                             "decode_gbs": round(nbytes * steps / dec / 1e6, 1),
+                             "decode_frac_of_hbm_peak": round(nbytes * steps / dec / 1e6 / HBM_PEAK_GBS, 4)})
+        for m in models.values():
+            m.close()
+        print(json.dumps({"metric": "fazinex_beside_llama2_f16", "size": name, "steps": steps, "n_gpus": 1,
+                          "config": {"width": dim, "layers": layers, "heads": heads, "kv_heads": kvh, "head": head,
+                                     "latent": rank, "ff": ffn, "vocab": vocab},
+                          "data": "synthetic: random-init N(0,0.02) weights, random prompt ids", "rows": rows}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--design", choices=("fazinex",),
+                    help="instead of the workload: this model design beside a Llama-2-shaped FP16 model of equal size")
+    ap.add_argument("--design-sizes", default="4096,2048", help="of " + ", ".join(sorted(DESIGN_SIZES)))
+    ap.add_argument("--design-prompts", default="32,2048", help="prompt lengths")
+    ap.add_argument("--design-repeats", type=int, default=3)
+    ap.add_argument("--design-only", choices=("fazinex", "llama2"), help="one side alone (for runs under a profiler)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)
@@ -190,6 +288,8 @@ def main():
         sys.exit("bench.py: this build runs on ONE GPU (batch-1 decode is a single dependency chain and "
                  "would shard by tensor parallelism, which is not built); got --gpus %d" % args.gpus)
 
+    if args.design:
+        return bench_design(args)
     if args.workload == "matmul-q8_0-4096":
         return bench_single_matmul(args)
 

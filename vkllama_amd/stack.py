@@ -1,0 +1,47 @@
+"""ctypes binding of the operators in include/vkl_stack.h (libvkllama_hip.so).
+The one-token step of such a stack is driven by the C++ model classes."""
+import ctypes as C
+
+from . import capi
+
+F32, BF16 = 0, 30
+vp, sz, u32, i32, f32 = C.c_void_p, C.c_size_t, C.c_uint32, C.c_int, C.c_float
+
+
+class OutSeg(C.Structure):
+    """vkl_out_seg"""
+    _fields_ = [("n0", i32), ("n", i32), ("y", vp), ("ys", sz), ("type", i32), ("act", i32), ("residual", vp),
+                ("cap", f32)]
+
+
+SIGNATURES = {
+    "vkl_project_bf16w": (i32, [vp, i32, sz, vp, i32, i32, i32, C.POINTER(OutSeg), i32, vp]),
+    "vkl_embed_norm_bf16": (i32, [vp, u32, i32, i32, vp, u32, vp, f32, vp, sz, vp]),
+    "vkl_rmsnorm_f32": (i32, [vp, sz, vp, i32, i32, vp, f32, vp, i32, sz, i32, vp]),
+    "vkl_attn_prefill_causal_bf16": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, sz, sz, sz, f32, f32, i32, vp, sz, vp, sz,
+                                           vp]),
+    "vkl_attn_rows": (i32, [vp, i32, sz, vp, i32, sz, i32, i32, i32, i32, u32, f32, f32, i32, vp, i32, sz, vp, vp]),
+    "vkl_attn_rows_scratch_bytes": (sz, [i32, i32, i32, i32]),
+    "vkl_head_matvec": (i32, [vp, i32, i32, i32, vp, i32, sz, sz, vp, i32, sz, sz, vp, sz, i32, vp]),
+    "vkl_stack_scratch_bytes": (sz, [vp]),
+    "vkl_stack_supported": (i32, [vp]),
+    "vkl_stack_step": (i32, [vp, vp, u32, vp, vp, vp]),
+    "vkl_stack_loop": (i32, [vp, vp, u32, i32, vp, vp]),
+    "vkl_stack_loop_sampled": (i32, [vp, vp, u32, i32, vp, i32, f32, C.c_uint64, vp]),
+    "vkl_stack_release": (None, [vp]),
+}
+
+_lib = None
+
+
+def lib():
+    global _lib
+    if _lib is None:
+        capi.lib()
+        _lib = capi.load_library(capi.HIP_LIB_PATH, SIGNATURES)
+    return _lib
+
+
+def segments(items):
+    """items: (n0, n, y, ys, type, act, residual, cap) each"""
+    return (OutSeg * len(items))(*[OutSeg(*it) for it in items])

@@ -1,19 +1,18 @@
-"""Replays a trace: feeds given token ids through a model step by step and writes
-logits.  Nothing is sampled; every step is a pass of the model over the tokens
-it brings, on the cache that earlier steps left.
+"""Replays recorded token ids: runs them through a model step by step, without
+sampling, and writes the logits that the recording asks for.  Every step is an
+ordinary pass of the model over new tokens, on the cache earlier steps left.
 
-    bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
+    bin/trace_run --model FOLDER --dtype float32 --out LOGITS --max-tokens 4096 < STEPS
 
-Steps come on standard input, one JSON object a line:
+Standard input holds one JSON object per line, for instance
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 7, "entries": [{"id": "chat-2", "tokens": [311, 40], "want": [1]}], "end": ["chat-2"]}
 
-An entry brings a request's next tokens and names the places among them whose
-logits are wanted; "end" lists the requests that are finished.  The logits of a
-step go to OUT/<step>.f32 (little-endian floats [wanted, vocab], no file if
-nothing is wanted), then a line "done <step>" is printed.  A model holds one
-sequence: requests follow one another, and a request that ends gives its cache
-rows to the next.
+"tokens" continues the request "id"; "want" numbers the tokens of this entry
+whose logits go to LOGITS/<step>.f32 (raw little-endian floats, one row of the
+vocabulary each; no file without any).  "done <step>" on standard output follows
+every step.  "end" closes requests.  A model holds one sequence, so requests
+follow one another, each on the cache rows of the one before.
 """
 import argparse
 import json
