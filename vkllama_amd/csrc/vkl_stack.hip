@@ -76,7 +76,7 @@ store_elem (void *p, int type, size_t i, float v)
     stg ((uint16_t *)p + i, f2bf (v));
 }
 
-// sum over a workgroup of 256 or 512 threads; red: 8 floats of LDS
+// sum over a workgroup of up to 1024 threads; red: a float of LDS per wave
 __device__ __forceinline__ float
 group_sum (float v, float *red)
 {
@@ -107,29 +107,66 @@ struct EmbedArgs
   size_t os;
 };
 
-__global__ __launch_bounds__ (256) void
+// one workgroup per token; a thread keeps its values of the row in registers
+// (rows of up to 16384 values; wider ones are read twice)
+__global__ __launch_bounds__ (1024) void
 embed_norm_kernel (const EmbedArgs a)
 {
-  __shared__ float red[8];
+  __shared__ float red[16];
+  constexpr int NV = 2; // 16-byte loads per thread
   const uint32_t i = blockIdx.x;
   uint32_t id = ldg (a.toks + (a.loop ? ldg (a.loop) : i));
   id = id < a.VH ? id : 0;
   const uint16_t *row = a.table + (size_t)id * a.K;
+  float *out = a.out + (size_t)i * a.os;
+  const int tid = threadIdx.x;
+  if ((a.K % 8) == 0 && a.W <= NV * 8192 && ((uintptr_t)a.table % 16) == 0)
+    {
+      float v[NV][8], ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+        {
+          const int c = (tid + j * 1024) * 8;
+          widen8 (ldg4 (row + min (c, a.K - 8)), v[j]);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            if (c + e < a.W)
+              ss = __builtin_fmaf (v[j][e], v[j][e], ss);
+        }
+      float w[NV][8];
+      if (a.w)
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            w[j][e] = ldg (a.w + min ((tid + j * 1024) * 8 + e, a.W - 1));
+      const float alpha = a.w ? 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps) : 1.f;
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          {
+            const int c = (tid + j * 1024) * 8 + e;
+            if (c < a.W)
+              stg (out + c, a.w ? v[j][e] * alpha * w[j][e] : v[j][e]);
+          }
+      return;
+    }
   float alpha = 1.f;
   if (a.w)
     {
       float ss = 0.f;
-      for (int c = threadIdx.x; c < a.W; c += 256)
+      for (int c = tid; c < a.W; c += 1024)
         {
           const float v = bf2f (ldg (row + c));
           ss = __builtin_fmaf (v, v, ss);
         }
       alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
     }
-  for (int c = threadIdx.x; c < a.W; c += 256)
+  for (int c = tid; c < a.W; c += 1024)
     {
       const float v = bf2f (ldg (row + c));
-      stg (a.out + (size_t)i * a.os + c, a.w ? v * alpha * ldg (a.w + c) : v);
+      stg (out + c, a.w ? v * alpha * ldg (a.w + c) : v);
     }
 }
 
@@ -146,20 +183,58 @@ struct NormArgs
   size_t os;
 };
 
+// one workgroup per row; NV 16-byte loads per thread keep the row in registers,
+// 0: a row of any length and alignment, read twice
+template <int NV>
 __global__ __launch_bounds__ (256) void
 rmsnorm_f32_kernel (const NormArgs a)
 {
   __shared__ float red[8];
   const size_t r = a.rows ? ldg (a.rows + blockIdx.x) : blockIdx.x;
   const float *x = a.x + r * a.xs;
+  const int tid = threadIdx.x;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < a.W; c += 256)
+  if constexpr (NV > 0)
+    {
+      float4 v[NV];
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+        {
+          // (W is a multiple of 4 here: a load is all inside or all padding)
+          const int c = (tid + j * 256) * 4;
+          v[j] = __builtin_bit_cast (float4, ldg4 (x + min (c, a.W - 4)));
+          if (c >= a.W)
+            v[j] = make_float4 (0.f, 0.f, 0.f, 0.f);
+          ss = __builtin_fmaf (v[j].x, v[j].x, ss), ss = __builtin_fmaf (v[j].y, v[j].y, ss);
+          ss = __builtin_fmaf (v[j].z, v[j].z, ss), ss = __builtin_fmaf (v[j].w, v[j].w, ss);
+        }
+      const float alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+        {
+          const int c = (tid + j * 256) * 4;
+          if (c >= a.Wp)
+            continue;
+          const float4 w = __builtin_bit_cast (float4, ldg4 (a.w + min (c, a.W - 4)));
+          const float o[4] = { v[j].x * alpha * w.x, v[j].y * alpha * w.y, v[j].z * alpha * w.z, v[j].w * alpha * w.w };
+          const size_t at = blockIdx.x * a.os + c;
+          if (a.otype == VKL_TYPE_F32)
+            stg ((vkl_u32x4 *)((float *)a.out + at), vkl_u32x4{ __float_as_uint (o[0]), __float_as_uint (o[1]),
+                                                              __float_as_uint (o[2]), __float_as_uint (o[3]) });
+          else
+            stg ((unsigned long long *)((uint16_t *)a.out + at),
+                 (unsigned long long)f2bf (o[0]) | ((unsigned long long)f2bf (o[1]) << 16)
+                     | ((unsigned long long)f2bf (o[2]) << 32) | ((unsigned long long)f2bf (o[3]) << 48));
+        }
+      return;
+    }
+  for (int c = tid; c < a.W; c += 256)
     {
       const float v = ldg (x + c);
       ss = __builtin_fmaf (v, v, ss);
     }
   const float alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps);
-  for (int c = threadIdx.x; c < a.Wp; c += 256)
+  for (int c = tid; c < a.Wp; c += 256)
     store_elem (a.out, a.otype, blockIdx.x * a.os + c, c < a.W ? ldg (x + c) * alpha * ldg (a.w + c) : 0.f);
 }
 
@@ -168,7 +243,7 @@ rmsnorm_f32_kernel (const NormArgs a)
 // ---------------------------------------------------------------------------
 constexpr int kRowThreads = 256;
 constexpr int kRowUnroll = 4;
-constexpr int kRowSplits = 64;
+constexpr int kRowSplits = 32;  // parts a context is cut into at most
 constexpr int kRowTarget = 512; // workgroups a launch aims for
 constexpr float kNoKey = -1.0e30f;
 
@@ -188,8 +263,17 @@ struct RowAttnArgs
   size_t os;
   int nsplit;
   float *pm, *pl, *pacc; // parts of a split context: [S][G*tiles][nsplit][HT] (x D)
-  uint32_t *cnt;         // [S][G*tiles]
+  uint32_t *cnt;         // [S][G*tiles]; null: the parts stay, the next launch combines them
 };
+
+// how a context of L positions is cut: parts of `chunk` rows, a multiple of the
+// rows a workgroup takes at a time
+__device__ __forceinline__ int
+row_chunk (int L, int nsplit, int step)
+{
+  const int c = (L + nsplit - 1) / nsplit;
+  return (c + step - 1) / step * step;
+}
 
 template <int LPR>
 __device__ __forceinline__ float
@@ -246,6 +330,24 @@ template <> struct RowVec<float>
   }
 };
 
+// 8 neighbouring values in either type
+__device__ __forceinline__ void
+load8 (const void *p, int type, size_t i, float (&f)[8])
+{
+  if (type == VKL_TYPE_F32)
+    {
+      RowVec<float> v;
+      v.load ((const float *)p + i);
+      v.get (f);
+    }
+  else
+    {
+      RowVec<uint16_t> v;
+      v.load ((const uint16_t *)p + i);
+      v.get (f);
+    }
+}
+
 // LPR lanes share a row, NCH chunks of 8 values per lane; HT query heads per
 // workgroup.  Every group of LPR lanes walks rows of its own with a running
 // maximum; the groups' results meet in LDS at the end.
@@ -263,8 +365,7 @@ attn_rows_kernel (const RowAttnArgs a)
   const int g = gt / a.tiles, t = gt - g * a.tiles;
   const uint32_t pos = a.pos.get () + (uint32_t)s;
   const int L = (int)pos + 1;
-  int chunk = (L + a.nsplit - 1) / a.nsplit;
-  chunk = (chunk + STEP - 1) / STEP * STEP;
+  const int chunk = row_chunk (L, a.nsplit, STEP);
   const int active = (L + chunk - 1) / chunk;
   const int c = blockIdx.x;
   if (c >= active)
@@ -280,6 +381,17 @@ attn_rows_kernel (const RowAttnArgs a)
   for (int n = 0; n < NCH; ++n)
     cc[n] = min (col[n], a.D - 8);
 
+  // the first rows travel while the queries are fetched
+  RowVec<CT> nx[U][NCH];
+  auto issue = [&] (int lb) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int n = 0; n < NCH; ++n)
+        nx[u][n].load (base + (size_t)min (lb + (u * 4 + wave) * RPW + grp, l1 - 1) * a.rs + cc[n]);
+  };
+  issue (l0);
+  __builtin_amdgcn_sched_barrier (0);
   const int h0 = g * a.rep + t * HT;
   float q[HT][NCH * 8];
   {
@@ -292,9 +404,13 @@ attn_rows_kernel (const RowAttnArgs a)
         const size_t qo = (size_t)s * a.qs + (size_t)(g * a.rep + min (t * HT + h, a.rep - 1)) * a.D;
 #pragma unroll
         for (int n = 0; n < NCH; ++n)
+          {
+            float v[8];
+            load8 (a.q, a.qtype, qo + cc[n], v);
 #pragma unroll
-          for (int e = 0; e < 8; ++e)
-            q[h][n * 8 + e] = col[n] < a.D ? load_elem (a.q, a.qtype, qo + cc[n] + e) * f : 0.f;
+            for (int e = 0; e < 8; ++e)
+              q[h][n * 8 + e] = col[n] < a.D ? v[e] * f : 0.f;
+          }
       }
   }
   float m[HT], l[HT], acc[HT][NCH * 8];
@@ -307,15 +423,6 @@ attn_rows_kernel (const RowAttnArgs a)
         acc[h][e] = 0.f;
     }
 
-  RowVec<CT> nx[U][NCH];
-  auto issue = [&] (int lb) {
-#pragma unroll
-    for (int u = 0; u < U; ++u)
-#pragma unroll
-      for (int n = 0; n < NCH; ++n)
-        nx[u][n].load (base + (size_t)min (lb + (u * 4 + wave) * RPW + grp, l1 - 1) * a.rs + cc[n]);
-  };
-  issue (l0);
   for (int lb = l0; lb < l1; lb += STEP)
     {
       float row[U][NCH * 8];
@@ -377,6 +484,7 @@ attn_rows_kernel (const RowAttnArgs a)
   for (int h = 0; h < HT; ++h)
     {
       float v = kNoKey;
+#pragma unroll
       for (int i = 0; i < NS; ++i)
         v = fmaxf (v, sm[i][h]);
       M[h] = v;
@@ -396,9 +504,12 @@ attn_rows_kernel (const RowAttnArgs a)
     {
       const int h = o / a.D, d = o - h * a.D;
       float v = 0.f, S = 0.f;
+#pragma unroll
       for (int i = 0; i < NS; ++i)
         v += lds_rows[(i * HT + h) * DA + d];
-      if (active == 1)
+      if (!a.cnt)
+        stg (a.pacc + ((pbase + c) * HT + h) * a.D + d, v);
+      else if (active == 1)
         {
           for (int i = 0; i < NS; ++i)
             S += sl[i][h];
@@ -410,16 +521,26 @@ attn_rows_kernel (const RowAttnArgs a)
           st_coherent_u32 ((uint32_t *)a.pacc + ((pbase + c) * HT + h) * a.D + d, __float_as_uint (v));
         }
     }
-  if (active == 1)
+  if (a.cnt && active == 1)
     return;
   if (tid < nh)
     {
       float S = 0.f, mm = kNoKey;
       for (int i = 0; i < NS; ++i)
         S += sl[i][tid], mm = fmaxf (mm, sm[i][tid]);
-      st_coherent_u32 ((uint32_t *)a.pm + (pbase + c) * HT + tid, __float_as_uint (mm));
-      st_coherent_u32 ((uint32_t *)a.pl + (pbase + c) * HT + tid, __float_as_uint (S));
+      if (!a.cnt)
+        {
+          stg (a.pm + (pbase + c) * HT + tid, mm);
+          stg (a.pl + (pbase + c) * HT + tid, S);
+        }
+      else
+        {
+          st_coherent_u32 ((uint32_t *)a.pm + (pbase + c) * HT + tid, __float_as_uint (mm));
+          st_coherent_u32 ((uint32_t *)a.pl + (pbase + c) * HT + tid, __float_as_uint (S));
+        }
     }
+  if (!a.cnt)
+    return;
   // count in once this workgroup's parts are in memory; the last one combines
   __builtin_amdgcn_s_waitcnt (0);
   __syncthreads ();
@@ -435,43 +556,71 @@ attn_rows_kernel (const RowAttnArgs a)
   __syncthreads ();
   if (last_s == 0u)
     return;
-  for (int i = tid; i < nh * active; i += kRowThreads)
-    {
-      const int h = i / active, p = i - h * active;
-      wgt[h][p] = __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pm + (pbase + p) * HT + h));
-    }
+  // what other workgroups wrote through is now read with ordinary loads
+  __builtin_amdgcn_fence (__ATOMIC_ACQUIRE, "agent");
+  // maxima and sums, one part per thread, and the first values are requested
+  // together: four neighbouring values per thread, the parts in two halves of the
+  // workgroup
+  static_assert (HT * kRowSplits <= kRowThreads, "one part per thread");
+  float *pls = lds_rows; // [HT][kRowSplits], the rows' area is free
+  float *sums = &sl[0][0]; // [nh], free as well
+  const int half = tid >> 7, q4 = a.D / 4, outs = nh * q4;
+  float4 pv[kRowSplits / 2];
+  auto request = [&] (int o0) {
+    const int oc = min (o0 + (tid & 127), outs - 1), h = oc / q4;
+    const float *src = a.pacc + (pbase * HT + h) * a.D + (oc - h * q4) * 4;
+#pragma unroll
+    for (int j = 0; j < kRowSplits / 2; ++j)
+      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (2 * j + half, active - 1) * HT * a.D));
+  };
+  const int th = min (tid / kRowSplits, HT - 1), tp = tid % kRowSplits;
+  const float pmv = ldg (a.pm + (pbase + min (tp, active - 1)) * HT + th);
+  const float plv = ldg (a.pl + (pbase + min (tp, active - 1)) * HT + th);
+  request (0);
+  if (tid < HT * kRowSplits)
+    wgt[th][tp] = pmv, pls[tid] = plv;
   __syncthreads ();
-  float *sums = &sl[0][0]; // [nh], free by now
   if (tid < nh)
     {
       float mm = kNoKey, S = 0.f;
       for (int p = 0; p < active; ++p)
         mm = fmaxf (mm, wgt[tid][p]);
-      for (int p = 0; p < active; ++p)
+#pragma unroll 8
+      for (int p = 0; p < kRowSplits; ++p)
         {
-          const float f = expf (wgt[tid][p] - mm);
+          const float f = p < active ? expf (wgt[tid][p] - mm) : 0.f;
           wgt[tid][p] = f;
-          S += f * __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pl + (pbase + p) * HT + tid));
+          S += f * pls[tid * kRowSplits + p];
         }
       sums[tid] = S;
     }
   __syncthreads ();
-  for (int o = tid; o < nh * a.D; o += kRowThreads)
+  float4 *swap = (float4 *)(lds_rows + HT * kRowSplits);
+  for (int o0 = 0; o0 < outs; o0 += kRowThreads / 2)
     {
-      const int h = o / a.D, d = o - h * a.D;
-      float v = 0.f;
-      for (int p0 = 0; p0 < active; p0 += 8)
+      const int o = o0 + (tid & 127), oc = min (o, outs - 1), h = oc / q4, d = (oc - h * q4) * 4;
+      float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int j = 0; j < kRowSplits / 2; ++j)
         {
-          float pv[8];
-#pragma unroll
-          for (int j = 0; j < 8; ++j)
-            pv[j] = __uint_as_float (ld_coherent_u32 (
-                (const uint32_t *)a.pacc + ((pbase + min (p0 + j, active - 1)) * HT + h) * a.D + d));
-#pragma unroll
-          for (int j = 0; j < 8; ++j)
-            v += p0 + j < active ? wgt[h][min (p0 + j, active - 1)] * pv[j] : 0.f;
+          const float f = wgt[h][2 * j + half];
+          v.x = __builtin_fmaf (f, pv[j].x, v.x), v.y = __builtin_fmaf (f, pv[j].y, v.y);
+          v.z = __builtin_fmaf (f, pv[j].z, v.z), v.w = __builtin_fmaf (f, pv[j].w, v.w);
         }
-      store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d, v / sums[h]);
+      if (half)
+        swap[tid & 127] = v;
+      if (o0 + kRowThreads / 2 < outs)
+        request (o0 + kRowThreads / 2);
+      __syncthreads ();
+      if (!half && o < outs)
+        {
+          const float4 w = swap[tid];
+          const float inv = 1.0f / sums[h], r[4] = { v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w };
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d + e, r[e] * inv);
+        }
+      __syncthreads ();
     }
 }
 
@@ -479,7 +628,7 @@ attn_rows_kernel (const RowAttnArgs a)
 int
 row_head_tile (int rep, int D)
 {
-  const int cap = D > 512 ? 4 : 8;
+  const int cap = D > 256 ? 4 : 8;
   int ht = 1;
   while (ht * 2 <= cap && ht < rep)
     ht *= 2;
@@ -527,7 +676,7 @@ launch_rows_ht (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
     case 2: return launch_rows_k<CT, LPR, NCH, 2> (a, grid, s);
     case 4: return launch_rows_k<CT, LPR, NCH, 4> (a, grid, s);
     default:
-      if constexpr (NCH == 1)
+      if constexpr (LPR <= 32)
         return launch_rows_k<CT, LPR, NCH, 8> (a, grid, s);
       return (int)hipErrorInvalidValue;
     }
@@ -561,13 +710,28 @@ size_t
 row_scratch_bytes (int H, int G, int D, int S)
 {
   const RowPlan p = row_plan (H, G, D, S);
-  return kRowCounterBytes + (p.nsplit > 1 ? p.parts * (2 + (size_t)D) * sizeof (float) : 0) + 256;
+  return kRowCounterBytes + p.parts * (2 + (size_t)D) * sizeof (float) + 256;
+}
+
+// the parts of a launch that leaves them to the next one
+struct RowParts
+{
+  const float *pm, *pl, *pacc;
+  int nsplit, ht, tiles, step; // tiles: head tiles of ht heads each (one group)
+};
+
+// rows a workgroup takes at a time (STEP of the kernel)
+int
+row_step (int D)
+{
+  const int lpr = D <= 32 ? 4 : D <= 64 ? 8 : D <= 128 ? 16 : D <= 256 ? 32 : 64;
+  return 4 * (64 / lpr) * kRowUnroll;
 }
 
 int
 rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype, size_t rs, int H, int G, int D,
                 int S, StepPos pos, float scale, float tcoef, int tevery, void *out, int otype, size_t os,
-                void *scratch, hipStream_t s)
+                void *scratch, RowParts *parts, hipStream_t s)
 {
   const RowPlan p = row_plan (H, G, D, S);
   RowAttnArgs a = {};
@@ -575,10 +739,12 @@ rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype
   a.G = G, a.D = D, a.rep = H / G, a.tiles = p.tiles;
   a.pos = pos, a.scale = scale, a.tcoef = tcoef, a.tevery = tevery;
   a.out = out, a.otype = otype, a.os = os, a.nsplit = p.nsplit;
-  a.cnt = (uint32_t *)scratch;
+  a.cnt = parts ? nullptr : (uint32_t *)scratch;
   a.pm = (float *)((uint8_t *)scratch + kRowCounterBytes);
   a.pl = a.pm + p.parts;
   a.pacc = a.pl + p.parts;
+  if (parts)
+    *parts = { a.pm, a.pl, a.pacc, p.nsplit, p.ht, p.tiles, row_step (D) };
   const dim3 grid ((unsigned)p.nsplit, (unsigned)(G * p.tiles), (unsigned)S);
   return ctype == VKL_TYPE_F32 ? launch_rows<float> (a, p.ht, grid, s) : launch_rows<uint16_t> (a, p.ht, grid, s);
 }
@@ -608,15 +774,19 @@ struct HeadArgs
   void *ncache;
   int ntype;
   StepPos pos;
+  // x as the parts an attention launch left (one token): combined here
+  RowParts parts;
 };
 
 constexpr int kHeadRows = 4; // row groups per wave
 
-template <int LPR>
+template <int LPR, bool PARTS>
 __global__ __launch_bounds__ (256) void
 head_matvec_kernel (const HeadArgs a)
 {
   __shared__ float red[8];
+  __shared__ __align__ (16) float xc[PARTS ? 1024 : 4];
+  __shared__ float wgt[kRowSplits];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   if ((int)blockIdx.x == a.heads * a.bph)
     {
@@ -638,6 +808,49 @@ head_matvec_kernel (const HeadArgs a)
   const int r0 = (b * 4 + wave) * RPW * kHeadRows + grp; // rows r0 + i * RPW
   const uint16_t *w = a.w + (size_t)h * a.R * a.K;
   const size_t xo = (size_t)s * a.xs + (size_t)h * a.xh;
+  if constexpr (PARTS)
+    {
+      const RowParts &p = a.parts;
+      const int L = (int)a.pos.get () + 1;
+      const int chunk = row_chunk (L, p.nsplit, p.step), active = (L + chunk - 1) / chunk;
+      const size_t pbase = (size_t)(h / p.ht) * p.nsplit;
+      const int hh = h % p.ht;
+      const int i = lane % kRowSplits, ic = min (i, active - 1);
+      const float mi = ldg (p.pm + (pbase + ic) * p.ht + hh), li = ldg (p.pl + (pbase + ic) * p.ht + hh);
+      const float M = wave_max (mi);
+      const float f = i < active ? expf (mi - M) : 0.f;
+      const float S = wave_sum (f * li) * ((float)kRowSplits / 64.f); // (every part stands in 64 / kRowSplits lanes)
+      if (tid < kRowSplits)
+        wgt[tid] = f / S;
+      __syncthreads ();
+      const int half = tid >> 7;
+      for (int k0 = 0; k0 < a.K; k0 += 512)
+        {
+          // four neighbouring values per thread, the parts in two halves of the workgroup
+          const int k = k0 + (tid & 127) * 4, kc = min (k, a.K - 4);
+          const float *src = p.pacc + (pbase * p.ht + hh) * a.K + kc;
+          float4 pv[kRowSplits / 2], v = make_float4 (0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+          for (int j = 0; j < kRowSplits / 2; ++j)
+            pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (2 * j + half, active - 1) * p.ht * a.K));
+#pragma unroll
+          for (int j = 0; j < kRowSplits / 2; ++j)
+            {
+              const float g = wgt[2 * j + half];
+              v.x = __builtin_fmaf (g, pv[j].x, v.x), v.y = __builtin_fmaf (g, pv[j].y, v.y);
+              v.z = __builtin_fmaf (g, pv[j].z, v.z), v.w = __builtin_fmaf (g, pv[j].w, v.w);
+            }
+          if (half && k < a.K)
+            *(float4 *)(xc + k) = v;
+          __syncthreads ();
+          if (!half && k < a.K)
+            {
+              const float4 w = *(const float4 *)(xc + k);
+              *(float4 *)(xc + k) = make_float4 (v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+            }
+        }
+      __syncthreads ();
+    }
   float acc[kHeadRows] = {};
   for (int k0 = 0; k0 < a.K; k0 += LPR * 8)
     {
@@ -647,18 +860,14 @@ head_matvec_kernel (const HeadArgs a)
       for (int i = 0; i < kHeadRows; ++i)
         wv[i] = ldg4 (w + (size_t)min (r0 + i * RPW, a.R - 1) * a.K + kc);
       float xv[8];
-      if (a.xtype == VKL_TYPE_F32)
+      if constexpr (PARTS)
         {
-          RowVec<float> v;
-          v.load ((const float *)a.x + xo + kc);
-          v.get (xv);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            xv[e] = xc[kc + e];
         }
       else
-        {
-          RowVec<uint16_t> v;
-          v.load ((const uint16_t *)a.x + xo + kc);
-          v.get (xv);
-        }
+        load8 (a.x, a.xtype, xo + kc, xv);
       if (k >= a.K)
 #pragma unroll
         for (int e = 0; e < 8; ++e)
@@ -690,14 +899,21 @@ head_matvec (HeadArgs a, int S, hipStream_t s)
   const int rows = 4 * (64 / lpr) * kHeadRows;
   a.bph = (a.R + rows - 1) / rows;
   const dim3 grid ((unsigned)(a.heads * a.bph + (a.nx ? 1 : 0)), (unsigned)S), block (256);
+#define VKL_HEAD(L)                                                           \
+  if (a.parts.pacc)                                                           \
+    head_matvec_kernel<L, true><<<grid, block, 0, s>>> (a);                   \
+  else                                                                        \
+    head_matvec_kernel<L, false><<<grid, block, 0, s>>> (a);                  \
+  break
   switch (lpr)
     {
-    case 4: head_matvec_kernel<4><<<grid, block, 0, s>>> (a); break;
-    case 8: head_matvec_kernel<8><<<grid, block, 0, s>>> (a); break;
-    case 16: head_matvec_kernel<16><<<grid, block, 0, s>>> (a); break;
-    case 32: head_matvec_kernel<32><<<grid, block, 0, s>>> (a); break;
-    default: head_matvec_kernel<64><<<grid, block, 0, s>>> (a); break;
+    case 4: VKL_HEAD (4);
+    case 8: VKL_HEAD (8);
+    case 16: VKL_HEAD (16);
+    case 32: VKL_HEAD (32);
+    default: VKL_HEAD (64);
     }
+#undef VKL_HEAD
   return (int)hipGetLastError ();
 }
 
@@ -742,6 +958,7 @@ struct GvArgs
   uint32_t *next_tok; // optional
   uint32_t *loop, *ids; // replayed loop: ids[index + 1], then both words advance
   int pick;
+  bool stream; // see NT of the kernel
 };
 
 __device__ __forceinline__ bool
@@ -752,7 +969,9 @@ amax_better (float v, uint32_t i, float bv, uint32_t bi)
 
 // XV: float4 per thread that hold the activation row while the first weights
 // are requested; 0: a row of any length, staged before them
-template <int MODE, int XV>
+// NT: the weights of a step exceed what the caches hold, they are requested past
+// them
+template <int MODE, int XV, bool NT>
 __global__ __launch_bounds__ (kGvThreads) void
 stack_gemv_kernel (const GvArgs a)
 {
@@ -781,7 +1000,10 @@ stack_gemv_kernel (const GvArgs a)
         const uint16_t *p = a.w + (size_t)min (row0 + r, a.N - 1) * a.K;
 #pragma unroll
         for (int u = 0; u < 4; ++u)
-          b[r * 4 + u] = ldg4_stream (p + min (sp * kGvSpan + u * 512 + lane * 8, a.K - 8));
+          {
+            const uint16_t *c = p + min (sp * kGvSpan + u * 512 + lane * 8, a.K - 8);
+            b[r * 4 + u] = NT ? ldg4_stream (c) : ldg4 (c);
+          }
       }
   };
   auto put = [&] (int c, const float4 v) { // c: a multiple of 4
@@ -1003,15 +1225,22 @@ gv_supported (int K)
   return (size_t)((K + kGvSpan - 1) / kGvSpan) * kGvSpan * sizeof (float) <= (size_t)kGvMaxLds;
 }
 
+template <int MODE, int XV, bool NT>
+int
+launch_gv_nt (const GvArgs &a, int grid, size_t lds, hipStream_t s)
+{
+  static LdsLimit limit;
+  if (int e = limit.raise ((const void *)stack_gemv_kernel<MODE, XV, NT>, lds))
+    return e;
+  stack_gemv_kernel<MODE, XV, NT><<<dim3 ((unsigned)grid), dim3 (kGvThreads), lds, s>>> (a);
+  return (int)hipGetLastError ();
+}
+
 template <int MODE, int XV>
 int
 launch_gv_k (const GvArgs &a, int grid, size_t lds, hipStream_t s)
 {
-  static LdsLimit limit;
-  if (int e = limit.raise ((const void *)stack_gemv_kernel<MODE, XV>, lds))
-    return e;
-  stack_gemv_kernel<MODE, XV><<<dim3 ((unsigned)grid), dim3 (kGvThreads), lds, s>>> (a);
-  return (int)hipGetLastError ();
+  return a.stream ? launch_gv_nt<MODE, XV, true> (a, grid, lds, s) : launch_gv_nt<MODE, XV, false> (a, grid, lds, s);
 }
 
 template <int MODE>
@@ -1041,7 +1270,7 @@ struct StackScratch
 {
   uint32_t *sync; // [0] arg-max counter, [16..17] loop state, [20..23] sampler parameters
   uint32_t *cnt;  // attention counters and parts
-  float *x, *q, *c, *g, *cat, *qa, *oa, *logits, *amax_v;
+  float *x, *q, *c, *g, *cat, *qa, *logits, *amax_v;
   uint32_t *amax_i;
   size_t bytes;
 };
@@ -1082,7 +1311,6 @@ carve_stack (const vkl_stack_model *m)
   s.g = (float *)take (g * 4);
   s.cat = (float *)take (cat * 4);
   s.qa = (float *)take (qa * 4);
-  s.oa = (float *)take (qa * 4);
   s.logits = (float *)take ((size_t)m->vocab * 4);
   s.amax_v = (float *)take (kMaxGrid * 4);
   s.amax_i = (uint32_t *)take (kMaxGrid * 4);
@@ -1130,8 +1358,24 @@ struct StepArgs
   uint32_t *next_tok;
   uint32_t *loop, *ids;
   bool sampled;
+  bool stream; // weights of the step beyond what the caches hold
   int n_cu;
 };
+
+// memory-side cache and L2s
+constexpr size_t kCacheBytes = (size_t)288 << 20;
+
+bool
+weights_stream (const vkl_stack_model &m)
+{
+  size_t n = (size_t)m.vocab * m.width_p;
+  for (int i = 0; i < m.n_runs; ++i)
+    {
+      const vkl_stack_layer &l = m.layers_h[i];
+      n += (size_t)l.n_in * m.width_p + (size_t)m.width * l.k_out;
+    }
+  return n * 2 > kCacheBytes;
+}
 
 int
 launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
@@ -1140,7 +1384,7 @@ launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
   const bool latent = l.mixer == VKL_MIX_LATENT;
   GvArgs a = {};
   a.w = (const uint16_t *)l.w_in, a.N = l.n_in, a.K = m.width_p;
-  a.x = p.s.x, a.norm = l.norm, a.W = m.width, a.eps = m.eps, a.pos = p.pos;
+  a.x = p.s.x, a.norm = l.norm, a.W = m.width, a.eps = m.eps, a.pos = p.pos, a.stream = p.stream;
   int n = 0;
   a.seg[n++] = { 0, l.H * l.dim, p.s.q, 1, 0, 0 };
   if (latent)
@@ -1165,23 +1409,24 @@ launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
       h.ncache = l.cache, h.ntype = m.ctype, h.pos = p.pos;
       if (int e = head_matvec (h, 1, st))
         return e;
-      if (int e = rows_attention (p.s.qa, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.rank_p, l.H, 1, l.rank_p, 1,
-                                  p.pos, l.scale, l.temp_coef, l.temp_every, p.s.oa, VKL_TYPE_F32, 0, p.s.cnt, st))
-        return e;
       HeadArgs v = {};
+      if (int e = rows_attention (p.s.qa, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.rank_p, l.H, 1, l.rank_p, 1,
+                                  p.pos, l.scale, l.temp_coef, l.temp_every, nullptr, VKL_TYPE_F32, 0, p.s.cnt,
+                                  &v.parts, st))
+        return e;
+      v.pos = p.pos;
       v.w = (const uint16_t *)l.w_uv, v.heads = l.H, v.R = l.vdim, v.K = l.rank_p;
-      v.x = p.s.oa, v.xtype = VKL_TYPE_F32, v.xh = (size_t)l.rank_p;
       v.y = p.s.cat, v.ytype = VKL_TYPE_F32, v.yh = (size_t)l.vdim;
       v.gate = p.s.g;
       if (int e = head_matvec (v, 1, st))
         return e;
     }
   else if (int e = rows_attention (p.s.q, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.G * l.dim, l.H, l.G, l.dim, 1,
-                                   p.pos, l.scale, l.temp_coef, l.temp_every, p.s.cat, VKL_TYPE_F32, 0, p.s.cnt, st))
+                                   p.pos, l.scale, l.temp_coef, l.temp_every, p.s.cat, VKL_TYPE_F32, 0, p.s.cnt, nullptr, st))
     return e;
   GvArgs o = {};
   o.w = (const uint16_t *)l.w_out, o.N = m.width, o.K = l.k_out;
-  o.x = p.s.cat, o.y = p.s.x;
+  o.x = p.s.cat, o.y = p.s.x, o.stream = p.stream;
   return launch_gv<GV_ADD> (o, p.n_cu, st);
 }
 
@@ -1192,14 +1437,14 @@ launch_stack_step (const StepArgs &p, hipStream_t st)
   EmbedArgs e = {};
   e.table = (const uint16_t *)m.embed, e.VH = (uint32_t)m.vocab, e.K = m.width_p, e.W = m.width;
   e.toks = p.toks, e.loop = p.loop, e.w = m.embed_norm, e.eps = m.eps, e.out = p.s.x, e.os = (size_t)m.width_p;
-  embed_norm_kernel<<<dim3 (1), dim3 (256), 0, st>>> (e);
+  embed_norm_kernel<<<dim3 (1), dim3 (1024), 0, st>>> (e);
   for (int i = 0; i < m.n_runs; ++i)
     if (int err = launch_stack_layer (p, m.layers_h[i], st))
       return err;
   GvArgs a = {};
   a.w = (const uint16_t *)m.embed, a.N = m.vocab, a.K = m.width_p;
   a.x = p.s.x, a.norm = m.final_norm, a.W = m.width, a.eps = m.eps;
-  a.y = p.logits ? p.logits : p.s.logits, a.cap = m.logit_cap;
+  a.y = p.logits ? p.logits : p.s.logits, a.cap = m.logit_cap, a.stream = p.stream;
   a.amax_v = p.s.amax_v, a.amax_i = p.s.amax_i, a.amax_cnt = p.s.sync;
   a.pick = (p.next_tok || p.loop) && !p.sampled;
   a.next_tok = p.next_tok, a.loop = p.loop, a.ids = p.ids;
@@ -1273,7 +1518,7 @@ stack_loop (const vkl_stack_model *m, uint32_t *ids, uint32_t pos0, int n_steps,
   if (n_steps == 0)
     return 0;
   StepArgs p = {};
-  p.m = m, p.s = carve_stack (m);
+  p.m = m, p.s = carve_stack (m), p.stream = weights_stream (*m);
   if (int e = compute_units (&p.n_cu))
     return e;
   p.loop = p.s.sync + 16, p.ids = ids, p.toks = ids;
@@ -1329,7 +1574,7 @@ vkl_embed_norm_bf16 (const void *table, uint32_t VH, int K, int W, const uint32_
   EmbedArgs a = {};
   a.table = (const uint16_t *)table, a.VH = VH, a.K = K, a.W = W, a.toks = toks, a.w = w, a.eps = eps;
   a.out = out, a.os = os;
-  embed_norm_kernel<<<dim3 (n), dim3 (256), 0, (hipStream_t)stream>>> (a);
+  embed_norm_kernel<<<dim3 (n), dim3 (1024), 0, (hipStream_t)stream>>> (a);
   return vkl_launch_status ();
 }
 
@@ -1340,7 +1585,20 @@ vkl_rmsnorm_f32 (const float *x, size_t xs, const uint32_t *rows, int n, int W, 
   VKL_CHECK_ARG (x && w && out && n > 0 && W > 0 && Wp >= W && xs >= (size_t)W && os >= (size_t)Wp);
   VKL_CHECK_ARG (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16);
   const NormArgs a = { x, xs, rows, W, Wp, w, eps, out, otype, os };
-  rmsnorm_f32_kernel<<<dim3 ((unsigned)n), dim3 (256), 0, (hipStream_t)stream>>> (a);
+  const dim3 grid ((unsigned)n), block (256);
+  hipStream_t st = (hipStream_t)stream;
+  const bool vec = (W % 4) == 0 && (Wp % 4) == 0 && (xs % 4) == 0 && (os % 4) == 0 && ((uintptr_t)x % 16) == 0
+                   && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 16) == 0;
+  if (vec && Wp <= 1024)
+    rmsnorm_f32_kernel<1><<<grid, block, 0, st>>> (a);
+  else if (vec && Wp <= 2048)
+    rmsnorm_f32_kernel<2><<<grid, block, 0, st>>> (a);
+  else if (vec && Wp <= 4096)
+    rmsnorm_f32_kernel<4><<<grid, block, 0, st>>> (a);
+  else if (vec && Wp <= 8192)
+    rmsnorm_f32_kernel<8><<<grid, block, 0, st>>> (a);
+  else
+    rmsnorm_f32_kernel<0><<<grid, block, 0, st>>> (a);
   return vkl_launch_status ();
 }
 
@@ -1364,7 +1622,7 @@ vkl_attn_rows (const void *q, int qtype, size_t qs, const void *rows, int ctype,
   VKL_CHECK_ARG ((qtype == VKL_TYPE_F32 || qtype == VKL_TYPE_BF16) && (ctype == VKL_TYPE_F32 || ctype == VKL_TYPE_BF16)
                  && (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16));
   return rows_attention (q, qtype, qs, rows, ctype, rs, H, G, dim, S, StepPos{ nullptr, pos0 }, scale, temp_coef,
-                         temp_every, out, otype, os, scratch, (hipStream_t)stream);
+                         temp_every, out, otype, os, scratch, nullptr, (hipStream_t)stream);
 }
 
 extern "C" int
@@ -1404,7 +1662,7 @@ vkl_stack_step (const vkl_stack_model *m, const uint32_t *tok, uint32_t pos, flo
     return e;
   VKL_CHECK_ARG (tok && pos < (uint32_t)m->maxlen);
   StepArgs p = {};
-  p.m = m, p.s = carve_stack (m);
+  p.m = m, p.s = carve_stack (m), p.stream = weights_stream (*m);
   if (int e = compute_units (&p.n_cu))
     return e;
   p.pos = { nullptr, pos }, p.toks = tok, p.logits = logits32, p.next_tok = next_tok;
