@@ -72,19 +72,20 @@ int vkl_attn_prefill_causal_bf16 (const void *q, const void *k, const void *v,
                                   float scale, float temp_coef, int temp_every,
                                   const float *gate, size_t gs, void *out,
                                   size_t ors, void *stream);
-/* The same where the values ARE the keys, all sums in fp32, for few query rows
- * (decode) and for the 32-bit format: q [S, H*dim] and out in qtype / otype,
- * rows [>= pos0 + S, G*dim] in ctype; query row s is at position pos0 + s.  One
- * pass over the rows: a row is used for the score and for the output while it
- * is in registers.  The context is split over workgroups, the last of which
- * combines the parts (scratch from vkl_attn_rows_scratch_bytes, zeroed once).
- * dim a multiple of 32 up to 1024. */
+/* The same where the values ARE the keys, for few query rows (decode) and for the
+ * 32-bit format: q [S, H*dim] and out in qtype / otype, rows [>= pos0 + S, G*dim]
+ * in ctype; query row s is at position pos0 + s.  One pass over the rows.  bf16
+ * rows that several heads share go through the matrix cores (queries and
+ * weights rounded to bf16 as operands), others through the vector units in fp32
+ * throughout.  The context is split over workgroups, the last of which combines
+ * the parts (scratch from vkl_attn_rows_scratch_bytes, zeroed once).  dim a
+ * multiple of 32 up to 1024. */
 int vkl_attn_rows (const void *q, int qtype, size_t qs, const void *rows,
                    int ctype, size_t rs, int H, int G, int dim, int S,
                    uint32_t pos0, float scale, float temp_coef, int temp_every,
                    void *out, int otype, size_t os, void *scratch,
                    void *stream);
-size_t vkl_attn_rows_scratch_bytes (int H, int G, int dim, int S);
+size_t vkl_attn_rows_scratch_bytes (int ctype, int H, int G, int dim, int S);
 /* y[s, h*yh + r] = f * sum_k w[h, r, k] x[s, h*xh + k], w bf16 [H, R, K], f = 1 or
  * sigmoid (gate[s*gs + h]); K a multiple of 32 */
 int vkl_head_matvec (const void *w, int H, int R, int K, const void *x,

@@ -114,7 +114,9 @@ def edge_targets(S, L):
 @pytest.mark.parametrize("ctype", [F32, BF16])
 @pytest.mark.parametrize("H,G,D,S,L", [(3, 3, 32, 1, 1), (8, 1, 32, 5, 70), (6, 2, 64, 1, 300), (12, 2, 96, 2, 129),
                                        (7, 7, 128, 3, 257), (8, 1, 160, 1, 1100), (5, 1, 256, 4, 64), (9, 1, 512, 1, 65),
-                                       (4, 2, 1024, 2, 150), (8, 1, 128, 1, 4099), (2, 1, 32, 1, 2048)])
+                                       (4, 2, 1024, 2, 150), (8, 1, 128, 1, 4099), (2, 1, 32, 1, 2048),
+                                       (33, 1, 448, 1, 900), (40, 1, 320, 2, 130), (32, 1, 512, 1, 4500), (10, 5, 384, 1, 640),
+                                       (70, 2, 192, 1, 333), (4, 4, 224, 2, 200), (6, 3, 288, 1, 90)])
 def test_row_attention(dev, rng, ctype, H, G, D, S, L):
     """Keys that are values, with keys planted at split and lane edges; the row
     after the last visible one holds values that would show."""
@@ -127,7 +129,7 @@ def test_row_attention(dev, rng, ctype, H, G, D, S, L):
     coef, every = 0.3, 40
     dq, dk = dev.upload(qb), dev.upload(kb)
     out = dev.alloc(S * H * D * 4)
-    n = K.lib().vkl_attn_rows_scratch_bytes(H, G, D, S)
+    n = K.lib().vkl_attn_rows_scratch_bytes(ctype, H, G, D, S)
     scratch = dev.alloc(n)
     scratch.zero()
     want = np.zeros((S, H, D))
@@ -140,7 +142,9 @@ def test_row_attention(dev, rng, ctype, H, G, D, S, L):
         capi.check(K.lib().vkl_attn_rows(dq.ptr, F32, H * D, dk.ptr, ctype, G * D, H, G, D, S, L - S, 0.5, coef, every,
                                          out.ptr, F32, H * D, scratch.ptr, dev.stream))
         got = out.read(np.float32, (S, H, D))
-        assert np.abs(got - want).max() < 3e-5 * np.abs(want).max(), np.abs(got - want).max()
+        # (bf16 rows that several heads share: operands rounded to bf16)
+        bound = 1.5e-2 if ctype == BF16 and H > G else 3e-5
+        assert np.abs(got - want).max() < bound * np.abs(want).max(), np.abs(got - want).max()
 
 
 @pytest.mark.parametrize("H,G,D,S,L", [(4, 4, 32, 1, 1), (8, 1, 64, 130, 130), (6, 2, 96, 200, 329), (4, 1, 128, 64, 1100),

@@ -243,7 +243,8 @@ rmsnorm_f32_kernel (const NormArgs a)
 // ---------------------------------------------------------------------------
 constexpr int kRowThreads = 256;
 constexpr int kRowUnroll = 4;
-constexpr int kRowSplits = 32;  // parts a context is cut into at most
+constexpr int kRowSplits = 64;  // parts a context is cut into at most (one per lane)
+constexpr int kRowHeads = 32;   // query heads of a workgroup at most
 constexpr int kRowTarget = 512; // workgroups a launch aims for
 constexpr float kNoKey = -1.0e30f;
 
@@ -254,7 +255,7 @@ struct RowAttnArgs
   size_t qs;
   const void *rows;
   size_t rs;
-  int G, D, rep, tiles; // rep: query heads per group; tiles: head tiles per group
+  int G, D, rep, tiles, ht; // rep: query heads per group; tiles of ht heads
   StepPos pos;
   float scale, tcoef;
   int tevery;
@@ -348,6 +349,100 @@ load8 (const void *p, int type, size_t i, float (&f)[8])
     }
 }
 
+// LDS of combine_parts in floats
+constexpr int kCombineLds = kRowHeads * kRowSplits + 4 * kRowThreads / 2;
+
+// The parts of nh heads (entries [part][ht] from pbase on) into their outputs, by
+// a whole workgroup: a wave per head for the weights, lane p holding part p, then
+// four neighbouring values per thread with the parts in two halves of the
+// workgroup.  The first values are requested together with the maxima and sums.
+__device__ __forceinline__ void
+combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, size_t out0, float *lds)
+{
+  constexpr int R = 16; // parts of a half in flight
+  float *wgt = lds; // [kRowHeads][kRowSplits]
+  float4 *swap = (float4 *)(lds + kRowHeads * kRowSplits);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int half = tid >> 7, q4 = a.D / 4, outs = nh * q4;
+  float4 pv[R];
+  auto request = [&] (int o0, int p0) {
+    const int oc = min (o0 + (tid & 127), outs - 1), h = oc / q4;
+    const float *src = a.pacc + (pbase * ht + h) * a.D + (oc - h * q4) * 4;
+#pragma unroll
+    for (int j = 0; j < R; ++j)
+      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (p0 + 2 * j + half, active - 1) * ht * a.D));
+  };
+  constexpr int HW = kRowHeads / 4; // heads per wave
+  float mv[HW], lv[HW];
+#pragma unroll
+  for (int i = 0; i < HW; ++i)
+    {
+      const size_t at = (pbase + min (lane, active - 1)) * ht + min (wave + 4 * i, nh - 1);
+      mv[i] = ldg (a.pm + at), lv[i] = ldg (a.pl + at);
+    }
+  request (0, 0);
+#pragma unroll
+  for (int i = 0; i < HW; ++i)
+    if (wave + 4 * i < nh)
+      {
+        const float M = wave_max (mv[i]);
+        const float f = lane < active ? expf (mv[i] - M) : 0.f;
+        wgt[(wave + 4 * i) * kRowSplits + lane] = f / wave_sum (f * lv[i]);
+      }
+  __syncthreads ();
+  for (int o0 = 0; o0 < outs; o0 += kRowThreads / 2)
+    {
+      const int o = o0 + (tid & 127), oc = min (o, outs - 1), h = oc / q4, d = (oc - h * q4) * 4;
+      float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
+      for (int p0 = 0; p0 < active; p0 += 2 * R)
+        {
+          if (o0 + p0 > 0)
+            request (o0, p0);
+#pragma unroll
+          for (int j = 0; j < R; ++j)
+            {
+              const float f = wgt[h * kRowSplits + p0 + 2 * j + half];
+              v.x = __builtin_fmaf (f, pv[j].x, v.x), v.y = __builtin_fmaf (f, pv[j].y, v.y);
+              v.z = __builtin_fmaf (f, pv[j].z, v.z), v.w = __builtin_fmaf (f, pv[j].w, v.w);
+            }
+        }
+      if (half)
+        swap[tid & 127] = v;
+      __syncthreads ();
+      if (!half && o < outs)
+        {
+          const float4 w = swap[tid];
+          const float r[4] = { v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w };
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            store_elem (a.out, a.otype, out0 + (size_t)h * a.D + d + e, r[e]);
+        }
+      __syncthreads ();
+    }
+}
+
+// Counts the workgroup in once its (written-through) parts are in memory; true
+// in the one that arrives last, which may then read all parts with ordinary loads.
+__device__ __forceinline__ bool
+last_of_parts (uint32_t *cnt, int active, uint32_t *flag)
+{
+  __builtin_amdgcn_s_waitcnt (0);
+  __syncthreads ();
+  if (threadIdx.x == 0)
+    {
+      const uint32_t old = __hip_atomic_fetch_add (cnt, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      const bool last = old + 1u == (uint32_t)active;
+      if (last)
+        st_coherent_u32 (cnt, 0u);
+      *flag = last ? 1u : 0u;
+    }
+  __syncthreads ();
+  if (*flag == 0u)
+    return false;
+  __builtin_amdgcn_fence (__ATOMIC_ACQUIRE, "agent");
+  return true;
+}
+
 // LPR lanes share a row, NCH chunks of 8 values per lane; HT query heads per
 // workgroup.  Every group of LPR lanes walks rows of its own with a running
 // maximum; the groups' results meet in LDS at the end.
@@ -359,7 +454,7 @@ attn_rows_kernel (const RowAttnArgs a)
   constexpr int NS = kRowThreads / LPR; // lane groups
   constexpr int DA = LPR * 8 * NCH;     // values of a row the lanes cover
   extern __shared__ __align__ (16) float lds_rows[]; // [NS][HT][DA]
-  __shared__ float sm[NS][HT], sl[NS][HT], wgt[HT][kRowSplits];
+  __shared__ float sm[NS][HT], sl[NS][HT];
   __shared__ uint32_t last_s;
   const int s = blockIdx.z, gt = blockIdx.y;
   const int g = gt / a.tiles, t = gt - g * a.tiles;
@@ -541,87 +636,9 @@ attn_rows_kernel (const RowAttnArgs a)
     }
   if (!a.cnt)
     return;
-  // count in once this workgroup's parts are in memory; the last one combines
-  __builtin_amdgcn_s_waitcnt (0);
-  __syncthreads ();
-  if (tid == 0)
-    {
-      uint32_t *cnt = a.cnt + (size_t)s * gridDim.y + gt;
-      const uint32_t old = __hip_atomic_fetch_add (cnt, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      const bool last = old + 1u == (uint32_t)active;
-      if (last)
-        st_coherent_u32 (cnt, 0u);
-      last_s = last ? 1u : 0u;
-    }
-  __syncthreads ();
-  if (last_s == 0u)
+  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, &last_s))
     return;
-  // what other workgroups wrote through is now read with ordinary loads
-  __builtin_amdgcn_fence (__ATOMIC_ACQUIRE, "agent");
-  // maxima and sums, one part per thread, and the first values are requested
-  // together: four neighbouring values per thread, the parts in two halves of the
-  // workgroup
-  static_assert (HT * kRowSplits <= kRowThreads, "one part per thread");
-  float *pls = lds_rows; // [HT][kRowSplits], the rows' area is free
-  float *sums = &sl[0][0]; // [nh], free as well
-  const int half = tid >> 7, q4 = a.D / 4, outs = nh * q4;
-  float4 pv[kRowSplits / 2];
-  auto request = [&] (int o0) {
-    const int oc = min (o0 + (tid & 127), outs - 1), h = oc / q4;
-    const float *src = a.pacc + (pbase * HT + h) * a.D + (oc - h * q4) * 4;
-#pragma unroll
-    for (int j = 0; j < kRowSplits / 2; ++j)
-      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (2 * j + half, active - 1) * HT * a.D));
-  };
-  const int th = min (tid / kRowSplits, HT - 1), tp = tid % kRowSplits;
-  const float pmv = ldg (a.pm + (pbase + min (tp, active - 1)) * HT + th);
-  const float plv = ldg (a.pl + (pbase + min (tp, active - 1)) * HT + th);
-  request (0);
-  if (tid < HT * kRowSplits)
-    wgt[th][tp] = pmv, pls[tid] = plv;
-  __syncthreads ();
-  if (tid < nh)
-    {
-      float mm = kNoKey, S = 0.f;
-      for (int p = 0; p < active; ++p)
-        mm = fmaxf (mm, wgt[tid][p]);
-#pragma unroll 8
-      for (int p = 0; p < kRowSplits; ++p)
-        {
-          const float f = p < active ? expf (wgt[tid][p] - mm) : 0.f;
-          wgt[tid][p] = f;
-          S += f * pls[tid * kRowSplits + p];
-        }
-      sums[tid] = S;
-    }
-  __syncthreads ();
-  float4 *swap = (float4 *)(lds_rows + HT * kRowSplits);
-  for (int o0 = 0; o0 < outs; o0 += kRowThreads / 2)
-    {
-      const int o = o0 + (tid & 127), oc = min (o, outs - 1), h = oc / q4, d = (oc - h * q4) * 4;
-      float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
-#pragma unroll
-      for (int j = 0; j < kRowSplits / 2; ++j)
-        {
-          const float f = wgt[h][2 * j + half];
-          v.x = __builtin_fmaf (f, pv[j].x, v.x), v.y = __builtin_fmaf (f, pv[j].y, v.y);
-          v.z = __builtin_fmaf (f, pv[j].z, v.z), v.w = __builtin_fmaf (f, pv[j].w, v.w);
-        }
-      if (half)
-        swap[tid & 127] = v;
-      if (o0 + kRowThreads / 2 < outs)
-        request (o0 + kRowThreads / 2);
-      __syncthreads ();
-      if (!half && o < outs)
-        {
-          const float4 w = swap[tid];
-          const float inv = 1.0f / sums[h], r[4] = { v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w };
-#pragma unroll
-          for (int e = 0; e < 4; ++e)
-            store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d + e, r[e] * inv);
-        }
-      __syncthreads ();
-    }
+  combine_parts (a, HT, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * a.D, lds_rows);
 }
 
 // heads per workgroup: as many as share a row, within the registers
@@ -635,23 +652,311 @@ row_head_tile (int rep, int D)
   return ht;
 }
 
+// the matrix-core form: bf16 rows that several heads share, of the sizes it is
+// instantiated for
+bool
+row_mfma (int ctype, int rep, int D)
+{
+  return ctype == VKL_TYPE_BF16 && rep >= 2 && (D <= 256 || (D <= 512 && D % 64 == 0));
+}
+
 struct RowPlan
 {
+  bool mfma;
   int ht, tiles, nsplit;
   size_t parts; // entries of pm / pl
 };
 
 RowPlan
-row_plan (int H, int G, int D, int S)
+row_plan (int ctype, int H, int G, int D, int S)
 {
   RowPlan p;
   const int rep = H / G;
-  p.ht = row_head_tile (rep, D);
+  p.mfma = row_mfma (ctype, rep, D);
+  p.ht = p.mfma ? std::min (rep, kRowHeads) : row_head_tile (rep, D);
   p.tiles = (rep + p.ht - 1) / p.ht;
   const long groups = (long)G * p.tiles * S;
-  p.nsplit = (int)std::max (1L, std::min ((long)kRowSplits, kRowTarget / groups));
+  p.nsplit = (int)std::max (1L, std::min ((long)(p.mfma ? kRowSplits : kRowSplits / 2), kRowTarget / groups));
   p.parts = (size_t)groups * p.nsplit * p.ht;
   return p;
+}
+
+// ---- the matrix-core form ----------------------------------------------------
+// A workgroup holds up to 32 query heads that share the rows of its part of the
+// context, and walks the part in tiles of 64 rows.  A tile lies in LDS twice: as
+// it is (first product: scores) and transposed (second product: the rows as
+// values).  v_mfma_f32_32x32x16_bf16 in the transposed form of the prompt kernel:
+//   S^T[row, head] = sum_d C[row, d] Q[head, d]   waves: 2 row blocks x 2 halves of d
+//   O^T[d, head] = sum_row C^T[d, row] P^T[row, head]   waves: blocks of 32 d in turn
+// The halves' scores meet in LDS in fp32; every wave then forms maximum, weights
+// and sum of all heads itself (lane l: head l % 32, rows 8 (l / 32) .. +7 of each
+// 16), which leaves the weights in its registers as the operand of the second
+// product.  Transposed rows are stored with their 16-byte groups of eight rows
+// XOR-swizzled by the block of d they come from, against bank conflicts.
+constexpr int kMfRows = 64;
+constexpr int kMfLdv = kMfRows + 8;
+constexpr int kMfLds = 33; // floats per row of the exchanged scores
+
+typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
+typedef float float16v __attribute__ ((ext_vector_type (16)));
+
+template <int NBLK>
+constexpr size_t
+mfma_rows_lds ()
+{
+  constexpr int D = 32 * NBLK;
+  const size_t need = (size_t)kMfRows * (D + 8) * 2 + (size_t)D * kMfLdv * 2 + 2 * kMfRows * kMfLds * 4;
+  return need > kCombineLds * 4 ? need : kCombineLds * 4;
+}
+
+template <int NBLK>
+__global__ __launch_bounds__ (kRowThreads, NBLK <= 4 ? 2 : 1) void
+attn_rows_mfma_kernel (const RowAttnArgs a)
+{
+  constexpr int D = 32 * NBLK, LDK = D + 8, CPR = D / 8;
+  constexpr int ITEMS = kMfRows / 2 * CPR;                     // (row pair, 8 values)
+  constexpr int IT = (ITEMS + kRowThreads - 1) / kRowThreads;
+  constexpr bool RAG = ITEMS % kRowThreads != 0;
+  constexpr int NB = (NBLK + 3) / 4;                           // blocks of d per wave
+  extern __shared__ __align__ (16) uint8_t lds_mf[];
+  uint16_t *Ks = (uint16_t *)lds_mf;                           // [64][LDK]
+  uint16_t *Vt = Ks + kMfRows * LDK;                           // [D][kMfLdv]
+  float *Sp = (float *)(Vt + D * kMfLdv);                      // [2][64][kMfLds]
+  __shared__ uint32_t last_s;
+  const int s = blockIdx.z, gt = blockIdx.y;
+  const int g = gt / a.tiles, t = gt - g * a.tiles;
+  const int ht = a.ht, nh = min (ht, a.rep - t * ht);
+  const uint32_t pos = a.pos.get () + (uint32_t)s;
+  const int L = (int)pos + 1;
+  const int chunk = row_chunk (L, a.nsplit, kMfRows);
+  const int active = (L + chunk - 1) / chunk;
+  const int c = blockIdx.x;
+  if (c >= active)
+    return;
+  const int l0 = c * chunk, l1 = min (L, l0 + chunk);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int lq = lane & 31, hh = lane >> 5;
+  const uint16_t *base = (const uint16_t *)a.rows + (size_t)g * D;
+
+  uint4 rv[IT][2];
+  auto load = [&] (int lb) {
+#pragma unroll
+    for (int i = 0; i < IT; ++i)
+      {
+        const int it = RAG ? min (tid + i * kRowThreads, ITEMS - 1) : tid + i * kRowThreads;
+        const int pair = it / CPR, ch = it - pair * CPR;
+        const uint16_t *p = base + ch * 8;
+        rv[i][0] = ldg4 (p + (size_t)min (lb + 2 * pair, l1 - 1) * a.rs);
+        rv[i][1] = ldg4 (p + (size_t)min (lb + 2 * pair + 1, l1 - 1) * a.rs);
+      }
+  };
+  auto store = [&] () {
+#pragma unroll
+    for (int i = 0; i < IT; ++i)
+      {
+        const int it = tid + i * kRowThreads;
+        if (RAG && it >= ITEMS)
+          continue;
+        const int pair = it / CPR, ch = it - pair * CPR;
+        *(uint4 *)(Ks + (2 * pair) * LDK + ch * 8) = rv[i][0];
+        *(uint4 *)(Ks + (2 * pair + 1) * LDK + ch * 8) = rv[i][1];
+        const uint32_t x[4] = { rv[i][0].x, rv[i][0].y, rv[i][0].z, rv[i][0].w };
+        const uint32_t y[4] = { rv[i][1].x, rv[i][1].y, rv[i][1].z, rv[i][1].w };
+        uint32_t *dst = (uint32_t *)(Vt + (ch * 8) * kMfLdv) + ((pair >> 2) ^ (ch & 7)) * 4 + (pair & 3);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          {
+            dst[(2 * e) * (kMfLdv / 2)] = (x[e] & 0xffffu) | (y[e] << 16);
+            dst[(2 * e + 1) * (kMfLdv / 2)] = (x[e] >> 16) | (y[e] & 0xffff0000u);
+          }
+      }
+  };
+  load (l0);
+  __builtin_amdgcn_sched_barrier (0);
+
+  const int blk = wave & 1, dh = wave >> 1;
+  float f = a.scale;
+  if (a.tcoef != 0.f)
+    f *= 1.0f + a.tcoef * logf ((float)((pos + 1u) / (uint32_t)a.tevery + 1u));
+  const int h0 = g * a.rep + t * ht;
+  bf8 qf[NBLK]; // this wave's half of d
+  {
+    const size_t qo = (size_t)s * a.qs + (size_t)(h0 + min (lq, nh - 1)) * D + dh * (D / 2) + hh * 8;
+#pragma unroll
+    for (int kt = 0; kt < NBLK; ++kt)
+      {
+        float v[8];
+        load8 (a.q, a.qtype, qo + kt * 16, v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          qf[kt][e] = (__bf16)v[e];
+      }
+  }
+  float m = kNoKey, sum = 0.f;
+  float16v oacc[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b)
+#pragma unroll
+    for (int r = 0; r < 16; ++r)
+      oacc[b][r] = 0.f;
+
+  for (int lb = l0; lb < l1; lb += kMfRows)
+    {
+      __syncthreads ();
+      store ();
+      __syncthreads ();
+      if (lb + kMfRows < l1)
+        load (lb + kMfRows);
+      {
+        float16v acc;
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          acc[r] = 0.f;
+        const uint16_t *kp = Ks + (32 * blk + lq) * LDK + dh * (D / 2) + hh * 8;
+#pragma unroll
+        for (int kt = 0; kt < NBLK; ++kt)
+          acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16 (*(const bf8 *)(kp + kt * 16), qf[kt], acc, 0, 0, 0);
+        float *sp = Sp + (dh * kMfRows + 32 * blk + 4 * hh) * kMfLds + lq;
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          sp[(8 * (r >> 2) + (r & 3)) * kMfLds] = acc[r];
+      }
+      __syncthreads ();
+      float sv[4][8], bm = kNoKey;
+#pragma unroll
+      for (int ks = 0; ks < 4; ++ks)
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          {
+            const int row = 16 * ks + 8 * hh + j;
+            const float sc = (Sp[row * kMfLds + lq] + Sp[(kMfRows + row) * kMfLds + lq]) * f;
+            sv[ks][j] = lb + row < l1 ? sc : kNoKey;
+            bm = fmaxf (bm, sv[ks][j]);
+          }
+      bm = fmaxf (bm, __shfl_xor (bm, 32, 64));
+      const float mn = fmaxf (m, bm);
+      if (__builtin_amdgcn_ballot_w64 (mn != m) != 0)
+        {
+          const float al = RowVec<uint16_t>::exponential (m - mn);
+          sum *= al;
+#pragma unroll
+          for (int b = 0; b < NB; ++b)
+#pragma unroll
+            for (int r = 0; r < 16; ++r)
+              oacc[b][r] *= al;
+          m = mn;
+        }
+      bf8 pf[4];
+#pragma unroll
+      for (int ks = 0; ks < 4; ++ks)
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          {
+            // (a masked row: exp of a hugely negative number; the sum takes the
+            // weight as the product consumes it)
+            const __bf16 e = (__bf16)RowVec<uint16_t>::exponential (sv[ks][j] - m);
+            sum += (float)e;
+            pf[ks][j] = e;
+          }
+#pragma unroll
+      for (int b = 0; b < NB; ++b)
+        {
+          const int db = wave + 4 * b;
+          if (NBLK % 4 != 0 && db >= NBLK)
+            continue;
+          const int d = 32 * db + lq;
+          const uint16_t *vp = Vt + d * kMfLdv;
+#pragma unroll
+          for (int ks = 0; ks < 4; ++ks)
+            oacc[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16 (
+                *(const bf8 *)(vp + (((2 * ks + hh) ^ ((d >> 3) & 7)) << 3)), pf[ks], oacc[b], 0, 0, 0);
+        }
+    }
+  sum += __shfl_xor (sum, 32, 64);
+  const size_t pbase = ((size_t)s * gridDim.y + gt) * a.nsplit;
+  const bool direct = a.cnt && active == 1;
+  const float inv = direct ? 1.0f / sum : 1.0f;
+  if (lq < nh)
+    {
+      if (!direct && wave == 0 && hh == 0)
+        {
+          const size_t at = (pbase + c) * ht + lq;
+          if (a.cnt)
+            {
+              st_coherent_u32 ((uint32_t *)a.pm + at, __float_as_uint (m));
+              st_coherent_u32 ((uint32_t *)a.pl + at, __float_as_uint (sum));
+            }
+          else
+            stg (a.pm + at, m), stg (a.pl + at, sum);
+        }
+#pragma unroll
+      for (int b = 0; b < NB; ++b)
+        {
+          const int db = wave + 4 * b;
+          if (NBLK % 4 != 0 && db >= NBLK)
+            continue;
+#pragma unroll
+          for (int q4 = 0; q4 < 4; ++q4)
+            {
+              const int d = 32 * db + 8 * q4 + 4 * hh;
+              const float v[4] = { oacc[b][4 * q4] * inv, oacc[b][4 * q4 + 1] * inv, oacc[b][4 * q4 + 2] * inv,
+                                   oacc[b][4 * q4 + 3] * inv };
+              if (direct)
+                {
+#pragma unroll
+                  for (int e = 0; e < 4; ++e)
+                    store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + lq) * D + d + e, v[e]);
+                  continue;
+                }
+              float *dst = a.pacc + ((pbase + c) * ht + lq) * D + d;
+              if (a.cnt)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                  st_coherent_u32 ((uint32_t *)dst + e, __float_as_uint (v[e]));
+              else
+                stg ((vkl_u32x4 *)dst, vkl_u32x4{ __float_as_uint (v[0]), __float_as_uint (v[1]),
+                                                  __float_as_uint (v[2]), __float_as_uint (v[3]) });
+            }
+        }
+    }
+  if (!a.cnt || active == 1)
+    return;
+  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, &last_s))
+    return;
+  combine_parts (a, ht, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * D, (float *)lds_mf);
+}
+
+template <int NBLK>
+int
+launch_mfma_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
+{
+  static LdsLimit limit;
+  constexpr size_t lds = mfma_rows_lds<NBLK> ();
+  if (int e = limit.raise ((const void *)attn_rows_mfma_kernel<NBLK>, lds))
+    return e;
+  attn_rows_mfma_kernel<NBLK><<<grid, dim3 (kRowThreads), lds, s>>> (a);
+  return (int)hipGetLastError ();
+}
+
+int
+launch_mfma (const RowAttnArgs &a, dim3 grid, hipStream_t s)
+{
+  switch (a.D / 32)
+    {
+    case 1: return launch_mfma_k<1> (a, grid, s);
+    case 2: return launch_mfma_k<2> (a, grid, s);
+    case 3: return launch_mfma_k<3> (a, grid, s);
+    case 4: return launch_mfma_k<4> (a, grid, s);
+    case 5: return launch_mfma_k<5> (a, grid, s);
+    case 6: return launch_mfma_k<6> (a, grid, s);
+    case 7: return launch_mfma_k<7> (a, grid, s);
+    case 8: return launch_mfma_k<8> (a, grid, s);
+    case 10: return launch_mfma_k<10> (a, grid, s);
+    case 12: return launch_mfma_k<12> (a, grid, s);
+    case 14: return launch_mfma_k<14> (a, grid, s);
+    case 16: return launch_mfma_k<16> (a, grid, s);
+    default: return (int)hipErrorInvalidValue;
+    }
 }
 
 template <typename CT, int LPR, int NCH, int HT>
@@ -659,7 +964,7 @@ int
 launch_rows_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
 {
   static LdsLimit limit;
-  const size_t lds = (size_t)kRowThreads * 8 * NCH * HT * sizeof (float);
+  const size_t lds = sizeof (float) * std::max ((size_t)kRowThreads * 8 * NCH * HT, (size_t)kCombineLds);
   if (int e = limit.raise ((const void *)attn_rows_kernel<CT, LPR, NCH, HT>, lds))
     return e;
   attn_rows_kernel<CT, LPR, NCH, HT><<<grid, dim3 (kRowThreads), lds, s>>> (a);
@@ -707,9 +1012,9 @@ constexpr size_t kRowCounterBytes = 4096;
 static_assert (kRowTarget / 2 * sizeof (uint32_t) <= kRowCounterBytes, "a counter per workgroup row");
 
 size_t
-row_scratch_bytes (int H, int G, int D, int S)
+row_scratch_bytes (int ctype, int H, int G, int D, int S)
 {
-  const RowPlan p = row_plan (H, G, D, S);
+  const RowPlan p = row_plan (ctype, H, G, D, S);
   return kRowCounterBytes + p.parts * (2 + (size_t)D) * sizeof (float) + 256;
 }
 
@@ -733,10 +1038,10 @@ rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype
                 int S, StepPos pos, float scale, float tcoef, int tevery, void *out, int otype, size_t os,
                 void *scratch, RowParts *parts, hipStream_t s)
 {
-  const RowPlan p = row_plan (H, G, D, S);
+  const RowPlan p = row_plan (ctype, H, G, D, S);
   RowAttnArgs a = {};
   a.q = q, a.qtype = qtype, a.qs = qs, a.rows = rows, a.rs = rs;
-  a.G = G, a.D = D, a.rep = H / G, a.tiles = p.tiles;
+  a.G = G, a.D = D, a.rep = H / G, a.tiles = p.tiles, a.ht = p.ht;
   a.pos = pos, a.scale = scale, a.tcoef = tcoef, a.tevery = tevery;
   a.out = out, a.otype = otype, a.os = os, a.nsplit = p.nsplit;
   a.cnt = parts ? nullptr : (uint32_t *)scratch;
@@ -744,8 +1049,10 @@ rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype
   a.pl = a.pm + p.parts;
   a.pacc = a.pl + p.parts;
   if (parts)
-    *parts = { a.pm, a.pl, a.pacc, p.nsplit, p.ht, p.tiles, row_step (D) };
+    *parts = { a.pm, a.pl, a.pacc, p.nsplit, p.ht, p.tiles, p.mfma ? kMfRows : row_step (D) };
   const dim3 grid ((unsigned)p.nsplit, (unsigned)(G * p.tiles), (unsigned)S);
+  if (p.mfma)
+    return launch_mfma (a, grid, s);
   return ctype == VKL_TYPE_F32 ? launch_rows<float> (a, p.ht, grid, s) : launch_rows<uint16_t> (a, p.ht, grid, s);
 }
 
@@ -815,13 +1122,15 @@ head_matvec_kernel (const HeadArgs a)
       const int chunk = row_chunk (L, p.nsplit, p.step), active = (L + chunk - 1) / chunk;
       const size_t pbase = (size_t)(h / p.ht) * p.nsplit;
       const int hh = h % p.ht;
-      const int i = lane % kRowSplits, ic = min (i, active - 1);
-      const float mi = ldg (p.pm + (pbase + ic) * p.ht + hh), li = ldg (p.pl + (pbase + ic) * p.ht + hh);
+      // lane p holds part p
+      static_assert (kRowSplits == 64, "one part per lane");
+      const size_t at = (pbase + min (lane, active - 1)) * p.ht + hh;
+      const float mi = ldg (p.pm + at), li = ldg (p.pl + at);
       const float M = wave_max (mi);
-      const float f = i < active ? expf (mi - M) : 0.f;
-      const float S = wave_sum (f * li) * ((float)kRowSplits / 64.f); // (every part stands in 64 / kRowSplits lanes)
-      if (tid < kRowSplits)
-        wgt[tid] = f / S;
+      const float f = lane < active ? expf (mi - M) : 0.f;
+      const float S = wave_sum (f * li);
+      if (wave == 0)
+        wgt[lane] = f / S;
       __syncthreads ();
       const int half = tid >> 7;
       for (int k0 = 0; k0 < a.K; k0 += 512)
@@ -829,16 +1138,20 @@ head_matvec_kernel (const HeadArgs a)
           // four neighbouring values per thread, the parts in two halves of the workgroup
           const int k = k0 + (tid & 127) * 4, kc = min (k, a.K - 4);
           const float *src = p.pacc + (pbase * p.ht + hh) * a.K + kc;
-          float4 pv[kRowSplits / 2], v = make_float4 (0.f, 0.f, 0.f, 0.f);
-#pragma unroll
-          for (int j = 0; j < kRowSplits / 2; ++j)
-            pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (2 * j + half, active - 1) * p.ht * a.K));
-#pragma unroll
-          for (int j = 0; j < kRowSplits / 2; ++j)
+          float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
+          for (int p0 = 0; p0 < active; p0 += 32)
             {
-              const float g = wgt[2 * j + half];
-              v.x = __builtin_fmaf (g, pv[j].x, v.x), v.y = __builtin_fmaf (g, pv[j].y, v.y);
-              v.z = __builtin_fmaf (g, pv[j].z, v.z), v.w = __builtin_fmaf (g, pv[j].w, v.w);
+              float4 pv[16];
+#pragma unroll
+              for (int j = 0; j < 16; ++j)
+                pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (p0 + 2 * j + half, active - 1) * p.ht * a.K));
+#pragma unroll
+              for (int j = 0; j < 16; ++j)
+                {
+                  const float g = wgt[p0 + 2 * j + half];
+                  v.x = __builtin_fmaf (g, pv[j].x, v.x), v.y = __builtin_fmaf (g, pv[j].y, v.y);
+                  v.z = __builtin_fmaf (g, pv[j].z, v.z), v.w = __builtin_fmaf (g, pv[j].w, v.w);
+                }
             }
           if (half && k < a.K)
             *(float4 *)(xc + k) = v;
@@ -1291,10 +1604,10 @@ carve_stack (const vkl_stack_model *m)
         {
           c = std::max (c, (size_t)l.rank_p), g = std::max (g, (size_t)l.H);
           qa = std::max (qa, (size_t)l.H * l.rank_p);
-          attn = std::max (attn, row_scratch_bytes (l.H, 1, l.rank_p, 1));
+          attn = std::max (attn, row_scratch_bytes (m->ctype, l.H, 1, l.rank_p, 1));
         }
       else
-        attn = std::max (attn, row_scratch_bytes (l.H, l.G, l.dim, 1));
+        attn = std::max (attn, row_scratch_bytes (m->ctype, l.H, l.G, l.dim, 1));
     }
   uint8_t *base = (uint8_t *)m->scratch;
   size_t off = 0;
@@ -1603,11 +1916,11 @@ vkl_rmsnorm_f32 (const float *x, size_t xs, const uint32_t *rows, int n, int W, 
 }
 
 extern "C" size_t
-vkl_attn_rows_scratch_bytes (int H, int G, int dim, int S)
+vkl_attn_rows_scratch_bytes (int ctype, int H, int G, int dim, int S)
 {
   if (H <= 0 || G <= 0 || H % G || dim <= 0 || S <= 0)
     return 0;
-  return row_scratch_bytes (H, G, dim, S);
+  return row_scratch_bytes (ctype, H, G, dim, S);
 }
 
 extern "C" int

@@ -98,7 +98,7 @@ absl::Status
 RowMixer::attend_rows_ (const void *q, int qtype, size_t qs, int run, int groups, int dim, int S, size_t offset,
                         void *out, int otype, size_t os)
 {
-  const size_t need = vkl_attn_rows_scratch_bytes (p_.heads, groups, dim, S);
+  const size_t need = vkl_attn_rows_scratch_bytes (type_ (), p_.heads, groups, dim, S);
   if (scratch_.bytes () < need)
     {
       scratch_ = Tensor (1, 1, (int)need, dev_, INT8);

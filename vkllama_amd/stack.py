@@ -21,7 +21,7 @@ SIGNATURES = {
     "vkl_attn_prefill_causal_bf16": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, sz, sz, sz, f32, f32, i32, vp, sz, vp, sz,
                                            vp]),
     "vkl_attn_rows": (i32, [vp, i32, sz, vp, i32, sz, i32, i32, i32, i32, u32, f32, f32, i32, vp, i32, sz, vp, vp]),
-    "vkl_attn_rows_scratch_bytes": (sz, [i32, i32, i32, i32]),
+    "vkl_attn_rows_scratch_bytes": (sz, [i32, i32, i32, i32, i32]),
     "vkl_head_matvec": (i32, [vp, i32, i32, i32, vp, i32, sz, sz, vp, i32, sz, sz, vp, sz, i32, vp]),
     "vkl_stack_scratch_bytes": (sz, [vp]),
     "vkl_stack_supported": (i32, [vp]),
