@@ -350,69 +350,81 @@ load8 (const void *p, int type, size_t i, float (&f)[8])
 }
 
 // LDS of combine_parts in floats
-constexpr int kCombineLds = kRowHeads * kRowSplits + 4 * kRowThreads / 2;
+template <int THREADS>
+constexpr int
+combine_lds ()
+{
+  return kRowHeads * kRowSplits + 4 * (THREADS - 128);
+}
 
 // The parts of nh heads (entries [part][ht] from pbase on) into their outputs, by
 // a whole workgroup: a wave per head for the weights, lane p holding part p, then
-// four neighbouring values per thread with the parts in two halves of the
-// workgroup.  The first values are requested together with the maxima and sums.
+// four neighbouring values per thread with the parts dealt to groups of 128
+// threads.  The first values are requested together with the maxima and sums.
+template <int THREADS>
 __device__ __forceinline__ void
 combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, size_t out0, float *lds)
 {
-  constexpr int R = 16; // parts of a half in flight
+  constexpr int NG = THREADS / 128;
+  constexpr int R = 32 / NG; // parts of a group in flight
   float *wgt = lds; // [kRowHeads][kRowSplits]
   float4 *swap = (float4 *)(lds + kRowHeads * kRowSplits);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int half = tid >> 7, q4 = a.D / 4, outs = nh * q4;
+  const int grp = tid >> 7, q4 = a.D / 4, outs = nh * q4;
   float4 pv[R];
   auto request = [&] (int o0, int p0) {
     const int oc = min (o0 + (tid & 127), outs - 1), h = oc / q4;
     const float *src = a.pacc + (pbase * ht + h) * a.D + (oc - h * q4) * 4;
 #pragma unroll
     for (int j = 0; j < R; ++j)
-      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (p0 + 2 * j + half, active - 1) * ht * a.D));
+      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (p0 + NG * j + grp, active - 1) * ht * a.D));
   };
-  constexpr int HW = kRowHeads / 4; // heads per wave
+  constexpr int NW = THREADS / 64, HW = kRowHeads / NW; // heads per wave
   float mv[HW], lv[HW];
 #pragma unroll
   for (int i = 0; i < HW; ++i)
     {
-      const size_t at = (pbase + min (lane, active - 1)) * ht + min (wave + 4 * i, nh - 1);
+      const size_t at = (pbase + min (lane, active - 1)) * ht + min (wave + NW * i, nh - 1);
       mv[i] = ldg (a.pm + at), lv[i] = ldg (a.pl + at);
     }
   request (0, 0);
 #pragma unroll
   for (int i = 0; i < HW; ++i)
-    if (wave + 4 * i < nh)
+    if (wave + NW * i < nh)
       {
         const float M = wave_max (mv[i]);
         const float f = lane < active ? expf (mv[i] - M) : 0.f;
-        wgt[(wave + 4 * i) * kRowSplits + lane] = f / wave_sum (f * lv[i]);
+        wgt[(wave + NW * i) * kRowSplits + lane] = f / wave_sum (f * lv[i]);
       }
   __syncthreads ();
-  for (int o0 = 0; o0 < outs; o0 += kRowThreads / 2)
+  for (int o0 = 0; o0 < outs; o0 += 128)
     {
       const int o = o0 + (tid & 127), oc = min (o, outs - 1), h = oc / q4, d = (oc - h * q4) * 4;
       float4 v = make_float4 (0.f, 0.f, 0.f, 0.f);
-      for (int p0 = 0; p0 < active; p0 += 2 * R)
+      for (int p0 = 0; p0 < active; p0 += NG * R)
         {
           if (o0 + p0 > 0)
             request (o0, p0);
 #pragma unroll
           for (int j = 0; j < R; ++j)
             {
-              const float f = wgt[h * kRowSplits + p0 + 2 * j + half];
+              const float f = wgt[h * kRowSplits + p0 + NG * j + grp];
               v.x = __builtin_fmaf (f, pv[j].x, v.x), v.y = __builtin_fmaf (f, pv[j].y, v.y);
               v.z = __builtin_fmaf (f, pv[j].z, v.z), v.w = __builtin_fmaf (f, pv[j].w, v.w);
             }
         }
-      if (half)
-        swap[tid & 127] = v;
+      if (grp)
+        swap[tid - 128] = v;
       __syncthreads ();
-      if (!half && o < outs)
+      if (!grp && o < outs)
         {
-          const float4 w = swap[tid];
-          const float r[4] = { v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w };
+          float r[4] = { v.x, v.y, v.z, v.w };
+#pragma unroll
+          for (int i = 0; i < NG - 1; ++i)
+            {
+              const float4 w = swap[tid + i * 128];
+              r[0] += w.x, r[1] += w.y, r[2] += w.z, r[3] += w.w;
+            }
 #pragma unroll
           for (int e = 0; e < 4; ++e)
             store_elem (a.out, a.otype, out0 + (size_t)h * a.D + d + e, r[e]);
@@ -638,7 +650,7 @@ attn_rows_kernel (const RowAttnArgs a)
     return;
   if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, &last_s))
     return;
-  combine_parts (a, HT, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * a.D, lds_rows);
+  combine_parts<kRowThreads> (a, HT, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * a.D, lds_rows);
 }
 
 // heads per workgroup: as many as share a row, within the registers
@@ -682,47 +694,55 @@ row_plan (int ctype, int H, int G, int D, int S)
 }
 
 // ---- the matrix-core form ----------------------------------------------------
-// A workgroup holds up to 32 query heads that share the rows of its part of the
-// context, and walks the part in tiles of 64 rows.  A tile lies in LDS twice: as
-// it is (first product: scores) and transposed (second product: the rows as
-// values).  v_mfma_f32_32x32x16_bf16 in the transposed form of the prompt kernel:
-//   S^T[row, head] = sum_d C[row, d] Q[head, d]   waves: 2 row blocks x 2 halves of d
-//   O^T[d, head] = sum_row C^T[d, row] P^T[row, head]   waves: blocks of 32 d in turn
-// The halves' scores meet in LDS in fp32; every wave then forms maximum, weights
-// and sum of all heads itself (lane l: head l % 32, rows 8 (l / 32) .. +7 of each
-// 16), which leaves the weights in its registers as the operand of the second
-// product.  Transposed rows are stored with their 16-byte groups of eight rows
-// XOR-swizzled by the block of d they come from, against bank conflicts.
+// A workgroup of eight waves holds up to 32 query heads that share the rows of its
+// part of the context, and walks the part in tiles of 64 rows.  A tile lies in LDS
+// twice: as it is (first product: scores) and transposed (second product: the rows
+// as values).
+//   S[row, head] = sum_d C[row, d] Q[head, d]: v_mfma_f32_16x16x32_bf16, waves = 4
+//     blocks of 16 rows x 2 halves of d; the halves meet in LDS in fp32
+//   weights: thread (head = tid % 32, rows 4 (tid / 32) .. +3), the maximum over
+//     the tile through LDS, weights to LDS as bf16 (over the tile, which is done
+//     with its first form)
+//   O^T[d, head] = sum_row C^T[d, row] P^T[row, head]: v_mfma_f32_32x32x16_bf16,
+//     waves = blocks of 32 d in turn
+// Transposed rows are stored with their 16-byte groups of eight rows XOR-swizzled by
+// the block of d they come from, against bank conflicts.
+constexpr int kMfThreads = 512, kMfWaves = 8;
 constexpr int kMfRows = 64;
 constexpr int kMfLdv = kMfRows + 8;
 constexpr int kMfLds = 33; // floats per row of the exchanged scores
 
 typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
+typedef float float4v __attribute__ ((ext_vector_type (4)));
 typedef float float16v __attribute__ ((ext_vector_type (16)));
 
 template <int NBLK>
 constexpr size_t
 mfma_rows_lds ()
 {
-  constexpr int D = 32 * NBLK;
-  const size_t need = (size_t)kMfRows * (D + 8) * 2 + (size_t)D * kMfLdv * 2 + 2 * kMfRows * kMfLds * 4;
-  return need > kCombineLds * 4 ? need : kCombineLds * 4;
+  constexpr int D = 32 * NBLK, DP = (D + 63) / 64 * 64;
+  const size_t need = (size_t)kMfRows * (DP + 8) * 2 + (size_t)D * kMfLdv * 2 + 2 * kMfRows * kMfLds * 4 + 16 * 32 * 4;
+  const size_t comb = combine_lds<kMfThreads> () * 4 + 16;
+  return need > comb ? need : comb;
 }
 
 template <int NBLK>
-__global__ __launch_bounds__ (kRowThreads, NBLK <= 4 ? 2 : 1) void
+__global__ __launch_bounds__ (kMfThreads) void
 attn_rows_mfma_kernel (const RowAttnArgs a)
 {
-  constexpr int D = 32 * NBLK, LDK = D + 8, CPR = D / 8;
+  constexpr int D = 32 * NBLK, DP = (D + 63) / 64 * 64, LDK = DP + 8, CPR = D / 8;
   constexpr int ITEMS = kMfRows / 2 * CPR;                     // (row pair, 8 values)
-  constexpr int IT = (ITEMS + kRowThreads - 1) / kRowThreads;
-  constexpr bool RAG = ITEMS % kRowThreads != 0;
-  constexpr int NB = (NBLK + 3) / 4;                           // blocks of d per wave
+  constexpr int IT = (ITEMS + kMfThreads - 1) / kMfThreads;
+  constexpr bool RAG = ITEMS % kMfThreads != 0;
+  constexpr int NB = (NBLK + kMfWaves - 1) / kMfWaves;         // blocks of d per wave
+  constexpr int KS = DP / 64;                                  // 32-wide steps of half a row
   extern __shared__ __align__ (16) uint8_t lds_mf[];
   uint16_t *Ks = (uint16_t *)lds_mf;                           // [64][LDK]
+  uint16_t *Pb = Ks;                                           // [32][kMfLdv], once the scores are out
   uint16_t *Vt = Ks + kMfRows * LDK;                           // [D][kMfLdv]
   float *Sp = (float *)(Vt + D * kMfLdv);                      // [2][64][kMfLds]
-  __shared__ uint32_t last_s;
+  float *red = Sp + 2 * kMfRows * kMfLds;                      // [16][32]
+  static_assert (32 * kMfLdv <= kMfRows * LDK, "the weights fit over the tile");
   const int s = blockIdx.z, gt = blockIdx.y;
   const int g = gt / a.tiles, t = gt - g * a.tiles;
   const int ht = a.ht, nh = min (ht, a.rep - t * ht);
@@ -738,26 +758,32 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
   const int lq = lane & 31, hh = lane >> 5;
   const uint16_t *base = (const uint16_t *)a.rows + (size_t)g * D;
 
-  uint4 rv[IT][2];
-  auto load = [&] (int lb) {
+  // item: four neighbouring row pairs x a run of chunks per wave
+  uint4 ra[IT][2], rb[IT][2]; // two tiles on their way
+  auto item = [&] (int i, int &pair, int &ch) {
+    const int it = RAG ? min (tid + i * kMfThreads, ITEMS - 1) : tid + i * kMfThreads;
+    const int q = it >> 2;
+    ch = q % CPR, pair = (q / CPR) * 4 + (it & 3);
+  };
+  auto load = [&] (int lb, uint4 (&rv)[IT][2]) {
 #pragma unroll
     for (int i = 0; i < IT; ++i)
       {
-        const int it = RAG ? min (tid + i * kRowThreads, ITEMS - 1) : tid + i * kRowThreads;
-        const int pair = it / CPR, ch = it - pair * CPR;
+        int pair, ch;
+        item (i, pair, ch);
         const uint16_t *p = base + ch * 8;
         rv[i][0] = ldg4 (p + (size_t)min (lb + 2 * pair, l1 - 1) * a.rs);
         rv[i][1] = ldg4 (p + (size_t)min (lb + 2 * pair + 1, l1 - 1) * a.rs);
       }
   };
-  auto store = [&] () {
+  auto store = [&] (const uint4 (&rv)[IT][2]) {
 #pragma unroll
     for (int i = 0; i < IT; ++i)
       {
-        const int it = tid + i * kRowThreads;
-        if (RAG && it >= ITEMS)
+        if (RAG && tid + i * kMfThreads >= ITEMS)
           continue;
-        const int pair = it / CPR, ch = it - pair * CPR;
+        int pair, ch;
+        item (i, pair, ch);
         *(uint4 *)(Ks + (2 * pair) * LDK + ch * 8) = rv[i][0];
         *(uint4 *)(Ks + (2 * pair + 1) * LDK + ch * 8) = rv[i][1];
         const uint32_t x[4] = { rv[i][0].x, rv[i][0].y, rv[i][0].z, rv[i][0].w };
@@ -770,29 +796,44 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
             dst[(2 * e + 1) * (kMfLdv / 2)] = (x[e] >> 16) | (y[e] & 0xffff0000u);
           }
       }
+    // columns that pad a row to a multiple of 64 (the weights may have lain there)
+    if (DP != D && tid < kMfRows * (DP - D) / 8)
+      *(uint4 *)(Ks + (tid / 4) * LDK + D + (tid & 3) * 8) = make_uint4 (0, 0, 0, 0);
   };
-  load (l0);
+  load (l0, ra);
+  load (min (l0 + kMfRows, l1 - 1), rb);
   __builtin_amdgcn_sched_barrier (0);
 
-  const int blk = wave & 1, dh = wave >> 1;
+  const int blk = wave & 3, dh = wave >> 2;
   float f = a.scale;
   if (a.tcoef != 0.f)
     f *= 1.0f + a.tcoef * logf ((float)((pos + 1u) / (uint32_t)a.tevery + 1u));
   const int h0 = g * a.rep + t * ht;
-  bf8 qf[NBLK]; // this wave's half of d
-  {
-    const size_t qo = (size_t)s * a.qs + (size_t)(h0 + min (lq, nh - 1)) * D + dh * (D / 2) + hh * 8;
+  // the queries go through LDS (where the transposed rows will lie): every value
+  // is fetched once, all waves need it
+  uint16_t *Qs = Vt; // [32][LDK]
+  static_assert (32 * LDK <= D * kMfLdv, "the queries fit over the transposed rows");
+  for (int i = tid; i < 32 * (DP / 8); i += kMfThreads)
+    {
+      const int h = i / (DP / 8), d = (i - h * (DP / 8)) * 8;
+      float v[8];
+      load8 (a.q, a.qtype, (size_t)s * a.qs + (size_t)(h0 + min (h, nh - 1)) * D + (DP == D ? d : min (d, D - 8)), v);
+      uint32_t w[4];
 #pragma unroll
-    for (int kt = 0; kt < NBLK; ++kt)
-      {
-        float v[8];
-        load8 (a.q, a.qtype, qo + kt * 16, v);
+      for (int e = 0; e < 4; ++e)
+        w[e] = DP == D || d < D ? f2bf (v[2 * e]) | ((uint32_t)f2bf (v[2 * e + 1]) << 16) : 0u;
+      *(uint4 *)(Qs + h * LDK + d) = make_uint4 (w[0], w[1], w[2], w[3]);
+    }
+  __syncthreads ();
+  // this wave's half of d: heads 0 .. 15 and 16 .. 31
+  bf8 qf[2][KS];
 #pragma unroll
-        for (int e = 0; e < 8; ++e)
-          qf[kt][e] = (__bf16)v[e];
-      }
-  }
-  float m = kNoKey, sum = 0.f;
+  for (int n = 0; n < 2; ++n)
+#pragma unroll
+    for (int kt = 0; kt < KS; ++kt)
+      qf[n][kt] = *(const bf8 *)(Qs + (16 * n + (lane & 15)) * LDK + dh * (DP / 2) + kt * 32 + (lane >> 4) * 8);
+  float m = kNoKey, sum = 0.f; // of head lq; the sum over this thread's rows
+  const int rg = tid >> 5;
   float16v oacc[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b)
@@ -800,40 +841,41 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
     for (int r = 0; r < 16; ++r)
       oacc[b][r] = 0.f;
 
-  for (int lb = l0; lb < l1; lb += kMfRows)
-    {
+  auto tile = [&] (int lb, uint4 (&rv)[IT][2]) {
       __syncthreads ();
-      store ();
+      store (rv);
       __syncthreads ();
-      if (lb + kMfRows < l1)
-        load (lb + kMfRows);
+      load (min (lb + 2 * kMfRows, l1 - 1), rv);
       {
-        float16v acc;
+        float4v acc[2] = { { 0.f, 0.f, 0.f, 0.f }, { 0.f, 0.f, 0.f, 0.f } };
+        const uint16_t *kp = Ks + (16 * blk + (lane & 15)) * LDK + dh * (DP / 2) + (lane >> 4) * 8;
 #pragma unroll
-        for (int r = 0; r < 16; ++r)
-          acc[r] = 0.f;
-        const uint16_t *kp = Ks + (32 * blk + lq) * LDK + dh * (D / 2) + hh * 8;
+        for (int kt = 0; kt < KS; ++kt)
+          {
+            const bf8 k = *(const bf8 *)(kp + kt * 32);
+            acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (k, qf[0][kt], acc[0], 0, 0, 0);
+            acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (k, qf[1][kt], acc[1], 0, 0, 0);
+          }
+        float *sp = Sp + (dh * kMfRows + 16 * blk + 4 * (lane >> 4)) * kMfLds + (lane & 15);
 #pragma unroll
-        for (int kt = 0; kt < NBLK; ++kt)
-          acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16 (*(const bf8 *)(kp + kt * 16), qf[kt], acc, 0, 0, 0);
-        float *sp = Sp + (dh * kMfRows + 32 * blk + 4 * hh) * kMfLds + lq;
-#pragma unroll
-        for (int r = 0; r < 16; ++r)
-          sp[(8 * (r >> 2) + (r & 3)) * kMfLds] = acc[r];
+        for (int r = 0; r < 4; ++r)
+          sp[r * kMfLds] = acc[0][r], sp[r * kMfLds + 16] = acc[1][r];
       }
       __syncthreads ();
-      float sv[4][8], bm = kNoKey;
+      float sv[4], bm = kNoKey;
 #pragma unroll
-      for (int ks = 0; ks < 4; ++ks)
+      for (int j = 0; j < 4; ++j)
+        {
+          const int row = 4 * rg + j;
+          const float sc = (Sp[row * kMfLds + lq] + Sp[(kMfRows + row) * kMfLds + lq]) * f;
+          sv[j] = lb + row < l1 ? sc : kNoKey;
+          bm = fmaxf (bm, sv[j]);
+        }
+      red[rg * 32 + lq] = bm;
+      __syncthreads ();
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          {
-            const int row = 16 * ks + 8 * hh + j;
-            const float sc = (Sp[row * kMfLds + lq] + Sp[(kMfRows + row) * kMfLds + lq]) * f;
-            sv[ks][j] = lb + row < l1 ? sc : kNoKey;
-            bm = fmaxf (bm, sv[ks][j]);
-          }
-      bm = fmaxf (bm, __shfl_xor (bm, 32, 64));
+      for (int i = 0; i < 16; ++i)
+        bm = fmaxf (bm, red[i * 32 + lq]);
       const float mn = fmaxf (m, bm);
       if (__builtin_amdgcn_ballot_w64 (mn != m) != 0)
         {
@@ -846,23 +888,29 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
               oacc[b][r] *= al;
           m = mn;
         }
+      {
+        // (a masked row: exp of a hugely negative number; the sum takes the weight
+        // as the product consumes it)
+        uint16_t e[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          {
+            e[j] = f2bf (RowVec<uint16_t>::exponential (sv[j] - m));
+            sum += bf2f (e[j]);
+          }
+        uint32_t *pp = (uint32_t *)(Pb + lq * kMfLdv + 4 * rg);
+        pp[0] = e[0] | ((uint32_t)e[1] << 16), pp[1] = e[2] | ((uint32_t)e[3] << 16);
+      }
+      __syncthreads ();
       bf8 pf[4];
 #pragma unroll
       for (int ks = 0; ks < 4; ++ks)
-#pragma unroll
-        for (int j = 0; j < 8; ++j)
-          {
-            // (a masked row: exp of a hugely negative number; the sum takes the
-            // weight as the product consumes it)
-            const __bf16 e = (__bf16)RowVec<uint16_t>::exponential (sv[ks][j] - m);
-            sum += (float)e;
-            pf[ks][j] = e;
-          }
+        pf[ks] = *(const bf8 *)(Pb + lq * kMfLdv + 16 * ks + 8 * hh);
 #pragma unroll
       for (int b = 0; b < NB; ++b)
         {
-          const int db = wave + 4 * b;
-          if (NBLK % 4 != 0 && db >= NBLK)
+          const int db = wave + kMfWaves * b;
+          if (NBLK % kMfWaves != 0 && db >= NBLK)
             continue;
           const int d = 32 * db + lq;
           const uint16_t *vp = Vt + d * kMfLdv;
@@ -871,8 +919,20 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
             oacc[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16 (
                 *(const bf8 *)(vp + (((2 * ks + hh) ^ ((d >> 3) & 7)) << 3)), pf[ks], oacc[b], 0, 0, 0);
         }
+  };
+  for (int lb = l0; lb < l1; lb += 2 * kMfRows)
+    {
+      tile (lb, ra);
+      if (lb + kMfRows < l1)
+        tile (lb + kMfRows, rb);
     }
-  sum += __shfl_xor (sum, 32, 64);
+  // the sums of a head's row groups
+  red[rg * 32 + lq] = sum;
+  __syncthreads ();
+  sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < 16; ++i)
+    sum += red[i * 32 + lq];
   const size_t pbase = ((size_t)s * gridDim.y + gt) * a.nsplit;
   const bool direct = a.cnt && active == 1;
   const float inv = direct ? 1.0f / sum : 1.0f;
@@ -892,8 +952,8 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
 #pragma unroll
       for (int b = 0; b < NB; ++b)
         {
-          const int db = wave + 4 * b;
-          if (NBLK % 4 != 0 && db >= NBLK)
+          const int db = wave + kMfWaves * b;
+          if (NBLK % kMfWaves != 0 && db >= NBLK)
             continue;
 #pragma unroll
           for (int q4 = 0; q4 < 4; ++q4)
@@ -921,9 +981,11 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
     }
   if (!a.cnt || active == 1)
     return;
-  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, &last_s))
+  // (the flag lies behind what combine_parts uses of LDS)
+  uint32_t *flag = (uint32_t *)((float *)lds_mf + combine_lds<kMfThreads> ());
+  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, flag))
     return;
-  combine_parts (a, ht, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * D, (float *)lds_mf);
+  combine_parts<kMfThreads> (a, ht, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * D, (float *)lds_mf);
 }
 
 template <int NBLK>
@@ -934,7 +996,7 @@ launch_mfma_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
   constexpr size_t lds = mfma_rows_lds<NBLK> ();
   if (int e = limit.raise ((const void *)attn_rows_mfma_kernel<NBLK>, lds))
     return e;
-  attn_rows_mfma_kernel<NBLK><<<grid, dim3 (kRowThreads), lds, s>>> (a);
+  attn_rows_mfma_kernel<NBLK><<<grid, dim3 (kMfThreads), lds, s>>> (a);
   return (int)hipGetLastError ();
 }
 
@@ -964,7 +1026,7 @@ int
 launch_rows_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
 {
   static LdsLimit limit;
-  const size_t lds = sizeof (float) * std::max ((size_t)kRowThreads * 8 * NCH * HT, (size_t)kCombineLds);
+  const size_t lds = sizeof (float) * std::max ((size_t)kRowThreads * 8 * NCH * HT, (size_t)combine_lds<kRowThreads> ());
   if (int e = limit.raise ((const void *)attn_rows_kernel<CT, LPR, NCH, HT>, lds))
     return e;
   attn_rows_kernel<CT, LPR, NCH, HT><<<grid, dim3 (kRowThreads), lds, s>>> (a);
@@ -1717,13 +1779,15 @@ launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
       HeadArgs h = {};
       h.w = (const uint16_t *)l.w_ukt, h.heads = l.H, h.R = l.rank_p, h.K = l.dim;
       h.x = p.s.q, h.xtype = VKL_TYPE_F32, h.xh = (size_t)l.dim;
-      h.y = p.s.qa, h.ytype = VKL_TYPE_F32, h.yh = (size_t)l.rank_p;
+      // (rounded here if the attention takes them as bf16 operands anyway)
+      const int qt = row_mfma (m.ctype, l.H, l.rank_p) ? VKL_TYPE_BF16 : VKL_TYPE_F32;
+      h.y = p.s.qa, h.ytype = qt, h.yh = (size_t)l.rank_p;
       h.nx = p.s.c, h.nw = l.c_norm, h.nW = l.rank, h.nWp = l.rank_p, h.neps = m.eps;
       h.ncache = l.cache, h.ntype = m.ctype, h.pos = p.pos;
       if (int e = head_matvec (h, 1, st))
         return e;
       HeadArgs v = {};
-      if (int e = rows_attention (p.s.qa, VKL_TYPE_F32, 0, l.cache, m.ctype, (size_t)l.rank_p, l.H, 1, l.rank_p, 1,
+      if (int e = rows_attention (p.s.qa, qt, 0, l.cache, m.ctype, (size_t)l.rank_p, l.H, 1, l.rank_p, 1,
                                   p.pos, l.scale, l.temp_coef, l.temp_every, nullptr, VKL_TYPE_F32, 0, p.s.cnt,
                                   &v.parts, st))
         return e;
