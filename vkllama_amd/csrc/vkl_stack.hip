@@ -349,6 +349,25 @@ load8 (const void *p, int type, size_t i, float (&f)[8])
     }
 }
 
+// 16 bytes past the XCD's L2, like st_coherent_u32 (the caller waits for the
+// store before it tells anybody)
+__device__ __forceinline__ void
+st_coherent_16 (float *p, const float (&v)[4])
+{
+  const vkl_u32x4 w = { __float_as_uint (v[0]), __float_as_uint (v[1]), __float_as_uint (v[2]), __float_as_uint (v[3]) };
+  asm volatile ("global_store_dwordx4 %0, %1, off sc1" ::"v"(p), "v"(w) : "memory");
+}
+
+// 16 bytes that another XCD wrote through, read past this XCD's L2
+__device__ __forceinline__ float4
+ld_coherent_16 (const float *p)
+{
+  const unsigned long long a = __hip_atomic_load ((const unsigned long long *)p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  const unsigned long long b = __hip_atomic_load ((const unsigned long long *)p + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  return make_float4 (__uint_as_float ((uint32_t)a), __uint_as_float ((uint32_t)(a >> 32)), __uint_as_float ((uint32_t)b),
+                      __uint_as_float ((uint32_t)(b >> 32)));
+}
+
 // LDS of combine_parts in floats
 template <int THREADS>
 constexpr int
@@ -377,7 +396,7 @@ combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, s
     const float *src = a.pacc + (pbase * ht + h) * a.D + (oc - h * q4) * 4;
 #pragma unroll
     for (int j = 0; j < R; ++j)
-      pv[j] = __builtin_bit_cast (float4, ldg4 (src + (size_t)min (p0 + NG * j + grp, active - 1) * ht * a.D));
+      pv[j] = ld_coherent_16 (src + (size_t)min (p0 + NG * j + grp, active - 1) * ht * a.D);
   };
   constexpr int NW = THREADS / 64, HW = kRowHeads / NW; // heads per wave
   float mv[HW], lv[HW];
@@ -385,7 +404,8 @@ combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, s
   for (int i = 0; i < HW; ++i)
     {
       const size_t at = (pbase + min (lane, active - 1)) * ht + min (wave + NW * i, nh - 1);
-      mv[i] = ldg (a.pm + at), lv[i] = ldg (a.pl + at);
+      mv[i] = __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pm + at));
+      lv[i] = __uint_as_float (ld_coherent_u32 ((const uint32_t *)a.pl + at));
     }
   request (0, 0);
 #pragma unroll
@@ -434,7 +454,7 @@ combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, s
 }
 
 // Counts the workgroup in once its (written-through) parts are in memory; true
-// in the one that arrives last, which may then read all parts with ordinary loads.
+// in the one that arrives last.
 __device__ __forceinline__ bool
 last_of_parts (uint32_t *cnt, int active, uint32_t *flag)
 {
@@ -449,10 +469,7 @@ last_of_parts (uint32_t *cnt, int active, uint32_t *flag)
       *flag = last ? 1u : 0u;
     }
   __syncthreads ();
-  if (*flag == 0u)
-    return false;
-  __builtin_amdgcn_fence (__ATOMIC_ACQUIRE, "agent");
-  return true;
+  return *flag != 0u;
 }
 
 // LPR lanes share a row, NCH chunks of 8 values per lane; HT query heads per
@@ -607,26 +624,31 @@ attn_rows_kernel (const RowAttnArgs a)
   __syncthreads ();
   const int nh = min (HT, a.rep - t * HT); // heads of this tile
   const size_t pbase = ((size_t)s * gridDim.y + gt) * a.nsplit;
-  for (int o = tid; o < nh * a.D; o += kRowThreads)
+  for (int o = tid * 4; o < nh * a.D; o += kRowThreads * 4)
     {
       const int h = o / a.D, d = o - h * a.D;
-      float v = 0.f, S = 0.f;
+      float v[4] = { 0.f, 0.f, 0.f, 0.f }, S = 0.f;
 #pragma unroll
       for (int i = 0; i < NS; ++i)
-        v += lds_rows[(i * HT + h) * DA + d];
+        {
+          const float4 w = *(const float4 *)(lds_rows + (i * HT + h) * DA + d);
+          v[0] += w.x, v[1] += w.y, v[2] += w.z, v[3] += w.w;
+        }
+      float *dst = a.pacc + ((pbase + c) * HT + h) * a.D + d;
       if (!a.cnt)
-        stg (a.pacc + ((pbase + c) * HT + h) * a.D + d, v);
+        stg ((vkl_u32x4 *)dst, vkl_u32x4{ __float_as_uint (v[0]), __float_as_uint (v[1]), __float_as_uint (v[2]),
+                                          __float_as_uint (v[3]) });
       else if (active == 1)
         {
           for (int i = 0; i < NS; ++i)
             S += sl[i][h];
-          store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d, v / S);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d + e, v[e] / S);
         }
       else
-        {
-          // (write-through: the workgroup that combines may be on another XCD)
-          st_coherent_u32 ((uint32_t *)a.pacc + ((pbase + c) * HT + h) * a.D + d, __float_as_uint (v));
-        }
+        // (write-through: the workgroup that combines may be on another XCD)
+        st_coherent_16 (dst, v);
     }
   if (a.cnt && active == 1)
     return;
@@ -758,12 +780,15 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
   const int lq = lane & 31, hh = lane >> 5;
   const uint16_t *base = (const uint16_t *)a.rows + (size_t)g * D;
 
+  auto swizzle = [] (int ch) { return (ch ^ (ch >> 3)) & 7; };
   // item: four neighbouring row pairs x a run of chunks per wave
   uint4 ra[IT][2], rb[IT][2]; // two tiles on their way
   auto item = [&] (int i, int &pair, int &ch) {
     const int it = RAG ? min (tid + i * kMfThreads, ITEMS - 1) : tid + i * kMfThreads;
-    const int q = it >> 2;
-    ch = q % CPR, pair = (q / CPR) * 4 + (it & 3);
+    if constexpr (CPR % 16 == 0)
+      ch = (it & 15) + 16 * ((it >> 6) % (CPR / 16)), pair = (it >> 6) / (CPR / 16) * 4 + ((it >> 4) & 3);
+    else
+      ch = (it >> 2) % CPR, pair = ((it >> 2) / CPR) * 4 + (it & 3);
   };
   auto load = [&] (int lb, uint4 (&rv)[IT][2]) {
 #pragma unroll
@@ -788,7 +813,7 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
         *(uint4 *)(Ks + (2 * pair + 1) * LDK + ch * 8) = rv[i][1];
         const uint32_t x[4] = { rv[i][0].x, rv[i][0].y, rv[i][0].z, rv[i][0].w };
         const uint32_t y[4] = { rv[i][1].x, rv[i][1].y, rv[i][1].z, rv[i][1].w };
-        uint32_t *dst = (uint32_t *)(Vt + (ch * 8) * kMfLdv) + ((pair >> 2) ^ (ch & 7)) * 4 + (pair & 3);
+        uint32_t *dst = (uint32_t *)(Vt + (ch * 8) * kMfLdv) + ((pair >> 2) ^ swizzle (ch)) * 4 + (pair & 3);
 #pragma unroll
         for (int e = 0; e < 4; ++e)
           {
@@ -917,7 +942,7 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
 #pragma unroll
           for (int ks = 0; ks < 4; ++ks)
             oacc[b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16 (
-                *(const bf8 *)(vp + (((2 * ks + hh) ^ ((d >> 3) & 7)) << 3)), pf[ks], oacc[b], 0, 0, 0);
+                *(const bf8 *)(vp + (((2 * ks + hh) ^ swizzle (d >> 3)) << 3)), pf[ks], oacc[b], 0, 0, 0);
         }
   };
   for (int lb = l0; lb < l1; lb += 2 * kMfRows)
@@ -969,10 +994,8 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
                   continue;
                 }
               float *dst = a.pacc + ((pbase + c) * ht + lq) * D + d;
-              if (a.cnt)
-#pragma unroll
-                for (int e = 0; e < 4; ++e)
-                  st_coherent_u32 ((uint32_t *)dst + e, __float_as_uint (v[e]));
+              if (a.cnt) // (through LDS, to leave it in whole lines)
+                *(float4 *)((float *)lds_mf + lq * D + d) = make_float4 (v[0], v[1], v[2], v[3]);
               else
                 stg ((vkl_u32x4 *)dst, vkl_u32x4{ __float_as_uint (v[0]), __float_as_uint (v[1]),
                                                   __float_as_uint (v[2]), __float_as_uint (v[3]) });
@@ -981,6 +1004,14 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
     }
   if (!a.cnt || active == 1)
     return;
+  static_assert (32 * D * 4 <= kMfRows * LDK * 2 + D * kMfLdv * 2, "a part fits over the tile");
+  __syncthreads ();
+  for (int o = tid * 4; o < nh * D; o += kMfThreads * 4)
+    {
+      const float4 w = *(const float4 *)((const float *)lds_mf + o);
+      const float v[4] = { w.x, w.y, w.z, w.w };
+      st_coherent_16 (a.pacc + (pbase + c) * ht * D + o, v);
+    }
   // (the flag lies behind what combine_parts uses of LDS)
   uint32_t *flag = (uint32_t *)((float *)lds_mf + combine_lds<kMfThreads> ());
   if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, flag))
