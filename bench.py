@@ -208,7 +208,9 @@ def fazinex_weights(cfg, seed):
 # --design fazinex: (width, layers, heads, key/value heads, head size, latent, ff), each beside a Llama-2-shaped model
 # with FP16 weights of the same width, heads, ff and layer count
 DESIGN_SIZES = {"4096": (4096, 8, 32, 8, 128, 512, 11008), "2048": (2048, 8, 16, 4, 128, 512, 5504),
-                "5120": (5120, 6, 40, 8, 128, 512, 13824)}
+                "5120": (5120, 6, 40, 8, 128, 512, 13824),
+                # as many key/value heads as query heads: caches of half the Llama-2 size
+                "4096-kv32": (4096, 8, 32, 32, 128, 512, 11008)}
 
 
 def bench_design(args):

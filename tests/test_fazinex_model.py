@@ -25,6 +25,8 @@ CONFIGS = {
     "one-layer-loop": config([latent(2, 96, 96, 200, ff=256), attention(8, 1, 80, ff=512)], 256, 128, loop=(1, 2, 2), cap=None),
     "all-looped": config([attention(3, 3, 16, q_temp=(0.9, 5), ff=40)], 67, 40, loop=(0, 1, 4), cap=5.0, eps=1e-2),
     "wide": config([attention(9, 3, 160, ff=1000), latent(16, 128, 64, 512, ff=700)], 517, 2112, loop=None),
+    "big-heads": config([attention(4, 2, 288, ff=64), latent(3, 300, 20, 600, ff=96), attention(2, 2, 520)], 97, 160,
+                        loop=(1, 3, 2)),
     "no-mlp": config([latent(1, 8, 8, 8), attention(1, 1, 8)], 33, 24, loop=(0, 2, 1)),
 }
 # scores far apart: every query depends on few keys, anywhere in its past

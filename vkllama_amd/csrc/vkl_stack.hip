@@ -1562,14 +1562,24 @@ stack_gemv_kernel (const GvArgs a)
           }
       }
   };
-  for (int it = 0; it < items; it += 2)
+  // (no branch around a request inside the loop: the waits then count exactly; the
+  // last one or two items stand behind it)
+  int it = 0;
+  for (; it + 2 < items; it += 2)
     {
       issue (it + 1, bufb);
       compute (it, bufa);
       issue (it + 2, bufa);
-      if (it + 1 < items)
-        compute (it + 1, bufb);
+      compute (it + 1, bufb);
     }
+  if (it + 1 < items)
+    {
+      issue (it + 1, bufb);
+      compute (it, bufa);
+      compute (it + 1, bufb);
+    }
+  else if (it < items)
+    compute (it, bufa);
   if (MODE != GV_LOGITS || !a.pick)
     return;
   // arg-max: the workgroup's best, then the last workgroup over all of them

@@ -131,6 +131,10 @@ Tensor::create ()
         "Tensor::create: negative extent (%d, %d, %d)", c_, h_, w_));
   release_ ();
   update_strides_ ();
+  // (strides are ints)
+  if ((size_t)h_ * (size_t)hs_ > 0x7fffffffu)
+    return absl::OutOfRangeError (absl::StrFormat (
+        "Tensor::create: a channel of (%d, %d) values exceeds 2 GiB", h_, w_));
   const size_t n = bytes ();
   void *p = nullptr;
   const int e = dev_->alloc (&p, n, visable_);
