@@ -248,6 +248,14 @@ constexpr int kRowHeads = 32;   // query heads of a workgroup at most
 constexpr int kRowTarget = 512; // workgroups a launch aims for
 constexpr float kNoKey = -1.0e30f;
 
+// The counters lie in front of the parts, in a block of fixed size, so that a
+// scratch area may serve launches of different shapes (each leaves its counters
+// at zero): only a split context has them, and there are at most kRowTarget / 2
+// of those workgroup rows then.
+// Every counter has a cache line of its own: arrivals at one line take turns.
+constexpr size_t kRowCounterStride = 32; // words
+constexpr size_t kRowCounterBytes = kRowTarget / 2 * kRowCounterStride * sizeof (uint32_t);
+
 struct RowAttnArgs
 {
   const void *q;
@@ -670,7 +678,7 @@ attn_rows_kernel (const RowAttnArgs a)
     }
   if (!a.cnt)
     return;
-  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, &last_s))
+  if (!last_of_parts (a.cnt + ((size_t)s * gridDim.y + gt) * kRowCounterStride, active, &last_s))
     return;
   combine_parts<kRowThreads> (a, HT, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * a.D, lds_rows);
 }
@@ -1014,7 +1022,7 @@ attn_rows_mfma_kernel (const RowAttnArgs a)
     }
   // (the flag lies behind what combine_parts uses of LDS)
   uint32_t *flag = (uint32_t *)((float *)lds_mf + combine_lds<kMfThreads> ());
-  if (!last_of_parts (a.cnt + (size_t)s * gridDim.y + gt, active, flag))
+  if (!last_of_parts (a.cnt + ((size_t)s * gridDim.y + gt) * kRowCounterStride, active, flag))
     return;
   combine_parts<kMfThreads> (a, ht, nh, active, pbase, (size_t)s * a.os + (size_t)h0 * D, (float *)lds_mf);
 }
@@ -1096,13 +1104,6 @@ launch_rows (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
     return launch_rows_ht<CT, 64, 1> (a, ht, grid, s);
   return launch_rows_ht<CT, 64, 2> (a, ht, grid, s);
 }
-
-// The counters lie in front of the parts, in a block of fixed size, so that a
-// scratch area may serve launches of different shapes (each leaves its counters
-// at zero): only a split context has them, and there are at most kRowTarget / 2
-// of those workgroup rows then.
-constexpr size_t kRowCounterBytes = 4096;
-static_assert (kRowTarget / 2 * sizeof (uint32_t) <= kRowCounterBytes, "a counter per workgroup row");
 
 size_t
 row_scratch_bytes (int ctype, int H, int G, int D, int S)
@@ -1202,7 +1203,9 @@ head_matvec_kernel (const HeadArgs a)
         store_elem (a.ncache, a.ntype, o + c, c < a.nW ? ldg (a.nx + c) * alpha * ldg (a.nw + c) : 0.f);
       return;
     }
-  const int h = blockIdx.x / a.bph, b = blockIdx.x - h * a.bph, s = blockIdx.y;
+  // (a head's workgroups are numbered so that, with a multiple of 8 heads, they
+  // share an XCD and what they read of the head)
+  const int h = blockIdx.x % a.heads, b = blockIdx.x / a.heads, s = blockIdx.y;
   constexpr int RPW = 64 / LPR;
   const int sub = lane % LPR, grp = lane / LPR;
   const int r0 = (b * 4 + wave) * RPW * kHeadRows + grp; // rows r0 + i * RPW
@@ -1327,15 +1330,27 @@ head_matvec (HeadArgs a, int S, hipStream_t s)
 // the weight-streaming product of the step
 // ---------------------------------------------------------------------------
 constexpr int kGvThreads = 512, kGvWaves = 8;
-constexpr int kGvSpan = 2048; // columns of an item: 4 loads of 512 columns per row
-constexpr int kGvRows = 2;    // rows of an item
-
 enum
 {
   GV_SEGS = 0,  // outputs by segment
   GV_ADD = 1,   // y[n] += sum
   GV_LOGITS = 2 // y[n] = soft cap, arg-max partials
 };
+
+// an item: 8 loads of 512 columns per lane; two rows of four, or, where rows are
+// few and long, one row of eight (every wave then has a row of its own)
+template <int MODE>
+constexpr int
+gv_rows ()
+{
+  return MODE == GV_ADD ? 1 : 2;
+}
+template <int MODE>
+constexpr int
+gv_span ()
+{
+  return 8 / gv_rows<MODE> () * 512;
+}
 
 struct GvSeg
 {
@@ -1387,28 +1402,29 @@ stack_gemv_kernel (const GvArgs a)
   __shared__ float bv_s[kGvWaves];
   __shared__ uint32_t bi_s[kGvWaves + 1];
   constexpr bool NORM = MODE != GV_ADD;
+  constexpr int ROWS = gv_rows<MODE> (), STEPS = 8 / ROWS, SPAN = gv_span<MODE> ();
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane (tid >> 6);
-  const int nspan = (a.K + kGvSpan - 1) / kGvSpan;
-  const int units = (a.N + kGvRows - 1) / kGvRows;
+  const int nspan = (a.K + SPAN - 1) / SPAN;
+  const int units = (a.N + ROWS - 1) / ROWS;
   const int w0 = blockIdx.x * kGvWaves + wave, nw = gridDim.x * kGvWaves;
   const int mine = w0 < units ? (units - w0 + nw - 1) / nw : 0;
   const int items = mine * nspan;
 
-  uint4 bufa[kGvRows * 4], bufb[kGvRows * 4];
-  auto issue = [&] (int it, uint4 (&b)[kGvRows * 4]) {
+  uint4 bufa[8], bufb[8];
+  auto issue = [&] (int it, uint4 (&b)[8]) {
     const int ic = min (it, max (items - 1, 0));
     const int un = ic / nspan, sp = ic - un * nspan;
-    const int row0 = min (w0 + un * nw, units - 1) * kGvRows;
+    const int row0 = min (w0 + un * nw, units - 1) * ROWS;
 #pragma unroll
-    for (int r = 0; r < kGvRows; ++r)
+    for (int r = 0; r < ROWS; ++r)
       {
         const uint16_t *p = a.w + (size_t)min (row0 + r, a.N - 1) * a.K;
 #pragma unroll
-        for (int u = 0; u < 4; ++u)
+        for (int u = 0; u < STEPS; ++u)
           {
-            const uint16_t *c = p + min (sp * kGvSpan + u * 512 + lane * 8, a.K - 8);
-            b[r * 4 + u] = NT ? ldg4_stream (c) : ldg4 (c);
+            const uint16_t *c = p + min (sp * SPAN + u * 512 + lane * 8, a.K - 8);
+            b[r * STEPS + u] = NT ? ldg4_stream (c) : ldg4 (c);
           }
       }
   };
@@ -1416,7 +1432,7 @@ stack_gemv_kernel (const GvArgs a)
     const int o = (c >> 9) * 512 + ((c >> 2) & 1) * 256 + ((c & 511) >> 3) * 4;
     *(float4 *)(xl + o) = v;
   };
-  const int kpad = nspan * kGvSpan;
+  const int kpad = nspan * SPAN;
   if constexpr (XV > 0)
     {
       float4 xv[XV], nv[XV];
@@ -1493,25 +1509,25 @@ stack_gemv_kernel (const GvArgs a)
   __syncthreads ();
 
   const uint32_t pos = MODE == GV_SEGS ? a.pos.get () : 0u;
-  float sum[kGvRows];
+  float sum[ROWS];
 #pragma unroll
-  for (int r = 0; r < kGvRows; ++r)
+  for (int r = 0; r < ROWS; ++r)
     sum[r] = 0.f;
   float best_v = -INFINITY;
   uint32_t best_i = 0xffffffffu;
-  auto compute = [&] (int it, const uint4 (&b)[kGvRows * 4]) {
+  auto compute = [&] (int it, const uint4 (&b)[8]) {
     const int un = it / nspan, sp = it - un * nspan;
 #pragma unroll
-    for (int u = 0; u < 4; ++u)
+    for (int u = 0; u < STEPS; ++u)
       {
-        const float *xp = xl + (sp * 4 + u) * 512 + lane * 4;
+        const float *xp = xl + (sp * STEPS + u) * 512 + lane * 4;
         const float4 x0 = *(const float4 *)xp, x1 = *(const float4 *)(xp + 256);
         const float xv[8] = { x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w };
 #pragma unroll
-        for (int r = 0; r < kGvRows; ++r)
+        for (int r = 0; r < ROWS; ++r)
           {
             float f[8];
-            widen8 (b[r * 4 + u], f);
+            widen8 (b[r * STEPS + u], f);
 #pragma unroll
             for (int e = 0; e < 8; ++e)
               sum[r] = __builtin_fmaf (f[e], xv[e], sum[r]);
@@ -1519,9 +1535,9 @@ stack_gemv_kernel (const GvArgs a)
       }
     if (sp != nspan - 1)
       return;
-    const int row0 = (w0 + un * nw) * kGvRows;
+    const int row0 = (w0 + un * nw) * ROWS;
 #pragma unroll
-    for (int r = 0; r < kGvRows; ++r)
+    for (int r = 0; r < ROWS; ++r)
       {
         float v = wave_sum (sum[r]);
         sum[r] = 0.f;
@@ -1638,7 +1654,7 @@ constexpr int kGvMaxLds = 128 << 10;
 bool
 gv_supported (int K)
 {
-  return (size_t)((K + kGvSpan - 1) / kGvSpan) * kGvSpan * sizeof (float) <= (size_t)kGvMaxLds;
+  return (size_t)((K + 4095) / 4096) * 4096 * sizeof (float) <= (size_t)kGvMaxLds; // (the longest span)
 }
 
 template <int MODE, int XV, bool NT>
@@ -1665,10 +1681,12 @@ launch_gv (const GvArgs &a, int n_cu, hipStream_t s)
 {
   if (!gv_supported (a.K))
     return (int)hipErrorInvalidValue;
-  const int units = (a.N + kGvRows - 1) / kGvRows;
+  constexpr int SPAN = gv_span<MODE> ();
+  const int units = (a.N + gv_rows<MODE> () - 1) / gv_rows<MODE> ();
   const int grid = std::min (2 * n_cu, (units + kGvWaves - 1) / kGvWaves);
-  const size_t lds = (size_t)((a.K + kGvSpan - 1) / kGvSpan) * kGvSpan * sizeof (float);
-  if (a.K <= 2048)
+  const size_t lds = (size_t)((a.K + SPAN - 1) / SPAN) * SPAN * sizeof (float);
+  // (the loads of the row have to cover its padding to whole spans)
+  if (SPAN == 2048 && a.K <= 2048)
     return launch_gv_k<MODE, 1> (a, grid, lds, s);
   if (a.K <= 4096)
     return launch_gv_k<MODE, 2> (a, grid, lds, s);
