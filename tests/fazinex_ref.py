@@ -28,8 +28,8 @@ def query_temperature(p, coef, every):
 
 
 def causal_attention(q, k, v, scale):
-    """q [T, H, d], k [T, G, d], v [T, G, e] -> [T, H, e]; query head h reads
-    key/value head h // (H / G); position i sees positions 0 .. i."""
+    """q [T, H, d], k [T, G, d], v [T, G, e] -> [T, H, e]; runs of H / G query
+    heads share a key/value head, a row attends to itself and what came before."""
     T, H, _ = q.shape
     G = k.shape[1]
     out = np.zeros((T, H, v.shape[2]))
@@ -41,8 +41,8 @@ def causal_attention(q, k, v, scale):
 
 
 def shared_kv_attention(h, get, m):
-    """The values are the keys as projected; positions enter through a factor
-    on the queries only."""
+    """One projection serves as keys and as values; besides the mask, positions
+    enter through a factor on the queries."""
     T = h.shape[0]
     H, G, d = m["heads"], m["kv_heads"], m["dim"]
     q = (h @ get("q").T).reshape(T, H, d)

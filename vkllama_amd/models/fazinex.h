@@ -2,9 +2,9 @@
 // feeds its token mixer and its feed-forward part in parallel; both add into an
 // fp32 residual stream:
 //   h = rms_norm (x) w;  x += mixer (h) + W_down relu (W_up h)^2
-// Mixers: shared key/value attention and gated latent attention (src/ops).  A
-// range of layers may run several times in a row, each run with a cache of its
-// own.  The embedding table, normed on the way in, is the output matrix too; the
+// Mixers: shared key/value attention and gated latent attention (src/ops).  The
+// configuration may have a stretch of layers repeated, each run with a cache of
+// its own.  The embedding table, normed on the way in, is the output matrix too; the
 // logits are soft-capped.
 //
 // A layer is two products: [queries | keys or latent | gates | feed-forward up]

@@ -1,5 +1,5 @@
-// SharedKVAttention: grouped-query attention whose values are the keys as
-// projected, without rotation; positions enter through the mask and a
+// SharedKVAttention: grouped-query attention in which one projection serves as
+// keys and as values, without rotation; positions enter through the mask and a
 // logarithmic factor on the queries.  Not part of the reference.
 #ifndef __VKLLAMA_SHARED_KV_ATTENTION_H__
 #define __VKLLAMA_SHARED_KV_ATTENTION_H__
