@@ -41,6 +41,7 @@
 // A second, small kernel in this file prepares the inputs of the first from
 // the projection outputs: RoPE of Q (in place) and K, and the K/V cache write.
 #include "../../include/vkl_hip.h"
+#include "../../include/vkl_stack.h"
 #include "vkl_common.h"
 
 namespace
@@ -67,6 +68,7 @@ struct AttnArgs
   int temp_every;
   const float *gate;  // optional [S, gs]: head h's output times sigmoid (gate[s, h])
   size_t gs;
+  int chunk, sink;    // CHUNKED kernels: see vkl_attn_prefill_chunked_bf16
 };
 
 // the two element types of the operands
@@ -228,7 +230,9 @@ score_block (const uint16_t *Ks, int blk, const typename E::v8 (&qf)[HD / 16], i
 }
 
 // (heads wider than 128 values: one workgroup per compute unit, twice the registers)
-template <int HD, class E>
+// CHUNKED: a query sees keys from the start of its own chunk of positions on, and
+// the softmax may have a sink (a score of 0 without a value)
+template <int HD, class E, bool CHUNKED = false>
 __global__ __launch_bounds__ (kThreads, HD <= 128 ? 2 : 1) void
 attn_prefill_kernel (const AttnArgs a)
 {
@@ -266,6 +270,11 @@ attn_prefill_kernel (const AttnArgs a)
   const int kmax = min (a.L, q0 + kBQ + shift);
   const int ntile = (kmax + kBKey - 1) / kBKey;
   const int wave_last = q0 + wave * 32 + 31 + shift; // last key any query of the wave sees
+  // first key of the chunk of this lane's query, of the wave's first and last
+  auto chunk_start = [&] (int row) { return CHUNKED && a.chunk ? (row + shift) / a.chunk * a.chunk : 0; };
+  const int klow = chunk_start (qrow), wave_low = chunk_start (q0 + wave * 32);
+  const int wave_high = chunk_start (q0 + wave * 32 + 31);
+  const int t0 = CHUNKED ? chunk_start (q0) / kBKey : 0;
   const int kvh = E::round_scores ? head : head / a.rep;
   const uint16_t *kb = a.k + (size_t)kvh * a.kcs;
   const uint16_t *vb = a.v + (size_t)kvh * a.vcs;
@@ -286,16 +295,18 @@ attn_prefill_kernel (const AttnArgs a)
   // One pass over the keys with a running maximum: the accumulated products
   // and the sum of exponentials are rescaled whenever the maximum grows, and
   // the division by the sum comes last.
-  float m = kNeg, sum = 0.f;
+  // (the sink is a key that every query has seen before the first tile; the sums of
+  // the two lane halves are added at the end, one of them has it)
+  float m = CHUNKED && a.sink ? 0.f : kNeg, sum = CHUNKED && a.sink && hh == 0 ? 1.f : 0.f;
   float16v oacc[DB];
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
     for (int r = 0; r < 16; ++r)
       oacc[db][r] = 0.f;
-  load_k<HD> (a, kb, 0, tl);
-  load_v<HD> (a, vb, 0, tl);
-  for (int t = 0; t < ntile; ++t)
+  load_k<HD> (a, kb, t0, tl);
+  load_v<HD> (a, vb, t0, tl);
+  for (int t = t0; t < ntile; ++t)
     {
       __syncthreads ();
       store_k<HD> (tl, Ks);
@@ -306,13 +317,14 @@ attn_prefill_kernel (const AttnArgs a)
           load_k<HD> (a, kb, t + 1, tl);
           load_v<HD> (a, vb, t + 1, tl);
         }
-      if (t * kBKey > wave_last)
+      if (t * kBKey > wave_last || (CHUNKED && t * kBKey + kBKey <= wave_low))
         continue;
       // scores of the tile's 64 keys, rounded to fp16 like the stand-alone
       // product; a key the query must not see counts as "never seen"
       float sv[2][16];
       float bm = kNeg;
-      const bool inner = t * kBKey + kBKey - 1 <= q0 + wave * 32 + shift; // every key visible to every query of the wave
+      const bool inner = t * kBKey + kBKey - 1 <= q0 + wave * 32 + shift // every key visible to every query of the wave
+                         && (!CHUNKED || t * kBKey >= wave_high);
 #pragma unroll
       for (int blk = 0; blk < 2; ++blk)
         {
@@ -323,7 +335,7 @@ attn_prefill_kernel (const AttnArgs a)
             {
               const int key = key0 + 8 * (r >> 2) + (r & 3);
               const float sc = E::round_scores ? vkl::h2f (vkl::f2h (acc[r] * scale)) : acc[r] * scale;
-              sv[blk][r] = inner || key <= qrow + shift ? sc : kNeg;
+              sv[blk][r] = inner || (key <= qrow + shift && (!CHUNKED || key >= klow)) ? sc : kNeg;
               bm = fmaxf (bm, sv[blk][r]);
             }
         }
@@ -351,7 +363,10 @@ attn_prefill_kernel (const AttnArgs a)
             // exp (kNeg - m) = 0.  The sum takes the weight as the product
             // below consumes it, rounded to fp16: the weights then add up to
             // one exactly.
-            const typename E::t e = (typename E::t)fast_exp (sv[blk][r] - m);
+            // (a query that has not seen any key yet has m = kNeg: the guard keeps
+            // its weights at zero)
+            const float w = CHUNKED && sv[blk][r] == kNeg ? 0.f : fast_exp (sv[blk][r] - m);
+            const typename E::t e = (typename E::t)w;
             sum += (float)e;
             pf[blk][r >> 3][r & 7] = e;
           }
@@ -521,41 +536,71 @@ vkl_attn_prefill_causal_f16 (const void *q, const void *k, const void *v,
   return vkl_launch_status ();
 }
 
+namespace
+{
+template <bool CHUNKED>
+int
+launch_prefill_bf16 (const AttnArgs &a, int hd, hipStream_t s)
+{
+  const dim3 grid ((unsigned)(a.ntq * a.H)), block (kThreads);
+  switch (hd)
+    {
+    case 32: attn_prefill_kernel<32, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 64: attn_prefill_kernel<64, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 96: attn_prefill_kernel<96, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 128: attn_prefill_kernel<128, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 160: attn_prefill_kernel<160, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 192: attn_prefill_kernel<192, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    case 224: attn_prefill_kernel<224, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    default: attn_prefill_kernel<256, Bf16Elem, CHUNKED><<<grid, block, 0, s>>> (a); break;
+    }
+  return vkl_launch_status ();
+}
+
+int
+prefill_args_bf16 (AttnArgs &a, const void *q, const void *k, const void *v, int H, int G, int S, int L, int hd,
+                   size_t qhs, size_t khs, size_t vhs, float scale, void *out, size_t ors)
+{
+  VKL_CHECK_ARG (q && k && v && out);
+  VKL_CHECK_ARG (H > 0 && G > 0 && (H % G) == 0 && S > 0 && L >= S);
+  VKL_CHECK_ARG (hd > 0 && (hd % 32) == 0 && hd <= 256);
+  VKL_CHECK_ARG (((uintptr_t)q % 16) == 0 && ((uintptr_t)k % 16) == 0 && ((uintptr_t)v % 16) == 0
+                 && ((uintptr_t)out % 8) == 0);
+  VKL_CHECK_ARG ((qhs % 8) == 0 && (khs % 8) == 0 && (vhs % 8) == 0 && (ors % 4) == 0);
+  VKL_CHECK_ARG (qhs >= (size_t)H * hd && khs >= (size_t)G * hd && vhs >= (size_t)G * hd && ors >= (size_t)H * hd);
+  a.q = (const uint16_t *)q, a.k = (const uint16_t *)k, a.v = (const uint16_t *)v;
+  a.out = (uint16_t *)out;
+  a.H = H, a.S = S, a.L = L, a.ntq = (S + kBQ - 1) / kBQ;
+  a.qcs = a.kcs = a.vcs = a.ohs = (size_t)hd;
+  a.qhs = qhs, a.khs = khs, a.vhs = vhs, a.ors = ors;
+  a.scale = scale, a.rep = H / G;
+  return 0;
+}
+} // namespace
+
 extern "C" int
 vkl_attn_prefill_causal_bf16 (const void *q, const void *k, const void *v, int H, int G, int S, int L, int hd,
                               size_t qhs, size_t khs, size_t vhs, float scale, float temp_coef,
                               int temp_every, const float *gate, size_t gs, void *out, size_t ors,
                               void *stream)
 {
-  VKL_CHECK_ARG (q && k && v && out);
-  VKL_CHECK_ARG (H > 0 && G > 0 && (H % G) == 0 && S > 0 && L >= S);
-  VKL_CHECK_ARG (hd > 0 && (hd % 32) == 0 && hd <= 256);
-  VKL_CHECK_ARG (temp_coef == 0.f || temp_every > 0);
-  VKL_CHECK_ARG (((uintptr_t)q % 16) == 0 && ((uintptr_t)k % 16) == 0 && ((uintptr_t)v % 16) == 0
-                 && ((uintptr_t)out % 8) == 0);
-  VKL_CHECK_ARG ((qhs % 8) == 0 && (khs % 8) == 0 && (vhs % 8) == 0 && (ors % 4) == 0);
-  VKL_CHECK_ARG (qhs >= (size_t)H * hd && khs >= (size_t)G * hd && vhs >= (size_t)G * hd
-                 && ors >= (size_t)H * hd && (!gate || gs >= (size_t)H));
   AttnArgs a = {};
-  a.q = (const uint16_t *)q, a.k = (const uint16_t *)k, a.v = (const uint16_t *)v;
-  a.out = (uint16_t *)out;
-  a.H = H, a.S = S, a.L = L, a.ntq = (S + kBQ - 1) / kBQ;
-  a.qcs = a.kcs = a.vcs = a.ohs = (size_t)hd;
-  a.qhs = qhs, a.khs = khs, a.vhs = vhs, a.ors = ors;
-  a.scale = scale, a.rep = H / G, a.temp_coef = temp_coef, a.temp_every = temp_every;
-  a.gate = gate, a.gs = gs;
-  const dim3 grid ((unsigned)(a.ntq * H)), block (kThreads);
-  hipStream_t s = (hipStream_t)stream;
-  switch (hd)
-    {
-    case 32: attn_prefill_kernel<32, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 64: attn_prefill_kernel<64, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 96: attn_prefill_kernel<96, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 128: attn_prefill_kernel<128, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 160: attn_prefill_kernel<160, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 192: attn_prefill_kernel<192, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    case 224: attn_prefill_kernel<224, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    default: attn_prefill_kernel<256, Bf16Elem><<<grid, block, 0, s>>> (a); break;
-    }
-  return vkl_launch_status ();
+  if (int e = prefill_args_bf16 (a, q, k, v, H, G, S, L, hd, qhs, khs, vhs, scale, out, ors))
+    return e;
+  VKL_CHECK_ARG ((temp_coef == 0.f || temp_every > 0) && (!gate || gs >= (size_t)H));
+  a.temp_coef = temp_coef, a.temp_every = temp_every, a.gate = gate, a.gs = gs;
+  return launch_prefill_bf16<false> (a, hd, (hipStream_t)stream);
+}
+
+extern "C" int
+vkl_attn_prefill_chunked_bf16 (const void *q, const void *k, const void *v, int H, int G, int S, int L, int hd,
+                               size_t qhs, size_t khs, size_t vhs, float scale, int chunk, int sink, void *out,
+                               size_t ors, void *stream)
+{
+  AttnArgs a = {};
+  if (int e = prefill_args_bf16 (a, q, k, v, H, G, S, L, hd, qhs, khs, vhs, scale, out, ors))
+    return e;
+  VKL_CHECK_ARG (chunk >= 0);
+  a.chunk = chunk, a.sink = sink;
+  return launch_prefill_bf16<true> (a, hd, (hipStream_t)stream);
 }

@@ -51,7 +51,7 @@ struct GemmSeg
   void *y;               // [M, n], row stride ys
   size_t ys;
   int f32;               // y in fp32, else bf16
-  int act;               // 0 none, 2 the square of relu
+  int act;               // VKL_ACT_...
   const float *residual; // fp32 y only: y = residual + v
   float cap;             // > 0: cap * tanh (v / cap)
   int vec;               // rows of y allow vector stores

@@ -2,6 +2,7 @@
 // eight neighbouring output columns per lane.
 #ifndef VKL_GEMM_FINISH_H
 #define VKL_GEMM_FINISH_H
+#include "vkl_act.h"
 #include "vkl_common.h"
 #include "vkl_gemm.h"
 
@@ -102,11 +103,7 @@ gemm_finish8 (const GemmArgs &a, float (&v)[8], const float (&g)[8], int m, int 
 __device__ __forceinline__ float
 seg_value (const GemmSeg &sg, float v)
 {
-  if (sg.act == 2)
-    {
-      v = fmaxf (v, 0.f);
-      v = v * v;
-    }
+  v = activate (sg.act, v);
   if (sg.cap > 0.f)
     v = sg.cap * tanhf (v / sg.cap);
   return v;

@@ -896,7 +896,7 @@ vkl_project_bf16w (const void *x, int xtype, size_t xs, const void *w, int M, in
       const vkl_out_seg &o = segs[i];
       VKL_CHECK_ARG (o.y && o.n > 0 && o.n0 >= end && (o.n0 % 8) == 0 && o.n0 + o.n <= N && o.ys >= (size_t)o.n);
       VKL_CHECK_ARG (i > 0 || o.n0 == 0);
-      VKL_CHECK_ARG (o.act == 0 || o.act == 2);
+      VKL_CHECK_ARG (o.act >= VKL_ACT_NONE && o.act <= VKL_ACT_GELU);
       VKL_CHECK_ARG (o.type == VKL_TYPE_F32 || (o.type == VKL_TYPE_BF16 && !o.residual));
       vkl::GemmSeg &g = a.seg[i];
       g.n0 = o.n0, g.n = o.n, g.y = o.y, g.ys = o.ys, g.f32 = o.type == VKL_TYPE_F32;

@@ -19,9 +19,8 @@
 //      concatenated inputs, added into the residual row
 // then final norm + tied output matrix + soft cap + arg-max.
 #include "../../include/vkl_stack.h"
-#include "vkl_common.h"
-#include "vkl_decode_dev.h"
 #include "vkl_gemm.h"
+#include "vkl_stack_dev.h"
 #include <algorithm>
 #include <mutex>
 #include <vector>
@@ -30,67 +29,6 @@ namespace vkl
 {
 namespace
 {
-// a position known on the host, or kept on the device by a replayed loop
-// ({index into the ids, position})
-struct StepPos
-{
-  const uint32_t *loop;
-  uint32_t val;
-  __device__ __forceinline__ uint32_t
-  get () const
-  {
-    return loop ? ldg (loop + 1) : val;
-  }
-};
-
-__device__ __forceinline__ void
-widen8 (const uint4 w, float (&f)[8])
-{
-  const uint32_t u[4] = { w.x, w.y, w.z, w.w };
-#pragma unroll
-  for (int i = 0; i < 4; ++i)
-    {
-      f[2 * i] = __uint_as_float (u[i] << 16);
-      f[2 * i + 1] = __uint_as_float (u[i] & 0xffff0000u);
-    }
-}
-
-__device__ __forceinline__ float
-sigmoid (float z)
-{
-  return 1.0f / (1.0f + expf (-z));
-}
-
-__device__ __forceinline__ float
-load_elem (const void *p, int type, size_t i)
-{
-  return type == VKL_TYPE_F32 ? ldg ((const float *)p + i) : bf2f (ldg ((const uint16_t *)p + i));
-}
-
-__device__ __forceinline__ void
-store_elem (void *p, int type, size_t i, float v)
-{
-  if (type == VKL_TYPE_F32)
-    stg ((float *)p + i, v);
-  else
-    stg ((uint16_t *)p + i, f2bf (v));
-}
-
-// sum over a workgroup of up to 1024 threads; red: a float of LDS per wave
-__device__ __forceinline__ float
-group_sum (float v, float *red)
-{
-  v = wave_sum (v);
-  if ((threadIdx.x & 63) == 0)
-    red[threadIdx.x >> 6] = v;
-  __syncthreads ();
-  float s = 0.f;
-  for (unsigned i = 0; i < blockDim.x / 64; ++i)
-    s += red[i];
-  __syncthreads ();
-  return s;
-}
-
 // ---------------------------------------------------------------------------
 // embedding and norms
 // ---------------------------------------------------------------------------
@@ -101,8 +39,8 @@ struct EmbedArgs
   int K, W;
   const uint32_t *toks;
   const uint32_t *loop; // replayed loop: the token is toks[loop[0]]
-  const float *w;
-  float eps;
+  const float *w; // null: the plain rows times scale
+  float eps, scale;
   float *out;
   size_t os;
 };
@@ -148,7 +86,7 @@ embed_norm_kernel (const EmbedArgs a)
           {
             const int c = (tid + j * 1024) * 8 + e;
             if (c < a.W)
-              stg (out + c, a.w ? v[j][e] * alpha * w[j][e] : v[j][e]);
+              stg (out + c, a.w ? v[j][e] * alpha * w[j][e] : v[j][e] * a.scale);
           }
       return;
     }
@@ -166,7 +104,7 @@ embed_norm_kernel (const EmbedArgs a)
   for (int c = tid; c < a.W; c += 1024)
     {
       const float v = bf2f (ldg (row + c));
-      stg (out + c, a.w ? v * alpha * ldg (a.w + c) : v);
+      stg (out + c, a.w ? v * alpha * ldg (a.w + c) : v * a.scale);
     }
 }
 
@@ -261,8 +199,9 @@ struct RowAttnArgs
   const void *q;
   int qtype;
   size_t qs;
-  const void *rows;
+  const void *rows, *vals; // vals: values of their own (null: the rows are keys and values)
   size_t rs;
+  int chunk, sink; // a position sees its own chunk (0: everything before it); a score 0 without a value
   int G, D, rep, tiles, ht; // rep: query heads per group; tiles of ht heads
   StepPos pos;
   float scale, tcoef;
@@ -388,6 +327,7 @@ combine_lds ()
 // a whole workgroup: a wave per head for the weights, lane p holding part p, then
 // four neighbouring values per thread with the parts dealt to groups of 128
 // threads.  The first values are requested together with the maxima and sums.
+// (a sink takes part in the maximum and in the sum)
 template <int THREADS>
 __device__ __forceinline__ void
 combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, size_t out0, float *lds)
@@ -420,9 +360,9 @@ combine_parts (const RowAttnArgs &a, int ht, int nh, int active, size_t pbase, s
   for (int i = 0; i < HW; ++i)
     if (wave + NW * i < nh)
       {
-        const float M = wave_max (mv[i]);
+        const float M = a.sink ? fmaxf (wave_max (mv[i]), 0.f) : wave_max (mv[i]);
         const float f = lane < active ? expf (mv[i] - M) : 0.f;
-        wgt[(wave + NW * i) * kRowSplits + lane] = f / wave_sum (f * lv[i]);
+        wgt[(wave + NW * i) * kRowSplits + lane] = f / (wave_sum (f * lv[i]) + (a.sink ? expf (-M) : 0.f));
       }
   __syncthreads ();
   for (int o0 = 0; o0 < outs; o0 += 128)
@@ -483,7 +423,8 @@ last_of_parts (uint32_t *cnt, int active, uint32_t *flag)
 // LPR lanes share a row, NCH chunks of 8 values per lane; HT query heads per
 // workgroup.  Every group of LPR lanes walks rows of its own with a running
 // maximum; the groups' results meet in LDS at the end.
-template <typename CT, int LPR, int NCH, int HT>
+// VALS: values of their own, chunks and a sink.
+template <typename CT, int LPR, int NCH, int HT, bool VALS>
 __global__ __launch_bounds__ (kRowThreads) void
 attn_rows_kernel (const RowAttnArgs a)
 {
@@ -496,7 +437,9 @@ attn_rows_kernel (const RowAttnArgs a)
   const int s = blockIdx.z, gt = blockIdx.y;
   const int g = gt / a.tiles, t = gt - g * a.tiles;
   const uint32_t pos = a.pos.get () + (uint32_t)s;
-  const int L = (int)pos + 1;
+  // the rows are counted from the first one that is visible
+  const uint32_t low = VALS && a.chunk ? pos / (uint32_t)a.chunk * (uint32_t)a.chunk : 0u;
+  const int L = (int)(pos - low) + 1;
   const int chunk = row_chunk (L, a.nsplit, STEP);
   const int active = (L + chunk - 1) / chunk;
   const int c = blockIdx.x;
@@ -507,20 +450,26 @@ attn_rows_kernel (const RowAttnArgs a)
   const int sub = lane % LPR, grp = lane / LPR, slot = tid / LPR;
 
   const int col[2] = { sub * 8, LPR * 8 + sub * 8 };
-  const CT *base = (const CT *)a.rows + (size_t)g * a.D;
+  const CT *base = (const CT *)a.rows + (size_t)low * a.rs + (size_t)g * a.D;
+  const CT *vbase = VALS ? (const CT *)a.vals + (size_t)low * a.rs + (size_t)g * a.D : nullptr;
   int cc[NCH]; // columns clamped into the row (lanes past its end contribute q = 0)
 #pragma unroll
   for (int n = 0; n < NCH; ++n)
     cc[n] = min (col[n], a.D - 8);
 
   // the first rows travel while the queries are fetched
-  RowVec<CT> nx[U][NCH];
+  RowVec<CT> nx[U][NCH], nv[VALS ? U : 1][NCH];
   auto issue = [&] (int lb) {
 #pragma unroll
     for (int u = 0; u < U; ++u)
 #pragma unroll
       for (int n = 0; n < NCH; ++n)
-        nx[u][n].load (base + (size_t)min (lb + (u * 4 + wave) * RPW + grp, l1 - 1) * a.rs + cc[n]);
+        {
+          const size_t o = (size_t)min (lb + (u * 4 + wave) * RPW + grp, l1 - 1) * a.rs + cc[n];
+          nx[u][n].load (base + o);
+          if constexpr (VALS)
+            nv[u][n].load (vbase + o);
+        }
   };
   issue (l0);
   __builtin_amdgcn_sched_barrier (0);
@@ -557,7 +506,7 @@ attn_rows_kernel (const RowAttnArgs a)
 
   for (int lb = l0; lb < l1; lb += STEP)
     {
-      float row[U][NCH * 8];
+      float row[U][NCH * 8], val[VALS ? U : 1][NCH * 8];
 #pragma unroll
       for (int u = 0; u < U; ++u)
 #pragma unroll
@@ -568,6 +517,13 @@ attn_rows_kernel (const RowAttnArgs a)
 #pragma unroll
             for (int e = 0; e < 8; ++e)
               row[u][n * 8 + e] = f[e];
+            if constexpr (VALS)
+              {
+                nv[u][n].get (f);
+#pragma unroll
+                for (int e = 0; e < 8; ++e)
+                  val[u][n * 8 + e] = f[e];
+              }
           }
       issue (min (lb + STEP, l1 - 1));
 #pragma unroll
@@ -600,7 +556,7 @@ attn_rows_kernel (const RowAttnArgs a)
               l[h] += p;
 #pragma unroll
               for (int e = 0; e < NCH * 8; ++e)
-                acc[h][e] = __builtin_fmaf (p, row[u][e], acc[h][e]);
+                acc[h][e] = __builtin_fmaf (p, VALS ? val[u][e] : row[u][e], acc[h][e]);
             }
         }
     }
@@ -611,11 +567,12 @@ attn_rows_kernel (const RowAttnArgs a)
     for (int h = 0; h < HT; ++h)
       sm[slot][h] = m[h];
   __syncthreads ();
+  const bool whole = a.cnt && active == 1; // no other part: the sink belongs here
   float M[HT];
 #pragma unroll
   for (int h = 0; h < HT; ++h)
     {
-      float v = kNoKey;
+      float v = VALS && a.sink && whole ? 0.f : kNoKey;
 #pragma unroll
       for (int i = 0; i < NS; ++i)
         v = fmaxf (v, sm[i][h]);
@@ -646,10 +603,17 @@ attn_rows_kernel (const RowAttnArgs a)
       if (!a.cnt)
         stg ((vkl_u32x4 *)dst, vkl_u32x4{ __float_as_uint (v[0]), __float_as_uint (v[1]), __float_as_uint (v[2]),
                                           __float_as_uint (v[3]) });
-      else if (active == 1)
+      else if (whole)
         {
           for (int i = 0; i < NS; ++i)
             S += sl[i][h];
+          if (VALS && a.sink)
+            {
+              float mm = 0.f;
+              for (int i = 0; i < NS; ++i)
+                mm = fmaxf (mm, sm[i][h]);
+              S += expf (-mm);
+            }
 #pragma unroll
           for (int e = 0; e < 4; ++e)
             store_elem (a.out, a.otype, (size_t)s * a.os + (size_t)(h0 + h) * a.D + d + e, v[e] / S);
@@ -658,7 +622,7 @@ attn_rows_kernel (const RowAttnArgs a)
         // (write-through: the workgroup that combines may be on another XCD)
         st_coherent_16 (dst, v);
     }
-  if (a.cnt && active == 1)
+  if (whole)
     return;
   if (tid < nh)
     {
@@ -697,9 +661,9 @@ row_head_tile (int rep, int D)
 // the matrix-core form: bf16 rows that several heads share, of the sizes it is
 // instantiated for
 bool
-row_mfma (int ctype, int rep, int D)
+row_mfma (int ctype, int rep, int D, bool vals = false)
 {
-  return ctype == VKL_TYPE_BF16 && rep >= 2 && (D <= 256 || (D <= 512 && D % 64 == 0));
+  return !vals && ctype == VKL_TYPE_BF16 && rep >= 2 && (D <= 256 || (D <= 512 && D % 64 == 0));
 }
 
 struct RowPlan
@@ -710,11 +674,11 @@ struct RowPlan
 };
 
 RowPlan
-row_plan (int ctype, int H, int G, int D, int S)
+row_plan (int ctype, int H, int G, int D, int S, bool vals = false)
 {
   RowPlan p;
   const int rep = H / G;
-  p.mfma = row_mfma (ctype, rep, D);
+  p.mfma = row_mfma (ctype, rep, D, vals);
   p.ht = p.mfma ? std::min (rep, kRowHeads) : row_head_tile (rep, D);
   p.tiles = (rep + p.ht - 1) / p.ht;
   const long groups = (long)G * p.tiles * S;
@@ -1060,55 +1024,55 @@ launch_mfma (const RowAttnArgs &a, dim3 grid, hipStream_t s)
     }
 }
 
-template <typename CT, int LPR, int NCH, int HT>
+template <typename CT, int LPR, int NCH, int HT, bool VALS>
 int
 launch_rows_k (const RowAttnArgs &a, dim3 grid, hipStream_t s)
 {
   static LdsLimit limit;
   const size_t lds = sizeof (float) * std::max ((size_t)kRowThreads * 8 * NCH * HT, (size_t)combine_lds<kRowThreads> ());
-  if (int e = limit.raise ((const void *)attn_rows_kernel<CT, LPR, NCH, HT>, lds))
+  if (int e = limit.raise ((const void *)attn_rows_kernel<CT, LPR, NCH, HT, VALS>, lds))
     return e;
-  attn_rows_kernel<CT, LPR, NCH, HT><<<grid, dim3 (kRowThreads), lds, s>>> (a);
+  attn_rows_kernel<CT, LPR, NCH, HT, VALS><<<grid, dim3 (kRowThreads), lds, s>>> (a);
   return (int)hipGetLastError ();
 }
 
-template <typename CT, int LPR, int NCH>
+template <typename CT, int LPR, int NCH, bool VALS>
 int
 launch_rows_ht (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
 {
   switch (ht)
     {
-    case 1: return launch_rows_k<CT, LPR, NCH, 1> (a, grid, s);
-    case 2: return launch_rows_k<CT, LPR, NCH, 2> (a, grid, s);
-    case 4: return launch_rows_k<CT, LPR, NCH, 4> (a, grid, s);
+    case 1: return launch_rows_k<CT, LPR, NCH, 1, VALS> (a, grid, s);
+    case 2: return launch_rows_k<CT, LPR, NCH, 2, VALS> (a, grid, s);
+    case 4: return launch_rows_k<CT, LPR, NCH, 4, VALS> (a, grid, s);
     default:
       if constexpr (LPR <= 32)
-        return launch_rows_k<CT, LPR, NCH, 8> (a, grid, s);
+        return launch_rows_k<CT, LPR, NCH, 8, VALS> (a, grid, s);
       return (int)hipErrorInvalidValue;
     }
 }
 
-template <typename CT>
+template <typename CT, bool VALS>
 int
 launch_rows (const RowAttnArgs &a, int ht, dim3 grid, hipStream_t s)
 {
   if (a.D <= 32)
-    return launch_rows_ht<CT, 4, 1> (a, ht, grid, s);
+    return launch_rows_ht<CT, 4, 1, VALS> (a, ht, grid, s);
   if (a.D <= 64)
-    return launch_rows_ht<CT, 8, 1> (a, ht, grid, s);
+    return launch_rows_ht<CT, 8, 1, VALS> (a, ht, grid, s);
   if (a.D <= 128)
-    return launch_rows_ht<CT, 16, 1> (a, ht, grid, s);
+    return launch_rows_ht<CT, 16, 1, VALS> (a, ht, grid, s);
   if (a.D <= 256)
-    return launch_rows_ht<CT, 32, 1> (a, ht, grid, s);
+    return launch_rows_ht<CT, 32, 1, VALS> (a, ht, grid, s);
   if (a.D <= 512)
-    return launch_rows_ht<CT, 64, 1> (a, ht, grid, s);
-  return launch_rows_ht<CT, 64, 2> (a, ht, grid, s);
+    return launch_rows_ht<CT, 64, 1, VALS> (a, ht, grid, s);
+  return launch_rows_ht<CT, 64, 2, VALS> (a, ht, grid, s);
 }
 
 size_t
-row_scratch_bytes (int ctype, int H, int G, int D, int S)
+row_scratch_bytes (int ctype, int H, int G, int D, int S, bool vals = false)
 {
-  const RowPlan p = row_plan (ctype, H, G, D, S);
+  const RowPlan p = row_plan (ctype, H, G, D, S, vals);
   return kRowCounterBytes + p.parts * (2 + (size_t)D) * sizeof (float) + 256;
 }
 
@@ -1127,27 +1091,141 @@ row_step (int D)
   return 4 * (64 / lpr) * kRowUnroll;
 }
 
+// an attention launch over p: the plan and the scratch area fill in the rest
 int
-rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype, size_t rs, int H, int G, int D,
-                int S, StepPos pos, float scale, float tcoef, int tevery, void *out, int otype, size_t os,
-                void *scratch, RowParts *parts, hipStream_t s)
+rows_launch (RowAttnArgs a, int ctype, int H, int S, void *scratch, RowParts *parts, hipStream_t s)
 {
-  const RowPlan p = row_plan (ctype, H, G, D, S);
-  RowAttnArgs a = {};
-  a.q = q, a.qtype = qtype, a.qs = qs, a.rows = rows, a.rs = rs;
-  a.G = G, a.D = D, a.rep = H / G, a.tiles = p.tiles, a.ht = p.ht;
-  a.pos = pos, a.scale = scale, a.tcoef = tcoef, a.tevery = tevery;
-  a.out = out, a.otype = otype, a.os = os, a.nsplit = p.nsplit;
+  const RowPlan p = row_plan (ctype, H, a.G, a.D, S, a.vals != nullptr);
+  a.rep = H / a.G, a.tiles = p.tiles, a.ht = p.ht, a.nsplit = p.nsplit;
   a.cnt = parts ? nullptr : (uint32_t *)scratch;
   a.pm = (float *)((uint8_t *)scratch + kRowCounterBytes);
   a.pl = a.pm + p.parts;
   a.pacc = a.pl + p.parts;
   if (parts)
-    *parts = { a.pm, a.pl, a.pacc, p.nsplit, p.ht, p.tiles, p.mfma ? kMfRows : row_step (D) };
-  const dim3 grid ((unsigned)p.nsplit, (unsigned)(G * p.tiles), (unsigned)S);
+    *parts = { a.pm, a.pl, a.pacc, p.nsplit, p.ht, p.tiles, p.mfma ? kMfRows : row_step (a.D) };
+  const dim3 grid ((unsigned)p.nsplit, (unsigned)(a.G * p.tiles), (unsigned)S);
   if (p.mfma)
     return launch_mfma (a, grid, s);
-  return ctype == VKL_TYPE_F32 ? launch_rows<float> (a, p.ht, grid, s) : launch_rows<uint16_t> (a, p.ht, grid, s);
+  if (a.vals)
+    return ctype == VKL_TYPE_F32 ? launch_rows<float, true> (a, p.ht, grid, s)
+                                 : launch_rows<uint16_t, true> (a, p.ht, grid, s);
+  return ctype == VKL_TYPE_F32 ? launch_rows<float, false> (a, p.ht, grid, s)
+                               : launch_rows<uint16_t, false> (a, p.ht, grid, s);
+}
+
+int
+rows_attention (const void *q, int qtype, size_t qs, const void *rows, int ctype, size_t rs, int H, int G, int D,
+                int S, StepPos pos, float scale, float tcoef, int tevery, void *out, int otype, size_t os,
+                void *scratch, RowParts *parts, hipStream_t s)
+{
+  RowAttnArgs a = {};
+  a.q = q, a.qtype = qtype, a.qs = qs, a.rows = rows, a.rs = rs, a.G = G, a.D = D;
+  a.pos = pos, a.scale = scale, a.tcoef = tcoef, a.tevery = tevery;
+  a.out = out, a.otype = otype, a.os = os;
+  return rows_launch (a, ctype, H, S, scratch, parts, s);
+}
+
+// keys and values of their own
+int
+kv_attention (const void *q, int qtype, size_t qs, const void *rows, const void *vals, int ctype, size_t rs, int H,
+              int G, int D, int S, StepPos pos, float scale, int chunk, int sink, void *out, int otype, size_t os,
+              void *scratch, hipStream_t s)
+{
+  RowAttnArgs a = {};
+  a.q = q, a.qtype = qtype, a.qs = qs, a.rows = rows, a.vals = vals, a.rs = rs, a.G = G, a.D = D;
+  a.pos = pos, a.scale = scale, a.chunk = chunk, a.sink = sink;
+  a.out = out, a.otype = otype, a.os = os;
+  return rows_launch (a, ctype, H, S, scratch, nullptr, s);
+}
+
+// ---------------------------------------------------------------------------
+// queries, keys and values between their projections and the attention
+// ---------------------------------------------------------------------------
+constexpr int kPrepMax = 1024; // values of a head at most
+
+struct PrepArgs
+{
+  vkl_attn_rows_prep p;
+  StepPos pos;
+  int S;
+};
+
+// one wave per head of a token: the query heads, the keys, the values
+__global__ __launch_bounds__ (256) void
+attn_prepare_kernel (const PrepArgs a)
+{
+  const vkl_attn_rows_prep &p = a.p;
+  const int per = p.H + 2 * p.G, lane = threadIdx.x & 63;
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (long)a.S * per)
+    return;
+  const int s = (int)(item / per), part = (int)(item - (long)s * per);
+  const size_t pos = (size_t)a.pos.get () + (size_t)s, crow = pos * (size_t)p.G * p.dim;
+  if (part >= p.H + p.G)
+    {
+      const int g = part - p.H - p.G;
+      if (!p.v)
+        return;
+      const size_t at = crow + (size_t)g * p.dim;
+      for (int c = lane; c < p.dim; c += 64)
+        {
+          float v = load_elem (p.v, p.kvtype, (size_t)s * p.kvs + (size_t)g * p.dim + c);
+          if (p.first)
+            v = (1.0f - p.mix) * v + p.mix * load_elem (p.first, p.ctype, at + c);
+          store_elem (p.vo, p.ctype, at + c, v);
+        }
+      return;
+    }
+  const bool key = part >= p.H;
+  const void *src = key ? p.k : p.q;
+  if (!src)
+    return;
+  const int type = key ? p.kvtype : p.qtype, h = key ? part - p.H : part;
+  const size_t at = (size_t)s * (key ? p.kvs : p.qs) + (size_t)h * p.dim;
+  float x[kPrepMax / 64], ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < kPrepMax / 64; ++j)
+    {
+      const int c = lane + 64 * j;
+      x[j] = 0.f;
+      if (64 * j >= p.dim || c >= p.n)
+        continue;
+      const float v = load_elem (src, type, at + c);
+      x[j] = v;
+      if (c < 2 * p.npair)
+        {
+          const int i = c < p.npair ? c : c - p.npair;
+          const float w = load_elem (src, type, at + (c < p.npair ? c + p.npair : c - p.npair));
+          // the angle to within a turn in double, its sine and cosine in float
+          double t = (double)pos * ldg (p.freq + i) * 0.15915494309189533577;
+          t -= rint (t);
+          float sn, cs;
+          sincosf ((float)(t * 6.28318530717958647693), &sn, &cs);
+          x[j] = c < p.npair ? v * cs - w * sn : v * cs + w * sn;
+        }
+      ss = __builtin_fmaf (x[j], x[j], ss);
+    }
+  const float alpha = 1.0f / sqrtf (wave_sum (ss) / (float)p.n + p.eps);
+#pragma unroll
+  for (int j = 0; j < kPrepMax / 64; ++j)
+    {
+      const int c = lane + 64 * j;
+      if (64 * j >= p.dim || c >= p.dim)
+        continue;
+      if (key)
+        store_elem (p.ko, p.ctype, crow + (size_t)h * p.dim + c, x[j] * alpha);
+      else
+        store_elem (p.qo, p.qotype, (size_t)s * p.qos + (size_t)h * p.dim + c, x[j] * alpha);
+    }
+}
+
+int
+attn_prepare (const vkl_attn_rows_prep &p, int S, StepPos pos, hipStream_t s)
+{
+  PrepArgs a = { p, pos, S };
+  const long items = (long)S * (p.H + 2 * p.G);
+  attn_prepare_kernel<<<dim3 ((unsigned)((items + 3) / 4)), dim3 (256), 0, s>>> (a);
+  return (int)hipGetLastError ();
 }
 
 // ---------------------------------------------------------------------------
@@ -1334,7 +1412,8 @@ enum
 {
   GV_SEGS = 0,  // outputs by segment
   GV_ADD = 1,   // y[n] += sum
-  GV_LOGITS = 2 // y[n] = soft cap, arg-max partials
+  GV_LOGITS = 2, // y[n] = soft cap, arg-max partials
+  GV_GATED = 3   // GV_ADD of a row that is normed and gated on the way in
 };
 
 // an item: 8 loads of 512 columns per lane; two rows of four, or, where rows are
@@ -1343,7 +1422,7 @@ template <int MODE>
 constexpr int
 gv_rows ()
 {
-  return MODE == GV_ADD ? 1 : 2;
+  return MODE == GV_ADD || MODE == GV_GATED ? 1 : 2;
 }
 template <int MODE>
 constexpr int
@@ -1366,6 +1445,7 @@ struct GvArgs
   int N, K;
   const float *x;    // [K]
   const float *norm; // [K] (zero beyond W), RMS norm over W values
+  const float *gate; // GV_GATED: times sigmoid (gate[c])
   int W;
   float eps;
   int nseg;
@@ -1401,7 +1481,7 @@ stack_gemv_kernel (const GvArgs a)
   __shared__ float red[16];
   __shared__ float bv_s[kGvWaves];
   __shared__ uint32_t bi_s[kGvWaves + 1];
-  constexpr bool NORM = MODE != GV_ADD;
+  constexpr bool NORM = MODE != GV_ADD, GATE = MODE == GV_GATED;
   constexpr int ROWS = gv_rows<MODE> (), STEPS = 8 / ROWS, SPAN = gv_span<MODE> ();
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane (tid >> 6);
@@ -1435,7 +1515,7 @@ stack_gemv_kernel (const GvArgs a)
   const int kpad = nspan * SPAN;
   if constexpr (XV > 0)
     {
-      float4 xv[XV], nv[XV];
+      float4 xv[XV], nv[XV], gv[XV];
 #pragma unroll
       for (int j = 0; j < XV; ++j)
         {
@@ -1443,6 +1523,8 @@ stack_gemv_kernel (const GvArgs a)
           xv[j] = __builtin_bit_cast (float4, ldg4 (a.x + c));
           if (NORM)
             nv[j] = __builtin_bit_cast (float4, ldg4 (a.norm + c));
+          if (GATE)
+            gv[j] = __builtin_bit_cast (float4, ldg4 (a.gate + c));
         }
       __builtin_amdgcn_sched_barrier (0);
       issue (0, bufa);
@@ -1470,6 +1552,8 @@ stack_gemv_kernel (const GvArgs a)
               v.x = v.x * alpha * nv[j].x, v.y = v.y * alpha * nv[j].y;
               v.z = v.z * alpha * nv[j].z, v.w = v.w * alpha * nv[j].w;
             }
+          if (GATE)
+            v.x *= sigmoid (gv[j].x), v.y *= sigmoid (gv[j].y), v.z *= sigmoid (gv[j].z), v.w *= sigmoid (gv[j].w);
           if (c >= a.K)
             v = make_float4 (0.f, 0.f, 0.f, 0.f);
           if (c < kpad)
@@ -1500,6 +1584,11 @@ stack_gemv_kernel (const GvArgs a)
                   const float4 n = __builtin_bit_cast (float4, ldg4 (a.norm + c));
                   v.x = v.x * alpha * n.x, v.y = v.y * alpha * n.y;
                   v.z = v.z * alpha * n.z, v.w = v.w * alpha * n.w;
+                }
+              if (GATE)
+                {
+                  const float4 g = __builtin_bit_cast (float4, ldg4 (a.gate + c));
+                  v.x *= sigmoid (g.x), v.y *= sigmoid (g.y), v.z *= sigmoid (g.z), v.w *= sigmoid (g.w);
                 }
             }
           put (c, v);
@@ -1544,7 +1633,7 @@ stack_gemv_kernel (const GvArgs a)
         const int n = row0 + r;
         if (n >= a.N)
           continue;
-        if (MODE == GV_ADD)
+        if (MODE == GV_ADD || MODE == GV_GATED)
           {
             if (lane == 0)
               stg (a.y + n, ldg (a.y + n) + v);
@@ -1565,12 +1654,7 @@ stack_gemv_kernel (const GvArgs a)
               if (i < a.nseg && n >= a.seg[i].n0 && n < a.seg[i].n0 + a.seg[i].n)
                 {
                   const GvSeg &sg = a.seg[i];
-                  float y = v;
-                  if (sg.act == 2)
-                    {
-                      y = fmaxf (y, 0.f);
-                      y = y * y;
-                    }
+                  const float y = activate (sg.act, v);
                   if (lane == 0)
                     store_elem (sg.y, sg.f32 ? VKL_TYPE_F32 : VKL_TYPE_BF16,
                                 (size_t)pos * sg.pos_stride + (n - sg.n0), y);
@@ -1704,24 +1788,42 @@ struct StackScratch
 {
   uint32_t *sync; // [0] arg-max counter, [16..17] loop state, [20..23] sampler parameters
   uint32_t *cnt;  // attention counters and parts
-  float *x, *q, *c, *g, *cat, *qa, *logits, *amax_v;
+  float *x, *q, *c, *g, *cat, *qa, *ff, *logits, *amax_v;
   uint32_t *amax_i;
   size_t bytes;
 };
 
 constexpr int kMaxGrid = 2048;
 
+size_t
+round64 (int n)
+{
+  return ((size_t)n + 63) / 64 * 64;
+}
+
 StackScratch
 carve_stack (const vkl_stack_model *m)
 {
   StackScratch s = {};
-  size_t q = 0, c = 0, g = 0, cat = 0, qa = 0, attn = 0;
+  size_t q = 0, c = 0, g = 0, cat = 0, qa = 0, attn = 0, ff = 0;
   for (int i = 0; i < m->n_runs; ++i)
     {
       const vkl_stack_layer &l = m->layers_h[i];
       q = std::max (q, (size_t)l.H * l.dim);
       cat = std::max (cat, (size_t)l.k_out);
-      if (l.mixer == VKL_MIX_LATENT)
+      ff = std::max (ff, (size_t)l.ff_p);
+      if (l.mixer == VKL_MIX_KV)
+        {
+          c = std::max (c, (size_t)2 * l.G * l.dim);
+          attn = std::max (attn, row_scratch_bytes (m->ctype, l.H, l.G, l.dim, 1, true));
+        }
+      else if (l.mixer == VKL_MIX_DELTA || l.mixer == VKL_MIX_DECAY)
+        {
+          c = std::max (c, (size_t)2 * l.G * l.dim + (size_t)l.H * l.vdim);
+          g = std::max (g, l.mixer == VKL_MIX_DELTA ? round64 (l.H) + round64 (l.r_a) + round64 (l.r_g)
+                                                    : (size_t)l.k_out);
+        }
+      else if (l.mixer == VKL_MIX_LATENT)
         {
           c = std::max (c, (size_t)l.rank_p), g = std::max (g, (size_t)l.H);
           qa = std::max (qa, (size_t)l.H * l.rank_p);
@@ -1745,6 +1847,7 @@ carve_stack (const vkl_stack_model *m)
   s.g = (float *)take (g * 4);
   s.cat = (float *)take (cat * 4);
   s.qa = (float *)take (qa * 4);
+  s.ff = (float *)take (ff * 4);
   s.logits = (float *)take ((size_t)m->vocab * 4);
   s.amax_v = (float *)take (kMaxGrid * 4);
   s.amax_i = (uint32_t *)take (kMaxGrid * 4);
@@ -1763,14 +1866,39 @@ check_stack (const vkl_stack_model *m)
   for (int i = 0; i < m->n_runs; ++i)
     {
       const vkl_stack_layer &l = m->layers_h[i];
-      VKL_CHECK_ARG (l.mixer == VKL_MIX_SHARED_KV || l.mixer == VKL_MIX_LATENT);
-      VKL_CHECK_ARG (l.norm && l.w_in && l.w_out && l.cache && l.H > 0 && l.G > 0 && (l.H % l.G) == 0);
+      VKL_CHECK_ARG (l.mixer >= VKL_MIX_SHARED_KV && l.mixer <= VKL_MIX_DECAY);
+      const bool recur = l.mixer == VKL_MIX_DELTA || l.mixer == VKL_MIX_DECAY;
+      VKL_CHECK_ARG (l.norm && l.w_in && l.w_out && (l.cache || recur) && l.H > 0 && l.G > 0 && (l.H % l.G) == 0);
       VKL_CHECK_ARG (l.dim > 0 && (l.dim % 32) == 0 && l.vdim > 0 && (l.vdim % 32) == 0);
       VKL_CHECK_ARG ((l.k_out % 64) == 0 && gv_supported (l.k_out) && l.ff >= 0);
-      VKL_CHECK_ARG (l.ff_col >= l.H * l.vdim && l.ff_col + l.ff <= l.k_out);
+      if (l.norm2)
+        VKL_CHECK_ARG (l.ff > 0 && l.w_up && l.w_down && (l.ff_p % 64) == 0 && l.ff_p >= l.ff && gv_supported (l.ff_p)
+                       && l.H * l.vdim <= l.k_out);
+      else
+        VKL_CHECK_ARG (l.ff_col >= l.H * l.vdim && l.ff_col + l.ff <= l.k_out);
       VKL_CHECK_ARG (l.temp_coef == 0.f || l.temp_every > 0);
-      VKL_CHECK_ARG (l.kv0 >= l.H * l.dim);
-      if (l.mixer == VKL_MIX_LATENT)
+      VKL_CHECK_ARG (l.kv0 >= (recur ? l.G : l.H) * l.dim);
+      if (l.mixer == VKL_MIX_KV)
+        {
+          VKL_CHECK_ARG (l.vcache && l.dim <= kPrepMax && l.vdim == l.dim && l.n > 0 && l.n <= l.dim && l.chunk >= 0);
+          VKL_CHECK_ARG (l.npair >= 0 && 2 * l.npair <= l.n && (l.npair == 0 || l.freq));
+          VKL_CHECK_ARG (l.v0 == l.kv0 + l.G * l.dim && l.v0 + l.G * l.dim <= l.n_in);
+        }
+      else if (recur)
+        {
+          // (the three kinds of rows are one stretch)
+          const int end = 2 * l.G * l.dim + l.H * l.vdim;
+          VKL_CHECK_ARG (recur_supported (l.H, l.H / l.G, l.dim, l.vdim) && l.state && l.gnorm);
+          VKL_CHECK_ARG (l.kv0 == l.G * l.dim && l.v0 == 2 * l.G * l.dim && l.n > 0 && l.n <= l.dim && l.vn > 0
+                         && l.vn <= l.vdim);
+          if (l.mixer == VKL_MIX_DECAY)
+            VKL_CHECK_ARG (l.G == l.H && l.log_decay && l.g0 >= end && l.g0 + l.H * l.vdim <= l.n_in);
+          else
+            VKL_CHECK_ARG (l.conv && l.ring && l.taps >= 1 && l.taps <= 16 && l.dt_bias && l.rate && l.w_a2 && l.w_g2
+                           && l.r_a > 0 && (l.r_a % 8) == 0 && l.r_g > 0 && (l.r_g % 8) == 0 && l.r_a + l.r_g <= 12288 && l.b0 >= end
+                           && l.a0 >= l.b0 + l.H && l.g0 >= l.a0 + l.r_a && l.g0 + l.r_g <= l.n_in);
+        }
+      else if (l.mixer == VKL_MIX_LATENT)
         {
           VKL_CHECK_ARG (l.w_ukt && l.w_uv && l.c_norm && l.rank > 0 && l.rank <= l.rank_p && (l.rank_p % 32) == 0
                          && l.rank_p <= 1024 && l.G == 1);
@@ -1807,8 +1935,95 @@ weights_stream (const vkl_stack_model &m)
     {
       const vkl_stack_layer &l = m.layers_h[i];
       n += (size_t)l.n_in * m.width_p + (size_t)m.width * l.k_out;
+      if (l.norm2)
+        n += (size_t)l.ff * m.width_p + (size_t)m.width * l.ff_p;
     }
   return n * 2 > kCacheBytes;
+}
+
+// a layer whose feed-forward part follows its mixer; a: the first product
+int
+launch_two_norm_layer (const StepArgs &p, const vkl_stack_layer &l, GvArgs a, hipStream_t st)
+{
+  const vkl_stack_model &m = *p.m;
+  GvArgs o = {};
+  o.w = (const uint16_t *)l.w_out, o.N = m.width, o.K = l.k_out;
+  o.x = p.s.cat, o.y = p.s.x, o.stream = p.stream;
+  if (l.mixer == VKL_MIX_KV)
+    {
+      a.nseg = 2;
+      a.seg[0] = { 0, l.H * l.dim, p.s.q, 1, VKL_ACT_NONE, 0 };
+      a.seg[1] = { l.kv0, 2 * l.G * l.dim, p.s.c, 1, VKL_ACT_NONE, 0 };
+      if (int e = launch_gv<GV_SEGS> (a, p.n_cu, st))
+        return e;
+      vkl_attn_rows_prep r = {};
+      r.H = l.H, r.G = l.G, r.dim = l.dim, r.n = l.n, r.npair = l.npair, r.freq = l.freq, r.eps = m.eps;
+      r.q = r.qo = p.s.q, r.qtype = r.qotype = r.kvtype = VKL_TYPE_F32;
+      r.k = p.s.c, r.v = p.s.c + l.G * l.dim, r.ko = l.cache, r.vo = l.vcache;
+      r.first = l.vfirst, r.mix = l.vmix, r.ctype = m.ctype;
+      if (int e = attn_prepare (r, 1, p.pos, st))
+        return e;
+      if (int e = kv_attention (p.s.q, VKL_TYPE_F32, 0, l.cache, l.vcache, m.ctype, (size_t)l.G * l.dim, l.H, l.G,
+                                l.dim, 1, p.pos, l.scale, l.chunk, l.sink, p.s.cat, VKL_TYPE_F32, 0, p.s.cnt, st))
+        return e;
+      if (int e = launch_gv<GV_ADD> (o, p.n_cu, st))
+        return e;
+    }
+  else
+    {
+      const bool delta = l.mixer == VKL_MIX_DELTA;
+      float *b = p.s.g, *a1 = b + round64 (l.H), *g1 = a1 + round64 (l.r_a);
+      a.seg[0] = { 0, 2 * l.G * l.dim + l.H * l.vdim, p.s.c, 1, delta ? VKL_ACT_NONE : VKL_ACT_SILU, 0 };
+      if (delta)
+        {
+          a.nseg = 4;
+          a.seg[1] = { l.b0, l.H, b, 1, VKL_ACT_NONE, 0 };
+          a.seg[2] = { l.a0, l.r_a, a1, 1, VKL_ACT_NONE, 0 };
+          a.seg[3] = { l.g0, l.r_g, g1, 1, VKL_ACT_NONE, 0 };
+        }
+      else
+        {
+          a.nseg = 2;
+          a.seg[1] = { l.g0, l.H * l.vdim, p.s.g, 1, VKL_ACT_NONE, 0 };
+        }
+      if (int e = launch_gv<GV_SEGS> (a, p.n_cu, st))
+        return e;
+      RecurStepArgs r = {};
+      r.H = l.H, r.rep = l.H / l.G, r.dim = l.dim, r.vdim = l.vdim, r.n = l.n, r.vn = l.vn, r.pos = p.pos;
+      r.qkv = p.s.c, r.state = l.state, r.out = p.s.cat, r.qscale = l.qscale;
+      if (delta)
+        {
+          r.conv = l.conv, r.ring = l.ring, r.taps = l.taps, r.b = b, r.a1 = a1, r.g1 = g1;
+          r.w_a2 = (const uint16_t *)l.w_a2, r.w_g2 = (const uint16_t *)l.w_g2, r.r_a = l.r_a, r.r_g = l.r_g;
+          r.dt_bias = l.dt_bias, r.rate = l.rate, r.gnorm = l.gnorm, r.unit_eps = l.unit_eps, r.eps = m.eps;
+          if (int e = delta_step_launch (r, st))
+            return e;
+          if (int e = launch_gv<GV_ADD> (o, p.n_cu, st))
+            return e;
+        }
+      else
+        {
+          r.log_decay = l.log_decay, r.out_pad = l.k_out - l.H * l.vdim;
+          if (int e = decay_step_launch (r, st))
+            return e;
+          o.norm = l.gnorm, o.gate = p.s.g, o.W = l.H * l.vn, o.eps = m.eps;
+          if (int e = launch_gv<GV_GATED> (o, p.n_cu, st))
+            return e;
+        }
+    }
+  if (!l.norm2)
+    return 0;
+  GvArgs u = {};
+  u.w = (const uint16_t *)l.w_up, u.N = l.ff, u.K = m.width_p;
+  u.x = p.s.x, u.norm = l.norm2, u.W = m.width, u.eps = m.eps, u.pos = p.pos, u.stream = p.stream;
+  u.nseg = 1;
+  u.seg[0] = { 0, l.ff, p.s.ff, 1, l.ff_act, 0 };
+  if (int e = launch_gv<GV_SEGS> (u, p.n_cu, st))
+    return e;
+  GvArgs d = {};
+  d.w = (const uint16_t *)l.w_down, d.N = m.width, d.K = l.ff_p;
+  d.x = p.s.ff, d.y = p.s.x, d.stream = p.stream;
+  return launch_gv<GV_ADD> (d, p.n_cu, st);
 }
 
 int
@@ -1820,6 +2035,8 @@ launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
   a.w = (const uint16_t *)l.w_in, a.N = l.n_in, a.K = m.width_p;
   a.x = p.s.x, a.norm = l.norm, a.W = m.width, a.eps = m.eps, a.pos = p.pos, a.stream = p.stream;
   int n = 0;
+  if (l.mixer == VKL_MIX_KV || l.mixer == VKL_MIX_DELTA || l.mixer == VKL_MIX_DECAY)
+    return launch_two_norm_layer (p, l, a, st);
   a.seg[n++] = { 0, l.H * l.dim, p.s.q, 1, 0, 0 };
   if (latent)
     {
@@ -1829,7 +2046,7 @@ launch_stack_layer (const StepArgs &p, const vkl_stack_layer &l, hipStream_t st)
   else
     a.seg[n++] = { l.kv0, l.G * l.dim, l.cache, m.ctype == VKL_TYPE_F32, 0, (size_t)l.G * l.dim };
   if (l.ff)
-    a.seg[n++] = { l.up0, l.ff, p.s.cat + l.ff_col, 1, 2, 0 };
+    a.seg[n++] = { l.up0, l.ff, p.s.cat + l.ff_col, 1, l.ff_act, 0 };
   a.nseg = n;
   if (int e = launch_gv<GV_SEGS> (a, p.n_cu, st))
     return e;
@@ -1872,13 +2089,13 @@ launch_stack_step (const StepArgs &p, hipStream_t st)
   const vkl_stack_model &m = *p.m;
   EmbedArgs e = {};
   e.table = (const uint16_t *)m.embed, e.VH = (uint32_t)m.vocab, e.K = m.width_p, e.W = m.width;
-  e.toks = p.toks, e.loop = p.loop, e.w = m.embed_norm, e.eps = m.eps, e.out = p.s.x, e.os = (size_t)m.width_p;
+  e.toks = p.toks, e.loop = p.loop, e.w = m.embed_norm, e.eps = m.eps, e.scale = m.embed_scale, e.out = p.s.x, e.os = (size_t)m.width_p;
   embed_norm_kernel<<<dim3 (1), dim3 (1024), 0, st>>> (e);
   for (int i = 0; i < m.n_runs; ++i)
     if (int err = launch_stack_layer (p, m.layers_h[i], st))
       return err;
   GvArgs a = {};
-  a.w = (const uint16_t *)m.embed, a.N = m.vocab, a.K = m.width_p;
+  a.w = (const uint16_t *)(m.head ? m.head : m.embed), a.N = m.vocab, a.K = m.width_p;
   a.x = p.s.x, a.norm = m.final_norm, a.W = m.width, a.eps = m.eps;
   a.y = p.logits ? p.logits : p.s.logits, a.cap = m.logit_cap, a.stream = p.stream;
   a.amax_v = p.s.amax_v, a.amax_i = p.s.amax_i, a.amax_cnt = p.s.sync;
@@ -1937,9 +2154,9 @@ stack_key (const vkl_stack_model *m, const void *ids, const void *logits, bool s
     for (size_t i = 0; i < n; ++i)
       h = (h ^ ((const uint8_t *)p)[i]) * 1099511628211ull;
   };
-  const void *ptrs[6] = { m->embed, m->embed_norm, m->final_norm, m->scratch, ids, logits };
+  const void *ptrs[7] = { m->embed, m->head, m->embed_norm, m->final_norm, m->scratch, ids, logits };
   const int dims[6] = { m->width, m->vocab, m->maxlen, m->n_runs, m->ctype, (int)sampled };
-  mix (ptrs, sizeof (ptrs)), mix (dims, sizeof (dims)), mix (&m->eps, 4), mix (&m->logit_cap, 4);
+  mix (ptrs, sizeof (ptrs)), mix (dims, sizeof (dims)), mix (&m->eps, 4), mix (&m->logit_cap, 4), mix (&m->embed_scale, 4);
   mix (m->layers_h, sizeof (vkl_stack_layer) * (size_t)m->n_runs);
   return h;
 }
@@ -2008,7 +2225,19 @@ vkl_embed_norm_bf16 (const void *table, uint32_t VH, int K, int W, const uint32_
 {
   VKL_CHECK_ARG (table && toks && out && VH > 0 && n > 0 && W > 0 && K >= W && os >= (size_t)W);
   EmbedArgs a = {};
-  a.table = (const uint16_t *)table, a.VH = VH, a.K = K, a.W = W, a.toks = toks, a.w = w, a.eps = eps;
+  a.table = (const uint16_t *)table, a.VH = VH, a.K = K, a.W = W, a.toks = toks, a.w = w, a.eps = eps, a.scale = 1.f;
+  a.out = out, a.os = os;
+  embed_norm_kernel<<<dim3 (n), dim3 (1024), 0, (hipStream_t)stream>>> (a);
+  return vkl_launch_status ();
+}
+
+extern "C" int
+vkl_embed_rows_bf16 (const void *table, uint32_t VH, int K, int W, const uint32_t *toks, uint32_t n, float scale,
+                     float *out, size_t os, void *stream)
+{
+  VKL_CHECK_ARG (table && toks && out && VH > 0 && n > 0 && W > 0 && K >= W && os >= (size_t)W);
+  EmbedArgs a = {};
+  a.table = (const uint16_t *)table, a.VH = VH, a.K = K, a.W = W, a.toks = toks, a.scale = scale;
   a.out = out, a.os = os;
   embed_norm_kernel<<<dim3 (n), dim3 (1024), 0, (hipStream_t)stream>>> (a);
   return vkl_launch_status ();
@@ -2059,6 +2288,39 @@ vkl_attn_rows (const void *q, int qtype, size_t qs, const void *rows, int ctype,
                  && (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16));
   return rows_attention (q, qtype, qs, rows, ctype, rs, H, G, dim, S, StepPos{ nullptr, pos0 }, scale, temp_coef,
                          temp_every, out, otype, os, scratch, nullptr, (hipStream_t)stream);
+}
+
+extern "C" size_t
+vkl_attn_kv_rows_scratch_bytes (int ctype, int H, int G, int dim, int S)
+{
+  if (H <= 0 || G <= 0 || H % G || dim <= 0 || S <= 0)
+    return 0;
+  return row_scratch_bytes (ctype, H, G, dim, S, true);
+}
+
+extern "C" int
+vkl_attn_kv_rows (const void *q, int qtype, size_t qs, const void *rows, const void *vals, int ctype, size_t rs, int H,
+                  int G, int dim, int S, uint32_t pos0, float scale, int chunk, int sink, void *out, int otype,
+                  size_t os, void *scratch, void *stream)
+{
+  VKL_CHECK_ARG (q && rows && vals && out && scratch && H > 0 && G > 0 && (H % G) == 0 && S > 0 && S <= 65535);
+  VKL_CHECK_ARG (dim > 0 && (dim % 32) == 0 && dim <= 1024 && rs >= (size_t)G * dim && (rs % 8) == 0 && chunk >= 0);
+  VKL_CHECK_ARG (((uintptr_t)rows % 16) == 0 && ((uintptr_t)vals % 16) == 0 && ((uintptr_t)q % 16) == 0
+                 && (qs % 8) == 0 && qs >= (size_t)H * dim && os >= (size_t)H * dim);
+  VKL_CHECK_ARG ((qtype == VKL_TYPE_F32 || qtype == VKL_TYPE_BF16) && (ctype == VKL_TYPE_F32 || ctype == VKL_TYPE_BF16)
+                 && (otype == VKL_TYPE_F32 || otype == VKL_TYPE_BF16));
+  return kv_attention (q, qtype, qs, rows, vals, ctype, rs, H, G, dim, S, StepPos{ nullptr, pos0 }, scale, chunk, sink,
+                       out, otype, os, scratch, (hipStream_t)stream);
+}
+
+extern "C" int
+vkl_attn_prepare (const vkl_attn_rows_prep *p, int S, uint32_t pos0, void *stream)
+{
+  VKL_CHECK_ARG (p && S > 0 && p->H > 0 && p->G > 0 && p->dim > 0 && p->dim <= kPrepMax && p->n > 0 && p->n <= p->dim);
+  VKL_CHECK_ARG (p->npair >= 0 && 2 * p->npair <= p->n && (p->npair == 0 || p->freq));
+  VKL_CHECK_ARG ((!p->q || (p->qo && p->qs >= (size_t)p->H * p->dim && p->qos >= (size_t)p->H * p->dim)) && (!p->k || p->ko)
+                 && (!p->v || p->vo) && p->kvs >= (size_t)p->G * p->dim);
+  return attn_prepare (*p, S, StepPos{ nullptr, pos0 }, (hipStream_t)stream);
 }
 
 extern "C" int

@@ -1,7 +1,7 @@
 // extern "C" wrappers around vkllama::Model and the synthetic-weight helpers
 // (include/vkl_model.h).
 #include "vkl_model.h"
-#include "models/fazinex.h"
+#include "models/stack_model.h"
 #include "models/gguflib.h"
 #include "models/llama2.h"
 #include "models/registry.h"
@@ -18,7 +18,7 @@ struct vkl_model
   vkllama::CausalModel *model = nullptr;
   // the family's own calls: null for a model of another family
   vkllama::Model *llama () const { return dynamic_cast<vkllama::Model *> (model); }
-  vkllama::Fazinex *fazinex () const { return dynamic_cast<vkllama::Fazinex *> (model); }
+  vkllama::StackModel *stack () const { return dynamic_cast<vkllama::StackModel *> (model); }
   std::string last_error;
   std::vector<gguf_value> values;
   std::vector<std::string> names;
@@ -247,9 +247,9 @@ vkl_model_residual_streams (vkl_model *m, const uint32_t *toks, size_t n_toks, s
 {
   if (!m || !m->model || !toks || !out)
     return (int)absl::StatusCode::kInvalidArgument;
-  if (!m->fazinex ())
+  if (!m->stack ())
     return fail (m, absl::UnimplementedError ("this model family keeps no fp32 residual stream"));
-  auto r = m->fazinex ()->residual_streams (std::vector<uint32_t> (toks, toks + n_toks), offset);
+  auto r = m->stack ()->residual_streams (std::vector<uint32_t> (toks, toks + n_toks), offset);
   if (!r.ok ())
     return fail (m, r.status ());
   if (r->size () != n)

@@ -30,6 +30,17 @@ CausalModel::check_span_ (size_t n, size_t offset) const
   return absl::OkStatus ();
 }
 
+absl::Status
+CausalModel::begin_pass_ (size_t offset)
+{
+  if (stateful_ && offset != 0 && offset != next_pos_)
+    return absl::FailedPreconditionError (absl::StrFormat (
+        "a pass at position %zu: the recurrent state is not there (a pass continues the last one or starts at 0)",
+        offset));
+  next_pos_ = (size_t)-1;
+  return absl::OkStatus ();
+}
+
 absl::StatusOr<std::vector<float> >
 CausalModel::operator() (std::vector<uint32_t> const &toks, const size_t offset)
 {
@@ -46,6 +57,7 @@ CausalModel::forward_rows (std::vector<uint32_t> const &toks, const size_t offse
   for (uint32_t r : rows)
     if (r >= toks.size ())
       return absl::OutOfRangeError (absl::StrFormat ("row %u of a pass over %zu tokens", r, toks.size ()));
+  VKLLAMA_STATUS_OK (begin_pass_ (offset));
   std::vector<float> out (rows.size () * vocab_);
   if (fused_decode_ && toks.size () == 1 && plan->usable ())
     {
@@ -64,6 +76,7 @@ CausalModel::forward_rows (std::vector<uint32_t> const &toks, const size_t offse
       VKLLAMA_STATUS_OK (rs);
       for (size_t i = 0; i < rows.size (); ++i)
         std::copy (one.begin (), one.end (), out.begin () + i * vocab_);
+      end_pass_ (offset + 1);
       return out;
     }
   auto logits = forward_ (toks, offset, rows);
@@ -72,6 +85,7 @@ CausalModel::forward_rows (std::vector<uint32_t> const &toks, const size_t offse
     if (int e = vkl_memcpy_d2h (out.data (), logits->data (), out.size () * sizeof (float), gpu_->stream ()))
       return absl::InternalError (vkl_error_string (e));
   VKLLAMA_STATUS_OK (wait_all_ ());
+  end_pass_ (offset + toks.size ());
   return out;
 }
 
@@ -148,6 +162,7 @@ CausalModel::generate_once_ (std::vector<uint32_t> const &prompt, size_t n_gen,
     }
   uint32_t *ids = (uint32_t *)next_tok_.data ();
   void *s = gpu_->stream ();
+  VKLLAMA_STATUS_OK (begin_pass_ (0));
 
   const auto t0 = clock::now ();
   // prompt pass; arg-max of its fp16 logits becomes ids[0]
@@ -211,6 +226,7 @@ CausalModel::generate_once_ (std::vector<uint32_t> const &prompt, size_t n_gen,
   VKLLAMA_STATUS_OK (plan->check ());
   // run deferred work the operator chain may have queued
   VKLLAMA_STATUS_OK (wait_all_ ());
+  end_pass_ (prompt.size () + n_gen - 1);
   out.resize (n_gen);
   if (int e = vkl_memcpy_d2h (out.data (), ids, n_gen * sizeof (uint32_t), s))
     return absl::InternalError (vkl_error_string (e));

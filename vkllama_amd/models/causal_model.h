@@ -71,14 +71,21 @@ protected:
   virtual absl::Status wait_all_ () = 0;
   virtual StepPlan *plan_ptr_ () = 0;
   absl::Status check_span_ (size_t n, size_t offset) const;
+  // A family with a recurrent state (stateful_) goes through a sequence in order: a
+  // pass starts where the last one ended, or at 0.  begin_pass_ checks that, and the
+  // state has no position until end_pass_ gives it the new one.
+  absl::Status begin_pass_ (size_t offset);
+  void end_pass_ (size_t next) { next_pos_ = next; }
 
   GPUDevice *gpu_ = nullptr;
   size_t vocab_ = 0, maxlen_ = 0;
   bool fused_decode_ = true;
   bool decode_graph_ = true;
   size_t decode_recoveries_ = 0;
+  bool stateful_ = false;
 
 private:
+  size_t next_pos_ = 0;
   Tensor next_tok_;
   // sampling on the device during generate_*(): off = arg-max
   bool samp_on_ = false;

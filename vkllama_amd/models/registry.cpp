@@ -1,5 +1,6 @@
 #include "models/registry.h"
 #include "models/fazinex.h"
+#include "models/fuzuvik.h"
 #include "models/llama2.h"
 #include <fstream>
 #include <sstream>
@@ -14,7 +15,7 @@ struct Entry
   const char *name;
   ModelFactory factory;
 };
-const Entry kEntries[] = { { "Fazinex", Fazinex::create } };
+const Entry kEntries[] = { { "Fazinex", Fazinex::create }, { "Fuzuvik", Fuzuvik::create } };
 
 absl::StatusOr<std::unique_ptr<CausalModel> >
 load_gguf (const std::string &path, const ModelOptions &opt)

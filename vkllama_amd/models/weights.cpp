@@ -10,6 +10,23 @@
 
 namespace vkllama
 {
+namespace
+{
+std::vector<float>
+widen (const uint8_t *data, size_t n)
+{
+  std::vector<float> out (n);
+  for (size_t i = 0; i < n; ++i)
+    {
+      uint16_t h;
+      memcpy (&h, data + 2 * i, 2);
+      const uint32_t u = (uint32_t)h << 16;
+      memcpy (&out[i], &u, 4);
+    }
+  return out;
+}
+}
+
 absl::StatusOr<WeightView>
 WeightSource::find (const std::string &name) const
 {
@@ -39,15 +56,17 @@ WeightSource::vector (const std::string &name, size_t n) const
   if (v->dtype != BF16 || v->shape.size () != 1 || v->shape[0] != n || v->bytes != n * 2)
     return absl::InvalidArgumentError (
         absl::StrFormat ("model tensor %s: a bf16 vector of %zu is needed", name, n));
-  std::vector<float> out (n);
-  for (size_t i = 0; i < n; ++i)
-    {
-      uint16_t h;
-      memcpy (&h, v->data + 2 * i, 2);
-      const uint32_t u = (uint32_t)h << 16;
-      memcpy (&out[i], &u, 4);
-    }
-  return out;
+  return widen (v->data, n);
+}
+
+absl::StatusOr<float>
+WeightSource::scalar (const std::string &name) const
+{
+  auto v = find (name);
+  VKLLAMA_STATUS_OK (v);
+  if (v->dtype != BF16 || v->bytes != 2)
+    return absl::InvalidArgumentError (absl::StrFormat ("model tensor %s: one bf16 value is needed", name));
+  return widen (v->data, 1)[0];
 }
 
 SafetensorsFile::~SafetensorsFile ()

@@ -28,6 +28,8 @@ public:
   // a bf16 matrix [rows, cols] / vector [n], checked
   absl::StatusOr<const uint16_t *> matrix (const std::string &name, size_t rows, size_t cols) const;
   absl::StatusOr<std::vector<float> > vector (const std::string &name, size_t n) const;
+  // a bf16 tensor of one value, whatever its shape
+  absl::StatusOr<float> scalar (const std::string &name) const;
   void add (const std::string &name, const WeightView &v) { views_[name] = v; }
 
 protected:

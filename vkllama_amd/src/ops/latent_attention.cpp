@@ -6,7 +6,7 @@
 namespace vkllama
 {
 // (keys and values share the padded head size: one attention kernel serves both)
-LatentAttention::LatentAttention (GPUDevice *dev, Command *command, const RowMixerParams &p)
+LatentAttention::LatentAttention (GPUDevice *dev, Command *command, const MixerParams &p)
     : RowMixer (dev, command, p)
 {
   dim_ = vdim_ = round_up (std::max (p.dim, p.vdim), 32);

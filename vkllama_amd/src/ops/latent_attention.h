@@ -15,7 +15,7 @@ namespace vkllama
 class LatentAttention : public RowMixer
 {
 public:
-  LatentAttention (GPUDevice *dev, Command *command, const RowMixerParams &p);
+  LatentAttention (GPUDevice *dev, Command *command, const MixerParams &p);
   absl::Status load (const WeightSource &w, const std::string &prefix) override;
   int in_rows () const override;
   absl::Status pack_in (const WeightSource &w, const std::string &prefix, PackedMatrix &m) const override;

@@ -7,7 +7,7 @@
 
 namespace vkllama
 {
-SharedKVAttention::SharedKVAttention (GPUDevice *dev, Command *command, const RowMixerParams &p)
+SharedKVAttention::SharedKVAttention (GPUDevice *dev, Command *command, const MixerParams &p)
     : RowMixer (dev, command, p)
 {
   dim_ = vdim_ = round_up (p.dim, 32);

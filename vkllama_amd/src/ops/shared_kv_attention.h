@@ -10,7 +10,7 @@ namespace vkllama
 class SharedKVAttention : public RowMixer
 {
 public:
-  SharedKVAttention (GPUDevice *dev, Command *command, const RowMixerParams &p);
+  SharedKVAttention (GPUDevice *dev, Command *command, const MixerParams &p);
   absl::Status load (const WeightSource &w, const std::string &prefix) override;
   int in_rows () const override;
   absl::Status pack_in (const WeightSource &w, const std::string &prefix, PackedMatrix &m) const override;
