@@ -196,17 +196,68 @@ def fazinex_weights(cfg, seed):
             r = m["kv_rank"]
             shapes += [(p + "mix.dkv", (r, w)), (p + "mix.dkv.norm", (r,)), (p + "mix.uk", (H * m["dim"], r)),
                        (p + "mix.uv", (H * m["vdim"], r)), (p + "mix.g", (H, w))]
+    return random_bf16(shapes, seed)
+
+
+def random_bf16(shapes, seed, fill={}):
+    """name -> bf16 bits: N(0, 0.02) matrices, vectors of ones (or of fill[last part of the name])"""
+    from vkllama_amd import model as M
     out = {}
     for i, (name, sh) in enumerate(shapes):
-        a = np.full(sh, 0x3F80, np.uint16)
+        a = np.full(sh, fill.get(name.split(".")[-1], 0x3F80), np.uint16)
         if len(sh) == 2:
             M.lib().vkl_synth_normal_bf16(seed + i, a.size, 0.02, a.ctypes.data)
         out[name] = a
     return out
 
 
-# --design fazinex: (width, layers, heads, key/value heads, head size, latent, ff), each beside a Llama-2-shaped model
-# with FP16 weights of the same width, heads, ff and layer count
+FUZUVIK_RANK, FUZUVIK_CHUNK = 128, 8192
+
+
+def fuzuvik_config(dim, n_layers, heads, kv_heads, head, ffn, vocab):
+    """Layers in turn: delta rule, decaying sums, two of chunked attention."""
+    mlp = {"kind": "dense", "ff": ffn}
+    delta = {"type": "channel_delta", "mlp": mlp,
+             "mixer": {"heads": heads, "kv_heads": heads, "dim": head, "vdim": head, "conv": 4}}
+    sums = {"type": "lightning", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": head, "vdim": head,
+                      "decay": [float(1.0 - 2.0 ** (-3.0 - 6.0 * h / heads)) for h in range(heads)]}}
+    attn = {"type": "attention", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": head, "vdim": head, "scale": head ** 0.5, "v_mix": True,
+                      "mask": {"size": FUZUVIK_CHUNK},
+                      "rot": {"base": 500000.0, "dims": head,
+                              "scaling": {"factor": 16.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    order = [delta, sums, attn, attn]
+    return {"architecture": "Fuzuvik", "vocab": vocab, "width": dim, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "layers": [order[i % 4] for i in range(n_layers)]}
+
+
+def fuzuvik_weights(cfg, seed):
+    w, V, r = cfg["width"], cfg["vocab"], FUZUVIK_RANK
+    shapes = [("embed", (V, w)), ("head", (V, w)), ("final.norm", (w,))]
+    for i, L in enumerate(cfg["layers"]):
+        m, p, f = L["mixer"], "l%d." % i, L["mlp"]["ff"]
+        H, G, d, e = m["heads"], m.get("kv_heads", m["heads"]), m["dim"], m["vdim"]
+        attn = L["type"] == "attention"
+        shapes += [(p + "norm1", (w,)), (p + "norm2", (w,)), (p + "mix.q", ((H if attn else G) * d, w)),
+                   (p + "mix.k", (G * d, w)), (p + "mix.v", ((G if attn else H) * e, w)), (p + "mix.o", (w, H * e)),
+                   (p + "mlp.up", (f, w)), (p + "mlp.down", (w, f))]
+        if attn:
+            shapes += [(p + "mix.vmix", (1,))]
+        elif L["type"] == "lightning":
+            shapes += [(p + "mix.g", (H * e, w)), (p + "mix.norm", (H * e,))]
+        else:
+            shapes += [(p + "mix.q.conv", (G * d, m["conv"])), (p + "mix.k.conv", (G * d, m["conv"])),
+                       (p + "mix.v.conv", (H * e, m["conv"])), (p + "mix.b", (H, w)), (p + "mix.A_log", (H,)),
+                       (p + "mix.norm", (e,)), (p + "mix.a1", (r, w)), (p + "mix.a2", (H * d, r)),
+                       (p + "mix.dt_bias", (H * d,)), (p + "mix.g1", (r, w)), (p + "mix.g2", (H * e, r))]
+    # decays near 0.95 per token, values mixed by a half
+    return random_bf16(shapes, seed, {"A_log": 0x0000, "dt_bias": 0xC040, "vmix": 0x3F00})
+
+
+# --design: (width, layers, heads, key/value heads, head size, latent, ff), each beside a model of the same width, heads,
+# ff and layer count: fazinex beside a Llama-2-shaped model with FP16 weights, fuzuvik beside fazinex
+DESIGN_BESIDE = {"fazinex": "llama2", "fuzuvik": "fazinex"}
 DESIGN_SIZES = {"4096": (4096, 8, 32, 8, 128, 512, 11008), "2048": (2048, 8, 16, 4, 128, 512, 5504),
                 "5120": (5120, 6, 40, 8, 128, 512, 13824),
                 # as many key/value heads as query heads: caches of half the Llama-2 size
@@ -214,21 +265,28 @@ DESIGN_SIZES = {"4096": (4096, 8, 32, 8, 128, 512, 11008), "2048": (2048, 8, 16,
 
 
 def bench_design(args):
-    """Prompt pass and greedy decoding of a Fazinex model and of a Llama-2-shaped FP16 model of equal size, random
-    weights, one JSON line per size.  The two are timed in turn, each figure is the best of the repetitions."""
+    """Prompt pass and greedy decoding of a model of the design and of its neighbour of equal size, random weights, one
+    JSON line per size.  The two are timed in turn, each figure is the best of the repetitions."""
     from vkllama_amd import model as M
     vocab, steps = 32000, args.steps
     for name in args.design_sizes.split(","):
         dim, layers, heads, kvh, head, rank, ffn = DESIGN_SIZES[name]
         prompts = [int(n) for n in args.design_prompts.split(",")]
         maxlen = max(prompts) + steps + 8
-        fcfg = fazinex_config(dim, layers, heads, kvh, head, rank, ffn, vocab)
+        sides = (args.design, DESIGN_BESIDE[args.design])
         models = {}
-        if args.design_only != "llama2":
-            w = fazinex_weights(fcfg, args.seed)
-            models["fazinex"] = M.CausalModel.create(fcfg, w, "bfloat16", maxlen)
+        for side in sides:
+            if args.design_only not in (None, side) or side == "llama2":
+                continue
+            if side == "fazinex":
+                cfg = fazinex_config(dim, layers, heads, kvh, head, rank, ffn, vocab)
+                w = fazinex_weights(cfg, args.seed)
+            else:
+                cfg = fuzuvik_config(dim, layers, heads, kvh, head, ffn, vocab)
+                w = fuzuvik_weights(cfg, args.seed)
+            models[side] = M.CausalModel.create(cfg, w, "bfloat16", maxlen)
             del w
-        if args.design_only != "fazinex":
+        if "llama2" in sides and args.design_only in (None, "llama2"):
             lcfg = dict(dim=dim, n_layers=layers, n_heads=heads, ffn=ffn, vocab=vocab, maxlen=maxlen, eps=1e-5, wtype=1)
             w = M.synth_weights(lcfg, seed=args.seed)
             models["llama2-f16"] = M.Llama2(lcfg, w)
@@ -256,7 +314,8 @@ def bench_design(args):
                              "decode_frac_of_hbm_peak": round(nbytes * steps / dec / 1e6 / HBM_PEAK_GBS, 4)})
         for m in models.values():
             m.close()
-        print(json.dumps({"metric": "fazinex_beside_llama2_f16", "size": name, "steps": steps, "n_gpus": 1,
+        beside = {"llama2": "llama2_f16"}.get(sides[1], sides[1])
+        print(json.dumps({"metric": "%s_beside_%s" % (args.design, beside), "size": name, "steps": steps, "n_gpus": 1,
                           "config": {"width": dim, "layers": layers, "heads": heads, "kv_heads": kvh, "head": head,
                                      "latent": rank, "ff": ffn, "vocab": vocab},
                           "data": "synthetic: random-init N(0,0.02) weights, random prompt ids", "rows": rows}), flush=True)
@@ -264,12 +323,12 @@ def bench_design(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=("fazinex",),
-                    help="instead of the workload: this model design beside a Llama-2-shaped FP16 model of equal size")
+    ap.add_argument("--design", choices=sorted(DESIGN_BESIDE),
+                    help="instead of the workload: this model design beside another one of equal size")
     ap.add_argument("--design-sizes", default="4096,2048", help="of " + ", ".join(sorted(DESIGN_SIZES)))
     ap.add_argument("--design-prompts", default="32,2048", help="prompt lengths")
     ap.add_argument("--design-repeats", type=int, default=3)
-    ap.add_argument("--design-only", choices=("fazinex", "llama2"), help="one side alone (for runs under a profiler)")
+    ap.add_argument("--design-only", choices=("fuzuvik", "fazinex", "llama2"), help="one side alone (for runs under a profiler)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)

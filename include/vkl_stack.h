@@ -153,12 +153,13 @@ int vkl_short_conv_silu (const void *x, int type, size_t xs, const float *w,
                          int n, int taps, float *ring, uint32_t pos0, int S,
                          void *out, size_t os, void *stream);
 /* Per head a state M [dim, vdim], zero before position 0:
- *   gated delta rule (z given): with q, k made unit vectors
+ *   gated delta rule (b given): with q, k made unit vectors
  *     (x / sqrt (sum x^2 + unit_eps)), q also times qscale,
  *     M <- diag (g) M,  u = beta (v - M^T k),  M <- M + k u^T,  out = M^T q,
- *     g = exp (-rate[h] softplus (z + dt_bias)), beta = sigmoid (b)
- *   decaying sums (z null): M <- exp (log_decay[h]) M + k v^T,  out = M^T q * qscale
- * Everything after q, k, v, z and b is fp32.  Head h reads query/key head
+ *     g = exp (-rate[h] softplus (z + dt_bias)), beta = sigmoid (b),
+ *     z given, or (chunked form only) z = a1 w_a2^T of low rank
+ *   decaying sums (b null): M <- exp (log_decay[h]) M + k v^T,  out = M^T q * qscale
+ * Everything after q, k, v, z (a1) and b is fp32.  Head h reads query/key head
  * h / rep.  dim and vdim are multiples of 32 up to 256, heads lie as densely. */
 typedef struct
 {
@@ -170,6 +171,10 @@ typedef struct
   const float *log_decay; /* [H] */
   const float *z;         /* [S, H*dim], row stride zs (a multiple of 4) */
   size_t zs;
+  const void *a1;         /* [S, r_a] in `type`, row stride as (a multiple of 8) */
+  size_t as;
+  const void *w_a2;       /* bf16 [H*dim, r_a], r_a a multiple of 64 */
+  int r_a;
   const float *b;         /* [S, H], row stride bs */
   size_t bs;
   const float *dt_bias;   /* [H*dim] */
@@ -187,6 +192,8 @@ typedef struct
 int vkl_recurrence (const vkl_recurrence_args *a, int S, uint32_t pos0,
                     int form, void *scratch, size_t scratch_bytes,
                     void *stream);
+/* whether VKL_RECUR_AUTO takes the chunked form (it needs scratch memory then) */
+int vkl_recurrence_chunked (const vkl_recurrence_args *a, int S);
 /* what the chunked form needs for S tokens at once (it takes them in pieces if
  * there is less, at least what 64 tokens need) */
 size_t vkl_recurrence_scratch_bytes (const vkl_recurrence_args *a, int S);
@@ -196,6 +203,14 @@ size_t vkl_recurrence_scratch_bytes (const vkl_recurrence_args *a, int S);
 int vkl_gated_norm (const float *x, size_t xs, int groups, int gw, int n,
                     const float *w, float eps, const void *gate, size_t gs,
                     int type, int S, void *out, size_t os, void *stream);
+
+/* the same per head of vdim values (a multiple of 32 up to 256, n of them valid)
+ * with gates of low rank: gate = g1 g2^T, g1 [S, r] in `type`, row stride gs, g2 bf16
+ * [H*vdim, r], r a multiple of 64; w [vdim] */
+int vkl_low_rank_gated_norm (const float *x, size_t xs, int H, int vdim, int n,
+                             const float *w, float eps, const void *g1,
+                             size_t gs, const void *g2, int r, int type, int S,
+                             void *out, size_t os, void *stream);
 
 /* ---- per-head products ------------------------------------------------------ */
 /* y[s, h*yh + r] = f * sum_k w[h, r, k] x[s, h*xh + k], w bf16 [H, R, K], f = 1 or

@@ -297,7 +297,9 @@ attn_prefill_kernel (const AttnArgs a)
   // the division by the sum comes last.
   // (the sink is a key that every query has seen before the first tile; the sums of
   // the two lane halves are added at the end, one of them has it)
-  float m = CHUNKED && a.sink ? 0.f : kNeg, sum = CHUNKED && a.sink && hh == 0 ? 1.f : 0.f;
+  // (a tile may hold no key of a query's chunk: its first maximum lies far above the
+  // score of a hidden key, whose weight is then zero)
+  float m = !CHUNKED ? kNeg : a.sink ? 0.f : 0.1f * kNeg, sum = CHUNKED && a.sink && hh == 0 ? 1.f : 0.f;
   float16v oacc[DB];
 #pragma unroll
   for (int db = 0; db < DB; ++db)
@@ -363,10 +365,7 @@ attn_prefill_kernel (const AttnArgs a)
             // exp (kNeg - m) = 0.  The sum takes the weight as the product
             // below consumes it, rounded to fp16: the weights then add up to
             // one exactly.
-            // (a query that has not seen any key yet has m = kNeg: the guard keeps
-            // its weights at zero)
-            const float w = CHUNKED && sv[blk][r] == kNeg ? 0.f : fast_exp (sv[blk][r] - m);
-            const typename E::t e = (typename E::t)w;
+            const typename E::t e = (typename E::t)fast_exp (sv[blk][r] - m);
             sum += (float)e;
             pf[blk][r >> 3][r & 7] = e;
           }

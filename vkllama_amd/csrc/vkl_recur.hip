@@ -20,7 +20,7 @@
 // 16 value columns).  The quotients D_i / D_j are formed from logarithms summed
 // within blocks of 16 tokens, relative to the edge of a block, so that no exponent
 // is positive; inside a block, where that is impossible, the factors are split at
-// the block's start as long as the block decays by less than e^-40, and formed
+// the block's start as long as the block decays by less than 2^-58, and formed
 // pair by pair otherwise.
 // Products run on v_mfma_f32_16x16x4_f32.  Its k index may be permuted: operands
 // hold k = 16 b + 4 (lane / 16) + e in step (b, e), so that a result block, of which
@@ -70,6 +70,17 @@ load4 (const void *p, int type, size_t i)
              __uint_as_float (hi & 0xffff0000u) };
 }
 
+__device__ __forceinline__ void
+store4 (void *p, int type, size_t i, f4 v)
+{
+  if (type == VKL_TYPE_F32)
+    stf4 ((float *)p + i, v);
+  else
+    stg ((unsigned long long *)((uint16_t *)p + i),
+         (unsigned long long)f2bf (v[0]) | ((unsigned long long)f2bf (v[1]) << 16) | ((unsigned long long)f2bf (v[2]) << 32)
+             | ((unsigned long long)f2bf (v[3]) << 48));
+}
+
 __device__ __forceinline__ float
 softplus (float z)
 {
@@ -81,6 +92,15 @@ __device__ __forceinline__ float
 log_decay_of (float rate, float z)
 {
   return fmaxf (-rate * softplus (z), -1.0e4f);
+}
+
+// In the chunked form logarithms are to base 2: their powers are one instruction.
+constexpr float kLog2e = 1.44269504088896340736f;
+
+__device__ __forceinline__ float
+power2 (float x)
+{
+  return __builtin_amdgcn_exp2f (x);
 }
 
 // sum over the lanes that hold the same column (four groups of 16)
@@ -109,52 +129,100 @@ struct ConvArgs
   size_t os;
 };
 
-// eight channels of one token per thread
-__global__ __launch_bounds__ (256) void
-short_conv_kernel (const ConvArgs a)
+// the input of eight channels at token s of the pass (negative: of the tokens before it)
+__device__ __forceinline__ void
+conv_input (const ConvArgs &a, int s, int c, f4 (&x)[2])
 {
-  const int n8 = a.n / 8;
-  const size_t it = (size_t)blockIdx.x * 256 + threadIdx.x;
-  if (it >= (size_t)a.S * n8)
-    return;
-  const int s = (int)(it / n8), c = (int)(it - (size_t)s * n8) * 8;
-  f4 lo = { 0.f, 0.f, 0.f, 0.f }, hi = lo;
-  for (int j = 0; j < a.taps; ++j)
+  x[0] = x[1] = f4{ 0.f, 0.f, 0.f, 0.f };
+  if (s >= 0)
     {
-      const int back = a.taps - 1 - j;
-      f4 x0, x1;
-      if (back <= s)
-        {
-          const size_t at = (size_t)(s - back) * a.xs + c;
-          x0 = load4 (a.x, a.type, at), x1 = load4 (a.x, a.type, at + 4);
-        }
-      else if ((uint32_t)(back - s) <= a.pos0)
-        {
-          const float *r = a.ring + (size_t)((a.pos0 - (uint32_t)(back - s)) % (uint32_t)a.taps) * a.n + c;
-          x0 = ldf4 (r), x1 = ldf4 (r + 4);
-        }
-      else
-        continue;
-      const f4 w0 = ldf4 (a.w + (size_t)j * a.n + c), w1 = ldf4 (a.w + (size_t)j * a.n + c + 4);
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        lo[e] = __builtin_fmaf (w0[e], x0[e], lo[e]), hi[e] = __builtin_fmaf (w1[e], x1[e], hi[e]);
+      const size_t at = (size_t)s * a.xs + c;
+      x[0] = load4 (a.x, a.type, at), x[1] = load4 (a.x, a.type, at + 4);
     }
+  else if ((uint32_t)-s <= a.pos0)
+    {
+      const float *r = a.ring + (size_t)((a.pos0 - (uint32_t)-s) % (uint32_t)a.taps) * a.n + c;
+      x[0] = ldf4 (r), x[1] = ldf4 (r + 4);
+    }
+}
+
+__device__ __forceinline__ void
+conv_output (const ConvArgs &a, int s, int c, const f4 (&y)[2])
+{
   const size_t o = (size_t)s * a.os + c;
+  f4 z[2];
+#pragma unroll
+  for (int h = 0; h < 2; ++h)
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      z[h][e] = silu (y[h][e]);
   if (a.type == VKL_TYPE_F32)
     {
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        lo[e] = silu (lo[e]), hi[e] = silu (hi[e]);
-      stf4 ((float *)a.out + o, lo), stf4 ((float *)a.out + o + 4, hi);
+      stf4 ((float *)a.out + o, z[0]), stf4 ((float *)a.out + o + 4, z[1]);
       return;
     }
   uint32_t h[8];
 #pragma unroll
   for (int e = 0; e < 4; ++e)
-    h[e] = f2bf (silu (lo[e])), h[4 + e] = f2bf (silu (hi[e]));
+    h[e] = f2bf (z[0][e]), h[4 + e] = f2bf (z[1][e]);
   stg ((vkl_u32x4 *)((uint16_t *)a.out + o), vkl_u32x4{ h[0] | (h[1] << 16), h[2] | (h[3] << 16), h[4] | (h[5] << 16),
                                                         h[6] | (h[7] << 16) });
+}
+
+constexpr int kConvRun = 4; // tokens of a thread
+
+// eight channels of a run of tokens per thread.  TAPS: the inputs of the window and
+// the weights stay in registers; 0: any number of taps
+template <int TAPS>
+__global__ __launch_bounds__ (256) void
+short_conv_kernel (const ConvArgs a)
+{
+  const int n8 = a.n / 8;
+  const size_t it = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const int s0 = (int)(it / n8) * kConvRun, c = (int)(it % n8) * 8;
+  if (s0 >= a.S)
+    return;
+  if constexpr (TAPS > 0)
+    {
+      f4 w[TAPS][2], x[kConvRun + TAPS - 1][2];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+        w[j][0] = ldf4 (a.w + (size_t)j * a.n + c), w[j][1] = ldf4 (a.w + (size_t)j * a.n + c + 4);
+#pragma unroll
+      for (int j = 0; j < kConvRun + TAPS - 1; ++j)
+        conv_input (a, min (s0 + j - (TAPS - 1), a.S - 1), c, x[j]);
+#pragma unroll
+      for (int t = 0; t < kConvRun; ++t)
+        {
+          f4 y[2] = { { 0.f, 0.f, 0.f, 0.f }, { 0.f, 0.f, 0.f, 0.f } };
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+#pragma unroll
+              for (int e = 0; e < 4; ++e)
+                y[h][e] = __builtin_fmaf (w[j][h][e], x[t + j][h][e], y[h][e]);
+          if (s0 + t < a.S)
+            conv_output (a, s0 + t, c, y);
+        }
+      return;
+    }
+  for (int s = s0; s < min (s0 + kConvRun, a.S); ++s)
+    {
+      f4 y[2] = { { 0.f, 0.f, 0.f, 0.f }, { 0.f, 0.f, 0.f, 0.f } };
+      for (int j = 0; j < a.taps; ++j)
+        {
+          f4 x[2];
+          conv_input (a, s - (a.taps - 1 - j), c, x);
+          const f4 w[2] = { ldf4 (a.w + (size_t)j * a.n + c), ldf4 (a.w + (size_t)j * a.n + c + 4) };
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              y[h][e] = __builtin_fmaf (w[h][e], x[h][e], y[h][e]);
+        }
+      conv_output (a, s, c, y);
+    }
 }
 
 // the last inputs into the ring, in a launch of their own: the one above reads it
@@ -279,6 +347,9 @@ chunk_floats (int dim, int vdim)
   return (size_t)3 * kChunk * dim + kChunk * kChunk + (size_t)kChunk * vdim + dim;
 }
 
+// Operands lie as the second launch's lanes load them: a block of 16 rows and 16 columns
+// (of the product's inner index) is 64 lanes of four values, lane = row % 16 +
+// 16 (column / 4) - or, for u, as a result lies: lane = column % 16 + 16 (row / 4).
 struct ChunkView
 {
   float *w, *qd, *kt, *p, *u, *dec;
@@ -288,21 +359,68 @@ __device__ __forceinline__ ChunkView
 chunk_view (float *ws, int dim, int vdim)
 {
   ChunkView c;
-  c.w = ws;                           // [64][dim]
-  c.qd = c.w + (size_t)kChunk * dim;  // [64][dim]
-  c.kt = c.qd + (size_t)kChunk * dim; // [dim][64]
-  c.p = c.kt + (size_t)kChunk * dim;  // [64][64]
-  c.u = c.p + kChunk * kChunk;        // [64][vdim]
+  c.w = ws;                            // [4 token blocks][dim / 16]
+  c.qd = c.w + (size_t)kChunk * dim;   // the same
+  c.kt = c.qd + (size_t)kChunk * dim;  // [dim / 16][4 token blocks]
+  c.p = c.kt + (size_t)kChunk * dim;   // [4][4]
+  c.u = c.p + kChunk * kChunk;         // [4][vdim / 16]
   c.dec = c.u + (size_t)kChunk * vdim; // [dim]
   return c;
 }
 
-constexpr int kLdA = kChunk + 4;
+constexpr int kLdA = kChunk + 4, kLdT = 20;
 
 inline size_t
 prep_lds_bytes (int dim)
 {
-  return ((size_t)3 * kChunk * (dim + 4) + kChunk * kLdA + (size_t)kBlocks * dim + 2 * kChunk) * sizeof (float);
+  return ((size_t)3 * kChunk * (dim + 4) + kChunk * kLdA + (size_t)kBlocks * dim + kChunk + kChunk * kLdT)
+         * sizeof (float);
+}
+
+typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
+
+// x W^T for the 16 columns of W rows w0 .. +15 and kChunk rows of x from row s0 on (n of
+// them exist), K a multiple of 64: acc[m][e] is row 16 m + 4 (lane / 16) + e, column
+// lane % 16
+__device__ __forceinline__ void
+low_rank_tile (const void *x, int type, size_t xs, int s0, int n, const uint16_t *w, int K, int lane,
+               f4 (&acc)[kBlocks])
+{
+  const int lo = lane & 15, q = lane >> 4;
+  size_t row[kBlocks];
+#pragma unroll
+  for (int m = 0; m < kBlocks; ++m)
+    {
+      acc[m] = f4{ 0.f, 0.f, 0.f, 0.f };
+      row[m] = (size_t)(s0 + min (16 * m + lo, n - 1)) * xs;
+    }
+  const uint16_t *wr = w + (size_t)lo * K;
+  if (type == VKL_TYPE_BF16)
+    {
+      for (int k0 = 0; k0 < K; k0 += 64)
+#pragma unroll
+        for (int k = k0 + 8 * q, u = 0; u < 2; ++u, k += 32)
+          {
+            const bf8 b = __builtin_bit_cast (bf8, ldg4 (wr + k));
+#pragma unroll
+            for (int m = 0; m < kBlocks; ++m)
+              acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (
+                  __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)x + row[m] + k)), b, acc[m], 0, 0, 0);
+          }
+      return;
+    }
+  for (int k = 4 * q; k < K; k += 16)
+    {
+      const f4 b = load4 (wr, VKL_TYPE_BF16, (size_t)k);
+#pragma unroll
+      for (int m = 0; m < kBlocks; ++m)
+        {
+          const f4 v = ldf4 ((const float *)x + row[m] + k);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            acc[m] = mfma4 (v[e], b[e], acc[m]);
+        }
+    }
 }
 
 template <bool DELTA>
@@ -318,95 +436,146 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
   float *A = ls + kChunk * LD;    // [64][kLdA]
   float *es = A + kChunk * kLdA;  // [4][D]: a block's sum
   float *beta = es + kBlocks * D; // [64]
+  float *T = beta + kChunk;       // [4][16][kLdT]: (1 + A)^-1 of the blocks on the diagonal
   __shared__ uint32_t steep;
   const int h = blockIdx.x % r.H, c = blockIdx.x / r.H, s0 = c * kChunk;
   const int n = min (kChunk, a.S - s0); // tokens; the rest of the chunk changes nothing
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int lo = lane & 15, hi = 4 * (lane >> 4);
   const ChunkView v = chunk_view (ws + ((size_t)c * r.H + h) * chunk_floats (D, r.vdim), D, r.vdim);
   if (tid == 0)
     steep = 0;
   const size_t qo = (size_t)(h / r.rep) * D;
-  // a wave per token: queries, keys, decays
   const float rate = DELTA ? ldg (r.rate + h) : 0.f;
-  const float ld = DELTA ? 0.f : fmaxf (ldg (r.log_decay + h), -1.0e4f);
-  for (int i = wave; i < kChunk; i += kPrepThreads / 64)
-    {
-      const bool in = i < n;
-      const size_t s = (size_t)(s0 + min (i, n - 1));
-      float x[2][2], qq = 0.f, kk = 0.f;
+  const float ld = DELTA ? 0.f : kLog2e * fmaxf (ldg (r.log_decay + h), -1.0e4f);
+  {
+    // queries and keys: 16 lanes per token, eight channels each
+    constexpr int PASS = kChunk / (kPrepThreads / 16);
+    const int d = 8 * lo, dc = min (d, D - 8);
+    f4 x[PASS][2][2], z[PASS][2];
+    float bv[PASS];
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
-        {
-          const int d = lane + 64 * j, dc = min (d, D - 1);
-          x[0][j] = in && d < D ? load_elem (r.q, r.type, s * r.qs + qo + dc) : 0.f;
-          x[1][j] = in && d < D ? load_elem (r.k, r.type, s * r.ks + qo + dc) : 0.f;
-          qq = __builtin_fmaf (x[0][j], x[0][j], qq), kk = __builtin_fmaf (x[1][j], x[1][j], kk);
-        }
-      float fq = r.qscale, fk = 1.f;
-      if (DELTA)
-        fq = r.qscale / sqrtf (wave_sum (qq) + r.unit_eps), fk = 1.0f / sqrtf (wave_sum (kk) + r.unit_eps);
+    for (int p = 0; p < PASS; ++p)
+      {
+        const int i = (p * 8 + wave) * 4 + (lane >> 4);
+        const size_t s = (size_t)(s0 + min (i, n - 1));
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
+        for (int e = 0; e < 2; ++e)
+          {
+            x[p][0][e] = load4 (r.q, r.type, s * r.qs + qo + dc + 4 * e);
+            x[p][1][e] = load4 (r.k, r.type, s * r.ks + qo + dc + 4 * e);
+            if (DELTA && !r.a1)
+              z[p][e] = ldf4 (r.z + s * r.zs + (size_t)h * D + dc + 4 * e);
+          }
+        if (DELTA)
+          bv[p] = ldg (r.b + s * r.bs + h);
+      }
+    if constexpr (DELTA)
+      if (r.a1 && 16 * wave < D)
         {
-          const int d = lane + 64 * j;
-          if (d >= D)
-            continue;
-          qs[i * LD + d] = x[0][j] * fq, ks[i * LD + d] = x[1][j] * fk;
-          float l = ld;
-          if (DELTA)
-            l = log_decay_of (rate, ldg (r.z + s * r.zs + (size_t)h * D + d) + ldg (r.dt_bias + (size_t)h * D + d));
-          ls[i * LD + d] = in ? l : 0.f;
+          f4 acc[kBlocks];
+          low_rank_tile (r.a1, r.type, r.as, s0, n, (const uint16_t *)r.w_a2 + ((size_t)h * D + 16 * wave) * r.r_a, r.r_a,
+                         lane, acc);
+          const float bias = ldg (r.dt_bias + (size_t)h * D + 16 * wave + lo);
+#pragma unroll
+          for (int m = 0; m < kBlocks; ++m)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              {
+                const int i = 16 * m + hi + e;
+                ls[i * LD + 16 * wave + lo] = i < n ? kLog2e * log_decay_of (rate, acc[m][e] + bias) : 0.f;
+              }
         }
-      if (DELTA && lane == 0)
-        beta[i] = in ? sigmoid (ldg (r.b + s * r.bs + h)) : 0.f;
-    }
+#pragma unroll
+    for (int p = 0; p < PASS; ++p)
+      {
+        const int i = (p * 8 + wave) * 4 + (lane >> 4);
+        const bool in = i < n;
+        float qq = 0.f, kk = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          {
+            const float qv = in && d < D ? x[p][0][e >> 2][e & 3] : 0.f, kv = in && d < D ? x[p][1][e >> 2][e & 3] : 0.f;
+            x[p][0][e >> 2][e & 3] = qv, x[p][1][e >> 2][e & 3] = kv;
+            qq = __builtin_fmaf (qv, qv, qq), kk = __builtin_fmaf (kv, kv, kk);
+          }
+        float fq = r.qscale, fk = 1.f;
+        if (DELTA)
+          {
+            fq = r.qscale / sqrtf (row_sum<16> (qq) + r.unit_eps), fk = 1.0f / sqrtf (row_sum<16> (kk) + r.unit_eps);
+            if (lo == 0)
+              beta[i] = in ? sigmoid (bv[p]) : 0.f;
+          }
+        if (d >= D)
+          continue;
+#pragma unroll
+        for (int e = 0; e < 2; ++e)
+          {
+            *(f4 *)(qs + i * LD + d + 4 * e) = x[p][0][e] * fq;
+            *(f4 *)(ks + i * LD + d + 4 * e) = x[p][1][e] * fk;
+            if (DELTA && r.a1)
+              continue;
+            f4 l;
+#pragma unroll
+            for (int g = 0; g < 4; ++g)
+              {
+                if (DELTA)
+                  l[g] = kLog2e * log_decay_of (rate, z[p][e][g] + ldg (r.dt_bias + (size_t)h * D + d + 4 * e + g));
+                else
+                  l[g] = ld;
+                l[g] = in ? l[g] : 0.f;
+              }
+            *(f4 *)(ls + i * LD + d + 4 * e) = l;
+          }
+      }
+  }
   __syncthreads ();
   for (int it = tid; it < kBlocks * D; it += kPrepThreads)
     {
       const int b = it / D, d = it - b * D;
-      float l = 0.f;
+      float x[16], l = 0.f;
+#pragma unroll
+      for (int i = 0; i < 16; ++i)
+        x[i] = ls[(16 * b + i) * LD + d];
+#pragma unroll
       for (int i = 0; i < 16; ++i)
         {
-          l += ls[(16 * b + i) * LD + d];
+          l += x[i];
           ls[(16 * b + i) * LD + d] = l;
         }
       es[it] = l;
-      if (l < -40.f)
+      if (l < -58.f)
         atomicOr (&steep, 1u << b);
     }
   __syncthreads ();
 
-  // P, and for the delta rule A: pairs of blocks (bi, bj <= bi)
-  const int lo = lane & 15, hi = 4 * (lane >> 4);
-  for (int t = wave; t < kBlocks * (kBlocks + 1) / 2; t += kPrepThreads / 64)
-    {
-      const int bi = t < 1 ? 0 : t < 3 ? 1 : t < 6 ? 2 : 3, bj = t - bi * (bi + 1) / 2;
-      if (bi == bj && ((steep >> bi) & 1u))
+  // P, and for the delta rule A, in blocks (bi, bj <= bi), transposed in the registers:
+  // a lane holds row lo, columns hi .. hi + 3.  Waves 0 .. 3 take the diagonal and
+  // invert it, the others the blocks below it.
+  const int DB = D / 16;
+  auto block = [&] (int bi, int bj) {
+    const int i = 16 * bi + lo;
+    f4 sp = { 0.f, 0.f, 0.f, 0.f }, sa = sp;
+    if (bi == bj && ((steep >> bi) & 1u))
+      // pair by pair
+      for (int d = 0; d < D; ++d)
         {
-          // pair by pair
-          for (int pr = lane; pr < 256; pr += 64)
+          const float q = qs[i * LD + d], k = ks[i * LD + d], l = ls[i * LD + d];
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
             {
-              const int i = 16 * bi + (pr >> 4), j = 16 * bi + (pr & 15);
-              float sa = 0.f, sp = 0.f;
-              if (j <= i)
-                for (int d = 0; d < D; ++d)
-                  {
-                    const float f = ks[j * LD + d] * expf (ls[i * LD + d] - ls[j * LD + d]);
-                    sp = __builtin_fmaf (qs[i * LD + d], f, sp);
-                    if (DELTA)
-                      sa = __builtin_fmaf (ks[i * LD + d], f, sa);
-                  }
-              stg (v.p + i * kChunk + j, sp);
+              const int j = 16 * bj + hi + e;
+              const float f = ks[j * LD + d] * power2 (fminf (l - ls[j * LD + d], 0.f));
+              sp[e] = __builtin_fmaf (q, f, sp[e]);
               if (DELTA)
-                A[i * kLdA + j] = j < i ? sa * beta[i] : 0.f;
+                sa[e] = __builtin_fmaf (k, f, sa[e]);
             }
-          continue;
         }
-      f4 accp = { 0.f, 0.f, 0.f, 0.f }, acca = accp;
+    else
       for (int d0 = hi; d0 < D; d0 += 16)
         {
-          const f4 li = *(const f4 *)(ls + (16 * bi + lo) * LD + d0), lj = *(const f4 *)(ls + (16 * bj + lo) * LD + d0);
-          const f4 qi = *(const f4 *)(qs + (16 * bi + lo) * LD + d0), kj = *(const f4 *)(ks + (16 * bj + lo) * LD + d0);
+          const f4 li = *(const f4 *)(ls + i * LD + d0), lj = *(const f4 *)(ls + (16 * bj + lo) * LD + d0);
+          const f4 qi = *(const f4 *)(qs + i * LD + d0), kj = *(const f4 *)(ks + (16 * bj + lo) * LD + d0);
           f4 mid = { 0.f, 0.f, 0.f, 0.f };
           if (bj < bi)
             mid = *(const f4 *)(es + bj * D + d0);
@@ -414,92 +583,143 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
             mid += *(const f4 *)(es + b * D + d0);
           f4 ki = { 0.f, 0.f, 0.f, 0.f };
           if (DELTA)
-            ki = *(const f4 *)(ks + (16 * bi + lo) * LD + d0);
+            ki = *(const f4 *)(ks + i * LD + d0);
 #pragma unroll
           for (int e = 0; e < 4; ++e)
             {
-              const float fi = expf (li[e]), x = kj[e] * expf (mid[e] - lj[e]);
-              accp = mfma4 (qi[e] * fi, x, accp);
+              const float fi = power2 (li[e]), x = kj[e] * power2 (mid[e] - lj[e]);
+              sp = mfma4 (x, qi[e] * fi, sp);
               if (DELTA)
-                acca = mfma4 (ki[e] * fi, x, acca);
+                sa = mfma4 (x, ki[e] * fi, sa);
             }
         }
+    const float bi_ = DELTA ? beta[i] : 0.f;
 #pragma unroll
-      for (int e = 0; e < 4; ++e)
+    for (int e = 0; e < 4; ++e)
+      {
+        const int j = 16 * bj + hi + e;
+        sp[e] = j <= i ? sp[e] : 0.f;
+        if (DELTA)
+          sa[e] = j < i ? sa[e] * bi_ : 0.f;
+      }
+    stf4 (v.p + ((size_t)(bi * kBlocks + bj) * 64 + lane) * 4, sp);
+    if (DELTA)
+      *(f4 *)(A + i * kLdA + 16 * bj + hi) = sa;
+  };
+  if (wave < kBlocks)
+    {
+      block (wave, wave);
+      if constexpr (DELTA)
         {
-          const int i = 16 * bi + hi + e, j = 16 * bj + lo;
-          stg (v.p + i * kChunk + j, j <= i ? accp[e] : 0.f);
-          if (DELTA)
-            A[i * kLdA + j] = j < i ? acca[e] * beta[i] : 0.f;
+          // column lo of the inverse (the lane groups do the same)
+          __builtin_amdgcn_fence (__ATOMIC_RELEASE, "wavefront");
+          __builtin_amdgcn_wave_barrier ();
+          const float *Ab = A + 16 * wave * kLdA + 16 * wave;
+          float x[16];
+#pragma unroll
+          for (int i = 0; i < 16; ++i)
+            {
+              float y = i == lo ? 1.f : 0.f;
+#pragma unroll
+              for (int j = 0; j < i; ++j)
+                y = __builtin_fmaf (-Ab[i * kLdA + j], x[j], y);
+              x[i] = y;
+              T[(16 * wave + i) * kLdT + lo] = y;
+            }
         }
     }
-  // queries with the decay since the start of the chunk, keys with the decay to its end
-  for (int it = tid; it < kChunk * D; it += kPrepThreads)
+  else if (wave < 6)
+    block (wave - 3, 0), block (3, wave - 4);
+  else
+    block (wave == 6 ? 3 : 2, wave == 6 ? 2 : 1);
+  // keys with the decay to the end of the chunk
+  for (int it = wave; it < DB * kBlocks; it += kPrepThreads / 64)
     {
-      const int i = it / D, d = it - i * D;
-      float l = ls[i * LD + d];
-      for (int b = 0; b < i / 16; ++b)
-        l += es[b * D + d];
-      stg (v.qd + it, qs[i * LD + d] * expf (l));
+      const int b = it % kBlocks, d = it / kBlocks * 16 + lo, j = 16 * b + hi;
+      float end = es[b * D + d];
+      for (int k = b + 1; k < kBlocks; ++k)
+        end += es[k * D + d];
+      f4 o;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        o[e] = ks[(j + e) * LD + d] * power2 (end - ls[(j + e) * LD + d]);
+      stf4 (v.kt + ((size_t)it * 64 + lane) * 4, o);
     }
-  for (int it = tid; it < kChunk * D; it += kPrepThreads)
+  // queries with the decay since its start
+  for (int it = wave; it < kBlocks * DB; it += kPrepThreads / 64)
     {
-      const int d = it / kChunk, j = it - d * kChunk;
-      float l = es[(j / 16) * D + d] - ls[j * LD + d];
-      for (int b = j / 16 + 1; b < kBlocks; ++b)
-        l += es[b * D + d];
-      stg (v.kt + it, ks[j * LD + d] * expf (l));
+      const int b = it / DB, d = it % DB * 16 + hi, i = 16 * b + lo;
+      f4 l = *(const f4 *)(ls + i * LD + d), o = *(const f4 *)(qs + i * LD + d);
+      for (int k = 0; k < b; ++k)
+        l += *(const f4 *)(es + k * D + d);
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        o[e] *= power2 (l[e]);
+      stf4 (v.qd + ((size_t)it * 64 + lane) * 4, o);
     }
   for (int d = tid; d < D; d += kPrepThreads)
     {
       float l = 0.f;
       for (int b = 0; b < kBlocks; ++b)
         l += es[b * D + d];
-      stg (v.dec + d, expf (l));
+      stg (v.dec + d, power2 (l));
     }
-  if (!DELTA)
-    return;
-  __syncthreads ();
-  // (1 + A) x = right side, a column per thread: diag (beta) V, diag (beta) K D
-  for (int col = tid; col < r.vdim + D; col += kPrepThreads)
+  if constexpr (DELTA)
     {
-      const bool val = col < r.vdim;
-      const int d = val ? 0 : col - r.vdim;
-      float x[kChunk], before = 0.f;
-#pragma unroll
-      for (int i = 0; i < kChunk; ++i)
+      __syncthreads ();
+      // (1 + A) X = [diag (beta) V | diag (beta) K D], 16 columns of X per wave, block row
+      // by block row: X_b = T_b (R_b - sum_{b' < b} A_bb' X_b').  The queries' place in LDS
+      // takes W, which leaves it in the other order.
+      const int VB = r.vdim / 16;
+      for (int g = wave; g < VB + DB; g += kPrepThreads / 64)
         {
-          float y;
-          if (val)
-            y = load_elem (r.v, r.type, (size_t)(s0 + min (i, n - 1)) * r.vs + (size_t)h * r.vdim + col);
-          else
-            {
-              if (i > 0 && i % 16 == 0)
-                before += es[(i / 16 - 1) * D + d];
-              y = ks[i * LD + d] * expf (ls[i * LD + d] + before);
-            }
-          x[i] = y * beta[i];
-        }
+          const bool val = g < VB;
+          const int col = 16 * (val ? g : g - VB) + lo;
+          f4 x[kBlocks];
+          float before = 0.f;
 #pragma unroll
-      for (int i = 1; i < kChunk; ++i)
-        {
-          float y = x[i];
-#pragma unroll
-          for (int j = 0; j < i; j += 4)
+          for (int b = 0; b < kBlocks; ++b)
             {
-              const f4 w = *(const f4 *)(A + i * kLdA + j);
 #pragma unroll
               for (int e = 0; e < 4; ++e)
-                if (j + e < i)
-                  y = __builtin_fmaf (-w[e], x[j + e], y);
+                {
+                  const int i = 16 * b + hi + e;
+                  const float y = val ? load_elem (r.v, r.type, (size_t)(s0 + min (i, n - 1)) * r.vs + (size_t)h * r.vdim + col)
+                                      : ks[i * LD + col] * power2 (ls[i * LD + col] + before);
+                  x[b][e] = y * beta[i];
+                }
+              if (!val)
+                before += es[b * D + col];
             }
-          x[i] = y;
-        }
-      float *dst = val ? v.u + col : v.w + d;
-      const int stride = val ? r.vdim : D;
 #pragma unroll
-      for (int i = 0; i < kChunk; ++i)
-        stg (dst + (size_t)i * stride, x[i]);
+          for (int b = 0; b < kBlocks; ++b)
+            {
+              f4 acc = x[b];
+#pragma unroll
+              for (int k = 0; k < b; ++k)
+                {
+                  const f4 m = *(const f4 *)(A + (16 * b + lo) * kLdA + 16 * k + hi);
+#pragma unroll
+                  for (int e = 0; e < 4; ++e)
+                    acc = mfma4 (-m[e], x[k][e], acc);
+                }
+              const f4 m = *(const f4 *)(T + (16 * b + lo) * kLdT + hi);
+              f4 y = { 0.f, 0.f, 0.f, 0.f };
+#pragma unroll
+              for (int e = 0; e < 4; ++e)
+                y = mfma4 (m[e], acc[e], y);
+              x[b] = y;
+              if (val)
+                stf4 (v.u + ((size_t)(b * VB + g) * 64 + lane) * 4, y);
+              else
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                  qs[(16 * b + hi + e) * LD + col] = y[e];
+            }
+        }
+      __syncthreads ();
+      for (int it = wave; it < kBlocks * DB; it += kPrepThreads / 64)
+        stf4 (v.w + ((size_t)it * 64 + lane) * 4, *(const f4 *)(qs + (16 * (it / DB) + lo) * LD + it % DB * 16 + hi));
     }
 }
 
@@ -507,8 +727,9 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
 // chunks: along the state
 // ---------------------------------------------------------------------------
 // wave w: tokens 16 w .. +15 of a chunk, and blocks w, w + 4 of the state's rows
+// (one workgroup per compute unit: the next chunk's operands travel in registers)
 template <int DB, bool DELTA>
-__global__ __launch_bounds__ (256) void
+__global__ __launch_bounds__ (256) __attribute__ ((amdgpu_waves_per_eu (1, 1))) void
 chunk_scan_kernel (const RecurArgs a, const float *ws)
 {
   constexpr int KB = (DB + 3) / 4, D = 16 * DB;
@@ -539,18 +760,18 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
   auto fetch = [&] (int c, Operands &o) {
     const float *base = ws + ((size_t)c * r.H + h) * per;
     const ChunkView v = chunk_view (const_cast<float *> (base), D, r.vdim);
-    const int row = 16 * wave + lo;
+    auto at = [&] (const float *m, int blk) { return ldf4 (m + ((size_t)blk * 64 + lane) * 4); };
 #pragma unroll
     for (int b = 0; b < DB; ++b)
       {
-        o.q[b] = ldf4 (v.qd + (size_t)row * D + 16 * b + hi);
+        o.q[b] = at (v.qd, wave * DB + b);
         if constexpr (DELTA)
-          o.w[b] = ldf4 (v.w + (size_t)row * D + 16 * b + hi);
+          o.w[b] = at (v.w, wave * DB + b);
       }
 #pragma unroll
     for (int b = 0; b < kBlocks; ++b)
       // (blocks right of the diagonal do not exist)
-      o.p[b] = ldf4 (v.p + row * kChunk + 16 * min (b, wave) + hi);
+      o.p[b] = at (v.p, wave * kBlocks + min (b, wave));
 #pragma unroll
     for (int i = 0; i < KB; ++i)
       {
@@ -558,21 +779,18 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
         o.dec[i] = ldf4 (v.dec + 16 * b + hi);
 #pragma unroll
         for (int j = 0; j < kBlocks; ++j)
-          o.k[i][j] = ldf4 (v.kt + (size_t)(16 * b + lo) * kChunk + 16 * j + hi);
+          o.k[i][j] = at (v.kt, b * kBlocks + j);
       }
+    if constexpr (DELTA)
+      o.u = at (v.u, wave * (r.vdim / 16) + vb);
+    else
 #pragma unroll
-    for (int e = 0; e < 4; ++e)
-      {
-        const int t = 16 * wave + hi + e;
-        if constexpr (DELTA)
-          o.u[e] = ldg (v.u + (size_t)t * r.vdim + col);
-        else
-          {
-            // (tokens past the end have keys of zero)
-            const int s = min (c * kChunk + t, a.S - 1);
-            o.u[e] = load_elem (r.v, r.type, (size_t)s * r.vs + (size_t)h * r.vdim + col);
-          }
-      }
+      for (int e = 0; e < 4; ++e)
+        {
+          // (tokens past the end have keys of zero)
+          const int s = min (c * kChunk + 16 * wave + hi + e, a.S - 1);
+          o.u[e] = load_elem (r.v, r.type, (size_t)s * r.vs + (size_t)h * r.vdim + col);
+        }
   };
   auto chunk = [&] (int c, const Operands &o) {
     f4 acc = { 0.f, 0.f, 0.f, 0.f }, sub = acc, acc2 = acc, sub2 = acc;
@@ -638,10 +856,12 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
   for (int c = 0; c < chunks; c += 2)
     {
       fetch (min (c + 1, chunks - 1), y);
+      __builtin_amdgcn_sched_barrier (0);
       chunk (c, x);
       if (c + 1 >= chunks)
         break;
       fetch (min (c + 2, chunks - 1), x);
+      __builtin_amdgcn_sched_barrier (0);
       chunk (c + 1, y);
     }
 #pragma unroll
@@ -748,13 +968,85 @@ gated_norm_kernel (const GatedNormArgs a)
 #pragma unroll
       for (int e = 0; e < 4; ++e)
         o[e] = v[e] * alpha * w[e] * sigmoid (g[e]);
-      const size_t at = s * a.os + g0 + c;
-      if (a.type == VKL_TYPE_F32)
-        stf4 ((float *)a.out + at, o);
-      else
-        stg ((unsigned long long *)((uint16_t *)a.out + at),
-             (unsigned long long)f2bf (o[0]) | ((unsigned long long)f2bf (o[1]) << 16)
-                 | ((unsigned long long)f2bf (o[2]) << 32) | ((unsigned long long)f2bf (o[3]) << 48));
+      store4 (a.out, a.type, s * a.os + g0 + c, o);
+    }
+}
+
+// The same per head with gates x W^T of low rank: a wave takes 16 tokens of a head, a
+// workgroup 64.
+struct LowRankNormArgs
+{
+  const float *x;
+  size_t xs;
+  int H, vdim, n;
+  const float *w;
+  float eps;
+  const void *g1;
+  size_t gs;
+  const uint16_t *g2;
+  int r, type, S;
+  void *out;
+  size_t os;
+};
+
+template <int VB>
+__global__ __launch_bounds__ (256) void
+low_rank_norm_kernel (const LowRankNormArgs a)
+{
+  const int lane = threadIdx.x & 63, lo = lane & 15, q = lane >> 4;
+  const int h = blockIdx.x % a.H, s0 = (blockIdx.x / a.H) * 64 + (threadIdx.x >> 6) * 16;
+  if (s0 >= a.S)
+    return;
+  // a lane holds token lo and columns 16 b + 4 q + 0..3
+  const size_t s = (size_t)min (s0 + lo, a.S - 1);
+  f4 o[VB], g[VB];
+  float ss = 0.f;
+#pragma unroll
+  for (int b = 0; b < VB; ++b)
+    {
+      g[b] = f4{ 0.f, 0.f, 0.f, 0.f };
+      o[b] = ldf4 (a.x + s * a.xs + (size_t)h * a.vdim + 16 * b + 4 * q);
+    }
+  const uint16_t *w = a.g2 + ((size_t)h * a.vdim + lo) * a.r;
+  if (a.type == VKL_TYPE_BF16)
+    for (int k = 8 * q; k < a.r; k += 32)
+      {
+        const bf8 x = __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)a.g1 + s * a.gs + k));
+#pragma unroll
+        for (int b = 0; b < VB; ++b)
+          g[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (__builtin_bit_cast (bf8, ldg4 (w + (size_t)16 * b * a.r + k)), x,
+                                                          g[b], 0, 0, 0);
+      }
+  else
+    for (int k = 4 * q; k < a.r; k += 16)
+      {
+        const f4 x = ldf4 ((const float *)a.g1 + s * a.gs + k);
+#pragma unroll
+        for (int b = 0; b < VB; ++b)
+          {
+            const f4 y = load4 (w, VKL_TYPE_BF16, (size_t)16 * b * a.r + k);
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              g[b] = mfma4 (y[e], x[e], g[b]);
+          }
+      }
+#pragma unroll
+  for (int b = 0; b < VB; ++b)
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      ss = __builtin_fmaf (o[b][e], o[b][e], ss);
+  const float alpha = 1.0f / sqrtf (rows_sum (ss) / (float)a.n + a.eps);
+  if (s0 + lo >= a.S)
+    return;
+#pragma unroll
+  for (int b = 0; b < VB; ++b)
+    {
+      const f4 wn = ldf4 (a.w + 16 * b + 4 * q);
+      f4 y;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        y[e] = o[b][e] * alpha * wn[e] * sigmoid (g[b][e]);
+      store4 (a.out, a.type, s * a.os + (size_t)h * a.vdim + 16 * b + 4 * q, y);
     }
 }
 
@@ -763,99 +1055,196 @@ gated_norm_kernel (const GatedNormArgs a)
 // ---------------------------------------------------------------------------
 constexpr int kStepThreads = 512, kStepWaves = 8;
 
-// y[i] = w[i, :] x for the rows i of one head, eight lanes per row
-template <typename F>
-__device__ __forceinline__ void
-head_rows (const uint16_t *w, int rows, int K, const float *x, F put)
-{
-  const int sub = threadIdx.x & 7;
-  for (int i0 = 0; i0 < rows; i0 += kStepThreads / 8)
-    {
-      const int i = i0 + (threadIdx.x >> 3), ic = min (i, rows - 1);
-      float acc = 0.f;
-      for (int k = sub * 8; k < K; k += 64)
-        {
-          float f[8];
-          widen8 (ldg4 (w + (size_t)ic * K + k), f);
-          const f4 x0 = *(const f4 *)(x + k), x1 = *(const f4 *)(x + k + 4);
-#pragma unroll
-          for (int e = 0; e < 4; ++e)
-            acc = __builtin_fmaf (f[e], x0[e], acc), acc = __builtin_fmaf (f[4 + e], x1[e], acc);
-        }
-      acc = row_sum<8> (acc);
-      if (sub == 0 && i < rows)
-        put (i, acc);
-    }
-}
+// y[i] = w[i, :] x for the rows i of one head.  Rows of 64 or 128 values are dealt out
+// in 16-byte chunks, so that the first of them are requested long before x is
+// there; other lengths take eight lanes per row.
+constexpr int kAhead = 4; // chunks of a thread
 
-// DJ: dim / 16.  A wave takes blocks of 16 value columns in turn; the state of the
-// first is requested before anything else.
+struct HeadRows
+{
+  const uint16_t *w;
+  int rows, K;
+  uint4 ahead[kAhead];
+
+  __device__ __forceinline__ bool
+  dealt () const
+  {
+    return K == 64 || K == 128;
+  }
+  __device__ __forceinline__ int
+  shift () const
+  {
+    return K == 64 ? 3 : 4;
+  }
+  __device__ __forceinline__ void
+  request ()
+  {
+    if (dealt ())
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u)
+        ahead[u] = ldg4 (w + (size_t)min ((int)threadIdx.x + u * kStepThreads, (rows << shift ()) - 1) * 8);
+  }
+  static __device__ __forceinline__ float
+  dot8 (const uint4 v, const float *x)
+  {
+    float f[8], acc = 0.f;
+    widen8 (v, f);
+    const f4 x0 = *(const f4 *)x, x1 = *(const f4 *)(x + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      acc = __builtin_fmaf (f[e], x0[e], acc), acc = __builtin_fmaf (f[4 + e], x1[e], acc);
+    return acc;
+  }
+  template <typename F>
+  __device__ __forceinline__ void
+  run (const float *x, F put) const
+  {
+    if (dealt ())
+      {
+        const int sh = shift (), all = rows << sh, mask = (1 << sh) - 1;
+        auto part = [&] (int c, const uint4 v) {
+          float y = row_sum<8> (dot8 (v, x + (c & mask) * 8));
+          if (sh == 4)
+            y += dpp_get<0x140> (y);
+          if ((c & mask) == 0 && c < all)
+            put (c >> sh, y);
+        };
+#pragma unroll
+        for (int u = 0; u < kAhead; ++u)
+          part ((int)threadIdx.x + u * kStepThreads, ahead[u]);
+#pragma unroll 1
+        for (int c = (int)threadIdx.x + kAhead * kStepThreads; c < all; c += kStepThreads)
+          part (c, ldg4 (w + (size_t)c * 8));
+        return;
+      }
+    const int sub = threadIdx.x & 7;
+#pragma unroll 1
+    for (int i0 = 0; i0 < rows; i0 += kStepThreads / 8)
+      {
+        const int i = i0 + (int)(threadIdx.x >> 3), ic = min (i, rows - 1);
+        float acc = 0.f;
+#pragma unroll 1
+        for (int k = sub * 8; k < K; k += 64)
+          acc += dot8 (ldg4 (w + (size_t)ic * K + k), x + k);
+        acc = row_sum<8> (acc);
+        if (sub == 0 && i < rows)
+          put (i, acc);
+      }
+  }
+};
+
+// DJ: dim / 16.  A wave takes blocks of 16 value columns in turn.  What the launch
+// reads is requested at its start, in one round trip.
 template <int DJ, bool DELTA>
 __global__ __launch_bounds__ (kStepThreads) void
 recur_step_kernel (const RecurStepArgs a)
 {
-  constexpr int D = 16 * DJ, MV = 256;
-  __shared__ __align__ (16) float q[D], k[D], g[D], v[MV], o[MV], z[MV];
+  constexpr int D = 16 * DJ, MV = 256, TAPS = 4; // taps requested ahead
+  __shared__ __align__ (16) float q[D], k[D], g[D], v[MV], o[MV], z[MV], bias[D];
   extern __shared__ __align__ (16) float lds_step[]; // a1 | g1
   __shared__ float red[kStepWaves];
   const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int lo = lane & 15, hi = 4 * (lane >> 4);
   const uint32_t pos = a.pos.get ();
-  float *st = a.state + (size_t)h * D * a.vdim + lo;
+  float *st = a.state + (size_t)h * D * a.vdim;
+  const uint32_t cell = (uint32_t)(hi * a.vdim + lo); // a lane's place in a block of the state
   f4 m[DJ];
   auto fetch = [&] (int vb) {
 #pragma unroll
     for (int j = 0; j < DJ; ++j)
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        m[j][e] = ldg (st + (size_t)(16 * j + hi + e) * a.vdim + 16 * vb);
+        m[j][e] = ldg (st + ((16 * j + e) * a.vdim + 16 * vb) + cell);
   };
-  const int blocks = a.vdim / 16;
-  fetch (min (wave, blocks - 1));
-  __builtin_amdgcn_sched_barrier (0);
   const int G = a.H / a.rep, hq = h / a.rep;
   const int nqk = G * D, n = 2 * nqk + a.H * a.vdim;
-  // q, k, v of the head
-  for (int c = tid; c < 2 * D + a.vdim; c += kStepThreads)
-    {
-      const int ch = c < D ? hq * D + c : c < 2 * D ? nqk + hq * D + c - D : 2 * nqk + h * a.vdim + c - 2 * D;
-      float x = ldg (a.qkv + ch);
-      if (DELTA)
+  // q, k, v of the head: a channel per thread, where there are more than threads in turns
+  auto channel = [&] (int c) {
+    return c < D ? hq * D + c : c < 2 * D ? nqk + hq * D + c - D : 2 * nqk + h * a.vdim + c - 2 * D;
+  };
+  auto request = [&] (int c, float &now, float (&w)[TAPS], float (&x)[TAPS]) {
+    const int ch = channel (min (c, 2 * D + a.vdim - 1));
+    now = ldg (a.qkv + ch);
+    if (DELTA)
+#pragma unroll
+      for (int b = 0; b < TAPS; ++b)
         {
-          const float now = x;
-          x = ldg (a.conv + (size_t)(a.taps - 1) * n + ch) * now;
-          for (int back = 1; back < a.taps; ++back)
-            if ((uint32_t)back <= pos)
-              x = __builtin_fmaf (ldg (a.conv + (size_t)(a.taps - 1 - back) * n + ch),
-                                  ldg (a.ring + (size_t)((pos - (uint32_t)back) % (uint32_t)a.taps) * n + ch), x);
-          x = silu (x);
-          // (the row of this position is none that the step reads; heads that share a
-          // query and key leave it to the first of them)
-          if (c >= 2 * D || h % a.rep == 0)
-            stg (a.ring + (size_t)(pos % (uint32_t)a.taps) * n + ch, now);
+          w[b] = ldg (a.conv + (size_t)max (a.taps - 1 - b, 0) * n + ch);
+          x[b] = ldg (a.ring + (size_t)((pos - (uint32_t)min (b, (int)pos)) % (uint32_t)a.taps) * n + ch);
         }
-      if (c < D)
-        q[c] = x;
-      else if (c < 2 * D)
-        k[c - D] = x;
-      else
-        v[c - 2 * D] = x;
+  };
+  auto finish = [&] (int c, float now, const float (&w)[TAPS], const float (&x)[TAPS]) {
+    float y = now;
+    if (DELTA)
+      {
+        const int ch = channel (c);
+        y = w[0] * now;
+#pragma unroll
+        for (int b = 1; b < TAPS; ++b)
+          if (b < a.taps && (uint32_t)b <= pos)
+            y = __builtin_fmaf (w[b], x[b], y);
+#pragma unroll 1
+        for (int b = TAPS; b < a.taps && (uint32_t)b <= pos; ++b)
+          y = __builtin_fmaf (ldg (a.conv + (size_t)(a.taps - 1 - b) * n + ch),
+                              ldg (a.ring + (size_t)((pos - (uint32_t)b) % (uint32_t)a.taps) * n + ch), y);
+        y = silu (y);
+        // (the row of this position is none that the step uses; heads that share a
+        // query and key leave it to the first of them)
+        if (c >= 2 * D || h % a.rep == 0)
+          stg (a.ring + (size_t)(pos % (uint32_t)a.taps) * n + ch, now);
+      }
+    if (c < D)
+      q[c] = y;
+    else if (c < 2 * D)
+      k[c - D] = y;
+    else
+      v[c - 2 * D] = y;
+  };
+  float now, cw[TAPS], cx[TAPS];
+  request (tid, now, cw, cx);
+  const int blocks = a.vdim / 16;
+  float a1v = 0.f, g1v = 0.f, bv = 0.f, rate = 0.f, bias_v = 0.f, gn = 0.f;
+  HeadRows decays, gates;
+  if constexpr (DELTA)
+    {
+      a1v = ldg (a.a1 + min (tid, a.r_a - 1)), g1v = ldg (a.g1 + min (tid, a.r_g - 1));
+      bv = ldg (a.b + h), rate = ldg (a.rate + h);
+      bias_v = ldg (a.dt_bias + (size_t)h * D + min (tid, D - 1));
+      gn = ldg (a.gnorm + min (tid, a.vdim - 1));
+      decays.w = a.w_a2 + (size_t)h * D * a.r_a, decays.rows = D, decays.K = a.r_a;
+      gates.w = a.w_g2 + (size_t)h * a.vdim * a.r_g, gates.rows = a.vdim, gates.K = a.r_g;
+      decays.request (), gates.request ();
+    }
+  fetch (min (wave, blocks - 1));
+  __builtin_amdgcn_sched_barrier (0);
+  if (tid < 2 * D + a.vdim)
+    finish (tid, now, cw, cx);
+#pragma unroll 1
+  for (int c = tid + kStepThreads; c < 2 * D + a.vdim; c += kStepThreads)
+    {
+      request (c, now, cw, cx);
+      finish (c, now, cw, cx);
     }
   float decay = 1.f, beta = 0.f, fq = a.qscale, fk = 1.f;
   if (DELTA)
     {
       float *a1 = lds_step, *g1 = lds_step + a.r_a;
-      for (int i = tid; i < a.r_a; i += kStepThreads)
+      if (tid < a.r_a)
+        a1[tid] = a1v;
+      if (tid < a.r_g)
+        g1[tid] = g1v;
+      if (tid < D)
+        bias[tid] = bias_v;
+#pragma unroll 1
+      for (int i = tid + kStepThreads; i < a.r_a; i += kStepThreads)
         a1[i] = ldg (a.a1 + i);
-      for (int i = tid; i < a.r_g; i += kStepThreads)
+#pragma unroll 1
+      for (int i = tid + kStepThreads; i < a.r_g; i += kStepThreads)
         g1[i] = ldg (a.g1 + i);
-      beta = sigmoid (ldg (a.b + h));
-      const float rate = ldg (a.rate + h);
+      beta = sigmoid (bv);
       __syncthreads ();
-      head_rows (a.w_a2 + (size_t)h * D * a.r_a, D, a.r_a, a1, [&] (int i, float y) {
-        g[i] = expf (log_decay_of (rate, y + ldg (a.dt_bias + (size_t)h * D + i)));
-      });
-      head_rows (a.w_g2 + (size_t)h * a.vdim * a.r_g, a.vdim, a.r_g, g1, [&] (int i, float y) { z[i] = sigmoid (y); });
+      decays.run (a1, [&] (int i, float y) { g[i] = expf (log_decay_of (rate, y + bias[i])); });
+      gates.run (g1, [&] (int i, float y) { z[i] = sigmoid (y); });
       float qq = 0.f, kk = 0.f;
       for (int d = lane; d < D; d += 64)
         qq = __builtin_fmaf (q[d], q[d], qq), kk = __builtin_fmaf (k[d], k[d], kk);
@@ -897,7 +1286,7 @@ recur_step_kernel (const RecurStepArgs a)
                 m[j][e] = pos ? m[j][e] * decay : 0.f;
               m[j][e] = __builtin_fmaf (kj[e] * fk, u, m[j][e]);
               out = __builtin_fmaf (m[j][e], qj[e], out);
-              stg (st + (size_t)(16 * j + hi + e) * a.vdim + 16 * vb, m[j][e]);
+              stg (st + ((16 * j + e) * a.vdim + 16 * vb) + cell, m[j][e]);
             }
         }
       out = rows_sum (out) * fq;
@@ -920,8 +1309,8 @@ recur_step_kernel (const RecurStepArgs a)
   for (int c = tid; c < a.vdim; c += kStepThreads)
     ss = __builtin_fmaf (o[c], o[c], ss);
   const float alpha = 1.0f / sqrtf (group_sum (ss, red) / (float)a.vn + a.eps);
-  for (int c = tid; c < a.vdim; c += kStepThreads)
-    stg (a.out + (size_t)h * a.vdim + c, o[c] * alpha * ldg (a.gnorm + c) * z[c]);
+  if (tid < a.vdim)
+    stg (a.out + (size_t)h * a.vdim + tid, o[tid] * alpha * gn * z[tid]);
 }
 
 template <bool DELTA>
@@ -983,8 +1372,15 @@ vkl_short_conv_silu (const void *x, int type, size_t xs, const float *w, int n, 
                  && ((uintptr_t)ring % 16) == 0);
   const ConvArgs a = { x, type, xs, w, n, taps, ring, pos0, S, out, os };
   hipStream_t s = (hipStream_t)stream;
-  const size_t items = (size_t)S * (n / 8), keep = (size_t)std::min (S, taps) * n;
-  short_conv_kernel<<<dim3 ((unsigned)((items + 255) / 256)), dim3 (256), 0, s>>> (a);
+  const size_t items = (size_t)((S + kConvRun - 1) / kConvRun) * (n / 8), keep = (size_t)std::min (S, taps) * n;
+  const dim3 grid ((unsigned)((items + 255) / 256)), block (256);
+  switch (taps)
+    {
+    case 2: short_conv_kernel<2><<<grid, block, 0, s>>> (a); break;
+    case 3: short_conv_kernel<3><<<grid, block, 0, s>>> (a); break;
+    case 4: short_conv_kernel<4><<<grid, block, 0, s>>> (a); break;
+    default: short_conv_kernel<0><<<grid, block, 0, s>>> (a); break;
+    }
   short_conv_keep_kernel<<<dim3 ((unsigned)((keep + 255) / 256)), dim3 (256), 0, s>>> (a);
   return vkl_launch_status ();
 }
@@ -998,6 +1394,12 @@ vkl_recurrence_scratch_bytes (const vkl_recurrence_args *a, int S)
 }
 
 extern "C" int
+vkl_recurrence_chunked (const vkl_recurrence_args *a, int S)
+{
+  return a && S >= kChunkMin && recur_supported (a->H, a->rep, a->dim, a->vdim) && a->dim <= 128;
+}
+
+extern "C" int
 vkl_recurrence (const vkl_recurrence_args *r, int S, uint32_t pos0, int form, void *scratch, size_t scratch_bytes,
                 void *stream)
 {
@@ -1006,20 +1408,25 @@ vkl_recurrence (const vkl_recurrence_args *r, int S, uint32_t pos0, int form, vo
   VKL_CHECK_ARG (r->q && r->k && r->v && r->state && r->out && r->qs >= nqk && r->ks >= nqk && r->vs >= nv && r->os >= nv);
   VKL_CHECK_ARG ((r->type == VKL_TYPE_F32 || r->type == VKL_TYPE_BF16) && (r->qs % 8) == 0 && (r->ks % 8) == 0
                  && ((uintptr_t)r->q % 16) == 0 && ((uintptr_t)r->k % 16) == 0);
-  const bool delta = r->z != nullptr;
+  const bool delta = r->b != nullptr;
   if (delta)
-    VKL_CHECK_ARG (r->b && r->dt_bias && r->rate && r->zs >= (size_t)r->H * r->dim && (r->zs % 4) == 0
-                   && ((uintptr_t)r->z % 16) == 0 && ((uintptr_t)r->dt_bias % 16) == 0 && r->bs >= (size_t)r->H);
+    {
+      VKL_CHECK_ARG (r->dt_bias && r->rate && (r->z || r->a1) && ((uintptr_t)r->dt_bias % 16) == 0 && r->bs >= (size_t)r->H);
+      VKL_CHECK_ARG (!r->z || (r->zs >= (size_t)r->H * r->dim && (r->zs % 4) == 0 && ((uintptr_t)r->z % 16) == 0));
+      VKL_CHECK_ARG (!r->a1 || (r->w_a2 && r->r_a > 0 && (r->r_a % 64) == 0 && r->as >= (size_t)r->r_a && (r->as % 8) == 0
+                                && ((uintptr_t)r->a1 % 16) == 0 && ((uintptr_t)r->w_a2 % 16) == 0));
+    }
   else
     VKL_CHECK_ARG (r->log_decay);
   VKL_CHECK_ARG (form >= VKL_RECUR_AUTO && form <= VKL_RECUR_CHUNKS && (form != VKL_RECUR_CHUNKS || r->dim <= 128));
   hipStream_t s = (hipStream_t)stream;
   RecurArgs a = { *r, S, pos0 == 0 };
   const size_t one = (size_t)r->H * chunk_floats (r->dim, r->vdim) * sizeof (float);
-  if (form == VKL_RECUR_TOKENS || r->dim > 128
-      || (form == VKL_RECUR_AUTO && (S < kChunkMin || !scratch || scratch_bytes < one)))
+  if (form == VKL_RECUR_TOKENS || (form == VKL_RECUR_AUTO && !vkl_recurrence_chunked (r, S)))
+    VKL_CHECK_ARG (!delta || r->z);
+  if (form == VKL_RECUR_TOKENS || (form == VKL_RECUR_AUTO && !vkl_recurrence_chunked (r, S)))
     return delta ? launch_tokens<true> (a, s) : launch_tokens<false> (a, s);
-  VKL_CHECK_ARG (scratch && scratch_bytes >= one && ((uintptr_t)scratch % 16) == 0);
+  VKL_CHECK_ARG (scratch && scratch_bytes >= one && ((uintptr_t)scratch % 16) == 0 && (r->vs % 8) == 0);
   const int piece = (int)std::min<size_t> (scratch_bytes / one, (size_t)1 << 20) * kChunk;
   const size_t es = r->type == VKL_TYPE_F32 ? 4 : 2;
   for (int at = 0; at < S; at += piece)
@@ -1032,11 +1439,42 @@ vkl_recurrence (const vkl_recurrence_args *r, int S, uint32_t pos0, int form, vo
       p.r.v = (const uint8_t *)r->v + (size_t)at * r->vs * es;
       p.r.out = r->out + (size_t)at * r->os;
       if (delta)
-        p.r.z = r->z + (size_t)at * r->zs, p.r.b = r->b + (size_t)at * r->bs;
+        p.r.b = r->b + (size_t)at * r->bs;
+      if (r->z)
+        p.r.z = r->z + (size_t)at * r->zs;
+      if (r->a1)
+        p.r.a1 = (const uint8_t *)r->a1 + (size_t)at * r->as * es;
       if (int e = delta ? launch_chunks<true> (p, (float *)scratch, s) : launch_chunks<false> (p, (float *)scratch, s))
         return e;
     }
   return 0;
+}
+
+extern "C" int
+vkl_low_rank_gated_norm (const float *x, size_t xs, int H, int vdim, int n, const float *w, float eps, const void *g1,
+                         size_t gs, const void *g2, int r, int type, int S, void *out, size_t os, void *stream)
+{
+  VKL_CHECK_ARG (x && w && g1 && g2 && out && H > 0 && vdim > 0 && (vdim % 32) == 0 && vdim <= 256 && n > 0 && n <= vdim);
+  VKL_CHECK_ARG (S > 0 && r > 0 && (r % 64) == 0 && gs >= (size_t)r && (gs % 8) == 0 && xs >= (size_t)H * vdim
+                 && os >= (size_t)H * vdim);
+  VKL_CHECK_ARG ((type == VKL_TYPE_F32 || type == VKL_TYPE_BF16) && ((uintptr_t)g1 % 16) == 0 && ((uintptr_t)g2 % 16) == 0
+                 && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 16) == 0 && (xs % 4) == 0
+                 && (os % 4) == 0);
+  const LowRankNormArgs a = { x, xs, H, vdim, n, w, eps, g1, gs, (const uint16_t *)g2, r, type, S, out, os };
+  const dim3 grid ((unsigned)((S + 63) / 64 * H)), block (256);
+  hipStream_t s = (hipStream_t)stream;
+  switch (vdim / 32)
+    {
+    case 1: low_rank_norm_kernel<2><<<grid, block, 0, s>>> (a); break;
+    case 2: low_rank_norm_kernel<4><<<grid, block, 0, s>>> (a); break;
+    case 3: low_rank_norm_kernel<6><<<grid, block, 0, s>>> (a); break;
+    case 4: low_rank_norm_kernel<8><<<grid, block, 0, s>>> (a); break;
+    case 5: low_rank_norm_kernel<10><<<grid, block, 0, s>>> (a); break;
+    case 6: low_rank_norm_kernel<12><<<grid, block, 0, s>>> (a); break;
+    case 7: low_rank_norm_kernel<14><<<grid, block, 0, s>>> (a); break;
+    default: low_rank_norm_kernel<16><<<grid, block, 0, s>>> (a); break;
+    }
+  return vkl_launch_status ();
 }
 
 extern "C" int

@@ -79,15 +79,23 @@ embed_norm_kernel (const EmbedArgs a)
           for (int e = 0; e < 8; ++e)
             w[j][e] = ldg (a.w + min ((tid + j * 1024) * 8 + e, a.W - 1));
       const float alpha = a.w ? 1.0f / sqrtf (group_sum (ss, red) / (float)a.W + a.eps) : 1.f;
+      const bool vec = (a.W % 8) == 0 && (a.os % 4) == 0 && ((uintptr_t)a.out % 16) == 0;
 #pragma unroll
       for (int j = 0; j < NV; ++j)
+        {
+          const int c = (tid + j * 1024) * 8;
+          vkl_u32x4 o[2];
 #pragma unroll
-        for (int e = 0; e < 8; ++e)
-          {
-            const int c = (tid + j * 1024) * 8 + e;
-            if (c < a.W)
-              stg (out + c, a.w ? v[j][e] * alpha * w[j][e] : v[j][e] * a.scale);
-          }
+          for (int e = 0; e < 8; ++e)
+            {
+              const float f = a.w ? v[j][e] * alpha * w[j][e] : v[j][e] * a.scale;
+              o[e >> 2][e & 3] = __float_as_uint (f);
+              if (!vec && c + e < a.W)
+                stg (out + c + e, f);
+            }
+          if (vec && c < a.W)
+            stg ((vkl_u32x4 *)(out + c), o[0]), stg ((vkl_u32x4 *)(out + c + 4), o[1]);
+        }
       return;
     }
   float alpha = 1.f;
@@ -1150,81 +1158,198 @@ struct PrepArgs
   int S;
 };
 
-// one wave per head of a token: the query heads, the keys, the values
+// A workgroup takes `run` heads of a token, of the query heads, the keys and the
+// values in a row; sines and cosines of the position are shared.  A wave per head.
 __global__ __launch_bounds__ (256) void
-attn_prepare_kernel (const PrepArgs a)
+attn_prepare_kernel (const PrepArgs a, int run, int runs)
 {
+  __shared__ float cs[kPrepMax / 2], sn[kPrepMax / 2];
   const vkl_attn_rows_prep &p = a.p;
   const int per = p.H + 2 * p.G, lane = threadIdx.x & 63;
-  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (item >= (long)a.S * per)
-    return;
-  const int s = (int)(item / per), part = (int)(item - (long)s * per);
+  const int s = blockIdx.x / runs, first = (blockIdx.x - s * runs) * run;
   const size_t pos = (size_t)a.pos.get () + (size_t)s, crow = pos * (size_t)p.G * p.dim;
-  if (part >= p.H + p.G)
+  for (int i = threadIdx.x; i < p.npair; i += 256)
     {
-      const int g = part - p.H - p.G;
-      if (!p.v)
-        return;
-      const size_t at = crow + (size_t)g * p.dim;
-      for (int c = lane; c < p.dim; c += 64)
+      // the angle to within a turn in double, its sine and cosine in float
+      double t = (double)pos * ldg (p.freq + i) * 0.15915494309189533577;
+      t -= rint (t);
+      sincosf ((float)(t * 6.28318530717958647693), sn + i, cs + i);
+    }
+  __syncthreads ();
+  for (int part = first + (threadIdx.x >> 6); part < min (first + run, per); part += 4)
+    {
+      if (part >= p.H + p.G)
         {
-          float v = load_elem (p.v, p.kvtype, (size_t)s * p.kvs + (size_t)g * p.dim + c);
-          if (p.first)
-            v = (1.0f - p.mix) * v + p.mix * load_elem (p.first, p.ctype, at + c);
-          store_elem (p.vo, p.ctype, at + c, v);
+          const int g = part - p.H - p.G;
+          if (!p.v)
+            continue;
+          const size_t at = crow + (size_t)g * p.dim;
+          for (int c = lane; c < p.dim; c += 64)
+            {
+              float v = load_elem (p.v, p.kvtype, (size_t)s * p.kvs + (size_t)g * p.dim + c);
+              if (p.first)
+                v = (1.0f - p.mix) * v + p.mix * load_elem (p.first, p.ctype, at + c);
+              store_elem (p.vo, p.ctype, at + c, v);
+            }
+          continue;
         }
+      const bool key = part >= p.H;
+      const void *src = key ? p.k : p.q;
+      if (!src)
+        continue;
+      const int type = key ? p.kvtype : p.qtype, h = key ? part - p.H : part;
+      const size_t at = (size_t)s * (key ? p.kvs : p.qs) + (size_t)h * p.dim;
+      float x[kPrepMax / 64], ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < kPrepMax / 64; ++j)
+        {
+          const int c = lane + 64 * j;
+          x[j] = 0.f;
+          if (64 * j >= p.dim || c >= p.n)
+            continue;
+          const float v = load_elem (src, type, at + c);
+          x[j] = v;
+          if (c < 2 * p.npair)
+            {
+              const bool low = c < p.npair;
+              const int i = low ? c : c - p.npair;
+              const float w = load_elem (src, type, at + (low ? c + p.npair : i));
+              x[j] = low ? v * cs[i] - w * sn[i] : v * cs[i] + w * sn[i];
+            }
+          ss = __builtin_fmaf (x[j], x[j], ss);
+        }
+      const float alpha = 1.0f / sqrtf (wave_sum (ss) / (float)p.n + p.eps);
+#pragma unroll
+      for (int j = 0; j < kPrepMax / 64; ++j)
+        {
+          const int c = lane + 64 * j;
+          if (64 * j >= p.dim || c >= p.dim)
+            continue;
+          if (key)
+            store_elem (p.ko, p.ctype, crow + (size_t)h * p.dim + c, x[j] * alpha);
+          else
+            store_elem (p.qo, p.qotype, (size_t)s * p.qos + (size_t)h * p.dim + c, x[j] * alpha);
+        }
+    }
+}
+
+// The same in vectors: LPH lanes per head, eight neighbouring values each; heads of up
+// to 8 LPH values, pairs and strides multiples of eight.
+__device__ __forceinline__ void
+store8 (void *p, int type, size_t i, const float (&f)[8])
+{
+  if (type == VKL_TYPE_F32)
+    {
+      vkl_u32x4 w[2];
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        w[e >> 2][e & 3] = __float_as_uint (f[e]);
+      stg ((vkl_u32x4 *)((float *)p + i), w[0]), stg ((vkl_u32x4 *)((float *)p + i + 4), w[1]);
       return;
     }
-  const bool key = part >= p.H;
-  const void *src = key ? p.k : p.q;
-  if (!src)
+  vkl_u32x4 w;
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    w[e] = f2bf (f[2 * e]) | ((uint32_t)f2bf (f[2 * e + 1]) << 16);
+  stg ((vkl_u32x4 *)((uint16_t *)p + i), w);
+}
+
+template <int LPH>
+__global__ __launch_bounds__ (256) void
+attn_prepare_vec_kernel (const PrepArgs a, int runs)
+{
+  constexpr int HPW = 256 / LPH; // heads of a workgroup
+  __shared__ __align__ (16) float cs[LPH * 4], sn[LPH * 4];
+  const vkl_attn_rows_prep &p = a.p;
+  const int per = p.H + 2 * p.G, sub = threadIdx.x % LPH, c = 8 * sub;
+  const int s = blockIdx.x / runs, part = (blockIdx.x - s * runs) * HPW + (int)threadIdx.x / LPH;
+  const size_t pos = (size_t)a.pos.get () + (size_t)s, crow = pos * (size_t)p.G * p.dim;
+  const bool value = part >= p.H + p.G, key = !value && part >= p.H;
+  const int h = value ? part - p.H - p.G : key ? part - p.H : part;
+  const void *src = value ? p.v : key ? p.k : p.q;
+  const int type = value || key ? p.kvtype : p.qtype;
+  const bool live = part < per && src && c < p.dim;
+  const size_t at = (size_t)s * (value || key ? p.kvs : p.qs) + (size_t)h * p.dim + c, cat = crow + (size_t)h * p.dim + c;
+  const bool turned = c < 2 * p.npair, low = c < p.npair;
+  float x[8] = {}, y[8] = {};
+  if (live)
+    {
+      load8 (src, type, at, x);
+      if (value && p.first)
+        load8 (p.first, p.ctype, cat, y);
+      else if (!value && turned)
+        load8 (src, type, low ? at + p.npair : at - p.npair, y);
+    }
+  if ((int)threadIdx.x < p.npair)
+    {
+      // the angle to within a turn in double, its sine and cosine in float
+      double t = (double)pos * ldg (p.freq + threadIdx.x) * 0.15915494309189533577;
+      t -= rint (t);
+      sincosf ((float)(t * 6.28318530717958647693), sn + threadIdx.x, cs + threadIdx.x);
+    }
+  __syncthreads ();
+  if (value)
+    {
+      if (!live)
+        return;
+      if (p.first)
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          x[e] = (1.0f - p.mix) * x[e] + p.mix * y[e];
+      store8 (p.vo, p.ctype, cat, x);
+      return;
+    }
+  float ss = 0.f;
+  const int i0 = turned ? (low ? c : c - p.npair) : 0;
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+    {
+      if (turned)
+        x[e] = low ? x[e] * cs[i0 + e] - y[e] * sn[i0 + e] : x[e] * cs[i0 + e] + y[e] * sn[i0 + e];
+      x[e] = c + e < p.n ? x[e] : 0.f;
+      ss = __builtin_fmaf (x[e], x[e], ss);
+    }
+  const float alpha = 1.0f / sqrtf (lanes_sum<LPH> (ss) / (float)p.n + p.eps);
+  if (!live)
     return;
-  const int type = key ? p.kvtype : p.qtype, h = key ? part - p.H : part;
-  const size_t at = (size_t)s * (key ? p.kvs : p.qs) + (size_t)h * p.dim;
-  float x[kPrepMax / 64], ss = 0.f;
 #pragma unroll
-  for (int j = 0; j < kPrepMax / 64; ++j)
-    {
-      const int c = lane + 64 * j;
-      x[j] = 0.f;
-      if (64 * j >= p.dim || c >= p.n)
-        continue;
-      const float v = load_elem (src, type, at + c);
-      x[j] = v;
-      if (c < 2 * p.npair)
-        {
-          const int i = c < p.npair ? c : c - p.npair;
-          const float w = load_elem (src, type, at + (c < p.npair ? c + p.npair : c - p.npair));
-          // the angle to within a turn in double, its sine and cosine in float
-          double t = (double)pos * ldg (p.freq + i) * 0.15915494309189533577;
-          t -= rint (t);
-          float sn, cs;
-          sincosf ((float)(t * 6.28318530717958647693), &sn, &cs);
-          x[j] = c < p.npair ? v * cs - w * sn : v * cs + w * sn;
-        }
-      ss = __builtin_fmaf (x[j], x[j], ss);
-    }
-  const float alpha = 1.0f / sqrtf (wave_sum (ss) / (float)p.n + p.eps);
-#pragma unroll
-  for (int j = 0; j < kPrepMax / 64; ++j)
-    {
-      const int c = lane + 64 * j;
-      if (64 * j >= p.dim || c >= p.dim)
-        continue;
-      if (key)
-        store_elem (p.ko, p.ctype, crow + (size_t)h * p.dim + c, x[j] * alpha);
-      else
-        store_elem (p.qo, p.qotype, (size_t)s * p.qos + (size_t)h * p.dim + c, x[j] * alpha);
-    }
+  for (int e = 0; e < 8; ++e)
+    x[e] *= alpha;
+  if (key)
+    store8 (p.ko, p.ctype, cat, x);
+  else
+    store8 (p.qo, p.qotype, (size_t)s * p.qos + (size_t)h * p.dim + c, x);
+}
+
+template <int LPH>
+void
+launch_prepare_vec (const PrepArgs &a, hipStream_t s)
+{
+  const int runs = (a.p.H + 2 * a.p.G + 256 / LPH - 1) / (256 / LPH);
+  attn_prepare_vec_kernel<LPH><<<dim3 ((unsigned)(a.S * runs)), dim3 (256), 0, s>>> (a, runs);
 }
 
 int
 attn_prepare (const vkl_attn_rows_prep &p, int S, StepPos pos, hipStream_t s)
 {
   PrepArgs a = { p, pos, S };
-  const long items = (long)S * (p.H + 2 * p.G);
-  attn_prepare_kernel<<<dim3 ((unsigned)((items + 3) / 4)), dim3 (256), 0, s>>> (a);
+  uintptr_t mis = 0;
+  for (const void *q : { p.q, (const void *)p.qo, p.k, p.v, (const void *)p.ko, (const void *)p.vo, p.first })
+    mis |= (uintptr_t)q % 16;
+  if (p.dim % 8 == 0 && p.dim <= 256 && p.npair % 8 == 0 && p.qs % 8 == 0 && p.qos % 8 == 0 && p.kvs % 8 == 0 && !mis)
+    {
+      if (p.dim <= 32)
+        launch_prepare_vec<4> (a, s);
+      else if (p.dim <= 64)
+        launch_prepare_vec<8> (a, s);
+      else if (p.dim <= 128)
+        launch_prepare_vec<16> (a, s);
+      else
+        launch_prepare_vec<32> (a, s);
+      return (int)hipGetLastError ();
+    }
+  const int per = p.H + 2 * p.G, run = S < 64 ? 4 : 16, runs = (per + run - 1) / run;
+  attn_prepare_kernel<<<dim3 ((unsigned)(S * runs)), dim3 (256), 0, s>>> (a, run, runs);
   return (int)hipGetLastError ();
 }
 
@@ -2317,7 +2442,7 @@ extern "C" int
 vkl_attn_prepare (const vkl_attn_rows_prep *p, int S, uint32_t pos0, void *stream)
 {
   VKL_CHECK_ARG (p && S > 0 && p->H > 0 && p->G > 0 && p->dim > 0 && p->dim <= kPrepMax && p->n > 0 && p->n <= p->dim);
-  VKL_CHECK_ARG (p->npair >= 0 && 2 * p->npair <= p->n && (p->npair == 0 || p->freq));
+  VKL_CHECK_ARG (p->npair >= 0 && 2 * p->npair <= p->n && (p->npair == 0 || p->freq) && S <= 1 << 20);
   VKL_CHECK_ARG ((!p->q || (p->qo && p->qs >= (size_t)p->H * p->dim && p->qos >= (size_t)p->H * p->dim)) && (!p->k || p->ko)
                  && (!p->v || p->vo) && p->kvs >= (size_t)p->G * p->dim);
   return attn_prepare (*p, S, StepPos{ nullptr, pos0 }, (hipStream_t)stream);

@@ -71,7 +71,7 @@ RecurrentMixer::recur_ (vkl_recurrence_args a, const void *qkv, int S, size_t of
   const size_t es = p_.dtype == FP32 ? 4 : 2, nqk = (size_t)qk_cols_ ();
   const int no = p_.heads * vdim_;
   VKLLAMA_STATUS_OK (grow_ (o_, S, no, dev_, FP32));
-  a.H = p_.heads, a.rep = p_.heads / p_.kv_heads, a.dim = dim_, a.vdim = vdim_;
+  sizes_ (a);
   a.q = qkv, a.k = (const uint8_t *)qkv + nqk * es, a.v = (const uint8_t *)qkv + 2 * nqk * es;
   a.type = type_ (), a.qs = a.ks = a.vs = (size_t)qkv_cols_ ();
   a.state = (float *)states_[(size_t)run].data ();
@@ -83,6 +83,12 @@ RecurrentMixer::recur_ (vkl_recurrence_args a, const void *qkv, int S, size_t of
     }
   return launch_status ("recurrence", vkl_recurrence (&a, S, (uint32_t)offset, VKL_RECUR_AUTO, scratch_.data (),
                                                       scratch_.bytes (), dev_->stream ()));
+}
+
+void
+RecurrentMixer::sizes_ (vkl_recurrence_args &a) const
+{
+  a.H = p_.heads, a.rep = p_.heads / p_.kv_heads, a.dim = dim_, a.vdim = vdim_;
 }
 
 void
@@ -202,26 +208,30 @@ ChannelDelta::mix (int S, size_t offset, int run, void *out, size_t os)
   const int nz = p_.heads * dim_, no = p_.heads * vdim_, n = qkv_cols_ ();
   void *s = dev_->stream ();
   VKLLAMA_STATUS_OK (grow_ (conv_out_, S, n, dev_, p_.dtype));
-  VKLLAMA_STATUS_OK (grow_ (z_, S, nz, dev_, FP32));
-  VKLLAMA_STATUS_OK (grow_ (gate_, S, no, dev_, p_.dtype));
   timer_.start (dev_);
   int err = vkl_short_conv_silu (qkv_.data (), type_ (), (size_t)n, (const float *)conv_.data (), n, p_.taps,
                                  (float *)rings_[(size_t)run].data (), (uint32_t)offset, S, conv_out_.data (),
                                  (size_t)n, s);
-  const vkl_out_seg zs = segment (0, nz, z_, VKL_TYPE_F32, VKL_ACT_NONE);
-  const vkl_out_seg gs = segment (0, no, gate_, type_ (), VKL_ACT_NONE);
-  if (!err)
-    err = vkl_project_bf16w (a1_.data (), type_ (), (size_t)r_a_, w_a2_.data (), S, nz, r_a_, &zs, 1, s);
-  if (!err)
-    err = vkl_project_bf16w (g1_.data (), type_ (), (size_t)r_g_, w_g2_.data (), S, no, r_g_, &gs, 1, s);
-  VKLLAMA_STATUS_OK (launch_status ("delta rule inputs", err));
   vkl_recurrence_args a = {};
   a.qscale = qscale_, a.unit_eps = kUnitEps;
-  a.z = (const float *)z_.data (), a.zs = (size_t)nz, a.b = (const float *)b_.data (), a.bs = b_.width ();
+  a.b = (const float *)b_.data (), a.bs = b_.width ();
   a.dt_bias = (const float *)dt_bias_.data (), a.rate = (const float *)rate_.data ();
+  sizes_ (a);
+  if (vkl_recurrence_chunked (&a, S))
+    a.a1 = a1_.data (), a.as = (size_t)r_a_, a.w_a2 = w_a2_.data (), a.r_a = r_a_;
+  else
+    {
+      VKLLAMA_STATUS_OK (grow_ (z_, S, nz, dev_, FP32));
+      const vkl_out_seg zs = segment (0, nz, z_, VKL_TYPE_F32, VKL_ACT_NONE);
+      if (!err)
+        err = vkl_project_bf16w (a1_.data (), type_ (), (size_t)r_a_, w_a2_.data (), S, nz, r_a_, &zs, 1, s);
+      a.z = (const float *)z_.data (), a.zs = (size_t)nz;
+    }
+  VKLLAMA_STATUS_OK (launch_status ("delta rule inputs", err));
   VKLLAMA_STATUS_OK (recur_ (a, conv_out_.data (), S, offset, run));
-  err = vkl_gated_norm ((const float *)o_.data (), (size_t)no, p_.heads, vdim_, p_.vdim, (const float *)norm_.data (),
-                        p_.eps, gate_.data (), (size_t)no, type_ (), S, out, os, s);
+  err = vkl_low_rank_gated_norm ((const float *)o_.data (), (size_t)no, p_.heads, vdim_, p_.vdim,
+                                 (const float *)norm_.data (), p_.eps, g1_.data (), (size_t)r_g_, w_g2_.data (), r_g_,
+                                 type_ (), S, out, os, s);
   timer_.stop (dev_);
   return launch_status ("delta rule output", err);
 }

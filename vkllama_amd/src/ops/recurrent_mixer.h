@@ -24,6 +24,7 @@ protected:
   absl::StatusOr<Tensor> upload_heads_ (const std::vector<float> &v, int n, int np);
   // runs the recurrence over qkv [S, qkv_cols_] into o_; a: what is particular to the mixer
   absl::Status recur_ (vkl_recurrence_args a, const void *qkv, int S, size_t offset, int run);
+  void sizes_ (vkl_recurrence_args &a) const;
   void describe_ (vkl_stack_layer &l, int run);
   std::vector<Tensor> states_;
   Tensor qkv_, o_, scratch_;
@@ -55,7 +56,7 @@ private:
   float qscale_ = 1.f;
   Tensor conv_, w_a2_, w_g2_, dt_bias_, rate_, norm_;
   std::vector<Tensor> rings_;   // the convolution's last inputs
-  Tensor conv_out_, b_, a1_, g1_, z_, gate_;
+  Tensor conv_out_, b_, a1_, g1_, z_;
 };
 
 // Linear attention whose state decays by a constant factor per head ("lightning"):

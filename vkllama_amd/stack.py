@@ -25,8 +25,8 @@ class AttnRowsPrep(C.Structure):
 class RecurrenceArgs(C.Structure):
     """vkl_recurrence_args"""
     _fields_ = [("H", i32), ("rep", i32), ("dim", i32), ("vdim", i32), ("q", vp), ("k", vp), ("v", vp), ("type", i32),
-                ("qs", sz), ("ks", sz), ("vs", sz), ("qscale", f32), ("log_decay", vp), ("z", vp), ("zs", sz), ("b", vp),
-                ("bs", sz), ("dt_bias", vp), ("rate", vp), ("unit_eps", f32), ("state", vp), ("out", vp), ("os", sz)]
+                ("qs", sz), ("ks", sz), ("vs", sz), ("qscale", f32), ("log_decay", vp), ("z", vp), ("zs", sz), ("a1", vp), ("a_s", sz),
+                ("w_a2", vp), ("r_a", i32), ("b", vp), ("bs", sz), ("dt_bias", vp), ("rate", vp), ("unit_eps", f32), ("state", vp), ("out", vp), ("os", sz)]
 
 
 RECUR_AUTO, RECUR_TOKENS, RECUR_CHUNKS = 0, 1, 2
@@ -48,6 +48,8 @@ SIGNATURES = {
     "vkl_short_conv_silu": (i32, [vp, i32, sz, vp, i32, i32, vp, u32, i32, vp, sz, vp]),
     "vkl_recurrence": (i32, [C.POINTER(RecurrenceArgs), i32, u32, i32, vp, sz, vp]),
     "vkl_recurrence_scratch_bytes": (sz, [C.POINTER(RecurrenceArgs), i32]),
+    "vkl_recurrence_chunked": (i32, [C.POINTER(RecurrenceArgs), i32]),
+    "vkl_low_rank_gated_norm": (i32, [vp, sz, i32, i32, i32, vp, f32, vp, sz, vp, i32, i32, i32, vp, sz, vp]),
     "vkl_gated_norm": (i32, [vp, sz, i32, i32, i32, vp, f32, vp, sz, i32, i32, vp, sz, vp]),
     "vkl_head_matvec": (i32, [vp, i32, i32, i32, vp, i32, sz, sz, vp, i32, sz, sz, vp, sz, i32, vp]),
     "vkl_stack_scratch_bytes": (sz, [vp]),
