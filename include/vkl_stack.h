@@ -119,7 +119,9 @@ typedef struct
   size_t kvs;
   int kvtype;
   void *ko, *vo;         /* rows of the caches, stride G*dim, in ctype: the row of position 0 */
-  const void *first;     /* such rows of another layer's values, in ctype */
+  const void *first;     /* such rows of another layer's values, in ctype, its heads
+                            fdim apart (as many heads; beyond fdim: zeros) */
+  int fdim;
   float mix;
   int ctype;
 } vkl_attn_rows_prep;
@@ -262,6 +264,7 @@ typedef struct
   const double *freq;
   void *vcache;         /* [maxlen, G*dim] */
   const void *vfirst;   /* values cache of another layer, or null */
+  int fdim;             /* head size of its rows */
   float vmix;
 
   /* VKL_MIX_DELTA: w_in rows q | k (kv0) | v (v0), convolved, | b (b0) | a1 (a0) |

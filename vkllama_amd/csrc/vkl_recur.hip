@@ -59,10 +59,14 @@ stf4 (float *p, f4 v)
   stg ((vkl_u32x4 *)p, __builtin_bit_cast (vkl_u32x4, v));
 }
 
+// Rows in one of the two formats: T is float, or uint16_t for bf16.  (The format is a
+// template parameter wherever many loads are in flight: a branch per load would
+// wait for each.)
+template <typename T>
 __device__ __forceinline__ f4
-load4 (const void *p, int type, size_t i)
+load4 (const void *p, size_t i)
 {
-  if (type == VKL_TYPE_F32)
+  if constexpr (sizeof (T) == 4)
     return ldf4 ((const float *)p + i);
   const unsigned long long w = ldg ((const unsigned long long *)((const uint16_t *)p + i));
   const uint32_t lo = (uint32_t)w, hi = (uint32_t)(w >> 32);
@@ -70,15 +74,43 @@ load4 (const void *p, int type, size_t i)
              __uint_as_float (hi & 0xffff0000u) };
 }
 
-__device__ __forceinline__ void
-store4 (void *p, int type, size_t i, f4 v)
+__device__ __forceinline__ float
+value_of (float v)
 {
-  if (type == VKL_TYPE_F32)
+  return v;
+}
+
+__device__ __forceinline__ float
+value_of (uint16_t v)
+{
+  return bf2f (v);
+}
+
+template <typename T>
+__device__ __forceinline__ float
+load1 (const void *p, size_t i)
+{
+  return value_of (ldg ((const T *)p + i));
+}
+
+template <typename T>
+__device__ __forceinline__ void
+store4 (void *p, size_t i, f4 v)
+{
+  if constexpr (sizeof (T) == 4)
     stf4 ((float *)p + i, v);
   else
     stg ((unsigned long long *)((uint16_t *)p + i),
          (unsigned long long)f2bf (v[0]) | ((unsigned long long)f2bf (v[1]) << 16) | ((unsigned long long)f2bf (v[2]) << 32)
              | ((unsigned long long)f2bf (v[3]) << 48));
+}
+
+// calls f with a value of the format's type
+template <typename F>
+int
+with_format (int type, F f)
+{
+  return type == VKL_TYPE_F32 ? f (float ()) : f (uint16_t ());
 }
 
 __device__ __forceinline__ float
@@ -130,6 +162,7 @@ struct ConvArgs
 };
 
 // the input of eight channels at token s of the pass (negative: of the tokens before it)
+template <typename T>
 __device__ __forceinline__ void
 conv_input (const ConvArgs &a, int s, int c, f4 (&x)[2])
 {
@@ -137,7 +170,7 @@ conv_input (const ConvArgs &a, int s, int c, f4 (&x)[2])
   if (s >= 0)
     {
       const size_t at = (size_t)s * a.xs + c;
-      x[0] = load4 (a.x, a.type, at), x[1] = load4 (a.x, a.type, at + 4);
+      x[0] = load4<T> (a.x, at), x[1] = load4<T> (a.x, at + 4);
     }
   else if ((uint32_t)-s <= a.pos0)
     {
@@ -146,6 +179,7 @@ conv_input (const ConvArgs &a, int s, int c, f4 (&x)[2])
     }
 }
 
+template <typename T>
 __device__ __forceinline__ void
 conv_output (const ConvArgs &a, int s, int c, const f4 (&y)[2])
 {
@@ -156,24 +190,14 @@ conv_output (const ConvArgs &a, int s, int c, const f4 (&y)[2])
 #pragma unroll
     for (int e = 0; e < 4; ++e)
       z[h][e] = silu (y[h][e]);
-  if (a.type == VKL_TYPE_F32)
-    {
-      stf4 ((float *)a.out + o, z[0]), stf4 ((float *)a.out + o + 4, z[1]);
-      return;
-    }
-  uint32_t h[8];
-#pragma unroll
-  for (int e = 0; e < 4; ++e)
-    h[e] = f2bf (z[0][e]), h[4 + e] = f2bf (z[1][e]);
-  stg ((vkl_u32x4 *)((uint16_t *)a.out + o), vkl_u32x4{ h[0] | (h[1] << 16), h[2] | (h[3] << 16), h[4] | (h[5] << 16),
-                                                        h[6] | (h[7] << 16) });
+  store4<T> (a.out, o, z[0]), store4<T> (a.out, o + 4, z[1]);
 }
 
 constexpr int kConvRun = 4; // tokens of a thread
 
 // eight channels of a run of tokens per thread.  TAPS: the inputs of the window and
 // the weights stay in registers; 0: any number of taps
-template <int TAPS>
+template <int TAPS, typename T>
 __global__ __launch_bounds__ (256) void
 short_conv_kernel (const ConvArgs a)
 {
@@ -190,7 +214,15 @@ short_conv_kernel (const ConvArgs a)
         w[j][0] = ldf4 (a.w + (size_t)j * a.n + c), w[j][1] = ldf4 (a.w + (size_t)j * a.n + c + 4);
 #pragma unroll
       for (int j = 0; j < kConvRun + TAPS - 1; ++j)
-        conv_input (a, min (s0 + j - (TAPS - 1), a.S - 1), c, x[j]);
+        {
+          const size_t at = (size_t)max (min (s0 + j - (TAPS - 1), a.S - 1), 0) * a.xs + c;
+          x[j][0] = load4<T> (a.x, at), x[j][1] = load4<T> (a.x, at + 4);
+        }
+      if (s0 < TAPS - 1) // (the first run reaches back before the pass)
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j)
+          if (s0 + j < TAPS - 1)
+            conv_input<T> (a, s0 + j - (TAPS - 1), c, x[j]);
 #pragma unroll
       for (int t = 0; t < kConvRun; ++t)
         {
@@ -203,7 +235,7 @@ short_conv_kernel (const ConvArgs a)
               for (int e = 0; e < 4; ++e)
                 y[h][e] = __builtin_fmaf (w[j][h][e], x[t + j][h][e], y[h][e]);
           if (s0 + t < a.S)
-            conv_output (a, s0 + t, c, y);
+            conv_output<T> (a, s0 + t, c, y);
         }
       return;
     }
@@ -213,7 +245,7 @@ short_conv_kernel (const ConvArgs a)
       for (int j = 0; j < a.taps; ++j)
         {
           f4 x[2];
-          conv_input (a, s - (a.taps - 1 - j), c, x);
+          conv_input<T> (a, s - (a.taps - 1 - j), c, x);
           const f4 w[2] = { ldf4 (a.w + (size_t)j * a.n + c), ldf4 (a.w + (size_t)j * a.n + c + 4) };
 #pragma unroll
           for (int h = 0; h < 2; ++h)
@@ -221,7 +253,7 @@ short_conv_kernel (const ConvArgs a)
             for (int e = 0; e < 4; ++e)
               y[h][e] = __builtin_fmaf (w[h][e], x[h][e], y[h][e]);
         }
-      conv_output (a, s, c, y);
+      conv_output<T> (a, s, c, y);
     }
 }
 
@@ -247,7 +279,7 @@ struct RecurArgs
   bool fresh; // the state is zero
 };
 
-template <int DJ, bool DELTA>
+template <int DJ, bool DELTA, typename T>
 __global__ __launch_bounds__ (64) void
 recur_tokens_kernel (const RecurArgs a)
 {
@@ -273,12 +305,13 @@ recur_tokens_kernel (const RecurArgs a)
 #pragma unroll
       for (int j = 0; j < DJ; ++j)
         {
-          q[j] = load4 (r.q, r.type, (size_t)s * r.qs + qo + 16 * j);
-          k[j] = load4 (r.k, r.type, (size_t)s * r.ks + qo + 16 * j);
+          q[j] = load4<T> (r.q, (size_t)s * r.qs + qo + 16 * j);
+          k[j] = load4<T> (r.k, (size_t)s * r.ks + qo + 16 * j);
           if (DELTA)
             g[j] = ldf4 (r.z + (size_t)s * r.zs + (size_t)h * r.dim + 16 * j + row);
         }
-      float v = load_elem (r.v, r.type, (size_t)s * r.vs + vo), o = 0.f;
+      const float v = load1<T> (r.v, (size_t)s * r.vs + vo);
+      float o = 0.f;
       if (DELTA)
         {
           float qq = 0.f, kk = 0.f, mk = 0.f;
@@ -382,8 +415,9 @@ typedef __bf16 bf8 __attribute__ ((ext_vector_type (8)));
 // x W^T for the 16 columns of W rows w0 .. +15 and kChunk rows of x from row s0 on (n of
 // them exist), K a multiple of 64: acc[m][e] is row 16 m + 4 (lane / 16) + e, column
 // lane % 16
+template <typename T>
 __device__ __forceinline__ void
-low_rank_tile (const void *x, int type, size_t xs, int s0, int n, const uint16_t *w, int K, int lane,
+low_rank_tile (const void *x, size_t xs, int s0, int n, const uint16_t *w, int K, int lane,
                f4 (&acc)[kBlocks])
 {
   const int lo = lane & 15, q = lane >> 4;
@@ -395,7 +429,7 @@ low_rank_tile (const void *x, int type, size_t xs, int s0, int n, const uint16_t
       row[m] = (size_t)(s0 + min (16 * m + lo, n - 1)) * xs;
     }
   const uint16_t *wr = w + (size_t)lo * K;
-  if (type == VKL_TYPE_BF16)
+  if constexpr (sizeof (T) == 2)
     {
       for (int k0 = 0; k0 < K; k0 += 64)
 #pragma unroll
@@ -411,7 +445,7 @@ low_rank_tile (const void *x, int type, size_t xs, int s0, int n, const uint16_t
     }
   for (int k = 4 * q; k < K; k += 16)
     {
-      const f4 b = load4 (wr, VKL_TYPE_BF16, (size_t)k);
+      const f4 b = load4<uint16_t> (wr, (size_t)k);
 #pragma unroll
       for (int m = 0; m < kBlocks; ++m)
         {
@@ -423,7 +457,7 @@ low_rank_tile (const void *x, int type, size_t xs, int s0, int n, const uint16_t
     }
 }
 
-template <bool DELTA>
+template <bool DELTA, typename T>
 __global__ __launch_bounds__ (kPrepThreads) void
 chunk_prep_kernel (const RecurArgs a, float *ws)
 {
@@ -436,7 +470,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
   float *A = ls + kChunk * LD;    // [64][kLdA]
   float *es = A + kChunk * kLdA;  // [4][D]: a block's sum
   float *beta = es + kBlocks * D; // [64]
-  float *T = beta + kChunk;       // [4][16][kLdT]: (1 + A)^-1 of the blocks on the diagonal
+  float *Ti = beta + kChunk;      // [4][16][kLdT]: (1 + A)^-1 of the blocks on the diagonal
   __shared__ uint32_t steep;
   const int h = blockIdx.x % r.H, c = blockIdx.x / r.H, s0 = c * kChunk;
   const int n = min (kChunk, a.S - s0); // tokens; the rest of the chunk changes nothing
@@ -462,8 +496,8 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
 #pragma unroll
         for (int e = 0; e < 2; ++e)
           {
-            x[p][0][e] = load4 (r.q, r.type, s * r.qs + qo + dc + 4 * e);
-            x[p][1][e] = load4 (r.k, r.type, s * r.ks + qo + dc + 4 * e);
+            x[p][0][e] = load4<T> (r.q, s * r.qs + qo + dc + 4 * e);
+            x[p][1][e] = load4<T> (r.k, s * r.ks + qo + dc + 4 * e);
             if (DELTA && !r.a1)
               z[p][e] = ldf4 (r.z + s * r.zs + (size_t)h * D + dc + 4 * e);
           }
@@ -474,7 +508,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
       if (r.a1 && 16 * wave < D)
         {
           f4 acc[kBlocks];
-          low_rank_tile (r.a1, r.type, r.as, s0, n, (const uint16_t *)r.w_a2 + ((size_t)h * D + 16 * wave) * r.r_a, r.r_a,
+          low_rank_tile<T> (r.a1, r.as, s0, n, (const uint16_t *)r.w_a2 + ((size_t)h * D + 16 * wave) * r.r_a, r.r_a,
                          lane, acc);
           const float bias = ldg (r.dt_bias + (size_t)h * D + 16 * wave + lo);
 #pragma unroll
@@ -624,7 +658,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
               for (int j = 0; j < i; ++j)
                 y = __builtin_fmaf (-Ab[i * kLdA + j], x[j], y);
               x[i] = y;
-              T[(16 * wave + i) * kLdT + lo] = y;
+              Ti[(16 * wave + i) * kLdT + lo] = y;
             }
         }
     }
@@ -676,21 +710,32 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
           const bool val = g < VB;
           const int col = 16 * (val ? g : g - VB) + lo;
           f4 x[kBlocks];
-          float before = 0.f;
-#pragma unroll
-          for (int b = 0; b < kBlocks; ++b)
+          if (val)
             {
 #pragma unroll
-              for (int e = 0; e < 4; ++e)
-                {
-                  const int i = 16 * b + hi + e;
-                  const float y = val ? load_elem (r.v, r.type, (size_t)(s0 + min (i, n - 1)) * r.vs + (size_t)h * r.vdim + col)
-                                      : ks[i * LD + col] * power2 (ls[i * LD + col] + before);
-                  x[b][e] = y * beta[i];
-                }
-              if (!val)
-                before += es[b * D + col];
+              for (int b = 0; b < kBlocks; ++b)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                  x[b][e] = load1<T> (r.v, (size_t)(s0 + min (16 * b + hi + e, n - 1)) * r.vs + (size_t)h * r.vdim + col);
             }
+          else
+            {
+              float before = 0.f;
+#pragma unroll
+              for (int b = 0; b < kBlocks; ++b)
+                {
+#pragma unroll
+                  for (int e = 0; e < 4; ++e)
+                    {
+                      const int i = 16 * b + hi + e;
+                      x[b][e] = ks[i * LD + col] * power2 (ls[i * LD + col] + before);
+                    }
+                  before += es[b * D + col];
+                }
+            }
+#pragma unroll
+          for (int b = 0; b < kBlocks; ++b)
+            x[b] *= *(const f4 *)(beta + 16 * b + hi);
 #pragma unroll
           for (int b = 0; b < kBlocks; ++b)
             {
@@ -703,7 +748,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
                   for (int e = 0; e < 4; ++e)
                     acc = mfma4 (-m[e], x[k][e], acc);
                 }
-              const f4 m = *(const f4 *)(T + (16 * b + lo) * kLdT + hi);
+              const f4 m = *(const f4 *)(Ti + (16 * b + lo) * kLdT + hi);
               f4 y = { 0.f, 0.f, 0.f, 0.f };
 #pragma unroll
               for (int e = 0; e < 4; ++e)
@@ -728,7 +773,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
 // ---------------------------------------------------------------------------
 // wave w: tokens 16 w .. +15 of a chunk, and blocks w, w + 4 of the state's rows
 // (one workgroup per compute unit: the next chunk's operands travel in registers)
-template <int DB, bool DELTA>
+template <int DB, bool DELTA, typename T>
 __global__ __launch_bounds__ (256) __attribute__ ((amdgpu_waves_per_eu (1, 1))) void
 chunk_scan_kernel (const RecurArgs a, const float *ws)
 {
@@ -736,7 +781,7 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
   __shared__ f4 ms[DB][64], us[kBlocks][64];
   const vkl_recurrence_args &r = a.r;
   const int h = blockIdx.x % r.H, vb = blockIdx.x / r.H;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane (threadIdx.x >> 6);
   const int lo = lane & 15, hi = 4 * (lane >> 4), col = vb * 16 + lo;
   float *st = r.state + (size_t)h * D * r.vdim + col;
 #pragma unroll
@@ -756,6 +801,7 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
   struct Operands
   {
     f4 w[DELTA ? DB : 1], q[DB], p[kBlocks], k[KB][kBlocks], u, dec[KB];
+    T v[4]; // u, as the values lie (decaying sums)
   };
   auto fetch = [&] (int c, Operands &o) {
     const float *base = ws + ((size_t)c * r.H + h) * per;
@@ -789,65 +835,83 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
         {
           // (tokens past the end have keys of zero)
           const int s = min (c * kChunk + 16 * wave + hi + e, a.S - 1);
-          o.u[e] = load_elem (r.v, r.type, (size_t)s * r.vs + (size_t)h * r.vdim + col);
+          o.v[e] = ldg ((const T *)r.v + (size_t)s * r.vs + (size_t)h * r.vdim + col);
         }
   };
   auto chunk = [&] (int c, const Operands &o) {
-    f4 acc = { 0.f, 0.f, 0.f, 0.f }, sub = acc, acc2 = acc, sub2 = acc;
+    f4 m[DB], u[kBlocks];
 #pragma unroll
     for (int b = 0; b < DB; ++b)
+      m[b] = ms[b][lane];
+    __builtin_amdgcn_sched_barrier (0);
+    f4 acc = { 0.f, 0.f, 0.f, 0.f }, sub = acc, acc2 = acc, sub2 = acc;
+    if constexpr (!DELTA)
       {
-        const f4 m = ms[b][lane];
 #pragma unroll
-        for (int e = 0; e < 4; e += 2)
-          {
-            acc = mfma4 (o.q[b][e], m[e], acc);
-            if constexpr (DELTA)
-              sub = mfma4 (o.w[b][e], m[e], sub);
-            acc2 = mfma4 (o.q[b][e + 1], m[e + 1], acc2);
-            if constexpr (DELTA)
-              sub2 = mfma4 (o.w[b][e + 1], m[e + 1], sub2);
-          }
+        for (int e = 0; e < 4; ++e)
+          u[0][e] = value_of (o.v[e]);
+        us[wave][lane] = u[0];
       }
-    us[wave][lane] = o.u - (sub + sub2);
-    __syncthreads ();
+    else
+      {
 #pragma unroll
-    for (int b = 0; b < kBlocks; ++b)
-      if (b <= wave)
-        {
-          const f4 u = us[b][lane];
+        for (int b = 0; b < DB; ++b)
 #pragma unroll
           for (int e = 0; e < 4; e += 2)
             {
-              acc = mfma4 (o.p[b][e], u[e], acc);
-              acc2 = mfma4 (o.p[b][e + 1], u[e + 1], acc2);
+              sub = mfma4 (o.w[b][e], m[b][e], sub);
+              sub2 = mfma4 (o.w[b][e + 1], m[b][e + 1], sub2);
             }
-        }
-    acc += acc2;
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      {
-        const int s = c * kChunk + 16 * wave + hi + e;
-        if (s < a.S)
-          stg (r.out + (size_t)s * r.os + (size_t)h * r.vdim + col, acc[e]);
+        us[wave][lane] = o.u - (sub + sub2);
       }
+    // (what needs u of the other waves comes after this product)
+#pragma unroll
+    for (int b = 0; b < DB; ++b)
+#pragma unroll
+      for (int e = 0; e < 4; e += 2)
+        {
+          acc = mfma4 (o.q[b][e], m[b][e], acc);
+          acc2 = mfma4 (o.q[b][e + 1], m[b][e + 1], acc2);
+        }
+    __syncthreads ();
+#pragma unroll
+    for (int b = 0; b < kBlocks; ++b)
+      u[b] = us[b][lane];
 #pragma unroll
     for (int i = 0; i < KB; ++i)
-      {
-        const int b = wave + 4 * i;
-        if (b >= DB)
-          continue;
-        f4 m = o.dec[i] * ms[b][lane];
+      m[i] = o.dec[i] * ms[min (wave + 4 * i, DB - 1)][lane];
+    __builtin_amdgcn_sched_barrier (0);
 #pragma unroll
-        for (int j = 0; j < kBlocks; ++j)
+    for (int j = 0; j < kBlocks; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int i = 0; i < KB; ++i)
+          m[i] = mfma4 (o.k[i][j][e], u[j][e], m[i]);
+#pragma unroll
+    for (int i = 0; i < KB; ++i)
+      if (wave + 4 * i < DB)
+        ms[wave + 4 * i][lane] = m[i];
+#pragma unroll
+    for (int b = 0; b < kBlocks; ++b)
+      if (b <= wave)
+#pragma unroll
+        for (int e = 0; e < 4; e += 2)
           {
-            const f4 u = us[j][lane];
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-              m = mfma4 (o.k[i][j][e], u[e], m);
+            acc = mfma4 (o.p[b][e], u[b][e], acc);
+            acc2 = mfma4 (o.p[b][e + 1], u[b][e + 1], acc2);
           }
-        ms[b][lane] = m;
-      }
+    acc += acc2;
+    float *out = r.out + (size_t)(c * kChunk + 16 * wave + hi) * r.os + (size_t)h * r.vdim + col;
+    if (c * kChunk + kChunk <= a.S)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        stg (out + (size_t)e * r.os, acc[e]);
+    else
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c * kChunk + 16 * wave + hi + e < a.S)
+          stg (out + (size_t)e * r.os, acc[e]);
     __syncthreads ();
   };
   Operands x, y;
@@ -877,32 +941,32 @@ chunk_scan_kernel (const RecurArgs a, const float *ws)
     }
 }
 
-template <bool DELTA>
+template <bool DELTA, typename T>
 int
 launch_tokens (const RecurArgs &a, hipStream_t s)
 {
   const dim3 grid ((unsigned)(a.r.H * (a.r.vdim / 16))), block (64);
   switch (a.r.dim / 32)
     {
-    case 1: recur_tokens_kernel<2, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 2: recur_tokens_kernel<4, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 3: recur_tokens_kernel<6, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 4: recur_tokens_kernel<8, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 5: recur_tokens_kernel<10, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 6: recur_tokens_kernel<12, DELTA><<<grid, block, 0, s>>> (a); break;
-    case 7: recur_tokens_kernel<14, DELTA><<<grid, block, 0, s>>> (a); break;
-    default: recur_tokens_kernel<16, DELTA><<<grid, block, 0, s>>> (a); break;
+    case 1: recur_tokens_kernel<2, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 2: recur_tokens_kernel<4, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 3: recur_tokens_kernel<6, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 4: recur_tokens_kernel<8, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 5: recur_tokens_kernel<10, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 6: recur_tokens_kernel<12, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    case 7: recur_tokens_kernel<14, DELTA, T><<<grid, block, 0, s>>> (a); break;
+    default: recur_tokens_kernel<16, DELTA, T><<<grid, block, 0, s>>> (a); break;
     }
   return (int)hipGetLastError ();
 }
 
-template <bool DELTA>
+template <bool DELTA, typename T>
 int
 launch_chunks (const RecurArgs &a, float *ws, hipStream_t s)
 {
   static LdsLimit limit;
   const size_t lds = prep_lds_bytes (a.r.dim);
-  const auto prep = chunk_prep_kernel<DELTA>;
+  const auto prep = chunk_prep_kernel<DELTA, T>;
   if (int e = limit.raise ((const void *)prep, lds))
     return e;
   const int chunks = (a.S + kChunk - 1) / kChunk;
@@ -912,10 +976,10 @@ launch_chunks (const RecurArgs &a, float *ws, hipStream_t s)
   const dim3 grid ((unsigned)(a.r.H * (a.r.vdim / 16))), block (256);
   switch (a.r.dim / 32)
     {
-    case 1: chunk_scan_kernel<2, DELTA><<<grid, block, 0, s>>> (a, ws); break;
-    case 2: chunk_scan_kernel<4, DELTA><<<grid, block, 0, s>>> (a, ws); break;
-    case 3: chunk_scan_kernel<6, DELTA><<<grid, block, 0, s>>> (a, ws); break;
-    default: chunk_scan_kernel<8, DELTA><<<grid, block, 0, s>>> (a, ws); break;
+    case 1: chunk_scan_kernel<2, DELTA, T><<<grid, block, 0, s>>> (a, ws); break;
+    case 2: chunk_scan_kernel<4, DELTA, T><<<grid, block, 0, s>>> (a, ws); break;
+    case 3: chunk_scan_kernel<6, DELTA, T><<<grid, block, 0, s>>> (a, ws); break;
+    default: chunk_scan_kernel<8, DELTA, T><<<grid, block, 0, s>>> (a, ws); break;
     }
   return (int)hipGetLastError ();
 }
@@ -939,12 +1003,12 @@ struct GatedNormArgs
 };
 
 // WIDE: a workgroup per row that is one group; else a wave per group
-template <bool WIDE>
+template <bool WIDE, typename T>
 __global__ __launch_bounds__ (256) void
 gated_norm_kernel (const GatedNormArgs a)
 {
   __shared__ float red[8];
-  constexpr int T = WIDE ? 256 : 64;
+  constexpr int N = WIDE ? 256 : 64;
   const int t = WIDE ? threadIdx.x : (threadIdx.x & 63);
   const size_t it = WIDE ? blockIdx.x : (size_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (!WIDE && it >= (size_t)a.S * a.groups)
@@ -952,7 +1016,7 @@ gated_norm_kernel (const GatedNormArgs a)
   const size_t s = it / a.groups, g0 = (it - s * a.groups) * (size_t)a.gw;
   const float *x = a.x + s * a.xs + g0;
   float ss = 0.f;
-  for (int c = t * 4; c < a.gw; c += T * 4)
+  for (int c = t * 4; c < a.gw; c += N * 4)
     {
       const f4 v = ldf4 (x + c);
 #pragma unroll
@@ -961,14 +1025,14 @@ gated_norm_kernel (const GatedNormArgs a)
     }
   ss = WIDE ? group_sum (ss, red) : wave_sum (ss);
   const float alpha = 1.0f / sqrtf (ss / (float)a.n + a.eps);
-  for (int c = t * 4; c < a.gw; c += T * 4)
+  for (int c = t * 4; c < a.gw; c += N * 4)
     {
-      const f4 v = ldf4 (x + c), w = ldf4 (a.w + c), g = load4 (a.gate, a.type, s * a.gs + g0 + c);
+      const f4 v = ldf4 (x + c), w = ldf4 (a.w + c), g = load4<T> (a.gate, s * a.gs + g0 + c);
       f4 o;
 #pragma unroll
       for (int e = 0; e < 4; ++e)
         o[e] = v[e] * alpha * w[e] * sigmoid (g[e]);
-      store4 (a.out, a.type, s * a.os + g0 + c, o);
+      store4<T> (a.out, s * a.os + g0 + c, o);
     }
 }
 
@@ -989,7 +1053,7 @@ struct LowRankNormArgs
   size_t os;
 };
 
-template <int VB>
+template <int VB, typename T>
 __global__ __launch_bounds__ (256) void
 low_rank_norm_kernel (const LowRankNormArgs a)
 {
@@ -1008,14 +1072,24 @@ low_rank_norm_kernel (const LowRankNormArgs a)
       o[b] = ldf4 (a.x + s * a.xs + (size_t)h * a.vdim + 16 * b + 4 * q);
     }
   const uint16_t *w = a.g2 + ((size_t)h * a.vdim + lo) * a.r;
-  if (a.type == VKL_TYPE_BF16)
-    for (int k = 8 * q; k < a.r; k += 32)
+  if constexpr (sizeof (T) == 2)
+    for (int k0 = 0; k0 < a.r; k0 += 64)
       {
-        const bf8 x = __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)a.g1 + s * a.gs + k));
+        bf8 x[2], y[2][VB];
 #pragma unroll
-        for (int b = 0; b < VB; ++b)
-          g[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (__builtin_bit_cast (bf8, ldg4 (w + (size_t)16 * b * a.r + k)), x,
-                                                          g[b], 0, 0, 0);
+        for (int u = 0; u < 2; ++u)
+          {
+            const int k = k0 + 32 * u + 8 * q;
+            x[u] = __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)a.g1 + s * a.gs + k));
+#pragma unroll
+            for (int b = 0; b < VB; ++b)
+              y[u][b] = __builtin_bit_cast (bf8, ldg4 (w + (size_t)16 * b * a.r + k));
+          }
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int b = 0; b < VB; ++b)
+            g[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (y[u][b], x[u], g[b], 0, 0, 0);
       }
   else
     for (int k = 4 * q; k < a.r; k += 16)
@@ -1024,7 +1098,7 @@ low_rank_norm_kernel (const LowRankNormArgs a)
 #pragma unroll
         for (int b = 0; b < VB; ++b)
           {
-            const f4 y = load4 (w, VKL_TYPE_BF16, (size_t)16 * b * a.r + k);
+            const f4 y = load4<uint16_t> (w, (size_t)16 * b * a.r + k);
 #pragma unroll
             for (int e = 0; e < 4; ++e)
               g[b] = mfma4 (y[e], x[e], g[b]);
@@ -1046,7 +1120,7 @@ low_rank_norm_kernel (const LowRankNormArgs a)
 #pragma unroll
       for (int e = 0; e < 4; ++e)
         y[e] = o[b][e] * alpha * wn[e] * sigmoid (g[b][e]);
-      store4 (a.out, a.type, s * a.os + (size_t)h * a.vdim + 16 * b + 4 * q, y);
+      store4<T> (a.out, s * a.os + (size_t)h * a.vdim + 16 * b + 4 * q, y);
     }
 }
 
@@ -1374,13 +1448,17 @@ vkl_short_conv_silu (const void *x, int type, size_t xs, const float *w, int n, 
   hipStream_t s = (hipStream_t)stream;
   const size_t items = (size_t)((S + kConvRun - 1) / kConvRun) * (n / 8), keep = (size_t)std::min (S, taps) * n;
   const dim3 grid ((unsigned)((items + 255) / 256)), block (256);
-  switch (taps)
-    {
-    case 2: short_conv_kernel<2><<<grid, block, 0, s>>> (a); break;
-    case 3: short_conv_kernel<3><<<grid, block, 0, s>>> (a); break;
-    case 4: short_conv_kernel<4><<<grid, block, 0, s>>> (a); break;
-    default: short_conv_kernel<0><<<grid, block, 0, s>>> (a); break;
-    }
+  with_format (type, [&] (auto t) {
+    typedef decltype (t) T;
+    switch (taps)
+      {
+      case 2: short_conv_kernel<2, T><<<grid, block, 0, s>>> (a); break;
+      case 3: short_conv_kernel<3, T><<<grid, block, 0, s>>> (a); break;
+      case 4: short_conv_kernel<4, T><<<grid, block, 0, s>>> (a); break;
+      default: short_conv_kernel<0, T><<<grid, block, 0, s>>> (a); break;
+      }
+    return 0;
+  });
   short_conv_keep_kernel<<<dim3 ((unsigned)((keep + 255) / 256)), dim3 (256), 0, s>>> (a);
   return vkl_launch_status ();
 }
@@ -1425,7 +1503,9 @@ vkl_recurrence (const vkl_recurrence_args *r, int S, uint32_t pos0, int form, vo
   if (form == VKL_RECUR_TOKENS || (form == VKL_RECUR_AUTO && !vkl_recurrence_chunked (r, S)))
     VKL_CHECK_ARG (!delta || r->z);
   if (form == VKL_RECUR_TOKENS || (form == VKL_RECUR_AUTO && !vkl_recurrence_chunked (r, S)))
-    return delta ? launch_tokens<true> (a, s) : launch_tokens<false> (a, s);
+    return with_format (r->type, [&] (auto t) {
+      return delta ? launch_tokens<true, decltype (t)> (a, s) : launch_tokens<false, decltype (t)> (a, s);
+    });
   VKL_CHECK_ARG (scratch && scratch_bytes >= one && ((uintptr_t)scratch % 16) == 0 && (r->vs % 8) == 0);
   const int piece = (int)std::min<size_t> (scratch_bytes / one, (size_t)1 << 20) * kChunk;
   const size_t es = r->type == VKL_TYPE_F32 ? 4 : 2;
@@ -1444,7 +1524,10 @@ vkl_recurrence (const vkl_recurrence_args *r, int S, uint32_t pos0, int form, vo
         p.r.z = r->z + (size_t)at * r->zs;
       if (r->a1)
         p.r.a1 = (const uint8_t *)r->a1 + (size_t)at * r->as * es;
-      if (int e = delta ? launch_chunks<true> (p, (float *)scratch, s) : launch_chunks<false> (p, (float *)scratch, s))
+      if (int e = with_format (r->type, [&] (auto t) {
+            return delta ? launch_chunks<true, decltype (t)> (p, (float *)scratch, s)
+                         : launch_chunks<false, decltype (t)> (p, (float *)scratch, s);
+          }))
         return e;
     }
   return 0;
@@ -1463,17 +1546,21 @@ vkl_low_rank_gated_norm (const float *x, size_t xs, int H, int vdim, int n, cons
   const LowRankNormArgs a = { x, xs, H, vdim, n, w, eps, g1, gs, (const uint16_t *)g2, r, type, S, out, os };
   const dim3 grid ((unsigned)((S + 63) / 64 * H)), block (256);
   hipStream_t s = (hipStream_t)stream;
-  switch (vdim / 32)
-    {
-    case 1: low_rank_norm_kernel<2><<<grid, block, 0, s>>> (a); break;
-    case 2: low_rank_norm_kernel<4><<<grid, block, 0, s>>> (a); break;
-    case 3: low_rank_norm_kernel<6><<<grid, block, 0, s>>> (a); break;
-    case 4: low_rank_norm_kernel<8><<<grid, block, 0, s>>> (a); break;
-    case 5: low_rank_norm_kernel<10><<<grid, block, 0, s>>> (a); break;
-    case 6: low_rank_norm_kernel<12><<<grid, block, 0, s>>> (a); break;
-    case 7: low_rank_norm_kernel<14><<<grid, block, 0, s>>> (a); break;
-    default: low_rank_norm_kernel<16><<<grid, block, 0, s>>> (a); break;
-    }
+  with_format (type, [&] (auto t) {
+    typedef decltype (t) T;
+    switch (vdim / 32)
+      {
+      case 1: low_rank_norm_kernel<2, T><<<grid, block, 0, s>>> (a); break;
+      case 2: low_rank_norm_kernel<4, T><<<grid, block, 0, s>>> (a); break;
+      case 3: low_rank_norm_kernel<6, T><<<grid, block, 0, s>>> (a); break;
+      case 4: low_rank_norm_kernel<8, T><<<grid, block, 0, s>>> (a); break;
+      case 5: low_rank_norm_kernel<10, T><<<grid, block, 0, s>>> (a); break;
+      case 6: low_rank_norm_kernel<12, T><<<grid, block, 0, s>>> (a); break;
+      case 7: low_rank_norm_kernel<14, T><<<grid, block, 0, s>>> (a); break;
+      default: low_rank_norm_kernel<16, T><<<grid, block, 0, s>>> (a); break;
+      }
+    return 0;
+  });
   return vkl_launch_status ();
 }
 
@@ -1488,9 +1575,13 @@ vkl_gated_norm (const float *x, size_t xs, int groups, int gw, int n, const floa
                  && ((uintptr_t)gate % 16) == 0 && ((uintptr_t)out % 16) == 0);
   const GatedNormArgs a = { x, xs, groups, gw, n, w, eps, gate, gs, type, out, os, S };
   hipStream_t s = (hipStream_t)stream;
-  if (groups == 1)
-    gated_norm_kernel<true><<<dim3 ((unsigned)S), dim3 (256), 0, s>>> (a);
-  else
-    gated_norm_kernel<false><<<dim3 ((unsigned)(((size_t)S * groups + 3) / 4)), dim3 (256), 0, s>>> (a);
+  with_format (type, [&] (auto t) {
+    typedef decltype (t) T;
+    if (groups == 1)
+      gated_norm_kernel<true, T><<<dim3 ((unsigned)S), dim3 (256), 0, s>>> (a);
+    else
+      gated_norm_kernel<false, T><<<dim3 ((unsigned)(((size_t)S * groups + 3) / 4)), dim3 (256), 0, s>>> (a);
+    return 0;
+  });
   return vkl_launch_status ();
 }

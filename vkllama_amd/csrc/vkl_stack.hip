@@ -1188,7 +1188,8 @@ attn_prepare_kernel (const PrepArgs a, int run, int runs)
             {
               float v = load_elem (p.v, p.kvtype, (size_t)s * p.kvs + (size_t)g * p.dim + c);
               if (p.first)
-                v = (1.0f - p.mix) * v + p.mix * load_elem (p.first, p.ctype, at + c);
+                v = (1.0f - p.mix) * v
+                    + (c < p.fdim ? p.mix * load_elem (p.first, p.ctype, (pos * p.G + g) * p.fdim + c) : 0.f);
               store_elem (p.vo, p.ctype, at + c, v);
             }
           continue;
@@ -1275,8 +1276,8 @@ attn_prepare_vec_kernel (const PrepArgs a, int runs)
   if (live)
     {
       load8 (src, type, at, x);
-      if (value && p.first)
-        load8 (p.first, p.ctype, cat, y);
+      if (value && p.first && c < p.fdim)
+        load8 (p.first, p.ctype, (pos * p.G + h) * p.fdim + c, y);
       else if (!value && turned)
         load8 (src, type, low ? at + p.npair : at - p.npair, y);
     }
@@ -1336,7 +1337,7 @@ attn_prepare (const vkl_attn_rows_prep &p, int S, StepPos pos, hipStream_t s)
   uintptr_t mis = 0;
   for (const void *q : { p.q, (const void *)p.qo, p.k, p.v, (const void *)p.ko, (const void *)p.vo, p.first })
     mis |= (uintptr_t)q % 16;
-  if (p.dim % 8 == 0 && p.dim <= 256 && p.npair % 8 == 0 && p.qs % 8 == 0 && p.qos % 8 == 0 && p.kvs % 8 == 0 && !mis)
+  if (p.dim % 8 == 0 && p.fdim % 8 == 0 && p.dim <= 256 && p.npair % 8 == 0 && p.qs % 8 == 0 && p.qos % 8 == 0 && p.kvs % 8 == 0 && !mis)
     {
       if (p.dim <= 32)
         launch_prepare_vec<4> (a, s);
@@ -2007,6 +2008,7 @@ check_stack (const vkl_stack_model *m)
         {
           VKL_CHECK_ARG (l.vcache && l.dim <= kPrepMax && l.vdim == l.dim && l.n > 0 && l.n <= l.dim && l.chunk >= 0);
           VKL_CHECK_ARG (l.npair >= 0 && 2 * l.npair <= l.n && (l.npair == 0 || l.freq));
+          VKL_CHECK_ARG (!l.vfirst || l.fdim > 0);
           VKL_CHECK_ARG (l.v0 == l.kv0 + l.G * l.dim && l.v0 + l.G * l.dim <= l.n_in);
         }
       else if (recur)
@@ -2085,7 +2087,7 @@ launch_two_norm_layer (const StepArgs &p, const vkl_stack_layer &l, GvArgs a, hi
       r.H = l.H, r.G = l.G, r.dim = l.dim, r.n = l.n, r.npair = l.npair, r.freq = l.freq, r.eps = m.eps;
       r.q = r.qo = p.s.q, r.qtype = r.qotype = r.kvtype = VKL_TYPE_F32;
       r.k = p.s.c, r.v = p.s.c + l.G * l.dim, r.ko = l.cache, r.vo = l.vcache;
-      r.first = l.vfirst, r.mix = l.vmix, r.ctype = m.ctype;
+      r.first = l.vfirst, r.fdim = l.fdim, r.mix = l.vmix, r.ctype = m.ctype;
       if (int e = attn_prepare (r, 1, p.pos, st))
         return e;
       if (int e = kv_attention (p.s.q, VKL_TYPE_F32, 0, l.cache, l.vcache, m.ctype, (size_t)l.G * l.dim, l.H, l.G,
@@ -2444,7 +2446,7 @@ vkl_attn_prepare (const vkl_attn_rows_prep *p, int S, uint32_t pos0, void *strea
   VKL_CHECK_ARG (p && S > 0 && p->H > 0 && p->G > 0 && p->dim > 0 && p->dim <= kPrepMax && p->n > 0 && p->n <= p->dim);
   VKL_CHECK_ARG (p->npair >= 0 && 2 * p->npair <= p->n && (p->npair == 0 || p->freq) && S <= 1 << 20);
   VKL_CHECK_ARG ((!p->q || (p->qo && p->qs >= (size_t)p->H * p->dim && p->qos >= (size_t)p->H * p->dim)) && (!p->k || p->ko)
-                 && (!p->v || p->vo) && p->kvs >= (size_t)p->G * p->dim);
+                 && (!p->v || p->vo) && (!p->first || p->fdim > 0) && p->kvs >= (size_t)p->G * p->dim);
   return attn_prepare (*p, S, StepPos{ nullptr, pos0 }, (hipStream_t)stream);
 }
 

@@ -24,7 +24,7 @@ ChunkedAttention::init () noexcept
   if (2 * p_.freq.size () > (size_t)p_.dim)
     return absl::InvalidArgumentError (absl::StrFormat (
         "attention: rotation over %zu values of a head of %d", 2 * p_.freq.size (), p_.dim));
-  if (first_ && (first_->p_.kv_heads != p_.kv_heads || first_->p_.vdim != p_.vdim || first_->dim_ != dim_))
+  if (first_ && (first_->p_.kv_heads != p_.kv_heads || first_->p_.vdim != p_.vdim))
     return absl::InvalidArgumentError ("attention: layers that mix values need key/value heads of the same sizes");
   kcaches_.resize ((size_t)p_.runs), vcaches_.resize ((size_t)p_.runs);
   for (int i = 0; i < p_.runs; ++i)
@@ -96,7 +96,7 @@ ChunkedAttention::mix (int S, size_t offset, int run, void *out, size_t os)
   r.q = r.qo = q_.data (), r.qs = r.qos = nq, r.qtype = r.qotype = r.kvtype = r.ctype = type_ ();
   r.k = row_ (kc, offset), r.ko = kc.data (), r.kvs = nk, r.vo = vc.data ();
   if (first_)
-    r.v = row_ (vc, offset), r.first = first_->vcaches_[0].data (), r.mix = mix_;
+    r.v = row_ (vc, offset), r.first = first_->vcaches_[0].data (), r.fdim = first_->dim_, r.mix = mix_;
   timer_.start (dev_);
   int err = vkl_attn_prepare (&r, S, (uint32_t)offset, dev_->stream ());
   if (!err && (p_.dtype == FP32 || dim_ > 256 || S <= kFewRows))
@@ -123,6 +123,6 @@ ChunkedAttention::describe (vkl_stack_layer &l, int run)
   l.kv0 = p_.heads * dim_, l.v0 = (p_.heads + p_.kv_heads) * dim_;
   l.npair = (int)p_.freq.size (), l.freq = (const double *)freq_.data ();
   l.cache = kcaches_[(size_t)run].data (), l.vcache = vcaches_[(size_t)run].data ();
-  l.vfirst = first_ ? first_->vcaches_[0].data () : nullptr, l.vmix = mix_;
+  l.vfirst = first_ ? first_->vcaches_[0].data () : nullptr, l.fdim = first_ ? first_->dim_ : 0, l.vmix = mix_;
 }
 }

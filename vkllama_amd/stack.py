@@ -18,7 +18,7 @@ class AttnRowsPrep(C.Structure):
     """vkl_attn_rows_prep"""
     _fields_ = [("H", i32), ("G", i32), ("dim", i32), ("n", i32), ("npair", i32), ("freq", vp), ("eps", f32),
                 ("q", vp), ("qs", sz), ("qo", vp), ("qos", sz), ("qtype", i32), ("qotype", i32),
-                ("k", vp), ("v", vp), ("kvs", sz), ("kvtype", i32), ("ko", vp), ("vo", vp), ("first", vp), ("mix", f32),
+                ("k", vp), ("v", vp), ("kvs", sz), ("kvtype", i32), ("ko", vp), ("vo", vp), ("first", vp), ("fdim", i32), ("mix", f32),
                 ("ctype", i32)]
 
 
