@@ -105,6 +105,22 @@ store4 (void *p, size_t i, f4 v)
              | ((unsigned long long)f2bf (v[3]) << 48));
 }
 
+template <typename T>
+__device__ __forceinline__ void
+store8 (void *p, size_t i, const float (&v)[8])
+{
+  if constexpr (sizeof (T) == 4)
+    {
+      stf4 ((float *)p + i, f4{ v[0], v[1], v[2], v[3] }), stf4 ((float *)p + i + 4, f4{ v[4], v[5], v[6], v[7] });
+      return;
+    }
+  vkl_u32x4 w;
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    w[e] = f2bf (v[2 * e]) | ((uint32_t)f2bf (v[2 * e + 1]) << 16);
+  stg ((vkl_u32x4 *)((uint16_t *)p + i), w);
+}
+
 // calls f with a value of the format's type
 template <typename F>
 int
@@ -133,6 +149,31 @@ __device__ __forceinline__ float
 power2 (float x)
 {
   return __builtin_amdgcn_exp2f (x);
+}
+
+// 1 / (1 + e^-x) on the hardware's power and reciprocal, good to a few units of the last
+// place: where every value of a large tensor takes one
+__device__ __forceinline__ float
+quick_sigmoid (float x)
+{
+  return __builtin_amdgcn_rcpf (1.0f + power2 (-kLog2e * x));
+}
+
+// log2_decay_of: kLog2e * log_decay_of, with hardware powers and logarithms.  ln (1 + x)
+// comes from its series where 1 + x would round x away.
+__device__ __forceinline__ float
+log2_decay_of (float rate, float z)
+{
+  const float x = power2 (-kLog2e * fabsf (z));
+  float s = __builtin_fmaf (x, -1.0f / 8, 1.0f / 7);
+  s = __builtin_fmaf (x, s, -1.0f / 6);
+  s = __builtin_fmaf (x, s, 1.0f / 5);
+  s = __builtin_fmaf (x, s, -1.0f / 4);
+  s = __builtin_fmaf (x, s, 1.0f / 3);
+  s = __builtin_fmaf (x, s, -1.0f / 2);
+  s = __builtin_fmaf (x, s, 1.0f) * x * kLog2e;
+  const float l = x < 0.1f ? s : __builtin_amdgcn_logf (1.0f + x);
+  return fmaxf (-rate * (kLog2e * fmaxf (z, 0.f) + l), -1.4427e4f);
 }
 
 // sum over the lanes that hold the same column (four groups of 16)
@@ -183,14 +224,11 @@ template <typename T>
 __device__ __forceinline__ void
 conv_output (const ConvArgs &a, int s, int c, const f4 (&y)[2])
 {
-  const size_t o = (size_t)s * a.os + c;
-  f4 z[2];
+  float z[8];
 #pragma unroll
-  for (int h = 0; h < 2; ++h)
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      z[h][e] = silu (y[h][e]);
-  store4<T> (a.out, o, z[0]), store4<T> (a.out, o + 4, z[1]);
+  for (int e = 0; e < 8; ++e)
+    z[e] = y[e / 4][e % 4] * quick_sigmoid (y[e / 4][e % 4]);
+  store8<T> (a.out, (size_t)s * a.os + c, z);
 }
 
 constexpr int kConvRun = 4; // tokens of a thread
@@ -517,7 +555,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
             for (int e = 0; e < 4; ++e)
               {
                 const int i = 16 * m + hi + e;
-                ls[i * LD + 16 * wave + lo] = i < n ? kLog2e * log_decay_of (rate, acc[m][e] + bias) : 0.f;
+                ls[i * LD + 16 * wave + lo] = i < n ? log2_decay_of (rate, acc[m][e] + bias) : 0.f;
               }
         }
 #pragma unroll
@@ -554,7 +592,7 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
             for (int g = 0; g < 4; ++g)
               {
                 if (DELTA)
-                  l[g] = kLog2e * log_decay_of (rate, z[p][e][g] + ldg (r.dt_bias + (size_t)h * D + d + 4 * e + g));
+                  l[g] = log2_decay_of (rate, z[p][e][g] + ldg (r.dt_bias + (size_t)h * D + d + 4 * e + g));
                 else
                   l[g] = ld;
                 l[g] = in ? l[g] : 0.f;
@@ -583,6 +621,17 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
     }
   __syncthreads ();
 
+  // (the values of this wave's first columns: on their way while P is formed)
+  T vr[kBlocks][4];
+  if constexpr (DELTA)
+    {
+      const int col = 16 * min (wave, r.vdim / 16 - 1) + lo;
+#pragma unroll
+      for (int b = 0; b < kBlocks; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          vr[b][e] = ldg ((const T *)r.v + (size_t)(s0 + min (16 * b + hi + e, n - 1)) * r.vs + (size_t)h * r.vdim + col);
+    }
   // P, and for the delta rule A, in blocks (bi, bj <= bi), transposed in the registers:
   // a lane holds row lo, columns hi .. hi + 3.  Waves 0 .. 3 take the diagonal and
   // invert it, the others the blocks below it.
@@ -650,13 +699,19 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
           __builtin_amdgcn_wave_barrier ();
           const float *Ab = A + 16 * wave * kLdA + 16 * wave;
           float x[16];
+          f4 rows[16][4];
+#pragma unroll
+          for (int i = 1; i < 16; ++i)
+#pragma unroll
+            for (int j = 0; j < i; j += 4)
+              rows[i][j / 4] = *(const f4 *)(Ab + i * kLdA + j);
 #pragma unroll
           for (int i = 0; i < 16; ++i)
             {
               float y = i == lo ? 1.f : 0.f;
 #pragma unroll
               for (int j = 0; j < i; ++j)
-                y = __builtin_fmaf (-Ab[i * kLdA + j], x[j], y);
+                y = __builtin_fmaf (-rows[i][j / 4][j % 4], x[j], y);
               x[i] = y;
               Ti[(16 * wave + i) * kLdT + lo] = y;
             }
@@ -710,7 +765,15 @@ chunk_prep_kernel (const RecurArgs a, float *ws)
           const bool val = g < VB;
           const int col = 16 * (val ? g : g - VB) + lo;
           f4 x[kBlocks];
-          if (val)
+          if (val && g == wave)
+            {
+#pragma unroll
+              for (int b = 0; b < kBlocks; ++b)
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                  x[b][e] = value_of (vr[b][e]);
+            }
+          else if (val)
             {
 #pragma unroll
               for (int b = 0; b < kBlocks; ++b)
@@ -1031,7 +1094,7 @@ gated_norm_kernel (const GatedNormArgs a)
       f4 o;
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        o[e] = v[e] * alpha * w[e] * sigmoid (g[e]);
+        o[e] = v[e] * alpha * w[e] * quick_sigmoid (g[e]);
       store4<T> (a.out, s * a.os + g0 + c, o);
     }
 }
@@ -1061,47 +1124,50 @@ low_rank_norm_kernel (const LowRankNormArgs a)
   const int h = blockIdx.x % a.H, s0 = (blockIdx.x / a.H) * 64 + (threadIdx.x >> 6) * 16;
   if (s0 >= a.S)
     return;
-  // a lane holds token lo and columns 16 b + 4 q + 0..3
+  // Columns are dealt to the result blocks so that a lane holds eight neighbours of token
+  // lo: row m of block b is column 32 (b / 2) + 8 (m / 4) + 4 (b % 2) + m % 4.
   const size_t s = (size_t)min (s0 + lo, a.S - 1);
+  const float *x = a.x + s * a.xs + (size_t)h * a.vdim + 8 * q;
   f4 o[VB], g[VB];
   float ss = 0.f;
 #pragma unroll
   for (int b = 0; b < VB; ++b)
     {
       g[b] = f4{ 0.f, 0.f, 0.f, 0.f };
-      o[b] = ldf4 (a.x + s * a.xs + (size_t)h * a.vdim + 16 * b + 4 * q);
+      o[b] = ldf4 (x + 32 * (b / 2) + 4 * (b % 2));
     }
-  const uint16_t *w = a.g2 + ((size_t)h * a.vdim + lo) * a.r;
+  const uint16_t *w = a.g2 + ((size_t)h * a.vdim + 8 * (lo / 4) + lo % 4) * a.r;
+  auto row = [&] (int b) { return (size_t)(32 * (b / 2) + 4 * (b % 2)) * a.r; };
   if constexpr (sizeof (T) == 2)
     for (int k0 = 0; k0 < a.r; k0 += 64)
       {
-        bf8 x[2], y[2][VB];
+        bf8 v[2], y[2][VB];
 #pragma unroll
         for (int u = 0; u < 2; ++u)
           {
             const int k = k0 + 32 * u + 8 * q;
-            x[u] = __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)a.g1 + s * a.gs + k));
+            v[u] = __builtin_bit_cast (bf8, ldg4 ((const uint16_t *)a.g1 + s * a.gs + k));
 #pragma unroll
             for (int b = 0; b < VB; ++b)
-              y[u][b] = __builtin_bit_cast (bf8, ldg4 (w + (size_t)16 * b * a.r + k));
+              y[u][b] = __builtin_bit_cast (bf8, ldg4 (w + row (b) + k));
           }
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
           for (int b = 0; b < VB; ++b)
-            g[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (y[u][b], x[u], g[b], 0, 0, 0);
+            g[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16 (y[u][b], v[u], g[b], 0, 0, 0);
       }
   else
     for (int k = 4 * q; k < a.r; k += 16)
       {
-        const f4 x = ldf4 ((const float *)a.g1 + s * a.gs + k);
+        const f4 v = ldf4 ((const float *)a.g1 + s * a.gs + k);
 #pragma unroll
         for (int b = 0; b < VB; ++b)
           {
-            const f4 y = load4<uint16_t> (w, (size_t)16 * b * a.r + k);
+            const f4 y = load4<uint16_t> (w, row (b) + k);
 #pragma unroll
             for (int e = 0; e < 4; ++e)
-              g[b] = mfma4 (y[e], x[e], g[b]);
+              g[b] = mfma4 (y[e], v[e], g[b]);
           }
       }
 #pragma unroll
@@ -1113,14 +1179,16 @@ low_rank_norm_kernel (const LowRankNormArgs a)
   if (s0 + lo >= a.S)
     return;
 #pragma unroll
-  for (int b = 0; b < VB; ++b)
+  for (int b = 0; b < VB; b += 2)
     {
-      const f4 wn = ldf4 (a.w + 16 * b + 4 * q);
-      f4 y;
+      float y[8];
 #pragma unroll
-      for (int e = 0; e < 4; ++e)
-        y[e] = o[b][e] * alpha * wn[e] * sigmoid (g[b][e]);
-      store4<T> (a.out, s * a.os + (size_t)h * a.vdim + 16 * b + 4 * q, y);
+      for (int i = 0; i < 8; ++i)
+        {
+          const f4 &v = o[b + i / 4], &z = g[b + i / 4];
+          y[i] = v[i % 4] * alpha * ldg (a.w + 16 * b + 8 * q + i) * quick_sigmoid (z[i % 4]);
+        }
+      store8<T> (a.out, s * a.os + (size_t)h * a.vdim + 16 * b + 8 * q, y);
     }
 }
 
@@ -1542,7 +1610,7 @@ vkl_low_rank_gated_norm (const float *x, size_t xs, int H, int vdim, int n, cons
                  && os >= (size_t)H * vdim);
   VKL_CHECK_ARG ((type == VKL_TYPE_F32 || type == VKL_TYPE_BF16) && ((uintptr_t)g1 % 16) == 0 && ((uintptr_t)g2 % 16) == 0
                  && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)out % 16) == 0 && (xs % 4) == 0
-                 && (os % 4) == 0);
+                 && (os % 8) == 0);
   const LowRankNormArgs a = { x, xs, H, vdim, n, w, eps, g1, gs, (const uint16_t *)g2, r, type, S, out, os };
   const dim3 grid ((unsigned)((S + 63) / 64 * H)), block (256);
   hipStream_t s = (hipStream_t)stream;
