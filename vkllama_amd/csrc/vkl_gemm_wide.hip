@@ -792,26 +792,48 @@ gemm_wide_launch (const GemmArgs &a, hipStream_t s)
 // ---------------------------------------------------------------------------
 namespace
 {
-// adds the parts of a split k range in order and applies the segments' epilogue
-__global__ __launch_bounds__ (256) void
+// adds the parts of a split k range in order and applies the segments' epilogue; the
+// values of four parts are requested at a time
+constexpr int kSegReduce = 64; // threads: few values, spread over many compute units
+__global__ __launch_bounds__ (kSegReduce) void
 wide_reduce_seg_kernel (const GemmSegArgs a, const float *ws, int parts)
 {
   const int n8 = (a.N + 7) / 8;
-  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const size_t i = (size_t)blockIdx.x * kSegReduce + threadIdx.x;
   if (i >= (size_t)a.M * n8)
     return;
   const int m = (int)(i / n8), n = (int)(i % n8) * 8;
+  const size_t at = (size_t)m * a.N, part = (size_t)a.M * a.N;
   float v[8], g[8];
 #pragma unroll
   for (int e = 0; e < 8; ++e)
     v[e] = 0.f, g[e] = 0.f;
-  for (int p = 0; p < parts; ++p)
-    {
-      const float *src = ws + ((size_t)p * a.M + m) * a.N;
+  if ((a.N % 8) == 0)
+    for (int p0 = 0; p0 < parts; p0 += 4)
+      {
+        float4 x[4][2];
 #pragma unroll
-      for (int e = 0; e < 8; ++e)
-        v[e] += ldg (src + min (n + e, a.N - 1));
-    }
+        for (int p = 0; p < 4; ++p)
+          {
+            const float *src = ws + (size_t)min (p0 + p, parts - 1) * part + at + n;
+            x[p][0] = __builtin_bit_cast (float4, ldg4 (src)), x[p][1] = __builtin_bit_cast (float4, ldg4 (src + 4));
+          }
+#pragma unroll
+        for (int p = 0; p < 4; ++p)
+          if (p0 + p < parts)
+            {
+              v[0] += x[p][0].x, v[1] += x[p][0].y, v[2] += x[p][0].z, v[3] += x[p][0].w;
+              v[4] += x[p][1].x, v[5] += x[p][1].y, v[6] += x[p][1].z, v[7] += x[p][1].w;
+            }
+      }
+  else
+    for (int p = 0; p < parts; ++p)
+      {
+        const float *src = ws + (size_t)p * part + at;
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          v[e] += ldg (src + min (n + e, a.N - 1));
+      }
   gemm_finish8<false> (a, v, g, m, n, 0, 0, nullptr);
 }
 
@@ -860,7 +882,7 @@ launch_wide_bf16 (const GemmSegArgs &a, int ksplit, hipStream_t s)
   if (ksplit > 1)
     {
       const size_t total = (size_t)a.M * ((a.N + 7) / 8);
-      wide_reduce_seg_kernel<<<dim3 ((unsigned)((total + 255) / 256)), dim3 (256), 0, s>>> (a, ws, ksplit);
+      wide_reduce_seg_kernel<<<dim3 ((unsigned)((total + kSegReduce - 1) / kSegReduce)), dim3 (kSegReduce), 0, s>>> (a, ws, ksplit);
     }
   return (int)hipGetLastError ();
 }

@@ -76,7 +76,7 @@ RecurrentMixer::recur_ (vkl_recurrence_args a, const void *qkv, int S, size_t of
   a.type = type_ (), a.qs = a.ks = a.vs = (size_t)qkv_cols_ ();
   a.state = (float *)states_[(size_t)run].data ();
   a.out = (float *)o_.data (), a.os = (size_t)no;
-  if (S > kFewRows)
+  if (vkl_recurrence_chunked (&a, S))
     {
       const size_t need = vkl_recurrence_scratch_bytes (&a, std::min (S, kPiece)), row = 4096;
       VKLLAMA_STATUS_OK (grow_ (scratch_, (int)((need + row - 1) / row), (int)row / 4, dev_, FP32));
